@@ -654,7 +654,8 @@ class LLMEngine:
             fields["states"] = self.states.states
         dec_ctx = [s.num_tokens for s in decode]
         if prefill:
-            fields.update(seq_fields(prefill, pre_ctx), cu_seqlens_q=i32(cu), cu_host=cu)
+            fields.update(seq_fields(prefill, pre_ctx), cu_seqlens_q=i32(cu), cu_host=cu,
+                          ctx_host=pre_ctx)
             if decode:
                 fields.update(seq_fields(decode, dec_ctx, "dec_"), num_prefill_tokens=Tp)
         else:

@@ -55,7 +55,9 @@ class ModelSpec:
 
 # ---- layer-listed decoders -------------------------------------------------
 # A HybridSpec spells its layers out one by one: each has a mixer (attention
-# beside a recurrence, or a recurrence alone) and an optional feed-forward.
+# beside a recurrence, a recurrence or latent attention alone) and an optional
+# feed-forward. What all layers share (residual gates, the convolution of the
+# mixer's input, the norms' weight) are fields of the HybridSpec.
 
 @dataclass(frozen=True)
 class BiasedAttentionSpec:
@@ -100,6 +102,18 @@ class RetentionSpec:
 
 
 @dataclass(frozen=True)
+class LatentAttentionSpec:
+    """Attention without positions over one cached latent per token, with a
+    sink in the softmax and a gate per head."""
+    heads: int
+    dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    kv_from: Optional[int] = None  # layer whose latents it reads; None: its own
+
+
+@dataclass(frozen=True)
 class MoESpec:
     experts: int
     top: int
@@ -108,9 +122,34 @@ class MoESpec:
 
 
 @dataclass(frozen=True)
+class DenseSpec:
+    """Ungated two-matrix feed-forward with the xIELU activation."""
+    ff: int
+
+
+MixerSpec = Union[ParallelMixerSpec, RetentionSpec, LatentAttentionSpec]
+
+
+@dataclass(frozen=True)
 class LayerSpec:
-    mixer: Union[ParallelMixerSpec, RetentionSpec]
-    mlp: Optional[MoESpec]
+    mixer: MixerSpec
+    mlp: Union[MoESpec, DenseSpec, None]
+
+
+@dataclass(frozen=True)
+class BigramSpec:
+    """Hashed table of token pairs: row (previous * mul_prev + token * mul_cur)
+    mod buckets; row ``buckets`` where there is no previous token."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass(frozen=True)
+class EmbeddingSpec:
+    """Scaled token rows plus pair rows, normed."""
+    scale: float
+    bigram: BigramSpec
 
 
 @dataclass
@@ -125,8 +164,25 @@ class HybridSpec:
     max_position: int = 131072
     arch: str = "kikalix"
     is_encoder: bool = False
+    #: None: bare token rows
+    embedding: Optional[EmbeddingSpec] = None
+    #: taps of the causal convolution added to every mixer's input (0: none)
+    input_conv: int = 0
+    #: each sublayer's result is scaled by a sigmoid gate of the sublayer's input
+    residual_gates: bool = False
+    #: what norms add to their stored weight
+    norm_offset: float = 1.0
 
     def __post_init__(self):
+        for i, layer in enumerate(self.layers):
+            j = getattr(layer.mixer, "kv_from", None)
+            if j is None:
+                continue
+            src = self.layers[j].mixer if 0 <= j < i else None
+            if not isinstance(src, LatentAttentionSpec) or src.kv_from is not None \
+                    or src.kv_rank != layer.mixer.kv_rank:
+                raise ValueError(f"layer {i}: kv_from {j} is no earlier layer with "
+                                 "latents of its own and the same rank")
         if self.loop is not None:
             start, stop, times = self.loop
             if not (0 <= start < stop <= len(self.layers) and times >= 1):
@@ -152,10 +208,20 @@ class HybridSpec:
         n = 2 * self.vocab_size * w + w
         if self.loop is not None:
             n += self.loop[2] * w
+        if self.embedding is not None:
+            n += (self.embedding.bigram.buckets + 2) * w
         for layer in self.layers:
             m = layer.mixer
+            n += self.input_conv * w
+            if self.residual_gates:
+                n += (1 if layer.mlp is None else 2) * (w + 1) * w
             if isinstance(m, RetentionSpec):
                 n += w * m.heads * (2 * m.dim + 3 * m.vdim) + w
+            elif isinstance(m, LatentAttentionSpec):
+                n += w * m.heads * (m.dim + m.vdim + 1) + w + m.heads
+                n += m.kv_rank * m.heads * (m.dim + m.vdim)
+                if m.kv_from is None:
+                    n += m.kv_rank * (w + 1)
             else:
                 a, r = m.left, m.right
                 qkv = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)
@@ -164,7 +230,9 @@ class HybridSpec:
                 n += ch * (w + r.conv) + w * (r.heads + r.decay_rank + r.gate_rank)
                 n += r.heads * (r.dim * (r.decay_rank + 1) + r.vdim * r.gate_rank + 1)
                 n += r.vdim + w * r.heads * r.vdim
-            if layer.mlp is not None:
+            if isinstance(layer.mlp, DenseSpec):
+                n += w + 2 * w * layer.mlp.ff + 2
+            elif layer.mlp is not None:
                 n += w + layer.mlp.experts * (3 * w * layer.mlp.ff + w + 1)
         return n
 
@@ -222,8 +290,31 @@ def _kikalix_spec(name: str, cfg: dict, shapes: Dict[str, Sequence[int]]) -> Hyb
         loop=(lp["start"], lp["stop"], lp["times"]) if lp else None)
 
 
+def _senotar_spec(name: str, cfg: dict, shapes: Dict[str, Sequence[int]]) -> HybridSpec:
+    layers = []
+    for i, entry in enumerate(cfg["layers"]):
+        if entry["type"] != "latent_attention":
+            raise ValueError(f"layer {i}: unknown mixer type {entry['type']!r}")
+        m, ff = entry["mixer"], entry.get("mlp")
+        if ff is not None and ff.get("kind", "dense") != "dense":
+            raise ValueError(f"layer {i}: unknown feed-forward {ff['kind']!r}")
+        layers.append(LayerSpec(
+            LatentAttentionSpec(
+                heads=m["heads"], dim=m["dim"], vdim=m["vdim"], kv_rank=m["kv_rank"],
+                scale=float(m["scale"]), kv_from=m.get("kv_from")),
+            DenseSpec(ff["ff"]) if ff is not None else None))
+    emb = cfg["embedding"]
+    bigram = emb["bigram"]
+    return HybridSpec(
+        name=name, arch="senotar", hidden_size=cfg["width"], vocab_size=cfg["vocab"],
+        layers=tuple(layers), rms_eps=float(cfg["norm"]["eps"]), norm_offset=0.0,
+        input_conv=cfg["canon"]["taps"], residual_gates=True,
+        embedding=EmbeddingSpec(float(emb["scale"]), BigramSpec(
+            bigram["buckets"], bigram["mul_prev"], bigram["mul_cur"])))
+
+
 #: config.json "architecture" -> reader(name, config, tensor shapes)
-_CONFIG_READERS = {"Kikalix": _kikalix_spec}
+_CONFIG_READERS = {"Kikalix": _kikalix_spec, "Senotar": _senotar_spec}
 
 
 def is_checkpoint_dir(path: str) -> bool:
@@ -371,3 +462,33 @@ register(HybridSpec(  # layer sizes of a 7B-class decoder, 8 experts like mixtra
         d_heads=16, d_kv_heads=16, d_dim=128, d_vdim=128, rank=128, r_heads=16,
         r_dim=256, r_vdim=256, experts=8, top=2, ff=14336),
 ))
+
+# ---- Senotar presets ---------------------------------------------------------
+
+def senotar_spec(name: str, pattern: str, *, width: int, vocab: int, heads: int, dim: int,
+                 vdim: int, kv_rank: int, ff: int, taps: int = 4, buckets: int = 65521,
+                 max_position: int = 131072) -> HybridSpec:
+    """Layers of one size from a pattern: 'o' has latents of its own, 's' reads
+    the last 'o' layer's; upper case: without a feed-forward."""
+    layers, own = [], None
+    for i, c in enumerate(pattern):
+        if c in "oO":
+            own = i
+        mixer = LatentAttentionSpec(heads, dim, vdim, kv_rank, dim ** -0.5,
+                                    None if c in "oO" else own)
+        layers.append(LayerSpec(mixer, None if c.isupper() else DenseSpec(ff)))
+    return HybridSpec(
+        name=name, arch="senotar", hidden_size=width, vocab_size=vocab, layers=tuple(layers),
+        max_position=max_position, input_conv=taps, residual_gates=True, norm_offset=0.0,
+        embedding=EmbeddingSpec(width ** 0.5, BigramSpec(buckets, 31, 17)))
+
+
+register(senotar_spec(  # CPU plumbing size
+    "tiny-senotar", "oOss", width=64, vocab=512, heads=3, dim=16, vdim=24, kv_rank=20,
+    ff=96, taps=3, buckets=97, max_position=2048))
+register(senotar_spec(  # GPU smoke size
+    "smoke-senotar", "ooss", width=512, vocab=1024, heads=8, dim=64, vdim=64, kv_rank=256,
+    ff=1024, buckets=509, max_position=8192))
+register(senotar_spec(  # layer sizes of a 7B-class decoder
+    "senotar-7b", "o" * 16 + "s" * 16, width=4096, vocab=32000, heads=32, dim=128,
+    vdim=128, kv_rank=512, ff=14336))

@@ -1,11 +1,13 @@
-"""Layer-listed decoder (Kikalix): mixers and feed-forwards chosen layer by
-layer, with a span of layers that may run several times.
+"""Layer-listed decoders (Kikalix, Senotar): mixers and feed-forwards chosen
+layer by layer, with a span of layers that may run several times.
 
 Same engine shape as the other decoders: packed varlen tokens, paged KV and
 per-step metadata. Two things differ. The residual stream is one fp32 tensor
 that every norm kernel updates in place (the preceding sub-layer's output, or
 the weighted expert rows, and the pass vector are added by the kernel that
-norms). And every layer RUN, not layer, owns a paged cache or recurrent state.
+norms). And every layer RUN, not layer, owns a paged cache or recurrent state;
+a mixer may instead read an earlier layer's cache. Beside the mixers', state is
+what an input convolution and a pair embedding remember of the last tokens.
 """
 from __future__ import annotations
 
@@ -16,9 +18,16 @@ import torch.nn as nn
 
 from .. import ops
 from ..parallel import dist as pdist
-from .config import HybridSpec, ParallelMixerSpec
+from .config import DenseSpec, HybridSpec, LatentAttentionSpec, ParallelMixerSpec
 from .llama import AttnMetadata
-from .mixers import ParallelMixer, RetentionMixer, RoutedGLU, _param
+from .mixers import (
+    DenseXieluMLP,
+    LatentAttention,
+    ParallelMixer,
+    RetentionMixer,
+    RoutedGLU,
+    _param,
+)
 
 
 class HybridLayer(nn.Module):
@@ -29,6 +38,8 @@ class HybridLayer(nn.Module):
         self.norm1 = _param(w, dtype=torch.float32)
         if isinstance(s.mixer, ParallelMixerSpec):
             self.mixer: nn.Module = ParallelMixer(s.mixer, w, spec.rms_eps, dtype)
+        elif isinstance(s.mixer, LatentAttentionSpec):
+            self.mixer = LatentAttention(s.mixer, w, spec.rms_eps, dtype)
         else:
             m = s.mixer
             key = (m.rot_dims, m.rot_base)
@@ -36,11 +47,29 @@ class HybridLayer(nn.Module):
                 rotations[key] = ops.torch_ref.rope_cos_sin_cache(
                     m.rot_dims, spec.max_position, m.rot_base)
             self.mixer = RetentionMixer(m, w, spec.rms_eps, dtype, rotations[key])
-        if s.mlp is not None:
-            self.norm2 = _param(w, dtype=torch.float32)
-            self.mlp = RoutedGLU(s.mlp, w, dtype)
-        else:
+        # convolution of the mixer's input, residual gate of its output
+        self.conv = _param(w, spec.input_conv, dtype=torch.float32) \
+            if spec.input_conv else None
+        self.gate = _param(w, w, dtype=dtype) if spec.residual_gates else None
+        self.gate_bias = _param(w, dtype=torch.float32) if spec.residual_gates else None
+        if s.mlp is None:
             self.mlp = None
+            return
+        self.norm2 = _param(w, dtype=torch.float32)
+        if isinstance(s.mlp, DenseSpec):
+            self.mlp = DenseXieluMLP(s.mlp, w, dtype, spec.residual_gates)
+        elif spec.residual_gates:
+            raise ValueError("routed experts have no residual gate")
+        else:
+            self.mlp = RoutedGLU(s.mlp, w, dtype)
+
+    def state_layout(self, dtype) -> List[tuple]:
+        """The input convolution's last inputs, if it has any, then the mixer's."""
+        own = []
+        if self.conv is not None:
+            w, taps = self.conv.shape
+            own = [(((taps - 1, w), dtype),)]
+        return own + self.mixer.state_layout(dtype)
 
 
 class HybridForCausalLM(nn.Module):
@@ -62,15 +91,22 @@ class HybridForCausalLM(nn.Module):
             self.lm_head = _param(spec.vocab_size, spec.hidden_size, dtype=dtype)
             self.loop_step = _param(spec.loop[2], spec.hidden_size,
                                     dtype=torch.float32) if spec.loop else None
+            if spec.embedding is not None:
+                self.pairs = _param(spec.embedding.bigram.buckets + 1, spec.hidden_size,
+                                    dtype=dtype)
+                self.embed_norm = _param(spec.hidden_size, dtype=torch.float32)
         # run -> its paged caches and state entries, in kv_layout / state_layout
         # order
         self._runs: List[tuple] = []
-        n_kv = n_state = 0
+        last_kv: Dict[int, slice] = {}
+        n_kv, n_state = 0, len(self._embed_state())
         for i, step in spec.runs():
-            m = self.layers[i].mixer
-            a, b = len(m.kv_layout(dtype, "cpu")), len(m.state_layout(dtype))
-            self._runs.append((i, step, slice(n_kv, n_kv + a),
-                               slice(n_state, n_state + b)))
+            layer = self.layers[i]
+            a = len(layer.mixer.kv_layout(dtype, "cpu"))
+            b = len(layer.state_layout(dtype))
+            source = getattr(spec.layers[i].mixer, "kv_from", None)
+            last_kv[i] = slice(n_kv, n_kv + a) if source is None else last_kv[source]
+            self._runs.append((i, step, last_kv[i], slice(n_state, n_state + b)))
             n_kv, n_state = n_kv + a, n_state + b
 
     def kv_layout(self) -> List[Tuple[int, int, int]]:
@@ -78,35 +114,58 @@ class HybridForCausalLM(nn.Module):
         return [e for i, _ in self.spec.runs()
                 for e in self.layers[i].mixer.kv_layout(self.dtype, dev)]
 
+    def _embed_state(self) -> List[tuple]:
+        # a pair embedding remembers the last token
+        return [(((1,), torch.int32),)] if self.spec.embedding is not None else []
+
     def state_layout(self) -> List[tuple]:
-        """Per recurrent run, the (shape, dtype) of each state tensor's slot."""
-        return [e for i, _ in self.spec.runs()
-                for e in self.layers[i].mixer.state_layout(self.dtype)]
+        """The embedding's state, then per run with a state the (shape, dtype) of
+        each of its tensors' slots."""
+        return self._embed_state() + [
+            e for i, _ in self.spec.runs() for e in self.layers[i].state_layout(self.dtype)]
+
+    def _embed(self, input_ids, meta, segments) -> torch.Tensor:
+        e = self.spec.embedding
+        if e is None:
+            return self.embed(input_ids).float()
+        return ops.embed_pairs(
+            input_ids, self.embed.weight, e.scale, self.pairs, e.bigram.mul_prev,
+            e.bigram.mul_cur, self.embed_norm, self.spec.rms_eps, meta.states[0][0],
+            segments)
 
     @torch.inference_mode()
     def forward(self, input_ids: torch.Tensor, kv_caches, meta: AttnMetadata,
                 trail=None) -> torch.Tensor:
         """Normed hidden states [T, H]; ``trail``, if a list, receives the
         residual stream after every layer run."""
-        eps = self.spec.rms_eps
-        x = self.embed(input_ids).float()
-        segments = meta.segments(x.shape[0])
+        segments = meta.segments(input_ids.shape[0])
+        x = self._embed(input_ids, meta, segments)
+        norm = {"eps": self.spec.rms_eps, "offset": self.spec.norm_offset,
+                "dtype": self.dtype}
         add: Dict[str, object] = {}  # what the next norm adds to the residual
         for i, step, kv, st in self._runs:
             layer = self.layers[i]
+            state = meta.states[st]
             if step is not None:
                 add["step"] = self.loop_step[step]
-            h = ops.residual_rmsnorm(x, layer.norm1, eps, dtype=self.dtype, **add)
-            add = {"delta": layer.mixer(h, meta, segments, kv_caches[kv],
-                                        meta.states[st])}
+            if layer.conv is None:
+                h = u = ops.residual_rmsnorm(x, layer.norm1, **norm, **add)
+            else:
+                h, u = ops.residual_rmsnorm_conv(x, layer.norm1, conv_w=layer.conv,
+                                                 ring=state[0][0], segments=segments,
+                                                 **norm, **add)
+                state = state[1:]
+            add = {"delta": layer.mixer(u, meta, segments, kv_caches[kv], state)}
+            if layer.gate is not None:
+                add["gate"] = (ops.linear(h, layer.gate), layer.gate_bias)
             if layer.mlp is not None:
-                h = ops.residual_rmsnorm(x, layer.norm2, eps, dtype=self.dtype, **add)
-                add = {"moe": layer.mlp(h)}
+                h = ops.residual_rmsnorm(x, layer.norm2, **norm, **add)
+                add = layer.mlp(h)
             if trail is not None:
                 y = x.clone()
-                ops.residual_rmsnorm(y, layer.norm1, eps, dtype=self.dtype, **add)
+                ops.residual_rmsnorm(y, layer.norm1, **norm, **add)
                 trail.append(y)
-        return ops.residual_rmsnorm(x, self.final_norm, eps, dtype=self.dtype, **add)
+        return ops.residual_rmsnorm(x, self.final_norm, **norm, **add)
 
     @torch.inference_mode()
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
@@ -115,32 +174,46 @@ class HybridForCausalLM(nn.Module):
     @torch.inference_mode()
     def load_tensors(self, get) -> None:
         """Fill every weight from ``get(name) -> tensor``."""
-        self.embed.weight.copy_(get("embed"))
-        self.final_norm.copy_(get("final.norm"))
-        self.lm_head.copy_(get("head"))
-        if self.loop_step is not None:
-            self.loop_step.copy_(get("loop.step"))
+        for name, t in self._plain_tensors().items():
+            t.copy_(get(name))
         for i, layer in enumerate(self.layers):
-            layer.norm1.copy_(get(f"l{i}.norm1"))
             layer.mixer.load(lambda n, i=i: get(f"l{i}.mix.{n}"))
-            if layer.mlp is not None:
-                layer.norm2.copy_(get(f"l{i}.norm2"))
-                layer.mlp.load(lambda n, i=i: get(f"l{i}.mlp.{n}"))
+            if layer.mlp is None:
+                continue
+            read = [lambda n, i=i: get(f"l{i}.mlp.{n}")]
+            if layer.gate is not None:
+                read.append(lambda n, i=i: get(f"l{i}.rg2{n}"))
+            layer.mlp.load(*read)
 
-    def named_tensors(self) -> Dict[str, torch.Tensor]:
-        """Inverse of ``load_tensors``."""
+    def _plain_tensors(self) -> Dict[str, torch.Tensor]:
+        """Weights held as they are stored, by name."""
         out = {"embed": self.embed.weight.data, "final.norm": self.final_norm.data,
                "head": self.lm_head.data}
         if self.loop_step is not None:
             out["loop.step"] = self.loop_step.data
+        if self.spec.embedding is not None:
+            out["bigram"], out["embed.norm"] = self.pairs.data, self.embed_norm.data
         for i, layer in enumerate(self.layers):
             out[f"l{i}.norm1"] = layer.norm1.data
-            parts = [("mix", layer.mixer)]
             if layer.mlp is not None:
                 out[f"l{i}.norm2"] = layer.norm2.data
-                parts.append(("mlp", layer.mlp))
-            for tag, m in parts:
-                out.update({f"l{i}.{tag}.{n}": t.data for n, t in m.tensors().items()})
+            if layer.conv is not None:
+                out[f"l{i}.canon1"] = layer.conv.data
+            if layer.gate is not None:
+                out[f"l{i}.rg1"], out[f"l{i}.rg1.b"] = layer.gate.data, layer.gate_bias.data
+        return out
+
+    def named_tensors(self) -> Dict[str, torch.Tensor]:
+        """Inverse of ``load_tensors``."""
+        out = self._plain_tensors()
+        for i, layer in enumerate(self.layers):
+            parts = [(f"l{i}.mix.", layer.mixer.tensors())]
+            if layer.mlp is not None:
+                parts.append((f"l{i}.mlp.", layer.mlp.tensors()))
+                if layer.gate is not None:
+                    parts.append((f"l{i}.rg2", layer.mlp.gate_tensors()))
+            for tag, tensors in parts:
+                out.update({tag + n: t.data for n, t in tensors.items()})
         return out
 
     @torch.inference_mode()
@@ -161,14 +234,26 @@ class HybridForCausalLM(nn.Module):
             return torch.randn(shape, generator=gen).to(dev)
 
         w = self.spec.hidden_size
+
+        def norm_weight():  # norms scale by about one
+            return 1.0 - self.spec.norm_offset + randn((w,)) * 0.1
+
         self.embed.weight.copy_(randn(self.embed.weight.shape))
         self.lm_head.copy_(randn(self.lm_head.shape) * w ** -0.5)
-        self.final_norm.copy_(randn((w,)) * 0.1)
+        self.final_norm.copy_(norm_weight())
         if self.loop_step is not None:
             self.loop_step.copy_(randn(self.loop_step.shape) * 0.1)
+        if self.spec.embedding is not None:
+            self.pairs.copy_(randn(self.pairs.shape))
+            self.embed_norm.copy_(norm_weight())
         for layer in self.layers:
-            layer.norm1.copy_(randn((w,)) * 0.1)
+            layer.norm1.copy_(norm_weight())
             layer.mixer.init_random(randn)
+            if layer.conv is not None:
+                layer.conv.copy_(randn(layer.conv.shape) * 0.3)
+            if layer.gate is not None:
+                layer.gate.copy_(randn((w, w)) * w ** -0.5)
+                layer.gate_bias.copy_(randn((w,)))
             if layer.mlp is not None:
-                layer.norm2.copy_(randn((w,)) * 0.1)
+                layer.norm2.copy_(norm_weight())
                 layer.mlp.init_random(randn)

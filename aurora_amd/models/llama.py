@@ -57,6 +57,7 @@ class AttnMetadata:
     state_slots: Optional[torch.Tensor] = None
     dec_state_slots: Optional[torch.Tensor] = None
     cu_host: Optional[List[int]] = None  # cu_seqlens_q without a device read
+    ctx_host: Optional[List[int]] = None  # context_lens of the prompt portions
 
     def segments(self, T: int) -> List[ops.Segment]:
         """The step's prompt portions and its single-token rows, each with its
@@ -70,7 +71,8 @@ class AttnMetadata:
                 context_lens=self.context_lens,
                 starts=self.context_lens - (cu[1:] - cu[:-1]),
                 state_slots=self.state_slots, cu=cu,
-                cu_host=self.cu_host or cu.tolist()))
+                cu_host=self.cu_host or cu.tolist(),
+                ctx_host=self.ctx_host or self.context_lens.tolist()))
         if T > Tp:
             mixed = self.mode == "mixed"
             out.append(ops.Segment(

@@ -13,7 +13,13 @@ import torch
 import torch.nn as nn
 
 from .. import ops
-from .config import MoESpec, ParallelMixerSpec, RetentionSpec
+from .config import (
+    DenseSpec,
+    LatentAttentionSpec,
+    MoESpec,
+    ParallelMixerSpec,
+    RetentionSpec,
+)
 
 
 def _param(*shape, dtype) -> nn.Parameter:
@@ -236,6 +242,145 @@ class RetentionMixer(nn.Module):
         return ops.linear(out, self.out_proj)
 
 
+class LatentAttention(nn.Module):
+    """Attention without positions over one cached latent per token: keys and
+    values are per-head linear maps of it. The softmax has a sink, every head a
+    sigmoid gate. A layer may read an earlier layer's latents instead of its
+    own. Heads and latents are padded with zeros to the kernels' widths."""
+
+    def __init__(self, spec: LatentAttentionSpec, hidden: int, eps: float, dtype):
+        super().__init__()
+        self.spec = spec
+        self.eps = eps
+        H, R = spec.heads, ops.latent_width(spec.kv_rank)
+        self.D, self.E, self.R = D, E, R = (
+            ops.latent_head_width(spec.dim), ops.latent_head_width(spec.vdim), R)
+        own = [("dkv", spec.kv_rank)] if spec.kv_from is None else []
+        self.cols = FusedColumns([("q", H * D)] + own + [("g", H)])
+        self.in_proj = _param(self.cols.total, hidden, dtype=dtype)
+        if own:
+            self.latent_norm = _param(spec.kv_rank, dtype=torch.float32)
+        self.uk = _param(H, D, R, dtype=dtype)
+        self.uk_t = _param(H, R, D, dtype=dtype)
+        self.uv = _param(H, E, R, dtype=dtype)
+        self.sink = _param(H, dtype=torch.float32)
+        self.out_proj = _param(hidden, H * E, dtype=dtype)
+        self._p: Optional[ops.LatentParams] = None
+
+    def kv_layout(self, dtype, device) -> List[Tuple[int, int, int]]:
+        return [(1, self.R, 0)] if self.spec.kv_from is None else []
+
+    def state_layout(self, dtype) -> List[tuple]:
+        return []
+
+    def load(self, get) -> None:
+        s, H, dev = self.spec, self.spec.heads, self.uk.device
+
+        def heads(t, n):  # [H*n, ...] -> [H, n, ...]
+            return t.to(dev).unflatten(0, (H, n))
+
+        q = torch.zeros(H, self.D, self.in_proj.shape[1], dtype=self.uk.dtype, device=dev)
+        q[:, :s.dim] = heads(get("q"), s.dim)
+        parts = {"q": q.flatten(0, 1), "g": get("g")}
+        if s.kv_from is None:
+            parts["dkv"] = get("dkv")
+            self.latent_norm.copy_(get("dkv.norm"))
+        self.cols.pack(parts, self.in_proj)
+        self.uk.zero_()
+        self.uv.zero_()
+        self.uk[:, :s.dim, :s.kv_rank] = heads(get("uk"), s.dim).to(self.uk.dtype)
+        self.uv[:, :s.vdim, :s.kv_rank] = heads(get("uv"), s.vdim).to(self.uv.dtype)
+        self.uk_t.copy_(self.uk.transpose(1, 2))
+        self.sink.copy_(get("sink"))
+        self.out_proj.zero_()
+        self.out_proj.unflatten(1, (H, self.E))[:, :, :s.vdim] = get("o").to(
+            device=dev, dtype=self.out_proj.dtype).unflatten(1, (H, s.vdim))
+
+    def tensors(self) -> Dict[str, torch.Tensor]:
+        s, H = self.spec, self.spec.heads
+        out = dict(self.cols.unpack(self.in_proj))
+        out["q"] = out["q"].unflatten(0, (H, self.D))[:, :s.dim].flatten(0, 1)
+        if s.kv_from is None:
+            out["dkv.norm"] = self.latent_norm
+        out["uk"] = self.uk[:, :s.dim, :s.kv_rank].flatten(0, 1)
+        out["uv"] = self.uv[:, :s.vdim, :s.kv_rank].flatten(0, 1)
+        out["sink"] = self.sink
+        out["o"] = self.out_proj.unflatten(1, (H, self.E))[:, :, :s.vdim].flatten(1)
+        return out
+
+    def init_random(self, randn) -> None:
+        s, H, hidden = self.spec, self.spec.heads, self.in_proj.shape[1]
+        shapes = {"q": (H * s.dim, hidden), "dkv": (s.kv_rank, hidden), "g": (H, hidden),
+                  "uk": (H * s.dim, s.kv_rank), "uv": (H * s.vdim, s.kv_rank),
+                  "o": (hidden, H * s.vdim)}
+        self.load(lambda n: randn(shapes[n]) * shapes[n][1] ** -0.5 if n in shapes
+                  else 1.0 + 0.1 * randn((s.kv_rank,)) if n == "dkv.norm" else randn((H,)))
+
+    def forward(self, h, meta, segments, kv, state):
+        s, at = self.spec, self.cols.at
+        if self._p is None or self._p.uk.device != self.uk.device:
+            self._p = ops.LatentParams(s.heads, self.D, self.E, s.scale, at["q"], at["g"],
+                                       self.uk.data, self.uk_t.data, self.uv.data,
+                                       self.sink.data)
+        cache = kv[0][0]
+        proj = ops.linear(h, self.in_proj)
+        if s.kv_from is None:
+            ops.latent_write(proj, at["dkv"], s.kv_rank, self.latent_norm, self.eps,
+                             meta.slot_mapping, cache)
+        out = torch.empty(h.shape[0], self.out_proj.shape[1], dtype=h.dtype,
+                          device=h.device)
+        for seg in segments:
+            ops.latent_attention(proj, self._p, cache, seg, out)
+        return ops.linear(out, self.out_proj)
+
+
+class DenseXieluMLP(nn.Module):
+    """Two matrices around an xIELU. With ``gated``, the residual gate's
+    projection of the same input shares the first product."""
+
+    def __init__(self, spec: DenseSpec, hidden: int, dtype, gated: bool):
+        super().__init__()
+        self.spec = spec
+        self.cols = FusedColumns(([("gate", hidden)] if gated else []) + [("up", spec.ff)])
+        self.in_proj = _param(self.cols.total, hidden, dtype=dtype)
+        self.gate_bias = _param(hidden, dtype=torch.float32) if gated else None
+        self.down = _param(hidden, spec.ff, dtype=dtype)
+        self.act = _param(2, dtype=torch.float32)
+
+    def load(self, get, get_gate=None) -> None:
+        """``get_gate`` reads the residual gate: its weight, and with ".b" its bias."""
+        parts = {"up": get("up")}
+        if self.gate_bias is not None:
+            parts["gate"] = get_gate("")
+            self.gate_bias.copy_(get_gate(".b"))
+        self.cols.pack(parts, self.in_proj)
+        self.down.copy_(get("down"))
+        self.act.copy_(get("act"))
+
+    def tensors(self) -> Dict[str, torch.Tensor]:
+        return {"up": self.cols.unpack(self.in_proj)["up"], "down": self.down,
+                "act": self.act}
+
+    def gate_tensors(self) -> Dict[str, torch.Tensor]:
+        return {"": self.cols.unpack(self.in_proj)["gate"], ".b": self.gate_bias}
+
+    def init_random(self, randn) -> None:
+        hidden, ff = self.down.shape
+        self.load(lambda n: {"up": lambda: randn((ff, hidden)) * hidden ** -0.5,
+                             "down": lambda: randn((hidden, ff)) * ff ** -0.5,
+                             "act": lambda: randn((2,)) * 0.5}[n](),
+                  lambda n: randn((hidden,)) if n else randn((hidden, hidden)) * hidden ** -0.5)
+
+    def forward(self, h) -> Dict[str, object]:
+        at, ff = self.cols.at, self.spec.ff
+        z = ops.linear(h, self.in_proj)
+        add: Dict[str, object] = {
+            "delta": ops.linear(ops.xielu(z[:, at["up"]:at["up"] + ff], self.act), self.down)}
+        if self.gate_bias is not None:
+            add["gate"] = (z[:, :h.shape[1]], self.gate_bias)
+        return add
+
+
 class RoutedGLU(nn.Module):
     """Top-k routed clamped-GLU experts with a biased fp32 router. Returns the
     chosen experts' rows unsummed; the next residual norm adds them up."""
@@ -276,7 +421,7 @@ class RoutedGLU(nn.Module):
             self.gate_up[e].copy_(randn((2 * ff, hidden)) * hidden ** -0.5)
             self.down[e].copy_(randn((hidden, ff)) * ff ** -0.5)
 
-    def forward(self, h):
+    def forward(self, h) -> Dict[str, object]:
         s = self.spec
-        return ops.moe_clamped_glu(h, self.router, self.router_bias, s.top,
-                                   self.gate_up, self.down, s.limit, self.ALPHA)
+        return {"moe": ops.moe_clamped_glu(h, self.router, self.router_bias, s.top,
+                                           self.gate_up, self.down, s.limit, self.ALPHA)}

@@ -33,6 +33,7 @@ def _load_named(model, path):
 _ARCHS = {
     "llama": (_llama, _load_llama),
     "kikalix": (_hybrid, _load_named),
+    "senotar": (_hybrid, _load_named),
 }
 
 

@@ -242,13 +242,22 @@ def softmax_sample(logits, temperature, top_p, top_k, generator=None):
 
 from .sequence import (  # noqa: E402
     DeltaRuleParams,
+    LatentParams,
     RetentionParams,
     Segment,
     bias_kv_write,
     biased_attention,
     cache_head_dims,
     delta_rule,
+    embed_pairs,
+    latent_attention,
+    latent_head_width,
+    latent_width,
+    latent_write,
     moe_clamped_glu,
     residual_rmsnorm,
+    residual_rmsnorm_conv,
     retention,
+    short_conv_add,
+    xielu,
 )

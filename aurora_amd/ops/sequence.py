@@ -1,5 +1,6 @@
 """Ops of the layer-listed decoders: biased window attention over paged KV,
-the gated delta rule, retention, and routed clamped-GLU experts.
+the gated delta rule, retention, routed clamped-GLU experts, latent attention,
+pair embeddings and the mixers' input convolution.
 
 Same dispatch rule as the rest of the package: GPU tensors run the gfx950
 kernels (bf16, or float32 throughout) and fail loudly without the extension;
@@ -17,6 +18,10 @@ from . import torch_ref
 #: head widths of the matrix-core attention kernels; the paged cache of a
 #: bf16 model on the GPU stores heads at the next of these, zero filled
 MATRIX_HEAD_DIMS = (64, 128)
+#: latent widths of the matrix-core latent attention kernel
+MATRIX_LATENT_WIDTHS = (64, 128, 256, 384, 512)
+#: widest latent of the kernel that serves float32 and everything else
+MAX_LATENT = 1024
 #: tokens per chunk of the recurrence kernels
 RECURRENCE_CHUNK = 16
 
@@ -63,6 +68,34 @@ class RetentionParams:
     eps: float
 
 
+def latent_width(rank: int) -> int:
+    """Width at which latents are cached, zero filled."""
+    if rank > MAX_LATENT:
+        raise ValueError(f"latent of {rank} numbers; at most {MAX_LATENT}")
+    return next((w for w in MATRIX_LATENT_WIDTHS if w >= rank), -(-rank // 64) * 64)
+
+
+def latent_head_width(dim: int) -> int:
+    """Width of a latent-attention head's rows in the projections' weights."""
+    return next((w for w in MATRIX_HEAD_DIMS if w >= dim), -(-dim // 32) * 32)
+
+
+@dataclass
+class LatentParams:
+    """Sizes, projection columns and weights of latent attention; all head and
+    latent widths are the padded ones."""
+    heads: int
+    dim: int
+    vdim: int
+    scale: float
+    q0: int
+    g0: int
+    uk: torch.Tensor    # [heads, dim, R]
+    uk_t: torch.Tensor  # [heads, R, dim]
+    uv: torch.Tensor    # [heads, vdim, R]
+    sink: torch.Tensor  # [heads] fp32
+
+
 @dataclass
 class Segment:
     """One regime of a step: prompt portions (``cu`` given) or single tokens
@@ -74,6 +107,7 @@ class Segment:
     state_slots: Optional[torch.Tensor]
     cu: Optional[torch.Tensor] = None
     cu_host: Optional[List[int]] = None
+    ctx_host: Optional[List[int]] = None
     _maps: Dict[object, object] = field(default_factory=dict)
 
     @property
@@ -120,13 +154,146 @@ def _hip(op: str):
 
 
 def residual_rmsnorm(x, weight, eps, delta=None, moe=None, step=None,
-                     offset: float = 1.0, dtype=None):
+                     offset: float = 1.0, dtype=None, gate=None):
     if not x.is_cuda:
-        return torch_ref.residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype)
-    y, place, gate = moe if moe is not None else (None, None, None)
+        return torch_ref.residual_rmsnorm(x, weight, eps, delta, moe, step, offset,
+                                          dtype, gate)
+    return _residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate)[0]
+
+
+def _residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate,
+                      conv=(None, None, None, None)):
+    y, place, share = moe if moe is not None else (None, None, None)
+    pre, bias = gate if gate is not None else (None, None)
     return _hip("residual_rmsnorm").residual_rmsnorm(
-        x, weight, delta, y, place, gate, step, float(eps), float(offset),
-        dtype == torch.bfloat16)
+        x, weight, delta, pre, bias, y, place, share, step, *conv, float(eps),
+        float(offset), dtype == torch.bfloat16)
+
+
+def residual_rmsnorm_conv(x, weight, eps, conv_w, ring, segments: List[Segment],
+                          delta=None, moe=None, step=None, offset: float = 1.0,
+                          dtype=None, gate=None):
+    """``residual_rmsnorm`` and ``short_conv_add`` of its result: (h, h + conv).
+    A step of single tokens does both in one kernel."""
+    if x.is_cuda and len(segments) == 1 and segments[0].decode:
+        seg = segments[0]
+        return tuple(_residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype,
+                                       gate, (conv_w, ring, seg.starts, seg.state_slots)))
+    h = residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate)
+    u = torch.empty_like(h)
+    for seg in segments:
+        short_conv_add(h, conv_w, ring, seg, u)
+    return h, u
+
+
+def short_conv_add(h, w, ring, seg: Segment, out):
+    hs, os_ = h[seg.rows], out[seg.rows]
+    if not h.is_cuda:
+        torch_ref.short_conv_add(hs, w, ring, seg.cu_or_rows(hs.shape[0]), seg.starts,
+                                 seg.state_slots, os_)
+        return
+    _hip("short_conv_add").short_conv_add(hs, w, ring, seg.cu, seg.starts,
+                                          seg.state_slots, os_)
+
+
+def embed_pairs(ids, table, scale, pairs, mul_prev: int, mul_cur: int, weight, eps,
+                prev, segments: List[Segment]):
+    """fp32 rows of normed token plus pair embeddings; advances ``prev``."""
+    out = torch.empty(ids.shape[0], table.shape[1], dtype=torch.float32, device=ids.device)
+    for seg in segments:
+        i, o = ids[seg.rows], out[seg.rows]
+        if ids.is_cuda:
+            _hip("embed_pairs").embed_pairs(
+                i, table, float(scale), pairs, mul_prev, mul_cur, weight, float(eps),
+                prev, seg.cu, seg.starts, seg.state_slots, o)
+        else:
+            torch_ref.embed_pairs(i, table, scale, pairs, mul_prev, mul_cur, weight, eps,
+                                  prev, seg.cu_or_rows(i.shape[0]), seg.starts,
+                                  seg.state_slots, o)
+    return out
+
+
+def latent_write(proj, col: int, rank: int, weight, eps, slots, cache):
+    if not proj.is_cuda:
+        return torch_ref.latent_write(proj, col, rank, weight, eps, slots, cache)
+    _hip("latent_write").latent_write(proj, col, rank, weight, float(eps), slots, cache)
+
+
+def head_linear(x, w, gate=None, out=None):
+    """Per-head product: x [T, H, K] (rows may be strided), w [H, N, K] ->
+    [T, H, N], times sigmoid(gate [T, H]) if given."""
+    T, H, _ = x.shape
+    if out is None:
+        out = torch.empty(T, H, w.shape[1], dtype=x.dtype, device=x.device)
+    if x.dtype == torch.bfloat16:
+        _hip("head_linear").head_linear(x, w, gate, out)
+        return out
+    y = torch.bmm(x.transpose(0, 1).contiguous(), w.transpose(1, 2).contiguous())
+    y = y.transpose(0, 1)
+    out.copy_(y if gate is None else y * torch.sigmoid(gate).unsqueeze(-1))
+    return out
+
+
+def expand_latents(seg: Segment, p: LatentParams, rank: int) -> bool:
+    """Whether it is cheaper to spell out every key and value of a prompt
+    portion's context than to attend in the latents' own space, where a pair of
+    tokens costs 2 rank instead of dim + vdim but a key costs nothing."""
+    if seg.decode or (p.dim, p.vdim) not in {(a, b) for a in MATRIX_HEAD_DIMS
+                                             for b in MATRIX_HEAD_DIMS}:
+        return False
+    lens = [b - a for a, b in zip(seg.cu_host, seg.cu_host[1:])]
+    keys = sum(seg.ctx_host)
+    pairs = sum(n * (c - n / 2) for n, c in zip(lens, seg.ctx_host))
+    fits = keys * p.heads * (p.dim + p.vdim) <= EXPANDED_LIMIT
+    return fits and pairs * (2 * rank - p.dim - p.vdim) > keys * rank * (p.dim + p.vdim)
+
+
+#: most numbers of spelled-out keys and values one step may hold
+EXPANDED_LIMIT = 1 << 31
+
+
+def latent_attention(proj, p: LatentParams, cache, seg: Segment, out):
+    """One segment's rows of gated latent attention into out [rows, H * vdim]."""
+    pr, o = proj[seg.rows], out[seg.rows]
+    T, H, R = pr.shape[0], p.heads, cache.shape[3]
+    q = pr[:, p.q0:p.q0 + H * p.dim].unflatten(1, (H, p.dim))
+    gate = pr[:, p.g0:p.g0 + H]
+    if not proj.is_cuda:
+        torch_ref.latent_attention(q, gate, p.uk, p.uv, p.sink, p.scale, cache,
+                                   seg.block_tables, seg.cu_or_rows(T),
+                                   seg.context_lens, o)
+        return
+    m = _hip("latent_attention")
+    matrix = proj.dtype == torch.bfloat16 and R in MATRIX_LATENT_WIDTHS
+    if matrix and expand_latents(seg, p, R):
+        first = [0]
+        for n in seg.ctx_host:
+            first.append(first[-1] + n)
+        c, rows = seg.latent_rows(cache)
+        k = torch.nn.functional.linear(c, p.uk.flatten(0, 1))
+        v = torch.nn.functional.linear(c, p.uv.flatten(0, 1))
+        bseq, boff = seg.block_map(m.biased_prefill_rows(1))
+        m.sink_attention_prefill(q, k.view(-1, H, 1, p.dim), v.view(-1, H, 1, p.vdim),
+                                 rows, seg.cu, seg.context_lens, bseq, boff, p.scale,
+                                 p.sink, gate, o)
+        return
+    qa = head_linear(q, p.uk_t)
+    if matrix:
+        oc = m.latent_attention(qa, cache, seg.block_tables, seg.cu, seg.context_lens,
+                                *seg.latent_map(H), p.scale, p.sink)
+    else:
+        oc = torch.empty_like(qa)
+        bseq, boff = (None, None) if seg.decode else seg.block_map(1)
+        m.latent_attention_rows(qa, cache, seg.block_tables, seg.cu, seg.context_lens,
+                                bseq, boff, p.scale, p.sink, oc)
+    head_linear(oc, p.uv, gate, o.unflatten(1, (H, p.vdim)))
+
+
+def xielu(z, act):
+    """Rows of ``z`` may be strided; act [2]: the two slopes before softplus."""
+    if not z.is_cuda:
+        return torch_ref.xielu(z, act)
+    return _hip("xielu").xielu(z, act)
 
 
 def bias_kv_write(proj, cols, bias, slots, k_cache, v_cache, heads, kv_heads, dim, vdim):

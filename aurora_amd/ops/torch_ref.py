@@ -254,11 +254,13 @@ def softmax_sample(
 # ---- layer-listed decoders: biased attention, recurrences, routed GLU --------
 
 def residual_rmsnorm(x, weight, eps, delta=None, moe=None, step=None,
-                     offset: float = 1.0, dtype=None):
-    """x (fp32, updated in place) += delta, or the routed experts' weighted
-    sum, then += step; returns rms(x) * (offset + weight) in ``dtype``."""
+                     offset: float = 1.0, dtype=None, gate=None):
+    """x (fp32, updated in place) += delta (times the sigmoid of ``gate`` =
+    (pre-activation, bias), if given), or the routed experts' weighted sum,
+    then += step; returns rms(x) * (offset + weight) in ``dtype``."""
     if delta is not None:
-        x += delta.float()
+        y = delta.float()
+        x += y if gate is None else y * torch.sigmoid(gate[0].float() + gate[1])
     if moe is not None:
         y, place, weights = moe
         x += (y.float()[place.long()] * weights.unsqueeze(-1)).sum(1)
@@ -432,3 +434,95 @@ def moe_clamped_glu(h, sel, w_gate_up, w_down, limit: float, alpha: float):
         a = (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(h.dtype)
         y[rows] = (a.float() @ w_down[e].float().t()).to(h.dtype)
     return y, torch.arange(T * top, dtype=torch.int32).view(T, top)
+
+
+# ---- layer-listed decoders: pair embedding, input convolution, latent attention
+
+def embed_pairs(ids, table, scale, pairs, mul_prev, mul_cur, weight, eps, prev,
+                cu, starts, slots, out):
+    """rms(table[id] * scale + pairs[row]) * weight per token, fp32 into
+    ``out``; row = (previous id * mul_prev + id * mul_cur) mod (rows - 1), the
+    last row at position 0. prev [slots, 1] holds each sequence's last id and
+    is advanced; slot < 0 rows have no past and store nothing."""
+    buckets = pairs.shape[0] - 1
+    for s in range(cu.numel() - 1):
+        a, b, start, slot = int(cu[s]), int(cu[s + 1]), int(starts[s]), int(slots[s])
+        if a == b:
+            continue
+        cur = ids[a:b].long()
+        row = torch.full_like(cur, buckets)
+        row[1:] = (cur[:-1] * mul_prev + cur[1:] * mul_cur) % buckets
+        if start > 0 and slot >= 0:
+            row[0] = (prev[slot, 0].long() * mul_prev + cur[0] * mul_cur) % buckets
+        x = table[cur].float() * scale + pairs[row].float()
+        out[a:b] = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * weight
+        if slot >= 0:
+            prev[slot, 0] = cur[-1]
+
+
+def short_conv_add(h, w, ring, cu, starts, slots, out):
+    """out = h + causal convolution of h per channel; w [W, taps]. The ring
+    [slots, taps - 1, W] holds position p's h at p mod (taps - 1)."""
+    taps = w.shape[1]
+    past = taps - 1
+    for s in range(cu.numel() - 1):
+        a, b, start, slot = int(cu[s]), int(cu[s + 1]), int(starts[s]), int(slots[s])
+        n = b - a
+        if n == 0:
+            continue
+        full = torch.zeros(past + n, h.shape[1])
+        full[past:] = h[a:b].float()
+        if slot >= 0:
+            for j in range(1, past + 1):
+                if start - j >= 0:
+                    full[past - j] = ring[slot, (start - j) % past].float()
+            for t in range(max(0, n - past), n):
+                ring[slot, (start + t) % past] = h[a + t].to(ring.dtype)
+        y = full[past:].clone()
+        for j in range(taps):
+            y += full[j:j + n] * w[:, j]
+        out[a:b] = y.to(out.dtype)
+
+
+def latent_write(proj, col, rank, weight, eps, slots, cache):
+    """Normed latent of every token into the paged cache [pages, 1, P, R],
+    zero filled past ``rank``."""
+    c = proj[:, col:col + rank].float()
+    c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * weight
+    P = cache.shape[2]
+    ok = slots >= 0
+    at = slots[ok].long()
+    cache[at // P, 0, at % P] = torch.nn.functional.pad(
+        c, (0, cache.shape[3] - rank)).to(cache.dtype)[ok]
+
+
+def latent_attention(q, gate, uk, uv, sink, scale, cache, block_tables, cu, ctx, out):
+    """q [T, H, D], gate [T, H] pre-activations, uk [H, D, R], uv [H, E, R]:
+    causal attention of every head to keys uk c and values uv c of the cached
+    latents c, the sink in the denominator, times sigmoid(gate) -> out [T, H*E]."""
+    H = q.shape[1]
+    P = cache.shape[2]
+    for s in range(cu.numel() - 1):
+        a, b, L = int(cu[s]), int(cu[s + 1]), int(ctx[s])
+        if a == b:
+            continue
+        c = _paged_rows(cache, block_tables[s, :(L + P - 1) // P].long(), L)[0]
+        k = torch.einsum("hdr,kr->hkd", uk.float(), c)
+        v = torch.einsum("her,kr->hke", uv.float(), c)
+        att = torch.einsum("qhd,hkd->hqk", q[a:b].float(), k) * scale
+        later = (torch.arange(L).unsqueeze(0)
+                 > torch.arange(L - (b - a), L).unsqueeze(1))
+        att.masked_fill_(later, float("-inf"))
+        att = torch.cat([att, sink.view(H, 1, 1).expand(H, b - a, 1)], -1)
+        o = torch.einsum("hqk,hke->qhe", att.softmax(-1)[..., :-1], v)
+        o = o * torch.sigmoid(gate[a:b].float()).unsqueeze(-1)
+        out[a:b] = o.reshape(b - a, -1).to(out.dtype)
+
+
+def xielu(z, act):
+    """softplus(act[0]) z^2 + z/2 above zero, (1/2 + softplus(act[1]))
+    (e^z - 1 - z) + z/2 below."""
+    x = z.float()
+    p, q = torch.nn.functional.softplus(act.float())
+    low = (0.5 + q) * (torch.expm1(x.clamp(max=0)) - x)
+    return (torch.where(x > 0, p * x * x, low) + 0.5 * x).to(z.dtype)
