@@ -21,7 +21,9 @@
 // two 32-key MFMA steps each.
 // BIAS adds a per-head linear distance penalty and a sliding window (tiles
 // and MFMA steps wholly outside a wave's window are skipped), lets keys and
-// values differ in width, and writes scaled columns of a wider output.
+// values differ in width, and writes scaled columns of a wider output. SINK
+// starts every row's softmax from a term without key or value and multiplies
+// the head by a sigmoid gate.
 // Covers fresh prefill and append-prefill (chunked agent turns) since K/V
 // are read from the paged cache with an absolute-position causal bound.
 #include "common.h"
@@ -41,9 +43,9 @@ union frag_u {
   bf16x8 v;
 };
 
-template <int D, int DV, int HG, bool FP8, bool BIAS>  // HG = query heads per workgroup
+template <int D, int DV, int HG, bool FP8, bool BIAS, bool SINK>  // HG = query heads per workgroup
 __global__ __launch_bounds__(512, 1) void prefill_kernel(
-    const __hip_bfloat16* __restrict__ q,   // [T, Hq, D]
+    const __hip_bfloat16* __restrict__ q,   // [T, qstride], heads D apart
     const void* __restrict__ kc,  // [NP, Hkv, P, D] bf16 | fp8 e4m3
     const void* __restrict__ vc,
     __hip_bfloat16* __restrict__ out,       // [T, ostride], heads dv apart
@@ -53,8 +55,10 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
     const int* __restrict__ block_tables,   // [S, MP]
     const int* __restrict__ ctx_lens,       // [S]
     int Hq, int Hkv, int P, int MP, float scale,
-    long ostride, int dv, float oscale,
-    const float* __restrict__ slopes, int window) {
+    long qstride, long ostride, int dv, float oscale,
+    const float* __restrict__ slopes, int window,
+    const float* __restrict__ sink,         // [Hq]
+    const __hip_bfloat16* __restrict__ gate, long gstride) {  // [T, gstride]
   constexpr int KVB = 64;           // keys staged per tile
   constexpr int NC = D / 16;        // Q^T fragments (MFMA K-chunks of QK^T)
   constexpr int NDT = DV / 32;      // 32-wide d-tiles of O
@@ -93,7 +97,7 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   // ---- Q fragments (B-operand of swapped QK^T): held for the whole block
   const int qrow = qoff + qsub * 32 + col;  // local q row in this seq
   const bool qvalid = qrow < qlen;
-  const long qbase = ((long)(q_start + (qvalid ? qrow : 0)) * Hq + h) * D;
+  const long qbase = (q_start + (qvalid ? qrow : 0)) * qstride + (long)h * D;
   frag_u qf[NC];
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
@@ -110,7 +114,7 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   }
 
   const int q_abs = ctx - qlen + qrow;  // absolute position of this lane's q
-  float m = -1e30f, l = 0.f;
+  float m = SINK ? sink[h] : -1e30f, l = SINK ? 1.f : 0.f;
   floatx16 o[NDT];
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
@@ -279,6 +283,10 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   }
 
   // ---- epilogue: divide by l (per q row), transpose via LDS, store rows
+  if constexpr (SINK) {  // divided by l, times the gate
+    const long grow = (q_start + (qvalid ? qrow : 0)) * gstride + h;
+    l *= 1.f + __expf(-bf16_to_f32(((const unsigned short*)gate)[grow]));
+  }
   if (half == 0) wsc[col] = l;
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
   __builtin_amdgcn_sched_barrier(0);
@@ -374,7 +382,7 @@ torch::Tensor attention_prefill_paged(torch::Tensor q, torch::Tensor kc,
   dim3 grid(NB, Hq / HG), block(512);
   auto stream = CUR_STREAM;
 #define PLAUNCH1(DD, HGV, F8)                                                 \
-  hipLaunchKernelGGL((prefill_kernel<DD, DD, HGV, F8, false>), grid, block,   \
+  hipLaunchKernelGGL((prefill_kernel<DD, DD, HGV, F8, false, false>), grid, block,   \
                      (prefill_lds<DD, DD>()), stream,                         \
                      (const __hip_bfloat16*)q.data_ptr(),                     \
                      kc.data_ptr(), vc.data_ptr(),                            \
@@ -382,7 +390,8 @@ torch::Tensor attention_prefill_paged(torch::Tensor q, torch::Tensor kc,
                      bseq_t.data_ptr<int>(), boff_t.data_ptr<int>(),          \
                      cu_q.data_ptr<int>(), bt.data_ptr<int>(),                \
                      ctx.data_ptr<int>(), Hq, Hkv, P, MP, (float)scale,       \
-                     (long)Hq * D, D, 1.f, nullptr, 0)
+                     (long)Hq * D, (long)Hq * D, D, 1.f, nullptr, 0, nullptr, \
+                     nullptr, 0)
 #define PLAUNCH(DD, HGV)                                                      \
   if (fp8) { PLAUNCH1(DD, HGV, true); } else { PLAUNCH1(DD, HGV, false); }
 #define PLAUNCH_D(DD)                                                         \
@@ -428,15 +437,15 @@ void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor v
   const int HG = heads_per_block(Hq / Hkv);
   dim3 grid(NB, Hq / HG), block(512);
 #define BLAUNCH(DD, DVV, HGV)                                                   \
-  hipLaunchKernelGGL((prefill_kernel<DD, DVV, HGV, false, true>), grid, block,  \
+  hipLaunchKernelGGL((prefill_kernel<DD, DVV, HGV, false, true, false>), grid, block, \
                      (prefill_lds<DD, DVV>()), CUR_STREAM,                      \
                      (const __hip_bfloat16*)q.data_ptr(), kc.data_ptr(),        \
                      vc.data_ptr(), (__hip_bfloat16*)out.data_ptr() + col,      \
                      bseq.data_ptr<int>(), boff.data_ptr<int>(),                \
                      cu_q.data_ptr<int>(), bt.data_ptr<int>(),                  \
                      ctx.data_ptr<int>(), Hq, Hkv, P, MP, (float)scale,         \
-                     out.stride(0), (int)dv, (float)oscale,                     \
-                     slopes.data_ptr<float>(), (int)window)
+                     (long)Hq * D, out.stride(0), (int)dv, (float)oscale,       \
+                     slopes.data_ptr<float>(), (int)window, nullptr, nullptr, 0)
 #define BLAUNCH_HG(DD, DVV)                    \
   switch (HG) {                                \
     case 1: BLAUNCH(DD, DVV, 1); break;        \
@@ -450,5 +459,51 @@ void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor v
   else TORCH_CHECK(false, "unsupported cache head widths ", D, ", ", DV);
 #undef BLAUNCH_HG
 #undef BLAUNCH
+  HIP_CHECK_KERNEL();
+}
+
+// q [T, H, D] (rows may be strided), kc [NP, H, P, D], vc [NP, H, P, DV], gate
+// [T, H] pre-activations (rows may be strided) -> out [T, H * DV]
+void sink_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
+                            torch::Tensor bt, torch::Tensor cu_q, torch::Tensor ctx,
+                            torch::Tensor bseq, torch::Tensor boff, double scale,
+                            torch::Tensor sink, torch::Tensor gate, torch::Tensor out) {
+  const int T = q.size(0), H = q.size(1), D = q.size(2);
+  const int P = kc.size(2), MP = bt.size(1), DV = vc.size(3);
+  TORCH_CHECK(q.is_cuda() && q.dtype() == torch::kBFloat16 && q.stride(2) == 1 &&
+              q.stride(1) == D && q.stride(0) % 8 == 0 &&
+              (reinterpret_cast<uintptr_t>(q.data_ptr()) & 15) == 0, "queries");
+  TORCH_CHECK(kc.dtype() == torch::kBFloat16 && vc.dtype() == torch::kBFloat16 &&
+              kc.is_contiguous() && vc.is_contiguous() && bt.is_contiguous() &&
+              kc.size(1) == H && vc.size(1) == H && kc.size(3) == D && vc.size(2) == P &&
+              vc.size(0) == kc.size(0), "keys and values");
+  TORCH_CHECK(out.dtype() == torch::kBFloat16 && out.is_contiguous() && out.size(0) == T &&
+              out.size(1) == (long)H * DV);
+  TORCH_CHECK(gate.dtype() == torch::kBFloat16 && gate.size(0) == T && gate.size(1) == H &&
+              gate.stride(1) == 1 && sink.numel() == H && sink.dtype() == torch::kFloat32);
+  TORCH_CHECK(bseq.dtype() == torch::kInt32 && boff.dtype() == torch::kInt32 &&
+              bseq.numel() == boff.numel() && cu_q.dtype() == torch::kInt32 &&
+              bt.dtype() == torch::kInt32 && ctx.dtype() == torch::kInt32 &&
+              cu_q.numel() == ctx.numel() + 1 && bt.size(0) == ctx.numel());
+  const int NB = bseq.numel();
+  if (T == 0 || NB == 0) return;
+  dim3 grid(NB, H), block(512);
+#define SLAUNCH(DD, DVV)                                                        \
+  hipLaunchKernelGGL((prefill_kernel<DD, DVV, 1, false, false, true>), grid,    \
+                     block, (prefill_lds<DD, DVV>()), CUR_STREAM,               \
+                     (const __hip_bfloat16*)q.data_ptr(), kc.data_ptr(),        \
+                     vc.data_ptr(), (__hip_bfloat16*)out.data_ptr(),            \
+                     bseq.data_ptr<int>(), boff.data_ptr<int>(),                \
+                     cu_q.data_ptr<int>(), bt.data_ptr<int>(),                  \
+                     ctx.data_ptr<int>(), H, H, P, MP, (float)scale,            \
+                     q.stride(0), out.stride(0), DV, 1.f, nullptr, 0,           \
+                     sink.data_ptr<float>(),                                    \
+                     (const __hip_bfloat16*)gate.data_ptr(), gate.stride(0))
+  if (D == 64 && DV == 64) { SLAUNCH(64, 64); }
+  else if (D == 64 && DV == 128) { SLAUNCH(64, 128); }
+  else if (D == 128 && DV == 64) { SLAUNCH(128, 64); }
+  else if (D == 128 && DV == 128) { SLAUNCH(128, 128); }
+  else TORCH_CHECK(false, "unsupported head widths ", D, ", ", DV);
+#undef SLAUNCH
   HIP_CHECK_KERNEL();
 }

@@ -1,5 +1,6 @@
-// Distance-biased window attention for any head width and for float32: one
-// wave per (query row, head), 64 keys at a time.
+// Attention for any head width and for float32: one wave per (query row, head),
+// 64 keys at a time; with a distance bias and a window, or over shared latents
+// (keys that are also the values) with a sink.
 //
 // The matrix-core kernels (attention_prefill / attention_decode) serve bf16
 // heads up to 128 wide; this one serves everything else. Each lane scores its
@@ -11,14 +12,16 @@
 
 #define CUR_STREAM c10::hip::getCurrentHIPStream().stream()
 #define ROWS_MAX_DV 512
+#define ROWS_MAX_LATENT 1024
 
-template <typename T>
+template <typename T, int MAX_DV>
 __global__ __launch_bounds__(256) void attention_rows_kernel(
     const T* __restrict__ q,  // [T, Hq, DK]
     const T* __restrict__ kc, const T* __restrict__ vc,  // [NP, Hkv, P, DK|DV]
     const int* __restrict__ bt, const int* __restrict__ cu,
     const int* __restrict__ ctx, const int* __restrict__ row_seq,
     const int* __restrict__ row_off, const float* __restrict__ slopes,
+    const float* __restrict__ sink,  // [Hq] each, or null
     T* __restrict__ out, long ostride, int T_, int Hq, int Hkv, int DK, int DV,
     int dv, int P, int MP, float scale, int window, float oscale) {
   extern __shared__ float qs[];
@@ -36,12 +39,13 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(
   const int len = cu ? cu[seq + 1] - cu[seq] : 1;
   const int pos = ctx[seq] - len + (row_off ? row_off[t] : 0);
   const int kvh = h / (Hq / Hkv);
-  const float slope = slopes[h];
+  const float slope = slopes ? slopes[h] : 0.f;
   const int* pages = bt + (long)seq * MP;
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
-  float m = -1e30f, l = 0.f, acc[ROWS_MAX_DV / WAVE];
+  // a sink is one more term of the denominator
+  float m = sink ? sink[h] : -1e30f, l = sink ? 1.f : 0.f, acc[MAX_DV / WAVE];
 #pragma unroll
-  for (int j = 0; j < ROWS_MAX_DV / WAVE; ++j) acc[j] = 0.f;
+  for (int j = 0; j < MAX_DV / WAVE; ++j) acc[j] = 0.f;
   for (int k0 = lo; k0 <= pos; k0 += WAVE) {
     const int key = k0 + lane;
     const bool seen = key <= pos;
@@ -56,18 +60,18 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(
     m = mn;
     l = l * alpha + wave_sum(p);
 #pragma unroll
-    for (int j = 0; j < ROWS_MAX_DV / WAVE; ++j) acc[j] *= alpha;
+    for (int j = 0; j < MAX_DV / WAVE; ++j) acc[j] *= alpha;
     const int n = min(WAVE, pos - k0 + 1);
     for (int i = 0; i < n; ++i) {
       const float pi = __shfl(p, i, WAVE);
       const long ri = __shfl(row, i, WAVE);
 #pragma unroll
-      for (int j = 0; j < ROWS_MAX_DV / WAVE; ++j)
+      for (int j = 0; j < MAX_DV / WAVE; ++j)
         if (lane + j * WAVE < dv) acc[j] += pi * ldf(vc + ri * DV + lane + j * WAVE);
     }
   }
 #pragma unroll
-  for (int j = 0; j < ROWS_MAX_DV / WAVE; ++j)
+  for (int j = 0; j < MAX_DV / WAVE; ++j)
     if (lane + j * WAVE < dv)
       stf(out + t * ostride + h * dv + lane + j * WAVE, acc[j] / l * oscale);
 }
@@ -102,10 +106,51 @@ void biased_attention_rows(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
   const dim3 grid(((long)T_ * Hq + 3) / 4);
   DISPATCH_ELEM(q.dtype() == torch::kBFloat16, {
     hipLaunchKernelGGL(
-        (attention_rows_kernel<T>), grid, dim3(256), 4 * DK * 4, CUR_STREAM, (const T*)q.data_ptr(),
+        (attention_rows_kernel<T, ROWS_MAX_DV>), grid, dim3(256), 4 * DK * 4, CUR_STREAM, (const T*)q.data_ptr(),
         (const T*)kc.data_ptr(), (const T*)vc.data_ptr(), bt.data_ptr<int>(),
-        cup, ctx.data_ptr<int>(), rsp, rop, slopes.data_ptr<float>(), (T*)out.data_ptr() + col, out.stride(0), T_, Hq, Hkv,
-        DK, DV, (int)dv, P, MP, (float)scale, (int)window, (float)oscale);
+        cup, ctx.data_ptr<int>(), rsp, rop, slopes.data_ptr<float>(),
+        (const float*)nullptr, (T*)out.data_ptr() + col, out.stride(0), T_, Hq, Hkv, DK,
+        DV, (int)dv, P, MP, (float)scale, (int)window, (float)oscale);
+  });
+  HIP_CHECK_KERNEL();
+}
+
+// q [T, H, R] against the latent cache [NP, 1, P, R], which is keys and values
+void latent_attention_rows(torch::Tensor q, torch::Tensor cache, torch::Tensor bt,
+                           c10::optional<torch::Tensor> cu, torch::Tensor ctx,
+                           c10::optional<torch::Tensor> row_seq,
+                           c10::optional<torch::Tensor> row_off, double scale,
+                           torch::Tensor sink, torch::Tensor out) {
+  const int T_ = q.size(0), H = q.size(1), R = q.size(2);
+  const int P = cache.size(2), MP = bt.size(1);
+  TORCH_CHECK(q.is_cuda() && q.is_contiguous() && cache.is_contiguous() &&
+              bt.is_contiguous() && out.is_contiguous() && out.sizes() == q.sizes());
+  TORCH_CHECK(cache.size(1) == 1 && cache.size(3) == R && R <= ROWS_MAX_LATENT,
+              "latents of ", R, " numbers");
+  TORCH_CHECK(sink.numel() == H && sink.dtype() == torch::kFloat32);
+  TORCH_CHECK(cache.dtype() == q.dtype() && out.dtype() == q.dtype());
+  TORCH_CHECK(bt.dtype() == torch::kInt32 && ctx.dtype() == torch::kInt32 &&
+              bt.size(0) == ctx.numel());
+  if (cu) {
+    TORCH_CHECK(row_seq && row_off && row_seq->numel() == T_ && row_off->numel() == T_ &&
+                cu->numel() == ctx.numel() + 1);
+  } else {
+    TORCH_CHECK(ctx.numel() == T_);
+  }
+  if (T_ == 0) return;
+  const dim3 grid(((long)T_ * H + 3) / 4);
+  DISPATCH_ELEM(q.dtype() == torch::kBFloat16, {
+    auto launch = [&](auto kern) {
+      hipLaunchKernelGGL(
+          kern, grid, dim3(256), 4 * R * 4, CUR_STREAM, (const T*)q.data_ptr(),
+          (const T*)cache.data_ptr(), (const T*)cache.data_ptr(), bt.data_ptr<int>(),
+          cu ? cu->data_ptr<int>() : nullptr, ctx.data_ptr<int>(),
+          cu ? row_seq->data_ptr<int>() : nullptr, cu ? row_off->data_ptr<int>() : nullptr,
+          (const float*)nullptr, sink.data_ptr<float>(), (T*)out.data_ptr(), (long)H * R, T_,
+          H, 1, R, R, R, P, MP, (float)scale, 0, 1.f);
+    };
+    if (R <= ROWS_MAX_DV) launch(attention_rows_kernel<T, ROWS_MAX_DV>);
+    else launch(attention_rows_kernel<T, ROWS_MAX_LATENT>);
   });
   HIP_CHECK_KERNEL();
 }

@@ -28,9 +28,32 @@ torch::Tensor moe_grouped_gemm(torch::Tensor xp, torch::Tensor w,
                                torch::Tensor starts, torch::Tensor counts);
 // ---- layer-listed decoders
 using OptT = c10::optional<torch::Tensor>;
-torch::Tensor residual_rmsnorm(torch::Tensor x, torch::Tensor weight, OptT delta, OptT y,
-                               OptT place, OptT gate, OptT step, double eps, double offset,
-                               bool to_bf16);
+std::vector<torch::Tensor> residual_rmsnorm(torch::Tensor x, torch::Tensor weight, OptT delta,
+                                            OptT gate_pre, OptT gate_bias, OptT y, OptT place,
+                                            OptT gate, OptT step, OptT conv_w, OptT ring,
+                                            OptT pos, OptT slots, double eps, double offset,
+                                            bool to_bf16);
+void embed_pairs(torch::Tensor ids, torch::Tensor table, double scale, torch::Tensor pairs,
+                 long mul_prev, long mul_cur, torch::Tensor weight, double eps,
+                 torch::Tensor prev, OptT cu, torch::Tensor starts, torch::Tensor slots,
+                 torch::Tensor out);
+long short_conv_rows();
+void short_conv_add(torch::Tensor h, torch::Tensor w, torch::Tensor ring, OptT cu, OptT bseq,
+                    OptT boff, torch::Tensor starts, torch::Tensor slots, torch::Tensor out);
+torch::Tensor xielu(torch::Tensor z, torch::Tensor act);
+void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight, double eps,
+                  torch::Tensor slots, torch::Tensor cache);
+void head_linear(torch::Tensor x, torch::Tensor w, OptT gate, torch::Tensor out);
+torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tensor bt, OptT cu,
+                               torch::Tensor ctx, OptT bseq, OptT boff, long rows,
+                               double scale, torch::Tensor sink);
+void latent_attention_rows(torch::Tensor q, torch::Tensor cache, torch::Tensor bt, OptT cu,
+                           torch::Tensor ctx, OptT row_seq, OptT row_off, double scale,
+                           torch::Tensor sink, torch::Tensor out);
+void sink_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
+                            torch::Tensor bt, torch::Tensor cu_q, torch::Tensor ctx,
+                            torch::Tensor bseq, torch::Tensor boff, double scale,
+                            torch::Tensor sink, torch::Tensor gate, torch::Tensor out);
 torch::Tensor bias_kv_write(torch::Tensor proj, long q0, long k0, long v0,
                             torch::Tensor bias, torch::Tensor slots, torch::Tensor kc,
                             torch::Tensor vc, long Hq, long Hkv, long d, long dv);
@@ -93,7 +116,20 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_grouped_gemm", &moe_grouped_gemm,
         "packed per-expert grouped GEMM (skips unrouted experts)");
   m.def("residual_rmsnorm", &residual_rmsnorm,
-        "fp32 residual add (dense or routed rows, pass vector) + RMSNorm");
+        "fp32 residual add (dense, gated or routed rows, pass vector) + RMSNorm, "
+        "+ input convolution of single tokens");
+  m.def("embed_pairs", &embed_pairs, "token + token-pair embedding, normed");
+  m.def("short_conv_rows", &short_conv_rows);
+  m.def("short_conv_add", &short_conv_add, "input plus its causal convolution");
+  m.def("xielu", &xielu, "xIELU activation");
+  m.def("latent_write", &latent_write, "latent norm + paged scatter");
+  m.def("head_linear", &head_linear, "per-head product with an optional gate");
+  m.def("latent_attention", &latent_attention,
+        "MFMA attention in the latents' space over the paged cache, with a sink");
+  m.def("latent_attention_rows", &latent_attention_rows,
+        "any latent width / float32 latent attention with a sink");
+  m.def("sink_attention_prefill", &sink_attention_prefill,
+        "MFMA flash prefill with a sink and a gate per head");
   m.def("bias_kv_write", &bias_kv_write, "bias + head split + paged KV scatter");
   m.def("biased_prefill_rows", &biased_prefill_rows);
   m.def("biased_attention_prefill", &biased_attention_prefill,

@@ -1,0 +1,512 @@
+// Latent attention on gfx950: one cached vector c per token and layer, from
+// which every head's key and value are linear maps (uk, uv).
+//
+// A head's score q.(uk c) is (uk' q).c, and its output uv (sum_j p_j c_j), so
+// attention can stay in the latents' space: all (token, head) rows of a
+// sequence attend to ONE key row that is also the value row. That is what
+// decoding does (a latent is read once for all heads; 2 R flops per byte and
+// head row, so it needs the matrix cores), and short prompt portions on a long
+// context. Long portions spell keys and values out and run the flash prefill
+// kernel (ops.sequence.expand_latents decides).
+//
+// latent_attention_kernel: a workgroup holds 16 or 32 rows and walks its
+// context in tiles of 64 latents, four waves:
+//  * every wave loads its own 16 latents of the next tile straight to LDS while
+//    the tile before is computed, and scores them: S^T = C Q^T, the rows'
+//    queries live in registers as B fragments;
+//  * the tile's row maxima and the bf16 weights go through LDS (two barriers a
+//    tile), then every wave owns R / 4 columns of O += P C. The value fragments
+//    are columns of the row-major tile: ds_read_b64_tr_b16 transposes on the
+//    way to the registers. Contraction slot 8 g + j holds key 4 g + j (j < 4)
+//    or 16 + 4 g + j - 4, on both operands, so the eight rows two lane groups
+//    read at a time are consecutive;
+//  * LDS rows are unpadded (direct loads fill them in lane order); 16-byte units
+//    are permuted within a row by unit_swizzle, applied to the source address.
+// Few rows: the context is split over blockIdx.y, partial sums are merged by
+// latent_combine_kernel. A row's softmax starts from its sink (split 0 only).
+#include "elem.h"
+#include <torch/extension.h>
+#include <c10/hip/HIPStream.h>
+
+#define CUR_STREAM c10::hip::getCurrentHIPStream().stream()
+#define LAT_KEYS 64                    // latents per tile
+#define LAT_PSTRIDE (LAT_KEYS + 8)     // row stride of the weights in LDS
+
+union lfrag {
+  shortx8 s;
+  shortx4 h[2];
+  bf16x8 v;
+};
+
+// XOR of a row's 16-byte unit index: 16 rows at one unit, and 8 rows at two
+// neighbouring units, fall into distinct banks
+template <int U>
+DEVINL int unit_swizzle(int row) {
+  return U == 8 ? (((row >> 1) & 3) << 1) | ((row >> 3) & 1)
+                : ((row & 7) << 1) | ((row >> 3) & 1);
+}
+
+// Transposing reads of the four 16-row slices (STEP bytes apart) of one 16-column
+// tile; then wait until the slices requested before these have arrived. Written
+// out because the compiler puts a wait for all global loads in flight, the next
+// tile's among them, before the builtin form of these reads.
+template <int STEP>
+DEVINL void read_columns(shortx4 (&next)[4], shortx4 (&ready)[4], unsigned addr) {
+  asm volatile(
+      "ds_read_b64_tr_b16 %0, %8\n\t"
+      "ds_read_b64_tr_b16 %1, %8 offset:%9\n\t"
+      "ds_read_b64_tr_b16 %2, %8 offset:%10\n\t"
+      "ds_read_b64_tr_b16 %3, %8 offset:%11\n\t"
+      "s_waitcnt lgkmcnt(4)"
+      : "=&v"(next[0]), "=&v"(next[1]), "=&v"(next[2]), "=&v"(next[3]), "+v"(ready[0]),
+        "+v"(ready[1]), "+v"(ready[2]), "+v"(ready[3])
+      : "v"(addr), "n"(STEP), "n"(2 * STEP), "n"(3 * STEP)
+      : "memory");
+}
+
+DEVINL void await_columns(shortx4 (&ready)[4]) {
+  asm volatile("s_waitcnt lgkmcnt(0)"
+               : "+v"(ready[0]), "+v"(ready[1]), "+v"(ready[2]), "+v"(ready[3])::"memory");
+}
+
+template <int R, int MT>
+__global__ __launch_bounds__(256, 1) void latent_attention_kernel(
+    const bf16_t* __restrict__ q,      // [T * H, R]
+    const bf16_t* __restrict__ cache,  // [NP, P, R]
+    const int* __restrict__ bt, int MP, const int* __restrict__ cu,
+    const int* __restrict__ ctx, const int* __restrict__ bseq,
+    const int* __restrict__ boff, const float* __restrict__ sink,
+    bf16_t* __restrict__ out,          // [T * H, R] (one split)
+    float* __restrict__ part,          // [CS, T * H, R] (several)
+    float* __restrict__ part_ml,       // [CS, T * H, 2]
+    int H, int P, long rows_all, float scale) {
+  constexpr int U = R / 8;             // 16-byte units per latent
+  constexpr int NT = R / 64;           // 16-column tiles of O per wave
+  constexpr int ROWS = 16 * MT;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  short* pbuf = (short*)(smem + 2 * LAT_KEYS * R * 2);
+  float* stat = (float*)(smem + 2 * LAT_KEYS * R * 2 + ROWS * LAT_PSTRIDE * 2);  // [4][ROWS]
+
+  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
+  const int col = lane & 15, g = lane >> 4;
+  const int tiles_per_seq = (H + ROWS - 1) / ROWS;  // single tokens
+  const int seq = cu ? bseq[blockIdx.x] : blockIdx.x / tiles_per_seq;
+  const int off = cu ? boff[blockIdx.x] : blockIdx.x % tiles_per_seq * ROWS;
+  const int n = cu ? cu[seq + 1] - cu[seq] : 1;
+  const long row0 = (long)(cu ? cu[seq] : seq) * H + off;
+  const int nrows = min(ROWS, n * H - off);
+  const int start = ctx[seq] - n;
+  const int kend = start + (off + nrows - 1) / H + 1;  // keys any row here sees
+  const int ntiles = (kend + LAT_KEYS - 1) / LAT_KEYS;
+  const int per = (ntiles + gridDim.y - 1) / gridDim.y;
+  const int tile0 = blockIdx.y * per, tile1 = min(ntiles, tile0 + per);
+  const int* pages = bt + (long)seq * MP;
+
+  // queries (B operand: lane's row col, contraction 8 g + j), positions, sinks
+  lfrag qf[MT][R / 32];
+  int pos[MT];
+  float m[MT], l[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+    const int r = min(t * 16 + col, nrows - 1);
+    const bf16_t* src = q + (row0 + r) * R + g * 8;
+#pragma unroll
+    for (int k = 0; k < R / 32; ++k) qf[t][k].s = *(const shortx8*)(src + k * 32);
+    pos[t] = start + (off + r) / H;
+    m[t] = blockIdx.y == 0 ? sink[(off + r) % H] : -1e30f;
+    l[t] = blockIdx.y == 0 && wave == 0 && g == 0 ? 1.f : 0.f;
+  }
+  floatx4 o[MT][NT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+#pragma unroll
+    for (int c = 0; c < NT; ++c) o[t][c] = floatx4{0.f, 0.f, 0.f, 0.f};
+
+  // byte offsets of the wave's columns: lane i of a group reads row i / 4, the
+  // 8 bytes i mod 4 of the 32
+  const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) char*)smem;
+  unsigned vcol[NT];
+#pragma unroll
+  for (int c = 0; c < NT; ++c) {
+    const int row = g * 4 + (col >> 2), unit = (wave * NT + c) * 2 + ((lane & 3) >> 1);
+    vcol[c] = row * R * 2 + (unit ^ unit_swizzle<U>(row)) * 16 + (lane & 1) * 8;
+  }
+
+  // this wave's 16 latents of a tile; past the end the last one again
+  auto issue = [&](int tile) {
+    const int key = min(tile * LAT_KEYS + wave * 16 + col, kend - 1);
+    const int slot = pages[key / P] * P + key % P;
+    char* dst = smem + (tile & 1) * (LAT_KEYS * R * 2) + wave * 16 * R * 2;
+#pragma unroll
+    for (int i = 0; i < R / 32; ++i) {
+      const int id = i * WAVE + lane, row = id / U, unit = id % U;
+      const long s = __shfl(slot, row, WAVE);
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) void*)(
+              cache + s * R + (unit ^ unit_swizzle<U>(row)) * 8),
+          (__attribute__((address_space(3))) void*)(dst + id * 16), 16, 0, 0);
+    }
+  };
+
+  if (tile0 < tile1) issue(tile0);
+  for (int tile = tile0; tile < tile1; ++tile) {
+    const char* cb = smem + (tile & 1) * (LAT_KEYS * R * 2);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    // scores of the wave's own keys: S^T rows 4 g + r, columns are query rows
+    floatx4 st[MT];
+#pragma unroll
+    for (int t = 0; t < MT; ++t) st[t] = floatx4{0.f, 0.f, 0.f, 0.f};
+    const char* krow = cb + (wave * 16 + col) * R * 2;
+#pragma unroll
+    for (int k = 0; k < R / 32; ++k) {
+      lfrag kf;
+      kf.s = *(const shortx8*)(krow + ((k * 4 + g) ^ unit_swizzle<U>(col)) * 16);
+#pragma unroll
+      for (int t = 0; t < MT; ++t)
+        st[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf.v, qf[t][k].v, st[t], 0, 0, 0);
+    }
+    const int key0 = tile * LAT_KEYS + wave * 16 + g * 4;
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+      float mx = -1e30f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        st[t][r] = key0 + r <= pos[t] ? st[t][r] * scale : -1e30f;
+        mx = fmaxf(mx, st[t][r]);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
+      if (g == 0) stat[wave * ROWS + t * 16 + col] = mx;
+    }
+    // the whole tile has landed, and nobody reads the other buffer any more
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    if (tile + 1 < tile1) issue(tile + 1);
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+      float mn = m[t];
+#pragma unroll
+      for (int w = 0; w < 4; ++w) mn = fmaxf(mn, stat[w * ROWS + t * 16 + col]);
+      const float alpha = __expf(m[t] - mn);
+      m[t] = mn;
+      floatx4 p;
+      float sum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        p[r] = key0 + r <= pos[t] ? __expf(st[t][r] - mn) : 0.f;
+        sum += p[r];
+      }
+      l[t] = l[t] * alpha + sum;
+      st4((bf16_t*)pbuf + (t * 16 + col) * LAT_PSTRIDE + wave * 16 + g * 4, p);
+      if (__any(alpha < 1.f)) {
+        floatx4 av;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) av[r] = __shfl(alpha, g * 4 + r, WAVE);
+#pragma unroll
+        for (int c = 0; c < NT; ++c) o[t][c] *= av;
+      }
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    lfrag pf[2][MT];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+      for (int t = 0; t < MT; ++t) {
+        const short* pr = pbuf + (t * 16 + col) * LAT_PSTRIDE + kk * 32 + g * 4;
+        pf[kk][t].h[0] = *(const shortx4*)pr;
+        pf[kk][t].h[1] = *(const shortx4*)(pr + 16);
+      }
+    // slice 2 kk + j holds contraction slots 8 g + 4 j ..+3 of step kk
+    const unsigned tile_at = lds0 + (tile & 1) * (LAT_KEYS * R * 2);
+    shortx4 cols[NT + 1][4] = {};
+    read_columns<16 * R * 2>(cols[1], cols[0], tile_at + vcol[0]);
+#pragma unroll
+    for (int c = 0; c < NT; ++c) {
+      if (c + 1 < NT)
+        read_columns<16 * R * 2>(cols[c + 2], cols[c + 1], tile_at + vcol[c + 1]);
+      else
+        await_columns(cols[c + 1]);
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        lfrag cf;
+        cf.h[0] = cols[c + 1][2 * kk];
+        cf.h[1] = cols[c + 1][2 * kk + 1];
+#pragma unroll
+        for (int t = 0; t < MT; ++t)
+          o[t][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[kk][t].v, cf.v, o[t][c], 0, 0, 0);
+      }
+    }
+  }
+
+  // the waves' sums of weights
+  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+    l[t] += __shfl_xor(l[t], 16, WAVE);
+    l[t] += __shfl_xor(l[t], 32, WAVE);
+    if (g == 0) stat[wave * ROWS + t * 16 + col] = l[t];
+  }
+  asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+  if (gridDim.y == 1) {
+    bf16_t* ob = (bf16_t*)smem;
+#pragma unroll
+    for (int t = 0; t < MT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = t * 16 + g * 4 + r;
+        float sum = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) sum += stat[w * ROWS + row];
+        const float inv = 1.f / sum;
+#pragma unroll
+        for (int c = 0; c < NT; ++c)
+          stf(ob + row * R + (wave * NT + c) * 16 + col, o[t][c][r] * inv);
+      }
+    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    for (int i = tid; i < nrows * U; i += 256)
+      *(shortx8*)(out + row0 * R + (long)i * 8) = *(const shortx8*)(ob + i * 8);
+    return;
+  }
+  const long prow = blockIdx.y * rows_all + row0;
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = t * 16 + g * 4 + r;
+      if (row >= nrows) continue;
+#pragma unroll
+      for (int c = 0; c < NT; ++c)
+        part[(prow + row) * R + (wave * NT + c) * 16 + col] = o[t][c][r];
+    }
+  if (wave == 0 && g == 0)
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+      const int row = t * 16 + col;
+      if (row >= nrows) continue;
+      float sum = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) sum += stat[w * ROWS + row];
+      part_ml[(prow + row) * 2] = m[t];
+      part_ml[(prow + row) * 2 + 1] = sum;
+    }
+}
+
+// merge the context splits: one wave per row
+__global__ __launch_bounds__(256) void latent_combine_kernel(
+    const float* __restrict__ part, const float* __restrict__ part_ml,
+    bf16_t* __restrict__ out, long rows, int CS, int R) {
+  const long row = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
+  if (row >= rows) return;
+  const int lane = threadIdx.x % WAVE;
+  float M = -1e30f, L = 0.f;
+  for (int s = 0; s < CS; ++s) M = fmaxf(M, part_ml[(s * rows + row) * 2]);
+  for (int s = 0; s < CS; ++s) {
+    const float* ml = part_ml + (s * rows + row) * 2;
+    L += __expf(ml[0] - M) * ml[1];
+  }
+  const float inv = 1.f / L;
+  for (int d = lane * 4; d < R; d += WAVE * 4) {
+    floatx4 a = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < CS; ++s)
+      a += ld4(part + (s * rows + row) * R + d) *
+           (__expf(part_ml[(s * rows + row) * 2] - M) * inv);
+    st4(out + row * R + d, a);
+  }
+}
+
+torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tensor bt,
+                               c10::optional<torch::Tensor> cu, torch::Tensor ctx,
+                               c10::optional<torch::Tensor> bseq,
+                               c10::optional<torch::Tensor> boff, long rows, double scale,
+                               torch::Tensor sink) {
+  const int T = q.size(0), H = q.size(1), R = q.size(2), S = ctx.numel();
+  const int P = cache.size(2), MP = bt.size(1);
+  TORCH_CHECK(q.is_cuda() && q.dtype() == torch::kBFloat16 && q.is_contiguous());
+  TORCH_CHECK(cache.dtype() == torch::kBFloat16 && cache.is_contiguous() &&
+              cache.size(1) == 1 && cache.size(3) == R, "latent cache");
+  TORCH_CHECK(cache.size(0) * P < (1L << 31), "cache slots");
+  TORCH_CHECK(bt.is_contiguous() && bt.dtype() == torch::kInt32 && bt.size(0) == S &&
+              ctx.dtype() == torch::kInt32);
+  TORCH_CHECK(sink.numel() == H && sink.dtype() == torch::kFloat32);
+  TORCH_CHECK(rows == 16 || rows == 32);
+  int blocks;
+  if (cu) {
+    TORCH_CHECK(bseq && boff && bseq->numel() == boff->numel() && cu->numel() == S + 1 &&
+                cu->dtype() == torch::kInt32 && bseq->dtype() == torch::kInt32 &&
+                boff->dtype() == torch::kInt32);
+    blocks = bseq->numel();
+  } else {
+    TORCH_CHECK(T == S);
+    blocks = S * ((H + rows - 1) / rows);
+  }
+  auto out = torch::empty_like(q);
+  if (T == 0 || blocks == 0) return out;
+  // one workgroup per CU
+  const int CS = std::max(1, std::min(32, 256 / blocks));
+  const long all = (long)T * H;
+  torch::Tensor part, ml;
+  if (CS > 1) {
+    part = torch::empty({CS, all, R}, q.options().dtype(torch::kFloat32));
+    ml = torch::empty({CS, all, 2}, q.options().dtype(torch::kFloat32));
+  }
+#define LATENT(RR, MT)                                                                   \
+  do {                                                                                   \
+    auto kern = latent_attention_kernel<RR, MT>;                                         \
+    constexpr int lds = 2 * LAT_KEYS * RR * 2 + 16 * MT * LAT_PSTRIDE * 2 + 4 * 16 * MT * 4; \
+    static const hipError_t once = hipFuncSetAttribute(                                  \
+        (const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds);             \
+    TORCH_CHECK(once == hipSuccess, "LDS of the latent attention kernel");               \
+    hipLaunchKernelGGL(kern, dim3(blocks, CS), dim3(256), lds, CUR_STREAM,               \
+                       (const bf16_t*)q.data_ptr(), (const bf16_t*)cache.data_ptr(),     \
+                       bt.data_ptr<int>(), MP, cu ? cu->data_ptr<int>() : nullptr,       \
+                       ctx.data_ptr<int>(), cu ? bseq->data_ptr<int>() : nullptr,        \
+                       cu ? boff->data_ptr<int>() : nullptr, sink.data_ptr<float>(),     \
+                       (bf16_t*)out.data_ptr(), CS > 1 ? part.data_ptr<float>() : nullptr, \
+                       CS > 1 ? ml.data_ptr<float>() : nullptr, H, P, all, (float)scale); \
+  } while (0)
+#define LATENT_R(RR)                       \
+  if (R == RR) {                           \
+    if (rows == 16) LATENT(RR, 1);         \
+    else LATENT(RR, 2);                    \
+  } else
+  LATENT_R(64) LATENT_R(128) LATENT_R(256) LATENT_R(384) LATENT_R(512)
+  TORCH_CHECK(false, "unsupported latent width ", R);
+#undef LATENT_R
+#undef LATENT
+  if (CS > 1)
+    hipLaunchKernelGGL(latent_combine_kernel, dim3((all + 3) / 4), dim3(256), 0, CUR_STREAM,
+                       part.data_ptr<float>(), ml.data_ptr<float>(), (bf16_t*)out.data_ptr(),
+                       all, CS, R);
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+// ------------------------------------------------------------------ latents
+
+// norm of a token's latent in fp32 and its place in the cache: one wave per token
+template <typename T>
+__global__ __launch_bounds__(256) void latent_write_kernel(
+    const T* __restrict__ proj, long stride, int rank, const float* __restrict__ weight,
+    float eps, const int* __restrict__ slots, T* __restrict__ cache, int T_, int R) {
+  const int t = blockIdx.x * 4 + threadIdx.x / WAVE;
+  if (t >= T_) return;
+  const int lane = threadIdx.x % WAVE;
+  const int slot = slots[t];
+  if (slot < 0) return;
+  const T* src = proj + t * stride;
+  float ss = 0.f;
+  for (int i = lane; i < rank; i += WAVE) {
+    const float v = ldf(src + i);
+    ss += v * v;
+  }
+  const float inv = rsqrtf(wave_sum(ss) / rank + eps);
+  T* dst = cache + (long)slot * R;
+  for (int i = lane; i < R; i += WAVE)
+    stf(dst + i, i < rank ? ldf(src + i) * inv * weight[i] : 0.f);
+}
+
+void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight, double eps,
+                  torch::Tensor slots, torch::Tensor cache) {
+  const int T_ = proj.size(0), R = cache.size(3);
+  TORCH_CHECK(proj.is_cuda() && proj.dim() == 2 && proj.stride(1) == 1 &&
+              col + rank <= proj.size(1) && rank <= R);
+  TORCH_CHECK(cache.is_contiguous() && cache.size(1) == 1 && cache.dtype() == proj.dtype());
+  TORCH_CHECK(weight.numel() == rank && weight.dtype() == torch::kFloat32);
+  TORCH_CHECK(slots.numel() == T_ && slots.dtype() == torch::kInt32);
+  if (T_ == 0) return;
+  DISPATCH_ELEM(proj.dtype() == torch::kBFloat16, {
+    hipLaunchKernelGGL((latent_write_kernel<T>), dim3((T_ + 3) / 4), dim3(256), 0, CUR_STREAM,
+                       (const T*)proj.data_ptr() + col, proj.stride(0), (int)rank,
+                       weight.data_ptr<float>(), (float)eps, slots.data_ptr<int>(),
+                       (T*)cache.data_ptr(), T_, R);
+  });
+  HIP_CHECK_KERNEL();
+}
+
+// --------------------------------------------------------- per-head products
+
+// out[t, h, n] = sum_k x[t, h, k] w[h, n, k], times sigmoid(gate[t, h]). Waves
+// take 16 outputs each (KS 1) or split the contraction (KS 4); TT 16-token
+// tiles per workgroup. K and N are multiples of 32.
+template <int TT, int KS>
+__global__ __launch_bounds__(256) void head_linear_kernel(
+    const bf16_t* __restrict__ x, long xt, long xh, const bf16_t* __restrict__ w,
+    const bf16_t* __restrict__ gate, long gt, bf16_t* __restrict__ out, long ot, long oh,
+    int T_, int N, int K) {
+  __shared__ float red[KS > 1 ? 4 : 1][TT][WAVE][4];
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  const int col = lane & 15, g = lane >> 4;
+  const int h = blockIdx.y, t0 = blockIdx.z * 16 * TT;
+  const int n0 = KS > 1 ? blockIdx.x * 16 : (blockIdx.x * 4 + wave) * 16;
+  if (n0 >= N) return;  // KS 1 only: whole waves, no barrier follows
+  const int steps = K / 32, lo = KS > 1 ? steps * wave / 4 : 0,
+            hi = KS > 1 ? steps * (wave + 1) / 4 : steps;
+  const bf16_t* wp = w + ((long)h * N + n0 + col) * K + g * 8;
+  const bf16_t* xp[TT];
+#pragma unroll
+  for (int t = 0; t < TT; ++t)
+    xp[t] = x + min(t0 + t * 16 + col, T_ - 1) * xt + h * xh + g * 8;
+  floatx4 acc[TT];
+#pragma unroll
+  for (int t = 0; t < TT; ++t) acc[t] = floatx4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = lo; k < hi; ++k) {
+    lfrag a, b;
+    a.s = *(const shortx8*)(wp + k * 32);
+#pragma unroll
+    for (int t = 0; t < TT; ++t) {
+      b.s = *(const shortx8*)(xp[t] + k * 32);
+      acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, acc[t], 0, 0, 0);
+    }
+  }
+  if constexpr (KS > 1) {
+#pragma unroll
+    for (int t = 0; t < TT; ++t) *(floatx4*)red[wave][t][lane] = acc[t];
+    __syncthreads();
+  }
+#pragma unroll
+  for (int t = 0; t < TT; ++t) {
+    if (KS > 1 && (t & 3) != wave) continue;  // the waves share the tiles
+    floatx4 y = acc[t];
+    if constexpr (KS > 1) {
+      y = *(const floatx4*)red[0][t][lane];
+#pragma unroll
+      for (int s = 1; s < 4; ++s) y += *(const floatx4*)red[s][t][lane];
+    }
+    const int tok = t0 + t * 16 + col;
+    if (tok >= T_) continue;
+    if (gate) y *= sigmoid_f(ldf(gate + tok * gt + h));
+    st4(out + tok * ot + h * oh + n0 + g * 4, y);
+  }
+}
+
+void head_linear(torch::Tensor x, torch::Tensor w, c10::optional<torch::Tensor> gate,
+                 torch::Tensor out) {
+  const int T_ = x.size(0), H = x.size(1), K = x.size(2), N = w.size(1);
+  TORCH_CHECK(x.is_cuda() && x.dtype() == torch::kBFloat16 && w.dtype() == x.dtype() &&
+              out.dtype() == x.dtype() && w.is_contiguous());
+  TORCH_CHECK(w.size(0) == H && w.size(2) == K && K % 32 == 0 && N % 32 == 0);
+  auto aligned = [](const torch::Tensor& t, long unit) {
+    return t.stride(2) == 1 && t.stride(0) % unit == 0 && t.stride(1) % unit == 0 &&
+           (reinterpret_cast<uintptr_t>(t.data_ptr()) & (unit * 2 - 1)) == 0;
+  };
+  TORCH_CHECK(aligned(x, 8) && aligned(out, 4) && out.size(0) == T_ && out.size(1) == H &&
+              out.size(2) == N);
+  if (gate)
+    TORCH_CHECK(gate->size(0) == T_ && gate->size(1) == H && gate->stride(1) == 1 &&
+                gate->dtype() == x.dtype());
+  if (T_ == 0) return;
+  auto launch = [&](auto kern, int tt, int ks) {
+    const dim3 grid(ks > 1 ? N / 16 : (N + 63) / 64, H, (T_ + 16 * tt - 1) / (16 * tt));
+    hipLaunchKernelGGL(kern, grid, dim3(256), 0, CUR_STREAM, (const bf16_t*)x.data_ptr(),
+                       x.stride(0), x.stride(1), (const bf16_t*)w.data_ptr(),
+                       gate ? (const bf16_t*)gate->data_ptr() : nullptr,
+                       gate ? gate->stride(0) : 0, (bf16_t*)out.data_ptr(), out.stride(0),
+                       out.stride(1), T_, N, K);
+  };
+  // a long contraction with few outputs: split it over the waves
+  const bool split = K >= 256 && T_ <= 64;
+  if (T_ <= 16) split ? launch(head_linear_kernel<1, 4>, 1, 4) : launch(head_linear_kernel<1, 1>, 1, 1);
+  else if (T_ <= 32) split ? launch(head_linear_kernel<2, 4>, 2, 4) : launch(head_linear_kernel<2, 1>, 2, 1);
+  else split ? launch(head_linear_kernel<4, 4>, 4, 4) : launch(head_linear_kernel<4, 1>, 4, 1);
+  HIP_CHECK_KERNEL();
+}

@@ -1,11 +1,13 @@
 // Residual-stream kernels of the layer-listed decoders.
 //
 // residual_rmsnorm: the residual is ONE fp32 tensor. The kernel that norms it
-// also adds what came before: a sub-layer's output, or the chosen experts'
-// rows with their routing weights (so no separate combine pass exists), and
-// the vector that marks a pass of a repeated span. One workgroup per row, the
-// row lives in LDS between the sum of squares and the scaling: x is read and
-// written once, everything else once.
+// also adds what came before: a sub-layer's output, scaled by its residual gate
+// if it has one, or the chosen experts' rows with their routing weights (so no
+// separate combine pass exists), and the vector that marks a pass of a repeated
+// span. In steps of single tokens it also adds the next mixer's input
+// convolution to the result. One workgroup per row, the row lives in LDS
+// between the sum of squares and the scaling: x is read and written once,
+// everything else once.
 //
 // bias_kv_write: splits the fused projection, adds the biases in fp32, and
 // scatters K/V to the paged cache; heads are stored at the cache's width.
@@ -15,24 +17,53 @@
 
 #define CUR_STREAM c10::hip::getCurrentHIPStream().stream()
 
+// the sub-layer's output is multiplied by sigmoid(pre + bias)
+template <typename T>
+struct ResidualGate {
+  const T* pre;  // [T, stride], null: no gate
+  long stride;
+  const float* bias;
+};
+
+// causal convolution of the normed rows, one token per sequence: the ring holds
+// position p's row at p mod (taps - 1); slot -1 has no past and stores nothing
+template <typename T>
+struct ConvTail {
+  const float* w;  // [W, taps], null: no convolution
+  int taps;
+  T* ring;         // [slots, taps - 1, W]
+  const int* pos;
+  const int* slots;
+  T* out;          // [T, W]
+};
+
 template <typename T, int V>
 __global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
     float* __restrict__ x, const float* __restrict__ weight,
-    const T* __restrict__ delta, const T* __restrict__ y,
+    const T* __restrict__ delta, ResidualGate<T> rg, const T* __restrict__ y,
     const int* __restrict__ place, const float* __restrict__ gate, int top,
-    const float* __restrict__ step, T* __restrict__ out, int W, float eps,
-    float offset) {
+    const float* __restrict__ step, T* __restrict__ out, ConvTail<T> cv, int W,
+    float eps, float offset) {
   extern __shared__ __attribute__((aligned(16))) float row[];
   __shared__ float red[4];
   const long base = (long)blockIdx.x * W;
   const int* pl = place + (long)blockIdx.x * top;
   const float* gt = gate + (long)blockIdx.x * top;
+  const T* pre = rg.pre ? rg.pre + blockIdx.x * rg.stride : nullptr;
   float ss = 0.f;
   for (int i = threadIdx.x * V; i < W; i += 256 * V) {
     float v[V];
     if constexpr (V == 4) {
       floatx4 a = ld4(x + base + i);
-      if (delta) a += ld4(delta + base + i);
+      if (delta) {
+        floatx4 d = ld4(delta + base + i);
+        if (pre) {
+          const floatx4 g = ld4(pre + i) + ld4(rg.bias + i);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) d[j] *= sigmoid_f(g[j]);
+        }
+        a += d;
+      }
       if (y) {
         for (int j = 0; j < top; ++j) a += gt[j] * ld4(y + (long)pl[j] * W + i);
       }
@@ -43,7 +74,10 @@ __global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
       if (delta || y || step) st4(x + base + i, a);
     } else {
       float a = x[base + i];
-      if (delta) a += ldf(delta + base + i);
+      if (delta) {
+        const float d = ldf(delta + base + i);
+        a += pre ? d * sigmoid_f(ldf(pre + i) + rg.bias[i]) : d;
+      }
       if (y)
         for (int j = 0; j < top; ++j) a += gt[j] * ldf(y + (long)pl[j] * W + i);
       if (step) a += step[i];
@@ -55,6 +89,11 @@ __global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
     for (int j = 0; j < V; ++j) ss += v[j] * v[j];
   }
   const float inv = rsqrtf(block_sum4(ss, red) / W + eps);
+  const int keep = cv.taps - 1;
+  const int slot = cv.w ? cv.slots[blockIdx.x] : -1;
+  const int pos = cv.w ? cv.pos[blockIdx.x] : 0;
+  T* ring = cv.ring + (long)max(slot, 0) * keep * W;
+  const int known = slot >= 0 ? min(keep, pos) : 0;  // rows of the past
   for (int i = threadIdx.x * V; i < W; i += 256 * V) {
     if constexpr (V == 4) {
       const floatx4 a = *reinterpret_cast<const floatx4*>(row + i);
@@ -62,26 +101,53 @@ __global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
     } else {
       stf(out + base + i, row[i] * inv * (offset + weight[i]));
     }
+    if (!cv.w) continue;
+    // from here on the row as stored
+    float u[V];
+    const float* w = cv.w + (long)i * cv.taps;
+#pragma unroll
+    for (int j = 0; j < V; ++j) {
+      u[j] = ldf(out + base + i + j);
+      u[j] += u[j] * w[j * cv.taps + keep];
+    }
+    for (int b = 1; b <= known; ++b) {
+      const T* p = ring + (long)((pos - b) % keep) * W + i;
+#pragma unroll
+      for (int j = 0; j < V; ++j) u[j] += w[j * cv.taps + keep - b] * ldf(p + j);
+    }
+#pragma unroll
+    for (int j = 0; j < V; ++j) stf(cv.out + base + i + j, u[j]);
+    if (keep > 0 && slot >= 0) {  // takes the place of the oldest row, now read
+      T* p = ring + (long)(pos % keep) * W + i;
+#pragma unroll
+      for (int j = 0; j < V; ++j) p[j] = out[base + i + j];
+    }
   }
 }
 
-torch::Tensor residual_rmsnorm(torch::Tensor x, torch::Tensor weight,
-                               c10::optional<torch::Tensor> delta,
-                               c10::optional<torch::Tensor> y,
-                               c10::optional<torch::Tensor> place,
-                               c10::optional<torch::Tensor> gate,
-                               c10::optional<torch::Tensor> step, double eps,
-                               double offset, bool to_bf16) {
+std::vector<torch::Tensor> residual_rmsnorm(
+    torch::Tensor x, torch::Tensor weight, c10::optional<torch::Tensor> delta,
+    c10::optional<torch::Tensor> gate_pre, c10::optional<torch::Tensor> gate_bias,
+    c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> place,
+    c10::optional<torch::Tensor> gate, c10::optional<torch::Tensor> step,
+    c10::optional<torch::Tensor> conv_w, c10::optional<torch::Tensor> ring,
+    c10::optional<torch::Tensor> pos, c10::optional<torch::Tensor> slots, double eps,
+    double offset, bool to_bf16) {
   TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.is_contiguous() &&
               x.dtype() == torch::kFloat32, "residual must be fp32 [T, W]");
   const int T_ = x.size(0), W = x.size(1);
   TORCH_CHECK(weight.numel() == W && weight.dtype() == torch::kFloat32);
   TORCH_CHECK(W <= 32768, "row too wide for LDS");
   const auto dt = to_bf16 ? torch::kBFloat16 : torch::kFloat32;
-  auto out = torch::empty({T_, W}, x.options().dtype(dt));
+  std::vector<torch::Tensor> out = {torch::empty({T_, W}, x.options().dtype(dt))};
   if (delta)
     TORCH_CHECK(delta->is_contiguous() && delta->sizes() == x.sizes() &&
                 delta->dtype() == dt, "delta");
+  if (gate_pre)
+    TORCH_CHECK(delta && gate_bias && gate_pre->sizes() == x.sizes() &&
+                gate_pre->stride(1) == 1 && gate_pre->dtype() == dt &&
+                gate_bias->numel() == W && gate_bias->dtype() == torch::kFloat32,
+                "residual gate");
   int top = 0;
   if (y) {
     TORCH_CHECK(place && gate && y->is_contiguous() && y->size(1) == W &&
@@ -91,19 +157,37 @@ torch::Tensor residual_rmsnorm(torch::Tensor x, torch::Tensor weight,
     top = place->size(1);
   }
   if (step) TORCH_CHECK(step->numel() == W && step->dtype() == torch::kFloat32);
+  if (conv_w) {
+    TORCH_CHECK(ring && pos && slots && conv_w->is_contiguous() && conv_w->size(0) == W &&
+                conv_w->dtype() == torch::kFloat32 && ring->dim() == 3 &&
+                ring->is_contiguous() && ring->dtype() == dt && ring->size(2) == W &&
+                ring->size(1) == conv_w->size(1) - 1, "input convolution");
+    TORCH_CHECK(pos->numel() == T_ && slots->numel() == T_ &&
+                pos->dtype() == torch::kInt32 && slots->dtype() == torch::kInt32);
+    out.push_back(torch::empty_like(out[0]));
+  }
   if (T_ == 0) return out;
   const size_t lds = (size_t)W * 4;
   DISPATCH_ELEM(to_bf16, {
+    ResidualGate<T> rg = {nullptr, 0, nullptr};
+    if (gate_pre)
+      rg = {(const T*)gate_pre->data_ptr(), gate_pre->stride(0), gate_bias->data_ptr<float>()};
+    ConvTail<T> cv = {nullptr, 1, nullptr, nullptr, nullptr, nullptr};
+    if (conv_w)
+      cv = {conv_w->data_ptr<float>(), (int)conv_w->size(1), (T*)ring->data_ptr(),
+            pos->data_ptr<int>(), slots->data_ptr<int>(), (T*)out[1].data_ptr()};
     auto launch = [&](auto kern) {
       hipLaunchKernelGGL(
           kern, dim3(T_), dim3(256), lds, CUR_STREAM, x.data_ptr<float>(),
-          weight.data_ptr<float>(), delta ? (const T*)delta->data_ptr() : nullptr,
+          weight.data_ptr<float>(), delta ? (const T*)delta->data_ptr() : nullptr, rg,
           y ? (const T*)y->data_ptr() : nullptr,
           y ? place->data_ptr<int>() : nullptr, y ? gate->data_ptr<float>() : nullptr,
-          top, step ? step->data_ptr<float>() : nullptr, (T*)out.data_ptr(), W,
+          top, step ? step->data_ptr<float>() : nullptr, (T*)out[0].data_ptr(), cv, W,
           (float)eps, (float)offset);
     };
-    if (W % 4 == 0) launch(residual_rmsnorm_kernel<T, 4>);
+    const bool vec = W % 4 == 0 && (!gate_pre || (gate_pre->stride(0) % 4 == 0 &&
+                     (reinterpret_cast<uintptr_t>(gate_pre->data_ptr()) & 15) == 0));
+    if (vec) launch(residual_rmsnorm_kernel<T, 4>);
     else launch(residual_rmsnorm_kernel<T, 1>);
   });
   HIP_CHECK_KERNEL();

@@ -148,6 +148,42 @@ class Segment:
         return seq, off, hit
 
 
+    def latent_map(self, heads: int):
+        """(sequence, first row, rows per block) of the blocks of (token, head)
+        rows of latent attention; single tokens need no map."""
+        if self.decode:
+            return None, None, 16 if heads <= 16 else 32
+        hit = self._maps.get(("latent", heads))
+        if hit is None:
+            seq, off = [], []
+            for s in range(len(self.cu_host) - 1):
+                n = (self.cu_host[s + 1] - self.cu_host[s]) * heads
+                off.extend(range(0, n, 32))
+                seq.extend([s] * -(-n // 32))
+            t = torch.tensor([seq, off], dtype=torch.int32).to(self.context_lens.device)
+            hit = (t[0], t[1], 32)
+            self._maps[("latent", heads)] = hit
+        return hit
+
+    def latent_rows(self, cache):
+        """Every context token's latent, packed, and the place of sequence s's
+        token t among them as a table [s, t]; places are found once per step."""
+        P = cache.shape[2]
+        hit = self._maps.get("context")
+        if hit is None:
+            dev = cache.device
+            table = torch.zeros(len(self.ctx_host), max(self.ctx_host), dtype=torch.int32)
+            place, n = [], 0
+            for s, c in enumerate(self.ctx_host):
+                table[s, :c] = torch.arange(n, n + c, dtype=torch.int32)
+                n += c
+                t = torch.arange(c, device=dev)
+                place.append(self.block_tables[s].long()[t // P] * P + t % P)
+            hit = (torch.cat(place), table.to(dev))
+            self._maps["context"] = hit
+        return cache.view(-1, cache.shape[3]).index_select(0, hit[0]), hit[1]
+
+
 def _hip(op: str):
     from . import _require_hip
     return _require_hip(op)
@@ -192,8 +228,9 @@ def short_conv_add(h, w, ring, seg: Segment, out):
         torch_ref.short_conv_add(hs, w, ring, seg.cu_or_rows(hs.shape[0]), seg.starts,
                                  seg.state_slots, os_)
         return
-    _hip("short_conv_add").short_conv_add(hs, w, ring, seg.cu, seg.starts,
-                                          seg.state_slots, os_)
+    m = _hip("short_conv_add")
+    bseq, boff = (None, None) if seg.decode else seg.block_map(m.short_conv_rows())
+    m.short_conv_add(hs, w, ring, seg.cu, bseq, boff, seg.starts, seg.state_slots, os_)
 
 
 def embed_pairs(ids, table, scale, pairs, mul_prev: int, mul_cur: int, weight, eps,
@@ -266,9 +303,6 @@ def latent_attention(proj, p: LatentParams, cache, seg: Segment, out):
     m = _hip("latent_attention")
     matrix = proj.dtype == torch.bfloat16 and R in MATRIX_LATENT_WIDTHS
     if matrix and expand_latents(seg, p, R):
-        first = [0]
-        for n in seg.ctx_host:
-            first.append(first[-1] + n)
         c, rows = seg.latent_rows(cache)
         k = torch.nn.functional.linear(c, p.uk.flatten(0, 1))
         v = torch.nn.functional.linear(c, p.uv.flatten(0, 1))

@@ -33,7 +33,7 @@ def gpu(*ts):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("W", [512, 50, 1028])
-@pytest.mark.parametrize("kind", ["plain", "delta", "moe"])
+@pytest.mark.parametrize("kind", ["plain", "delta", "moe", "gated"])
 def test_residual_rmsnorm(dtype, W, kind):
     T, top = 7, 3
     x, w, step = rnd(T, W), rnd(W, scale=0.2), rnd(W)
@@ -45,6 +45,9 @@ def test_residual_rmsnorm(dtype, W, kind):
         args["moe"] = (rnd(T * top, W, dtype=dtype),
                        torch.randperm(T * top).view(T, top).int(),
                        torch.rand(T, top).softmax(-1))
+    if kind == "gated":  # the pre-activations are columns of a wider product
+        args["delta"] = rnd(T, W, dtype=dtype)
+        args["gate"] = (rnd(T, W + 12, dtype=dtype)[:, :W], rnd(W))
     xr, xg = x.clone(), x.cuda()
     want = torch_ref.residual_rmsnorm(xr, w, 1e-5, dtype=dtype, **args)
     dev = {k: tuple(gpu(*v)) if isinstance(v, tuple) else v.cuda() for k, v in args.items()}
@@ -72,13 +75,14 @@ def _segment(lens, starts, P, slots=None, decode=False, shuffle=True):
     return ops.Segment(
         rows=slice(0, cu[-1]), block_tables=bt, context_lens=i32(ctx), starts=i32(starts),
         state_slots=i32(slots if slots is not None else list(range(len(lens)))),
-        cu=None if decode else i32(cu), cu_host=None if decode else cu), sum(need)
+        cu=None if decode else i32(cu), cu_host=None if decode else cu,
+        ctx_host=ctx), sum(need)
 
 
 def _to(seg, dev):
     mv = lambda t: None if t is None else t.to(dev)  # noqa: E731
     return ops.Segment(seg.rows, mv(seg.block_tables), mv(seg.context_lens), mv(seg.starts),
-                       mv(seg.state_slots), mv(seg.cu), seg.cu_host)
+                       mv(seg.state_slots), mv(seg.cu), seg.cu_host, seg.ctx_host)
 
 
 ATTN = [  # heads, kv_heads, dim, vdim, window
@@ -214,3 +218,143 @@ def test_routed_experts(dtype, T, W, F, E, top):
     yg, pg = m.moe_clamped_glu(*gpu(h), sel.cuda(), *gpu(gu, dn), 0.9, 1.702)
     assert sorted(pg.flatten().tolist()) == list(range(T * top))
     close(yg.cpu()[pg.cpu().long()], y[place.long()], dtype)
+
+
+# ------------------------------------- embeddings, input convolution, activation
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W", [320, 50])
+def test_embed_pairs(dtype, W):
+    V, B = 200, 31
+    table, pairs, w = rnd(V, W, dtype=dtype), rnd(B + 1, W, dtype=dtype), rnd(W)
+    prev = torch.randint(0, V, (6, 1), dtype=torch.int32)
+    pg = prev.cuda()
+    # factors whose products leave 32 bits behind
+    mul = (2 ** 33 + 7, 2 ** 31 - 1)
+    for lens, starts, slots, dec in (
+            ([37, 2, 16, 1, 2], [0, 5, 100, 0, 1], [4, 0, 2, 5, 1], False),
+            ([1, 1, 1, 1], [37, 7, 0, 0], [4, 0, -1, 3], True)):
+        seg, _ = _segment(lens, starts, 64, slots, dec)
+        ids = torch.randint(0, V, (sum(lens),))
+        want = ops.embed_pairs(ids, table, 3.5, pairs, *mul, w, 1e-5, prev, [seg])
+        got = ops.embed_pairs(ids.cuda(), table.cuda(), 3.5, pairs.cuda(), *mul, w.cuda(),
+                              1e-5, pg, [_to(seg, "cuda")])
+        close(got, want, torch.float32)
+        assert torch.equal(pg.cpu(), prev)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("W", [320, 50, 2056])
+@pytest.mark.parametrize("taps", [1, 2, 3, 4, 5, 6, 7, 16])
+def test_short_conv_and_its_fused_form(dtype, W, taps):
+    w, nw = rnd(W, taps, scale=0.5), rnd(W)
+    ring = rnd(6, taps - 1, W, dtype=dtype)
+    rg = ring.cuda()
+    for lens, starts, slots, dec in (
+            ([37, 2, 16, 1, 33], [0, 5, 100, 0, 2], [4, 0, 2, 5, 1], False),
+            ([1, 1, 1, 1], [37, 7, 116, 1], [4, 0, 2, 5], True),
+            ([1, 1, 1, 1], [38, 8, 0, 0], [4, 0, -1, 3], True)):
+        seg, _ = _segment(lens, starts, 64, slots, dec)
+        x = rnd(sum(lens), W)
+        delta, gate = rnd(*x.shape, dtype=dtype), (rnd(*x.shape, dtype=dtype), rnd(W))
+        xg = x.cuda()
+        kw = dict(dtype=dtype, offset=0.0)
+        h, u = ops.residual_rmsnorm_conv(x, nw, 1e-5, w, ring, [seg], delta=delta, gate=gate, **kw)
+        hg, ug = ops.residual_rmsnorm_conv(
+            xg, nw.cuda(), 1e-5, w.cuda(), rg, [_to(seg, "cuda")], delta=delta.cuda(),
+            gate=(gate[0].cuda(), gate[1].cuda()), **kw)
+        close(hg, h, dtype)
+        close(ug, u, dtype)
+        close(rg, ring, dtype) if taps > 1 else None
+        rg.copy_(ring)  # the next step starts from equal pasts
+    # portions beside single tokens: one segment after the other
+    seg, _ = _segment([20, 3], [0, 9], 64, [1, 2])
+    one, _ = _segment([1, 1], [4, 30], 64, [3, 0], True)
+    one.rows = slice(23, 25)
+    x = rnd(25, W)
+    xg = x.cuda()
+    h, u = ops.residual_rmsnorm_conv(x, nw, 1e-5, w, ring, [seg, one], **kw)
+    hg, ug = ops.residual_rmsnorm_conv(xg, nw.cuda(), 1e-5, w.cuda(), rg,
+                                       [_to(seg, "cuda"), _to(one, "cuda")], **kw)
+    close(ug, u, dtype)
+    close(rg, ring, dtype) if taps > 1 else None
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("F", [256, 36])
+def test_xielu(dtype, F):
+    z = torch.cat([rnd(9, F), rnd(9, F, scale=1e-3), rnd(9, F, scale=30.0)]).to(dtype)
+    wide = torch.cat([z, z], 1)
+    for act in ([0.3, -0.7], [-40.0, 30.0]):
+        a = torch.tensor(act)
+        want = ops.xielu(z.float(), a).to(dtype)
+        close(ops.xielu(wide.cuda()[:, F:], a.cuda()), want, dtype)
+        close(ops.xielu(z.cuda(), a.cuda()), want, dtype)
+
+
+# ---------------------------------------------------------- latent attention
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,H,K,N", [(1, 3, 64, 128), (17, 2, 512, 64), (40, 5, 256, 96),
+                                     (64, 1, 32, 32), (150, 4, 128, 512), (70, 2, 320, 128)])
+def test_head_linear(dtype, T, H, K, N):
+    x, w = rnd(T, 8 + H * K, dtype=dtype), rnd(H, N, K, dtype=dtype, scale=K ** -0.5)
+    gate = rnd(T, H + 2, dtype=dtype)[:, :H]
+    xh = x[:, 8:].unflatten(1, (H, K))
+    want = torch.einsum("thk,hnk->thn", xh.float(), w.float())
+    xg = x.cuda()[:, 8:].unflatten(1, (H, K))
+    close(sequence.head_linear(xg, w.cuda()), want, dtype)
+    out = torch.zeros(T, H * N, dtype=dtype, device="cuda")
+    sequence.head_linear(xg, w.cuda(), gate.cuda(), out.unflatten(1, (H, N)))
+    close(out.cpu().unflatten(1, (H, N)), want * torch.sigmoid(gate.float()).unsqueeze(-1), dtype)
+
+
+LATENT = [  # heads, dim, vdim, rank
+    (4, 64, 64, 128), (3, 20, 100, 50), (16, 128, 128, 512), (17, 64, 128, 256),
+    (40, 128, 64, 300), (1, 160, 72, 384), (6, 32, 32, 520), (2, 128, 128, 700), (33, 40, 24, 64)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,d,e,rank", LATENT)
+@pytest.mark.parametrize("regime", ["decode", "portions", "long", "many"])
+def test_latent_attention(dtype, H, d, e, rank, regime, monkeypatch):
+    """Padded sizes as the mixer makes them; each regime's own form, and for
+    portions both."""
+    P = 48
+    decode = regime in ("decode", "many")
+    lens, starts = {"decode": ([1] * 4, [0, 63, 500, 129]),
+                    "many": ([1] * 70, [(37 * i) % 200 for i in range(70)]),
+                    "portions": ([2, 33, 7, 64], [300, 129, 0, 31]),
+                    "long": ([200, 300], [0, 70])}[regime]
+    seg, pages = _segment(lens, starts, P, decode=decode)
+    T, R = sum(lens), ops.latent_width(rank)
+    D, E = ops.latent_head_width(d), ops.latent_head_width(e)
+    cache = torch.zeros(pages, 1, P, R, dtype=dtype)
+    cache[..., :rank] = rnd(pages, 1, P, rank, dtype=dtype)
+    c0 = H * D
+    g0 = c0 + -(-rank // 8) * 8
+    proj = rnd(T, g0 + -(-H // 8) * 8, dtype=dtype)
+    w = rnd(rank)
+    slots = torch.tensor([int(seg.block_tables[s, p // P]) * P + p % P
+                          for s in range(len(lens))
+                          for p in range(starts[s], starts[s] + lens[s])], dtype=torch.int32)
+    cg = cache.cuda()
+    ops.latent_write(proj, c0, rank, w, 1e-5, slots, cache)
+    ops.latent_write(proj.cuda(), c0, rank, w.cuda(), 1e-5, slots.cuda(), cg)
+    close(cg, cache, dtype)
+    cg.copy_(cache)
+    uk, uv = torch.zeros(H, D, R, dtype=dtype), torch.zeros(H, E, R, dtype=dtype)
+    uk[:, :d, :rank] = rnd(H, d, rank, dtype=dtype, scale=rank ** -0.5)
+    uv[:, :e, :rank] = rnd(H, e, rank, dtype=dtype, scale=rank ** -0.5)
+    p = ops.LatentParams(H, D, E, 2.0 * d ** -0.5, 0, g0, uk,
+                         uk.transpose(1, 2).contiguous(), uv, rnd(H, scale=2.0))
+    out = torch.zeros(T, H * E, dtype=dtype)
+    ops.latent_attention(proj, p, cache, seg, out)
+    pg, sg = _params_to(p, "cuda"), _to(seg, "cuda")
+    for expand in [False] if decode else [False, True]:
+        if expand and (D > 128 or E > 128 or R not in sequence.MATRIX_LATENT_WIDTHS):
+            continue
+        monkeypatch.setattr(sequence, "expand_latents", lambda *a: expand)
+        og = torch.zeros(T, H * E, dtype=dtype, device="cuda")
+        ops.latent_attention(proj.cuda(), pg, cg, sg, og)
+        close(og, out, dtype)
