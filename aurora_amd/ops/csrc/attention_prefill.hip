@@ -68,7 +68,7 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   // the 128-B row)
   constexpr int SWZ = (D / 8) - 1;
   constexpr int QS = 8 / HG;          // 32-row q sub-blocks per WG
-  const int nb = blockIdx.x;
+  const int nb = gridDim.x - 1 - blockIdx.x;  // late rows see most keys: first
   const int seq = block_seq[nb];
   const int qoff = block_qoff[nb];
   const int q_start = cu_q[seq];

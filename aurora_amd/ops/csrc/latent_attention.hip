@@ -14,23 +14,34 @@
 //  * every wave loads its own 16 latents of the next tile straight to LDS while
 //    the tile before is computed, and scores them: S^T = C Q^T, the rows'
 //    queries live in registers as B fragments;
-//  * the tile's row maxima and the bf16 weights go through LDS (two barriers a
-//    tile), then every wave owns R / 4 columns of O += P C. The value fragments
-//    are columns of the row-major tile: ds_read_b64_tr_b16 transposes on the
-//    way to the registers. Contraction slot 8 g + j holds key 4 g + j (j < 4)
-//    or 16 + 4 g + j - 4, on both operands, so the eight rows two lane groups
-//    read at a time are consecutive;
-//  * LDS rows are unpadded (direct loads fill them in lane order); 16-byte units
-//    are permuted within a row by unit_swizzle, applied to the source address.
+//  * the bf16 weights go through LDS (one barrier a tile), then every wave owns
+//    R / 4 columns of O += P C. The value fragments are columns of the row-major
+//    tile: ds_read_b64_tr_b16 transposes on the way to the registers.
+//    Contraction slot 8 g + j holds key 4 g + j (j < 4) or 16 + 4 g + j - 4, on
+//    both operands;
+//  * a wave's 16 latents lie in LDS as R / 32 blocks of [16 rows][64 bytes], so
+//    that one load fills a block, a lane's source moves by 64 bytes from load to
+//    load, a score fragment is a block read in order, and all reads of a tile
+//    are one address plus constants. In rows 4-7 and 12-15 the two halves of the
+//    64 bytes change places, which spreads the column reads over all banks;
+//  * weights are taken against a reference that need not be the maximum: it only
+//    moves, and only then the waves exchange maxima and rescale O, when a score
+//    exceeds it by more than LAT_SLACK, so weights stay below 2^LAT_SLACK.
 // Few rows: the context is split over blockIdx.y, partial sums are merged by
 // latent_combine_kernel. A row's softmax starts from its sink (split 0 only).
+// Scores, maxima and sinks are in units of log 2.
 #include "elem.h"
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 
+#include <type_traits>
+
 #define CUR_STREAM c10::hip::getCurrentHIPStream().stream()
 #define LAT_KEYS 64                    // latents per tile
 #define LAT_PSTRIDE (LAT_KEYS + 8)     // row stride of the weights in LDS
+#define LAT_SLACK 10.f
+#define LAT_SPLITS 128                 // most parts of a context
+#define LOG2E 1.44269504f
 
 union lfrag {
   shortx8 s;
@@ -38,35 +49,56 @@ union lfrag {
   bf16x8 v;
 };
 
-// XOR of a row's 16-byte unit index: 16 rows at one unit, and 8 rows at two
-// neighbouring units, fall into distinct banks
-template <int U>
-DEVINL int unit_swizzle(int row) {
-  return U == 8 ? (((row >> 1) & 3) << 1) | ((row >> 3) & 1)
-                : ((row & 7) << 1) | ((row >> 3) & 1);
+template <int N, typename F>
+DEVINL void static_for(F&& f) {
+  if constexpr (N > 0) {
+    static_for<N - 1>(f);
+    f(std::integral_constant<int, N - 1>{});
+  }
 }
 
-// Transposing reads of the four 16-row slices (STEP bytes apart) of one 16-column
-// tile; then wait until the slices requested before these have arrived. Written
-// out because the compiler puts a wait for all global loads in flight, the next
-// tile's among them, before the builtin form of these reads.
-template <int STEP>
-DEVINL void read_columns(shortx4 (&next)[4], shortx4 (&ready)[4], unsigned addr) {
+// Reads of two neighbouring blocks; then wait until the two before have arrived.
+template <int AT>
+DEVINL void read_blocks(shortx8& a, shortx8& b, shortx8& ready_a, shortx8& ready_b,
+                        unsigned addr) {
   asm volatile(
-      "ds_read_b64_tr_b16 %0, %8\n\t"
-      "ds_read_b64_tr_b16 %1, %8 offset:%9\n\t"
-      "ds_read_b64_tr_b16 %2, %8 offset:%10\n\t"
-      "ds_read_b64_tr_b16 %3, %8 offset:%11\n\t"
-      "s_waitcnt lgkmcnt(4)"
-      : "=&v"(next[0]), "=&v"(next[1]), "=&v"(next[2]), "=&v"(next[3]), "+v"(ready[0]),
-        "+v"(ready[1]), "+v"(ready[2]), "+v"(ready[3])
-      : "v"(addr), "n"(STEP), "n"(2 * STEP), "n"(3 * STEP)
+      "ds_read_b128 %0, %4 offset:%5\n\t"
+      "ds_read_b128 %1, %4 offset:%6\n\t"
+      "s_waitcnt lgkmcnt(2)"
+      : "=&v"(a), "=&v"(b), "+v"(ready_a), "+v"(ready_b)
+      : "v"(addr), "n"(AT), "n"(AT + 1024)
       : "memory");
 }
 
+DEVINL void await_blocks(shortx8& a, shortx8& b) {
+  asm volatile("s_waitcnt lgkmcnt(0)" : "+v"(a), "+v"(b)::"memory");
+}
+
+// Transposing reads of the four 16-row slices (STEP bytes apart) of one 16-column
+// tile; then wait until the slices requested two calls before have arrived.
+// Written out because the compiler puts a wait for all global loads in flight,
+// the next tile's among them, before the builtin form of these reads.
+template <int AT, int STEP>
+DEVINL void read_columns(shortx4 (&next)[4], shortx4 (&ready)[4], unsigned addr) {
+  asm volatile(
+      "ds_read_b64_tr_b16 %0, %8 offset:%9\n\t"
+      "ds_read_b64_tr_b16 %1, %8 offset:%10\n\t"
+      "ds_read_b64_tr_b16 %2, %8 offset:%11\n\t"
+      "ds_read_b64_tr_b16 %3, %8 offset:%12\n\t"
+      "s_waitcnt lgkmcnt(8)"
+      : "=&v"(next[0]), "=&v"(next[1]), "=&v"(next[2]), "=&v"(next[3]), "+v"(ready[0]),
+        "+v"(ready[1]), "+v"(ready[2]), "+v"(ready[3])
+      : "v"(addr), "n"(AT), "n"(AT + STEP), "n"(AT + 2 * STEP), "n"(AT + 3 * STEP)
+      : "memory");
+}
+
+// the slices requested PENDING calls before the last have arrived
+template <int PENDING>
 DEVINL void await_columns(shortx4 (&ready)[4]) {
-  asm volatile("s_waitcnt lgkmcnt(0)"
-               : "+v"(ready[0]), "+v"(ready[1]), "+v"(ready[2]), "+v"(ready[3])::"memory");
+  asm volatile("s_waitcnt lgkmcnt(%4)"
+               : "+v"(ready[0]), "+v"(ready[1]), "+v"(ready[2]), "+v"(ready[3])
+               : "n"(4 * PENDING)
+               : "memory");
 }
 
 template <int R, int MT>
@@ -80,27 +112,71 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
     float* __restrict__ part,          // [CS, T * H, R] (several)
     float* __restrict__ part_ml,       // [CS, T * H, 2]
     int H, int P, long rows_all, float scale) {
-  constexpr int U = R / 8;             // 16-byte units per latent
   constexpr int NT = R / 64;           // 16-column tiles of O per wave
   constexpr int ROWS = 16 * MT;
+  constexpr int SLICE = 16 * R * 2;    // bytes of a wave's 16 latents
+  constexpr int TILE = 4 * SLICE;
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  short* pbuf = (short*)(smem + 2 * LAT_KEYS * R * 2);
-  float* stat = (float*)(smem + 2 * LAT_KEYS * R * 2 + ROWS * LAT_PSTRIDE * 2);  // [4][ROWS]
+  short* pbuf = (short*)(smem + 2 * TILE);  // [2][ROWS][LAT_PSTRIDE]
+  float* stat = (float*)(smem + 2 * TILE + 2 * ROWS * LAT_PSTRIDE * 2);  // [4][ROWS]
+  float* exceed = stat + 4 * ROWS;          // [2][4]: 1 where a wave saw a score too high
 
-  const int tid = threadIdx.x, wave = tid / WAVE, lane = tid % WAVE;
+  const int tid = threadIdx.x, lane = tid % WAVE;
+  const int wave = __builtin_amdgcn_readfirstlane(tid / WAVE);
   const int col = lane & 15, g = lane >> 4;
   const int tiles_per_seq = (H + ROWS - 1) / ROWS;  // single tokens
-  const int seq = cu ? bseq[blockIdx.x] : blockIdx.x / tiles_per_seq;
-  const int off = cu ? boff[blockIdx.x] : blockIdx.x % tiles_per_seq * ROWS;
+  const int nb = gridDim.x - 1 - blockIdx.x;  // a portion's late rows see most: first
+  const int seq = cu ? bseq[nb] : nb / tiles_per_seq;
+  const int off = cu ? boff[nb] : nb % tiles_per_seq * ROWS;
   const int n = cu ? cu[seq + 1] - cu[seq] : 1;
   const long row0 = (long)(cu ? cu[seq] : seq) * H + off;
   const int nrows = min(ROWS, n * H - off);
   const int start = ctx[seq] - n;
+  const int first_pos = start + off / H;
   const int kend = start + (off + nrows - 1) / H + 1;  // keys any row here sees
   const int ntiles = (kend + LAT_KEYS - 1) / LAT_KEYS;
   const int per = (ntiles + gridDim.y - 1) / gridDim.y;
   const int tile0 = blockIdx.y * per, tile1 = min(ntiles, tile0 + per);
   const int* pages = bt + (long)seq * MP;
+  const float scale2 = scale * LOG2E;
+
+  // this lane's latent of the next tile to look up (four lanes share one), as
+  // page and place; past the end the last one again. Pages are looked up a tile
+  // ahead of the loads that need them.
+  const int last_pg = (kend - 1) / P, last_in = (kend - 1) % P;
+  const int step_pg = LAT_KEYS / P, step_in = LAT_KEYS % P;
+  int key = tile0 * LAT_KEYS + wave * 16 + (lane >> 2), pg = key / P, in = key % P;
+  int page = 0, in_page = 0;
+  auto lookup = [&]() {
+    const bool past = key >= kend;
+    page = pages[past ? last_pg : pg];
+    in_page = past ? last_in : in;
+    key += LAT_KEYS;
+    pg += step_pg;
+    in += step_in;
+    if (in >= P) {
+      in -= P;
+      ++pg;
+    }
+  };
+  const int src_unit = (lane & 3) ^ (((lane >> 4) & 1) << 1);
+  // this wave's 16 latents of the tile looked up; the constant offset of a load
+  // moves its source and its destination
+  auto issue = [&](int tile) {
+    const bf16_t* src = cache + ((long)page * P + in_page) * R + src_unit * 8;
+    char* dst = smem + (tile & 1) * TILE + wave * SLICE;
+    static_for<R / 32>([&](auto I) {
+      constexpr int i = decltype(I)::value;
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) void*)src,
+          (__attribute__((address_space(3))) void*)(dst + i * (1024 - 64)), 16, i * 64, 0);
+    });
+    lookup();
+  };
+  if (tile0 < tile1) {
+    lookup();
+    issue(tile0);
+  }
 
   // queries (B operand: lane's row col, contraction 8 g + j), positions, sinks
   lfrag qf[MT][R / 32];
@@ -113,7 +189,7 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
 #pragma unroll
     for (int k = 0; k < R / 32; ++k) qf[t][k].s = *(const shortx8*)(src + k * 32);
     pos[t] = start + (off + r) / H;
-    m[t] = blockIdx.y == 0 ? sink[(off + r) % H] : -1e30f;
+    m[t] = blockIdx.y == 0 ? sink[(off + r) % H] * LOG2E : -1e30f;
     l[t] = blockIdx.y == 0 && wave == 0 && g == 0 ? 1.f : 0.f;
   }
   floatx4 o[MT][NT];
@@ -122,119 +198,138 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
 #pragma unroll
     for (int c = 0; c < NT; ++c) o[t][c] = floatx4{0.f, 0.f, 0.f, 0.f};
 
-  // byte offsets of the wave's columns: lane i of a group reads row i / 4, the
-  // 8 bytes i mod 4 of the 32
-  const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) char*)smem;
-  unsigned vcol[NT];
-#pragma unroll
-  for (int c = 0; c < NT; ++c) {
-    const int row = g * 4 + (col >> 2), unit = (wave * NT + c) * 2 + ((lane & 3) >> 1);
-    vcol[c] = row * R * 2 + (unit ^ unit_swizzle<U>(row)) * 16 + (lane & 1) * 8;
+  // where a lane's score fragments lie, and its pieces of the wave's columns:
+  // lane i of a group reads row i / 4 of the group's four, 8 bytes of 32
+  const unsigned smem_at = (unsigned)(size_t)(__attribute__((address_space(3))) char*)smem;
+  const unsigned score_at = smem_at + wave * SLICE + col * 64 + (g ^ (((col >> 2) & 1) << 1)) * 16;
+  unsigned vcol[2];
+  {
+    const int row = g * 4 + (col >> 2), flip = (row >> 2) & 1, ct = wave * NT;
+    const unsigned at = smem_at + ct / 2 * 1024 + row * 64 + (lane & 3) * 8;
+    vcol[0] = at + ((ct & 1) ^ flip) * 32;
+    vcol[1] = at + ((ct & 1) ^ flip ^ 1) * 32;
   }
 
-  // this wave's 16 latents of a tile; past the end the last one again
-  auto issue = [&](int tile) {
-    const int key = min(tile * LAT_KEYS + wave * 16 + col, kend - 1);
-    const int slot = pages[key / P] * P + key % P;
-    char* dst = smem + (tile & 1) * (LAT_KEYS * R * 2) + wave * 16 * R * 2;
+  auto score = [&](floatx4 (&st)[MT], shortx8 a, shortx8 b, int k) {
+    lfrag fa, fb;
+    fa.s = a;
+    fb.s = b;
 #pragma unroll
-    for (int i = 0; i < R / 32; ++i) {
-      const int id = i * WAVE + lane, row = id / U, unit = id % U;
-      const long s = __shfl(slot, row, WAVE);
-      __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) void*)(
-              cache + s * R + (unit ^ unit_swizzle<U>(row)) * 8),
-          (__attribute__((address_space(3))) void*)(dst + id * 16), 16, 0, 0);
-    }
+    for (int t = 0; t < MT; ++t)
+      st[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa.v, qf[t][k].v, st[t], 0, 0, 0);
+#pragma unroll
+    for (int t = 0; t < MT; ++t)
+      st[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fb.v, qf[t][k + 1].v, st[t], 0, 0, 0);
   };
 
-  if (tile0 < tile1) issue(tile0);
   for (int tile = tile0; tile < tile1; ++tile) {
-    const char* cb = smem + (tile & 1) * (LAT_KEYS * R * 2);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    const int buf = (tile & 1) * TILE;
+    asm volatile("s_waitcnt vmcnt(0)" : "+v"(page)::"memory");
     // scores of the wave's own keys: S^T rows 4 g + r, columns are query rows
     floatx4 st[MT];
 #pragma unroll
     for (int t = 0; t < MT; ++t) st[t] = floatx4{0.f, 0.f, 0.f, 0.f};
-    const char* krow = cb + (wave * 16 + col) * R * 2;
-#pragma unroll
-    for (int k = 0; k < R / 32; ++k) {
-      lfrag kf;
-      kf.s = *(const shortx8*)(krow + ((k * 4 + g) ^ unit_swizzle<U>(col)) * 16);
-#pragma unroll
-      for (int t = 0; t < MT; ++t)
-        st[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf.v, qf[t][k].v, st[t], 0, 0, 0);
-    }
+    const unsigned krow = score_at + buf;
+    shortx8 kf[(R / 64 + 1) * 2];  // block k is kf[k + 2]
+    kf[0] = kf[1] = shortx8{};
+    static_for<R / 64>([&](auto K) {
+      constexpr int k = decltype(K)::value * 2;
+      read_blocks<k * 1024>(kf[k + 2], kf[k + 3], kf[k], kf[k + 1], krow);
+      if constexpr (k > 0) score(st, kf[k], kf[k + 1], k - 2);
+    });
+    await_blocks(kf[R / 32], kf[R / 32 + 1]);
+    score(st, kf[R / 32], kf[R / 32 + 1], R / 32 - 2);
+    const bool some_hidden = tile * LAT_KEYS + LAT_KEYS - 1 > first_pos;
     const int key0 = tile * LAT_KEYS + wave * 16 + g * 4;
+    short* pb = pbuf + (tile & 1) * (ROWS * LAT_PSTRIDE);
 #pragma unroll
     for (int t = 0; t < MT; ++t) {
-      float mx = -1e30f;
+      st[t] *= scale2;
+      if (some_hidden)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        st[t][r] = key0 + r <= pos[t] ? st[t][r] * scale : -1e30f;
-        mx = fmaxf(mx, st[t][r]);
-      }
-      mx = fmaxf(mx, __shfl_xor(mx, 16, WAVE));
-      mx = fmaxf(mx, __shfl_xor(mx, 32, WAVE));
-      if (g == 0) stat[wave * ROWS + t * 16 + col] = mx;
+        for (int r = 0; r < 4; ++r)
+          if (key0 + r > pos[t]) st[t][r] = -INFINITY;
     }
-    // the whole tile has landed, and nobody reads the other buffer any more
+    auto weigh = [&](int t) {  // stores the weights, returns their sum
+      floatx4 p;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) p[r] = __builtin_amdgcn_exp2f(st[t][r] - m[t]);
+      *(bf16x4*)(pb + (t * 16 + col) * LAT_PSTRIDE + wave * 16 + g * 4) =
+          __builtin_convertvector(p, bf16x4);
+      return (p[0] + p[1]) + (p[2] + p[3]);
+    };
+    float mx[MT], sum[MT];
+    bool high = false;
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+      mx[t] = fmaxf(fmaxf(st[t][0], st[t][1]), fmaxf(st[t][2], st[t][3]));
+      high = high || mx[t] > m[t] + LAT_SLACK;
+      sum[t] = weigh(t);
+    }
+    float* flag = exceed + (tile & 1) * 4;
+    const float too_high = __any(high) ? 1.f : 0.f;
+    if (lane == 0) flag[wave] = too_high;
+    // the whole tile and its weights are there, and nobody reads the other buffer
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
     if (tile + 1 < tile1) issue(tile + 1);
+    if (__any((flag[0] + flag[1]) + (flag[2] + flag[3]) > 0.f)) {
+      // all waves: move the references to the largest scores so far
 #pragma unroll
-    for (int t = 0; t < MT; ++t) {
-      float mn = m[t];
-#pragma unroll
-      for (int w = 0; w < 4; ++w) mn = fmaxf(mn, stat[w * ROWS + t * 16 + col]);
-      const float alpha = __expf(m[t] - mn);
-      m[t] = mn;
-      floatx4 p;
-      float sum = 0.f;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        p[r] = key0 + r <= pos[t] ? __expf(st[t][r] - mn) : 0.f;
-        sum += p[r];
+      for (int t = 0; t < MT; ++t) {
+        mx[t] = fmaxf(mx[t], __shfl_xor(mx[t], 16, WAVE));
+        mx[t] = fmaxf(mx[t], __shfl_xor(mx[t], 32, WAVE));
+        if (g == 0) stat[wave * ROWS + t * 16 + col] = mx[t];
       }
-      l[t] = l[t] * alpha + sum;
-      st4((bf16_t*)pbuf + (t * 16 + col) * LAT_PSTRIDE + wave * 16 + g * 4, p);
-      if (__any(alpha < 1.f)) {
+      asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+#pragma unroll
+      for (int t = 0; t < MT; ++t) {
+        float mn = m[t];
+#pragma unroll
+        for (int w = 0; w < 4; ++w) mn = fmaxf(mn, stat[w * ROWS + t * 16 + col]);
+        const float alpha = __builtin_amdgcn_exp2f(m[t] - mn);
+        m[t] = mn;
+        l[t] *= alpha;
         floatx4 av;
 #pragma unroll
         for (int r = 0; r < 4; ++r) av[r] = __shfl(alpha, g * 4 + r, WAVE);
 #pragma unroll
         for (int c = 0; c < NT; ++c) o[t][c] *= av;
+        sum[t] = weigh(t);
       }
+      asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
     }
-    asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+#pragma unroll
+    for (int t = 0; t < MT; ++t) l[t] += sum[t];
     lfrag pf[2][MT];
 #pragma unroll
     for (int kk = 0; kk < 2; ++kk)
 #pragma unroll
       for (int t = 0; t < MT; ++t) {
-        const short* pr = pbuf + (t * 16 + col) * LAT_PSTRIDE + kk * 32 + g * 4;
+        const short* pr = pb + (t * 16 + col) * LAT_PSTRIDE + kk * 32 + g * 4;
         pf[kk][t].h[0] = *(const shortx4*)pr;
         pf[kk][t].h[1] = *(const shortx4*)(pr + 16);
       }
     // slice 2 kk + j holds contraction slots 8 g + 4 j ..+3 of step kk
-    const unsigned tile_at = lds0 + (tile & 1) * (LAT_KEYS * R * 2);
-    shortx4 cols[NT + 1][4] = {};
-    read_columns<16 * R * 2>(cols[1], cols[0], tile_at + vcol[0]);
-#pragma unroll
-    for (int c = 0; c < NT; ++c) {
-      if (c + 1 < NT)
-        read_columns<16 * R * 2>(cols[c + 2], cols[c + 1], tile_at + vcol[c + 1]);
+    const unsigned va[2] = {vcol[0] + buf, vcol[1] + buf};
+    shortx4 cols[NT + 2][4] = {};  // tile c is cols[c + 2]
+    read_columns<0, SLICE>(cols[2], cols[0], va[0]);
+    if constexpr (NT > 1) read_columns<0, SLICE>(cols[3], cols[1], va[1]);
+    static_for<NT>([&](auto C) {
+      constexpr int c = decltype(C)::value;
+      if constexpr (c + 2 < NT)
+        read_columns<(c + 2) / 2 * 1024, SLICE>(cols[c + 4], cols[c + 2], va[c & 1]);
       else
-        await_columns(cols[c + 1]);
+        await_columns<NT - 1 - c>(cols[c + 2]);
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
         lfrag cf;
-        cf.h[0] = cols[c + 1][2 * kk];
-        cf.h[1] = cols[c + 1][2 * kk + 1];
+        cf.h[0] = cols[c + 2][2 * kk];
+        cf.h[1] = cols[c + 2][2 * kk + 1];
 #pragma unroll
         for (int t = 0; t < MT; ++t)
           o[t][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[kk][t].v, cf.v, o[t][c], 0, 0, 0);
       }
-    }
+    });
   }
 
   // the waves' sums of weights
@@ -262,17 +357,18 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
           stf(ob + row * R + (wave * NT + c) * 16 + col, o[t][c][r] * inv);
       }
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-    for (int i = tid; i < nrows * U; i += 256)
+    for (int i = tid; i < nrows * (R / 8); i += 256)
       *(shortx8*)(out + row0 * R + (long)i * 8) = *(const shortx8*)(ob + i * 8);
     return;
   }
+  // (a split without keys has no sums, and nobody reads any)
   const long prow = blockIdx.y * rows_all + row0;
 #pragma unroll
   for (int t = 0; t < MT; ++t)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int row = t * 16 + g * 4 + r;
-      if (row >= nrows) continue;
+      if (row >= nrows || tile0 >= tile1) continue;
 #pragma unroll
       for (int c = 0; c < NT; ++c)
         part[(prow + row) * R + (wave * NT + c) * 16 + col] = o[t][c][r];
@@ -290,27 +386,40 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
     }
 }
 
-// merge the context splits: one wave per row
+// merge the context splits: one workgroup per row, R / 4 threads each on some of
+// the splits
 __global__ __launch_bounds__(256) void latent_combine_kernel(
     const float* __restrict__ part, const float* __restrict__ part_ml,
     bf16_t* __restrict__ out, long rows, int CS, int R) {
-  const long row = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
-  if (row >= rows) return;
-  const int lane = threadIdx.x % WAVE;
-  float M = -1e30f, L = 0.f;
-  for (int s = 0; s < CS; ++s) M = fmaxf(M, part_ml[(s * rows + row) * 2]);
-  for (int s = 0; s < CS; ++s) {
-    const float* ml = part_ml + (s * rows + row) * 2;
-    L += __expf(ml[0] - M) * ml[1];
+  __shared__ float weight[LAT_SPLITS];
+  __shared__ __attribute__((aligned(16))) float sums[1024];
+  __shared__ float red[4];
+  const long row = blockIdx.x;
+  const int tid = threadIdx.x, wave = tid / WAVE;
+  float m = -1e30f, l = 0.f;
+  if (tid < CS) {
+    m = part_ml[(tid * rows + row) * 2];
+    l = part_ml[(tid * rows + row) * 2 + 1];
   }
-  const float inv = 1.f / L;
-  for (int d = lane * 4; d < R; d += WAVE * 4) {
-    floatx4 a = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < CS; ++s)
-      a += ld4(part + (s * rows + row) * R + d) *
-           (__expf(part_ml[(s * rows + row) * 2] - M) * inv);
-    st4(out + row * R + d, a);
+  float M = wave_max(m);
+  if (tid % WAVE == 0) red[wave] = M;
+  __syncthreads();
+  M = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+  const float w = __builtin_amdgcn_exp2f(m - M);
+  if (tid < CS) weight[tid] = l != 0.f ? w : 0.f;  // a split without keys left no sums
+  const float L = block_sum4(w * l, red);
+  const int per = R / 4, groups = 256 / per, grp = tid / per, d = tid % per * 4;
+  floatx4 a = {0.f, 0.f, 0.f, 0.f};
+  if (grp < groups) {
+#pragma unroll 4
+    for (int s = grp; s < CS; s += groups)
+      if (weight[s] != 0.f) a += ld4(part + (s * rows + row) * R + d) * weight[s];
+    *(floatx4*)(sums + grp * R + d) = a;
   }
+  __syncthreads();
+  if (grp != 0) return;
+  for (int i = 1; i < groups; ++i) a += *(const floatx4*)(sums + i * R + d);
+  st4(out + row * R + d, a * (1.f / L));
 }
 
 torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tensor bt,
@@ -340,8 +449,8 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
   }
   auto out = torch::empty_like(q);
   if (T == 0 || blocks == 0) return out;
-  // one workgroup per CU
-  const int CS = std::max(1, std::min(32, 256 / blocks));
+  // one workgroup per CU, or as many as its LDS holds
+  const int CS = std::max(1, std::min(LAT_SPLITS, (R > 256 ? 256 : 512) / blocks));
   const long all = (long)T * H;
   torch::Tensor part, ml;
   if (CS > 1) {
@@ -351,7 +460,8 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
 #define LATENT(RR, MT)                                                                   \
   do {                                                                                   \
     auto kern = latent_attention_kernel<RR, MT>;                                         \
-    constexpr int lds = 2 * LAT_KEYS * RR * 2 + 16 * MT * LAT_PSTRIDE * 2 + 4 * 16 * MT * 4; \
+    constexpr int lds = 2 * LAT_KEYS * RR * 2 + \
+                        2 * 16 * MT * LAT_PSTRIDE * 2 + 4 * 16 * MT * 4 + 32;              \
     static const hipError_t once = hipFuncSetAttribute(                                  \
         (const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds);             \
     TORCH_CHECK(once == hipSuccess, "LDS of the latent attention kernel");               \
@@ -373,7 +483,7 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
 #undef LATENT_R
 #undef LATENT
   if (CS > 1)
-    hipLaunchKernelGGL(latent_combine_kernel, dim3((all + 3) / 4), dim3(256), 0, CUR_STREAM,
+    hipLaunchKernelGGL(latent_combine_kernel, dim3(all), dim3(256), 0, CUR_STREAM,
                        part.data_ptr<float>(), ml.data_ptr<float>(), (bf16_t*)out.data_ptr(),
                        all, CS, R);
   HIP_CHECK_KERNEL();
@@ -383,7 +493,7 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
 // ------------------------------------------------------------------ latents
 
 // norm of a token's latent in fp32 and its place in the cache: one wave per token
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void latent_write_kernel(
     const T* __restrict__ proj, long stride, int rank, const float* __restrict__ weight,
     float eps, const int* __restrict__ slots, T* __restrict__ cache, int T_, int R) {
@@ -393,15 +503,28 @@ __global__ __launch_bounds__(256) void latent_write_kernel(
   const int slot = slots[t];
   if (slot < 0) return;
   const T* src = proj + t * stride;
+  T* dst = cache + (long)slot * R;
   float ss = 0.f;
-  for (int i = lane; i < rank; i += WAVE) {
-    const float v = ldf(src + i);
-    ss += v * v;
+  for (int i = lane * V; i < rank; i += WAVE * V) {
+    if constexpr (V == 4) {
+      const floatx4 v = ld4(src + i);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss += v[j] * v[j];
+    } else {
+      const float v = ldf(src + i);
+      ss += v * v;
+    }
   }
   const float inv = rsqrtf(wave_sum(ss) / rank + eps);
-  T* dst = cache + (long)slot * R;
-  for (int i = lane; i < R; i += WAVE)
-    stf(dst + i, i < rank ? ldf(src + i) * inv * weight[i] : 0.f);
+  for (int i = lane * V; i < R; i += WAVE * V) {
+    if constexpr (V == 4) {
+      floatx4 y = {0.f, 0.f, 0.f, 0.f};
+      if (i < rank) y = ld4(src + i) * inv * ld4(weight + i);
+      st4(dst + i, y);
+    } else {
+      stf(dst + i, i < rank ? ldf(src + i) * inv * weight[i] : 0.f);
+    }
+  }
 }
 
 void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight, double eps,
@@ -414,10 +537,16 @@ void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight,
   TORCH_CHECK(slots.numel() == T_ && slots.dtype() == torch::kInt32);
   if (T_ == 0) return;
   DISPATCH_ELEM(proj.dtype() == torch::kBFloat16, {
-    hipLaunchKernelGGL((latent_write_kernel<T>), dim3((T_ + 3) / 4), dim3(256), 0, CUR_STREAM,
-                       (const T*)proj.data_ptr() + col, proj.stride(0), (int)rank,
-                       weight.data_ptr<float>(), (float)eps, slots.data_ptr<int>(),
-                       (T*)cache.data_ptr(), T_, R);
+    auto launch = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3((T_ + 3) / 4), dim3(256), 0, CUR_STREAM,
+                         (const T*)proj.data_ptr() + col, proj.stride(0), (int)rank,
+                         weight.data_ptr<float>(), (float)eps, slots.data_ptr<int>(),
+                         (T*)cache.data_ptr(), T_, R);
+    };
+    const bool vec = ((rank | col | proj.stride(0) | R) & 3) == 0 &&
+                     (reinterpret_cast<uintptr_t>(proj.data_ptr()) & 15) == 0;
+    if (vec) launch(latent_write_kernel<T, 4>);
+    else launch(latent_write_kernel<T, 1>);
   });
   HIP_CHECK_KERNEL();
 }
@@ -426,13 +555,14 @@ void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight,
 
 // out[t, h, n] = sum_k x[t, h, k] w[h, n, k], times sigmoid(gate[t, h]). Waves
 // take 16 outputs each (KS 1) or split the contraction (KS 4); TT 16-token
-// tiles per workgroup. K and N are multiples of 32.
-template <int TT, int KS>
+// tiles per workgroup. K and N are multiples of 32; STEPS: 32-wide steps of a
+// wave if known, all of whose loads are then in flight at once.
+template <int TT, int KS, int STEPS>
 __global__ __launch_bounds__(256) void head_linear_kernel(
     const bf16_t* __restrict__ x, long xt, long xh, const bf16_t* __restrict__ w,
     const bf16_t* __restrict__ gate, long gt, bf16_t* __restrict__ out, long ot, long oh,
     int T_, int N, int K) {
-  __shared__ float red[KS > 1 ? 4 : 1][TT][WAVE][4];
+  __shared__ __attribute__((aligned(16))) float red[KS > 1 ? 4 : 1][TT][WAVE][4];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, g = lane >> 4;
   const int h = blockIdx.y, t0 = blockIdx.z * 16 * TT;
@@ -440,22 +570,36 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   if (n0 >= N) return;  // KS 1 only: whole waves, no barrier follows
   const int steps = K / 32, lo = KS > 1 ? steps * wave / 4 : 0,
             hi = KS > 1 ? steps * (wave + 1) / 4 : steps;
-  const bf16_t* wp = w + ((long)h * N + n0 + col) * K + g * 8;
+  const bf16_t* wp = w + ((long)h * N + n0 + col) * K + lo * 32 + g * 8;
   const bf16_t* xp[TT];
 #pragma unroll
   for (int t = 0; t < TT; ++t)
-    xp[t] = x + min(t0 + t * 16 + col, T_ - 1) * xt + h * xh + g * 8;
+    xp[t] = x + min(t0 + t * 16 + col, T_ - 1) * xt + h * xh + lo * 32 + g * 8;
   floatx4 acc[TT];
 #pragma unroll
   for (int t = 0; t < TT; ++t) acc[t] = floatx4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k = lo; k < hi; ++k) {
-    lfrag a, b;
-    a.s = *(const shortx8*)(wp + k * 32);
+  if constexpr (STEPS > 0) {
+    lfrag a[STEPS], b[STEPS][TT];
 #pragma unroll
-    for (int t = 0; t < TT; ++t) {
-      b.s = *(const shortx8*)(xp[t] + k * 32);
-      acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, acc[t], 0, 0, 0);
+    for (int k = 0; k < STEPS; ++k) {
+      a[k].s = *(const shortx8*)(wp + k * 32);
+#pragma unroll
+      for (int t = 0; t < TT; ++t) b[k][t].s = *(const shortx8*)(xp[t] + k * 32);
+    }
+#pragma unroll
+    for (int k = 0; k < STEPS; ++k)
+#pragma unroll
+      for (int t = 0; t < TT; ++t)
+        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a[k].v, b[k][t].v, acc[t], 0, 0, 0);
+  } else {
+    for (int k = 0; k < hi - lo; ++k) {
+      lfrag a, b;
+      a.s = *(const shortx8*)(wp + k * 32);
+#pragma unroll
+      for (int t = 0; t < TT; ++t) {
+        b.s = *(const shortx8*)(xp[t] + k * 32);
+        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a.v, b.v, acc[t], 0, 0, 0);
+      }
     }
   }
   if constexpr (KS > 1) {
@@ -503,10 +647,21 @@ void head_linear(torch::Tensor x, torch::Tensor w, c10::optional<torch::Tensor> 
                        gate ? gate->stride(0) : 0, (bf16_t*)out.data_ptr(), out.stride(0),
                        out.stride(1), T_, N, K);
   };
-  // a long contraction with few outputs: split it over the waves
+  // a long contraction for few tokens: split it over the waves
   const bool split = K >= 256 && T_ <= 64;
-  if (T_ <= 16) split ? launch(head_linear_kernel<1, 4>, 1, 4) : launch(head_linear_kernel<1, 1>, 1, 1);
-  else if (T_ <= 32) split ? launch(head_linear_kernel<2, 4>, 2, 4) : launch(head_linear_kernel<2, 1>, 2, 1);
-  else split ? launch(head_linear_kernel<4, 4>, 4, 4) : launch(head_linear_kernel<4, 1>, 4, 1);
+  const int steps = K / 32 % (split ? 4 : 1) ? 0 : K / 32 / (split ? 4 : 1);
+#define HEAD_LINEAR(TT, KS)                                            \
+  do {                                                                 \
+    if (steps == 2) launch(head_linear_kernel<TT, KS, 2>, TT, KS);     \
+    else if (steps == 4) launch(head_linear_kernel<TT, KS, 4>, TT, KS); \
+    else launch(head_linear_kernel<TT, KS, 0>, TT, KS);                \
+  } while (0)
+#define HEAD_LINEAR_T(TT) \
+  do { if (split) HEAD_LINEAR(TT, 4); else HEAD_LINEAR(TT, 1); } while (0)
+  if (T_ <= 16) HEAD_LINEAR_T(1);
+  else if (T_ <= 32) HEAD_LINEAR_T(2);
+  else HEAD_LINEAR_T(4);
+#undef HEAD_LINEAR_T
+#undef HEAD_LINEAR
   HIP_CHECK_KERNEL();
 }

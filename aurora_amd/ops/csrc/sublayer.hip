@@ -17,7 +17,7 @@
 // ---------------------------------------------------------------- embedding
 
 // One workgroup per token: table row * scale + pair row, normed, in fp32.
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void embed_pairs_kernel(
     const long* __restrict__ ids, const T* __restrict__ table, float scale,
     const T* __restrict__ pairs, long buckets, long mul_prev, long mul_cur,
@@ -50,16 +50,26 @@ __global__ __launch_bounds__(256) void embed_pairs_kernel(
   const T* a = table + id * W;
   const T* b = pairs + pair * W;
   float ss = 0.f;
-  for (int i = threadIdx.x; i < W; i += 256) {
-    const float v = ldf(a + i) * scale + ldf(b + i);
-    row[i] = v;
-    ss += v * v;
+  for (int i = threadIdx.x * V; i < W; i += 256 * V) {
+    if constexpr (V == 4) {
+      const floatx4 v = ld4(a + i) * scale + ld4(b + i);
+      *(floatx4*)(row + i) = v;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss += v[j] * v[j];
+    } else {
+      const float v = ldf(a + i) * scale + ldf(b + i);
+      row[i] = v;
+      ss += v * v;
+    }
   }
   const float inv = rsqrtf(block_sum4(ss, red) / W + eps);
   // every thread has read the past by now
   if (t == first && slot >= 0 && threadIdx.x == 0) prev[slot] = (int)ids[last];
-  for (int i = threadIdx.x; i < W; i += 256)
-    out[(long)t * W + i] = row[i] * inv * weight[i];
+  float* y = out + (long)t * W;
+  for (int i = threadIdx.x * V; i < W; i += 256 * V) {
+    if constexpr (V == 4) st4(y + i, *(const floatx4*)(row + i) * inv * ld4(weight + i));
+    else y[i] = row[i] * inv * weight[i];
+  }
 }
 
 void embed_pairs(torch::Tensor ids, torch::Tensor table, double scale,
@@ -84,12 +94,17 @@ void embed_pairs(torch::Tensor ids, torch::Tensor table, double scale,
   }
   if (T_ == 0) return;
   DISPATCH_ELEM(table.dtype() == torch::kBFloat16, {
-    hipLaunchKernelGGL((embed_pairs_kernel<T>), dim3(T_), dim3(256), (size_t)W * 4,
-                       CUR_STREAM, (const long*)ids.data_ptr(), (const T*)table.data_ptr(),
-                       (float)scale, (const T*)pairs.data_ptr(), pairs.size(0) - 1, mul_prev,
-                       mul_cur, weight.data_ptr<float>(), (float)eps, prev.data_ptr<int>(),
-                       cu ? cu->data_ptr<int>() : nullptr, starts.data_ptr<int>(),
-                       slots.data_ptr<int>(), out.data_ptr<float>(), S, W);
+    auto launch = [&](auto kern) {
+      hipLaunchKernelGGL(kern, dim3(T_), dim3(256), (size_t)W * 4, CUR_STREAM,
+                         (const long*)ids.data_ptr(), (const T*)table.data_ptr(),
+                         (float)scale, (const T*)pairs.data_ptr(), pairs.size(0) - 1,
+                         mul_prev, mul_cur, weight.data_ptr<float>(), (float)eps,
+                         prev.data_ptr<int>(), cu ? cu->data_ptr<int>() : nullptr,
+                         starts.data_ptr<int>(), slots.data_ptr<int>(),
+                         out.data_ptr<float>(), S, W);
+    };
+    if (W % 4 == 0) launch(embed_pairs_kernel<T, 4>);
+    else launch(embed_pairs_kernel<T, 1>);
   });
   HIP_CHECK_KERNEL();
 }
@@ -247,7 +262,10 @@ __global__ __launch_bounds__(256) void xielu_kernel(const T* __restrict__ z, lon
   if (i >= total) return;
   const T* p = z + i / F * stride + i % F;
   auto f = [&](float x) {
-    const float low = down * (expm1f(fminf(x, 0.f)) - x);
+    // 16-bit results do not tell e^z - 1 from its accurate form: next to z / 2
+    // the difference is below their rounding
+    const float y = fminf(x, 0.f);
+    const float low = down * ((sizeof(T) == 2 ? __expf(y) - 1.f : expm1f(y)) - y);
     return (x > 0.f ? up * x * x : low) + 0.5f * x;
   };
   if constexpr (V % 4 == 0) {

@@ -271,22 +271,30 @@ def head_linear(x, w, gate=None, out=None):
     return out
 
 
-def expand_latents(seg: Segment, p: LatentParams, rank: int) -> bool:
-    """Whether it is cheaper to spell out every key and value of a prompt
-    portion's context than to attend in the latents' own space, where a pair of
-    tokens costs 2 rank instead of dim + vdim but a key costs nothing."""
-    if seg.decode or (p.dim, p.vdim) not in {(a, b) for a in MATRIX_HEAD_DIMS
-                                             for b in MATRIX_HEAD_DIMS}:
-        return False
-    lens = [b - a for a, b in zip(seg.cu_host, seg.cu_host[1:])]
-    keys = sum(seg.ctx_host)
-    pairs = sum(n * (c - n / 2) for n, c in zip(lens, seg.ctx_host))
-    fits = keys * p.heads * (p.dim + p.vdim) <= EXPANDED_LIMIT
-    return fits and pairs * (2 * rank - p.dim - p.vdim) > keys * rank * (p.dim + p.vdim)
-
-
 #: most numbers of spelled-out keys and values one step may hold
 EXPANDED_LIMIT = 1 << 31
+
+
+def expand_latents(seg: Segment, p: LatentParams, rank: int) -> bool:
+    """Whether it is faster to spell out every key and value of a prompt
+    portion's context than to attend in the latents' own space, where a pair of
+    tokens costs 2 rank instead of dim + vdim but a key costs nothing."""
+    if seg.decode or p.dim not in MATRIX_HEAD_DIMS or p.vdim not in MATRIX_HEAD_DIMS:
+        return False
+    width = p.dim + p.vdim
+    keys = sum(seg.ctx_host)
+    if keys * p.heads * width > EXPANDED_LIMIT:
+        return False
+    pairs = sum((b - a) * (c - (b - a) / 2) for a, b, c in
+                zip(seg.cu_host, seg.cu_host[1:], seg.ctx_host))
+    rows = seg.cu_host[-1]
+    # measured rates in flops per us: the latent kernel and the per-head products
+    # around it; library products and the flash kernel, which also takes 0.4 us
+    # per key and 10^3 of width at least
+    latent = pairs * p.heads * 4 * rank / 6e8 + rows * p.heads * 2 * rank * width / 2e8
+    product = keys * p.heads * 2 * rank * width / 6e8
+    flash = max(pairs * p.heads * 2 * width / 3e8, max(seg.ctx_host) * width * 4e-4)
+    return product + flash < latent
 
 
 def latent_attention(proj, p: LatentParams, cache, seg: Segment, out):

@@ -25,7 +25,8 @@ Two modes:
   eng.step() decode turns) — quoted alongside for comparability.
 
 * ``--mode layers``: prefill and decode throughput of a few full-width layers
-  of the Kikalix decoder beside as many of a Mixtral-style one of equal width,
+  of a layer-listed decoder (``--design``: Kikalix beside a Mixtral-style model,
+  Senotar beside a Llama-style one) and as many of the other of equal width,
   heads, experts and feed-forward (random weights), each through its engine's
   own batch building, kernels and decode graphs, the two timed in turn.
 
@@ -65,6 +66,8 @@ def parse_args():
                     help="layers per model in --mode layers")
     ap.add_argument("--size", default="all",
                     help="one of the --mode layers sizes, or all")
+    ap.add_argument("--design", choices=("kikalix", "senotar"), default="kikalix",
+                    help="design of --mode layers")
     ap.add_argument("--rag", type=int, default=int(os.environ.get("BENCH_RAG", "1")),
                     help="per-turn on-GPU RAG retrieval + input-rail check (1=on)")
     ap.add_argument("--rag-docs", type=int,
@@ -406,7 +409,7 @@ async def main_e2e_async(args, rank, world, use_cuda):
 
 
 # --------------------------------------------------------------------------
-# layers mode: Kikalix layers beside Mixtral-style layers of equal size
+# layers mode: a design's layers beside the closest model's of equal size
 # --------------------------------------------------------------------------
 
 #: width, heads, kv heads, experts, top, ff: layers of a 7B-class decoder with
@@ -415,6 +418,12 @@ LAYER_SIZES = {
     "4096-8x14336": (4096, 32, 8, 8, 2, 14336),
     "2048-64x1408": (2048, 16, 8, 64, 6, 1408),
     "1024-16x512": (1024, 8, 2, 16, 2, 512),
+}
+#: width, heads, kv heads of the Llama-style layers, latent rank, ff
+SENOTAR_SIZES = {
+    "4096-14336": (4096, 32, 8, 512, 14336),
+    "2048-5632": (2048, 16, 4, 512, 5632),
+    "1024-2816": (1024, 16, 4, 256, 2816),
 }
 PREFILL_SEQS, PREFILL_LEN, DECODE_SEQS, DECODE_STEPS = 4, 2048, 64, 32
 
@@ -436,6 +445,21 @@ def layer_pair(size: str, n_layers: int):
         head_dim=d, intermediate_size=ff, vocab_size=32000, max_position=8192,
         n_experts=experts, experts_per_token=top)
     return hybrid, mixtral
+
+
+def senotar_pair(size: str, n_layers: int):
+    """(Senotar spec, Llama-style spec) of one size; every second Senotar layer
+    reads the latents of the one before it."""
+    from aurora_amd.models.config import ModelSpec, senotar_spec
+    w, h, kv, rank, ff = SENOTAR_SIZES[size]
+    d = w // h
+    senotar = senotar_spec(
+        f"senotar-{size}", ("os" * n_layers)[:n_layers], width=w, vocab=32000, heads=h,
+        dim=d, vdim=d, kv_rank=rank, ff=ff, max_position=8192)
+    llama = ModelSpec(
+        name=f"llama-{size}", hidden_size=w, n_layers=n_layers, n_heads=h, n_kv_heads=kv,
+        head_dim=d, intermediate_size=ff, vocab_size=32000, max_position=8192)
+    return senotar, llama
 
 
 def layer_bench_engine(spec, seed: int = 0):
@@ -481,11 +505,13 @@ def layer_bench_once(eng, rng):
 
 
 def main_layers(args):
-    sizes = list(LAYER_SIZES) if args.size == "all" else [args.size]
+    table, pair = {"kikalix": (LAYER_SIZES, layer_pair),
+                   "senotar": (SENOTAR_SIZES, senotar_pair)}[args.design]
+    sizes = list(table) if args.size == "all" else [args.size]
     result = {}
     for size in sizes:
-        engines = {s.arch if s.arch != "llama" else "mixtral": layer_bench_engine(s)
-                   for s in layer_pair(size, args.layers)}
+        engines = {s.name.split("-")[0]: layer_bench_engine(s)
+                   for s in pair(size, args.layers)}
         rng = torch.Generator().manual_seed(5)
         best = {k: [float("inf"), float("inf")] for k in engines}
         for it in range(args.warmup + args.steps):

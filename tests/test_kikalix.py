@@ -15,10 +15,11 @@ import pytest
 import torch
 from safetensors.torch import save_file
 
+import decoder_rig
 import kikalix_oracle as oracle
 from aurora_amd import ops
 from aurora_amd.engine.engine import EngineConfig, LLMEngine
-from aurora_amd.engine.replay import TraceReplayer, make_engine
+from aurora_amd.engine.replay import TraceReplayer
 from aurora_amd.engine.sampling_params import SamplingParams
 from aurora_amd.models.config import get_spec, spec_from_checkpoint
 
@@ -123,55 +124,16 @@ def weights(cfg, seed=0, ranks=(10, 6)):
     return {k: v.to(torch.bfloat16) for k, v in t.items()}
 
 
-class Rig:
-    """A checkpoint on disk, its oracle, and engines over it."""
-
+class Rig(decoder_rig.Rig):
     def __init__(self, path, name, device, dtype="float32"):
-        self.cfg, self.device, self.dtype = config(name), device, dtype
+        cfg = config(name)
         if dtype == "bfloat16":
             # every expert is used, so that no close call of a router can fall
             # the other way by rounding; the choice itself is tested in float32
-            for layer in self.cfg["layers"]:
+            for layer in cfg["layers"]:
                 if layer["mlp"]:
                     layer["mlp"]["router"]["top"] = layer["mlp"]["router"]["experts"]
-        self.path = str(path)
-        self.t = weights(self.cfg)
-        with open(os.path.join(self.path, "config.json"), "w") as f:
-            json.dump(self.cfg, f)
-        save_file(self.t, os.path.join(self.path, "model.safetensors"))
-        self._oracle = {}
-
-    def tokens(self, n, seed):
-        gen = torch.Generator().manual_seed(100 + seed)
-        return torch.randint(0, self.cfg["vocab"], (n,), generator=gen).tolist()
-
-    def logits(self, toks):
-        key = tuple(toks)
-        if key not in self._oracle:
-            self._oracle[key] = oracle.forward(self.cfg, self.t, toks)[0]
-        return self._oracle[key]
-
-    def replayer(self, max_tokens=1024, page=16, requests=4):
-        return TraceReplayer(make_engine(self.path, self.dtype, max_tokens, self.device,
-                                         requests, page))
-
-    def check(self, got, want, tol=None):
-        """Every row's relative error."""
-        tol = tol or (1e-4 if self.dtype == "float32" else 0.1)
-        got, want = got.double().cpu(), want.double()
-        err = (got - want).norm(dim=-1) / want.norm(dim=-1)
-        assert err.max() < tol, [round(float(e), 5)
-                                 for e in err.sort(descending=True).values[:20]]
-
-    def run(self, rp, rid, toks, cuts):
-        """Logits of every token of a request fed in portions of ``cuts``."""
-        out, at = [], 0
-        for c in cuts:
-            out.append(rp.step([(rid, toks[at:at + c], list(range(c)))]).cpu())
-            at += c
-        assert at == len(toks)
-        rp.step([], [rid])
-        return torch.cat(out)
+        super().__init__(path, cfg, weights(cfg), oracle, device, dtype)
 
 
 CASES = [pytest.param((n, d, t), id=f"{n}-{d}-{t}",
@@ -200,14 +162,7 @@ def test_residual_after_every_run(rig):
     """The residual stream, run by run: a fault shows where it happens."""
     toks = rig.tokens(37, 1)
     want = oracle.forward(rig.cfg, rig.t, toks)[1]
-    rp = rig.replayer()
-    eng, trail = rp.engine, []
-    forward = eng.model.forward
-    eng.model.forward = lambda *a: forward(*a, trail=trail)
-    try:
-        rp.step([("a", toks, [0])])
-    finally:
-        eng.model.forward = forward
+    trail = rig.trail(toks)
     assert len(trail) == len(want)
     for got, w in zip(trail, want):
         rig.check(got, w, 3e-5 if rig.dtype == "float32" else 0.06)
@@ -233,18 +188,7 @@ def test_unequal_batch(rig):
     rp = rig.replayer(max_tokens=320)
     plan = [{"a": 40, "d": 5}, {"a": 1, "b": 20}, {"b": 1, "a": 1, "c": 50},
             {"c": 2}, {"b": 1, "c": 1}, {"c": 17, "a": 1, "b": 11}, {"a": 27, "c": 20}]
-    at, got = dict.fromkeys(toks, 0), {r: [] for r in toks}
-    for step in plan:
-        entries = [(r, toks[r][at[r]:at[r] + n], list(range(n))) for r, n in step.items()]
-        for r, n in step.items():
-            at[r] += n
-        rows = rp.step(entries, [r for r in step if at[r] == len(toks[r])]).cpu()
-        for r, n in step.items():
-            got[r].append(rows[:n])
-            rows = rows[n:]
-    for r in toks:
-        rig.check(torch.cat(got[r]), rig.logits(toks[r]))
-    assert not rp.live
+    rig.run_plan(rp, toks, plan)
 
 
 def test_reused_pages_and_slots(rig):
@@ -267,18 +211,12 @@ def test_long_decoding(rig):
 def test_greedy_generation(rig):
     """Through add_request, the scheduler (prompts cut at 32 tokens, batches
     of prompts beside decoding) and the sampler."""
-    eng = LLMEngine(EngineConfig(model=rig.path, dtype=rig.dtype, device=rig.device,
-                                 page_size=16, kv_cache_pages=64, max_num_seqs=3,
-                                 max_batched_tokens=32, max_model_len=256))
+    eng = rig.engine(kv_cache_pages=64, max_num_seqs=3, max_batched_tokens=32,
+                     max_model_len=256)
     prompts = [rig.tokens(n, 20 + n) for n in (3, 70, 25, 40)]
     out = eng.generate(prompts, SamplingParams(temperature=0.0, max_tokens=12, ignore_eos=True))
     assert eng.states.num_free() == eng.states.num_slots
-    for p, got in zip(prompts, out):
-        assert len(got) == 12
-        # the chosen token's oracle logit is the highest, up to rounding
-        lg = rig.logits(p + got)[len(p) - 1:-1]
-        gap = lg.max(-1).values - lg[torch.arange(12), torch.tensor(got)]
-        assert gap.max() < (1e-3 if rig.dtype == "float32" else 0.35), gap
+    rig.check_greedy(prompts, out, 12)
 
 
 # ----------------------------------------------------- the engine's own workings
@@ -286,13 +224,6 @@ def test_greedy_generation(rig):
 @pytest.fixture(scope="module")
 def cpu_rig(tmp_path_factory):
     return Rig(tmp_path_factory.mktemp("ckpt"), "odd", "cpu")
-
-
-def _greedy(rig, prompt, n):
-    toks = list(prompt)
-    for _ in range(n):
-        toks.append(int(oracle.forward(rig.cfg, rig.t, toks)[0][-1].argmax()))
-    return toks[len(prompt):]
 
 
 def test_preemption_recomputes_state(cpu_rig):
@@ -313,28 +244,22 @@ def test_preemption_recomputes_state(cpu_rig):
 def test_session_continues_from_its_state(cpu_rig):
     eng = LLMEngine(EngineConfig(model=cpu_rig.path, device="cpu", page_size=16,
                                  kv_cache_pages=32, max_num_seqs=2, max_model_len=256))
-    p = SamplingParams(temperature=0.0, max_tokens=5, ignore_eos=True)
 
     def turn(rid, toks):
-        eng.add_request(rid, toks, p, session_id="s")
-        out = []
-        while eng.has_work():
-            for o in eng.step():
-                out += o.new_token_ids
-        return out
+        return decoder_rig.turn(eng, rid, toks, 5, session="s")
 
     first = cpu_rig.tokens(21, 50)
     out1 = turn("t1", first)
-    assert out1 == _greedy(cpu_rig, first, 5)
+    assert out1 == cpu_rig.greedy(first, 5)
     # extends the session: only the new tokens run
     before = eng.counters["prompt_tokens"]
     second = first + out1 + cpu_rig.tokens(9, 51)
-    assert turn("t2", second) == _greedy(cpu_rig, second, 5)
+    assert turn("t2", second) == cpu_rig.greedy(second, 5)
     assert eng.counters["prompt_tokens"] - before == len(second) - (len(first) + 4)
     # departs from it inside what the state has seen: everything runs again
     before = eng.counters["prompt_tokens"]
     third = second[:15] + cpu_rig.tokens(9, 52)
-    assert turn("t3", third) == _greedy(cpu_rig, third, 5)
+    assert turn("t3", third) == cpu_rig.greedy(third, 5)
     assert eng.counters["prompt_tokens"] - before == len(third)
 
 
@@ -342,15 +267,10 @@ def test_sessions_give_up_slots(cpu_rig):
     eng = LLMEngine(EngineConfig(model=cpu_rig.path, device="cpu", page_size=16,
                                  kv_cache_pages=32, max_num_seqs=2, state_slots=2,
                                  max_model_len=256))
-    p = SamplingParams(temperature=0.0, max_tokens=3, ignore_eos=True)
     for i in range(4):
         prompt = cpu_rig.tokens(10 + i, 60 + i)
-        eng.add_request(f"r{i}", prompt, p, session_id=f"s{i}")
-        out = []
-        while eng.has_work():
-            for o in eng.step():
-                out += o.new_token_ids
-        assert out == _greedy(cpu_rig, prompt, 3)
+        out = decoder_rig.turn(eng, f"r{i}", prompt, 3, session=f"s{i}")
+        assert out == cpu_rig.greedy(prompt, 3)
     assert len(eng.sessions) == 2
 
 
@@ -359,8 +279,8 @@ def test_equal_prompts_share_no_pages(cpu_rig):
                                  kv_cache_pages=64, max_num_seqs=4, max_model_len=256))
     prompt = cpu_rig.tokens(50, 70)
     p = SamplingParams(temperature=0.0, max_tokens=4, ignore_eos=True)
-    assert eng.generate([prompt] * 2, p) == [_greedy(cpu_rig, prompt, 4)] * 2
-    assert eng.generate([prompt], p) == [_greedy(cpu_rig, prompt, 4)]
+    assert eng.generate([prompt] * 2, p) == [cpu_rig.greedy(prompt, 4)] * 2
+    assert eng.generate([prompt], p) == [cpu_rig.greedy(prompt, 4)]
     assert eng.counters["prefix_cache_pages"] == 0
 
 
