@@ -48,7 +48,7 @@ class HybridLayer(nn.Module):
                     m.rot_dims, spec.max_position, m.rot_base)
             self.mixer = RetentionMixer(m, w, spec.rms_eps, dtype, rotations[key])
         # convolution of the mixer's input, residual gate of its output
-        self.conv = _param(w, spec.input_conv, dtype=torch.float32) \
+        self.conv = _param(spec.input_conv, w, dtype=torch.float32) \
             if spec.input_conv else None
         self.gate = _param(w, w, dtype=dtype) if spec.residual_gates else None
         self.gate_bias = _param(w, dtype=torch.float32) if spec.residual_gates else None
@@ -67,7 +67,7 @@ class HybridLayer(nn.Module):
         """The input convolution's last inputs, if it has any, then the mixer's."""
         own = []
         if self.conv is not None:
-            w, taps = self.conv.shape
+            taps, w = self.conv.shape
             own = [(((taps - 1, w), dtype),)]
         return own + self.mixer.state_layout(dtype)
 
@@ -186,7 +186,7 @@ class HybridForCausalLM(nn.Module):
             layer.mlp.load(*read)
 
     def _plain_tensors(self) -> Dict[str, torch.Tensor]:
-        """Weights held as they are stored, by name."""
+        """Weights held as they are stored (or views of them), by name."""
         out = {"embed": self.embed.weight.data, "final.norm": self.final_norm.data,
                "head": self.lm_head.data}
         if self.loop_step is not None:
@@ -198,7 +198,7 @@ class HybridForCausalLM(nn.Module):
             if layer.mlp is not None:
                 out[f"l{i}.norm2"] = layer.norm2.data
             if layer.conv is not None:
-                out[f"l{i}.canon1"] = layer.conv.data
+                out[f"l{i}.canon1"] = layer.conv.data.t()
             if layer.gate is not None:
                 out[f"l{i}.rg1"], out[f"l{i}.rg1.b"] = layer.gate.data, layer.gate_bias.data
         return out

@@ -48,14 +48,19 @@ DEVINL float softplus_f(float x) {
   return fmaxf(x, 0.f) + s;
 }
 
-// sum over a workgroup of 4 waves; every thread gets it (red: 4 floats of LDS)
-DEVINL float block_sum4(float x, float* red) {
+// sum over a workgroup of NW waves; every thread gets it (red: NW floats of LDS)
+template <int NW>
+DEVINL float block_sum(float x, float* red) {
   x = wave_sum(x);
   __syncthreads();
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = x;
   __syncthreads();
-  return red[0] + red[1] + red[2] + red[3];
+  float y = red[0];
+#pragma unroll
+  for (int i = 1; i < NW; ++i) y += red[i];
+  return y;
 }
+DEVINL float block_sum4(float x, float* red) { return block_sum<4>(x, red); }
 
 #define DISPATCH_ELEM(IS_BF16, ...)                     \
   do {                                                  \

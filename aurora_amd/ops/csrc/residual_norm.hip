@@ -29,7 +29,7 @@ struct ResidualGate {
 // position p's row at p mod (taps - 1); slot -1 has no past and stores nothing
 template <typename T>
 struct ConvTail {
-  const float* w;  // [W, taps], null: no convolution
+  const float* w;  // [taps, W], the last row the present; null: no convolution
   int taps;
   T* ring;         // [slots, taps - 1, W]
   const int* pos;
@@ -37,21 +37,22 @@ struct ConvTail {
   T* out;          // [T, W]
 };
 
-template <typename T, int V>
-__global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
+// NTHR threads per row: 1024 where few wide rows would leave the chip waiting
+template <typename T, int V, int NTHR>
+__global__ __launch_bounds__(NTHR) void residual_rmsnorm_kernel(
     float* __restrict__ x, const float* __restrict__ weight,
     const T* __restrict__ delta, ResidualGate<T> rg, const T* __restrict__ y,
     const int* __restrict__ place, const float* __restrict__ gate, int top,
     const float* __restrict__ step, T* __restrict__ out, ConvTail<T> cv, int W,
     float eps, float offset) {
   extern __shared__ __attribute__((aligned(16))) float row[];
-  __shared__ float red[4];
+  __shared__ float red[NTHR / WAVE];
   const long base = (long)blockIdx.x * W;
   const int* pl = place + (long)blockIdx.x * top;
   const float* gt = gate + (long)blockIdx.x * top;
   const T* pre = rg.pre ? rg.pre + blockIdx.x * rg.stride : nullptr;
   float ss = 0.f;
-  for (int i = threadIdx.x * V; i < W; i += 256 * V) {
+  for (int i = threadIdx.x * V; i < W; i += NTHR * V) {
     float v[V];
     if constexpr (V == 4) {
       floatx4 a = ld4(x + base + i);
@@ -88,13 +89,13 @@ __global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
 #pragma unroll
     for (int j = 0; j < V; ++j) ss += v[j] * v[j];
   }
-  const float inv = rsqrtf(block_sum4(ss, red) / W + eps);
+  const float inv = rsqrtf(block_sum<NTHR / WAVE>(ss, red) / W + eps);
   const int keep = cv.taps - 1;
   const int slot = cv.w ? cv.slots[blockIdx.x] : -1;
   const int pos = cv.w ? cv.pos[blockIdx.x] : 0;
   T* ring = cv.ring + (long)max(slot, 0) * keep * W;
   const int known = slot >= 0 ? min(keep, pos) : 0;  // rows of the past
-  for (int i = threadIdx.x * V; i < W; i += 256 * V) {
+  for (int i = threadIdx.x * V; i < W; i += NTHR * V) {
     if constexpr (V == 4) {
       const floatx4 a = *reinterpret_cast<const floatx4*>(row + i);
       st4(out + base + i, a * inv * (offset + ld4(weight + i)));
@@ -102,25 +103,25 @@ __global__ __launch_bounds__(256) void residual_rmsnorm_kernel(
       stf(out + base + i, row[i] * inv * (offset + weight[i]));
     }
     if (!cv.w) continue;
-    // from here on the row as stored
-    float u[V];
-    const float* w = cv.w + (long)i * cv.taps;
-#pragma unroll
-    for (int j = 0; j < V; ++j) {
-      u[j] = ldf(out + base + i + j);
-      u[j] += u[j] * w[j * cv.taps + keep];
-    }
-    for (int b = 1; b <= known; ++b) {
-      const T* p = ring + (long)((pos - b) % keep) * W + i;
-#pragma unroll
-      for (int j = 0; j < V; ++j) u[j] += w[j * cv.taps + keep - b] * ldf(p + j);
-    }
-#pragma unroll
-    for (int j = 0; j < V; ++j) stf(cv.out + base + i + j, u[j]);
-    if (keep > 0 && slot >= 0) {  // takes the place of the oldest row, now read
-      T* p = ring + (long)(pos % keep) * W + i;
-#pragma unroll
-      for (int j = 0; j < V; ++j) p[j] = out[base + i + j];
+    // from here on the row as stored; its place in the ring is the oldest row's,
+    // read before
+    const float* w = cv.w + (long)keep * W + i;
+    T* mine = slot >= 0 && keep > 0 ? ring + (long)(pos % keep) * W + i : nullptr;
+    if constexpr (V == 4) {
+      const floatx4 y = ld4(out + base + i);
+      floatx4 u = y + y * ld4(w);
+#pragma unroll 4
+      for (int b = 1; b <= known; ++b)
+        u += ld4(w - (long)b * W) * ld4(ring + (long)((pos - b) % keep) * W + i);
+      st4(cv.out + base + i, u);
+      if (mine) st4(mine, y);
+    } else {
+      const float y = ldf(out + base + i);
+      float u = y + y * *w;
+      for (int b = 1; b <= known; ++b)
+        u += w[-(long)b * W] * ldf(ring + (long)((pos - b) % keep) * W + i);
+      stf(cv.out + base + i, u);
+      if (mine) stf(mine, y);
     }
   }
 }
@@ -158,10 +159,10 @@ std::vector<torch::Tensor> residual_rmsnorm(
   }
   if (step) TORCH_CHECK(step->numel() == W && step->dtype() == torch::kFloat32);
   if (conv_w) {
-    TORCH_CHECK(ring && pos && slots && conv_w->is_contiguous() && conv_w->size(0) == W &&
+    TORCH_CHECK(ring && pos && slots && conv_w->is_contiguous() && conv_w->size(1) == W &&
                 conv_w->dtype() == torch::kFloat32 && ring->dim() == 3 &&
                 ring->is_contiguous() && ring->dtype() == dt && ring->size(2) == W &&
-                ring->size(1) == conv_w->size(1) - 1, "input convolution");
+                ring->size(1) == conv_w->size(0) - 1, "input convolution");
     TORCH_CHECK(pos->numel() == T_ && slots->numel() == T_ &&
                 pos->dtype() == torch::kInt32 && slots->dtype() == torch::kInt32);
     out.push_back(torch::empty_like(out[0]));
@@ -174,11 +175,11 @@ std::vector<torch::Tensor> residual_rmsnorm(
       rg = {(const T*)gate_pre->data_ptr(), gate_pre->stride(0), gate_bias->data_ptr<float>()};
     ConvTail<T> cv = {nullptr, 1, nullptr, nullptr, nullptr, nullptr};
     if (conv_w)
-      cv = {conv_w->data_ptr<float>(), (int)conv_w->size(1), (T*)ring->data_ptr(),
+      cv = {conv_w->data_ptr<float>(), (int)conv_w->size(0), (T*)ring->data_ptr(),
             pos->data_ptr<int>(), slots->data_ptr<int>(), (T*)out[1].data_ptr()};
-    auto launch = [&](auto kern) {
+    auto launch = [&](auto kern, int threads) {
       hipLaunchKernelGGL(
-          kern, dim3(T_), dim3(256), lds, CUR_STREAM, x.data_ptr<float>(),
+          kern, dim3(T_), dim3(threads), lds, CUR_STREAM, x.data_ptr<float>(),
           weight.data_ptr<float>(), delta ? (const T*)delta->data_ptr() : nullptr, rg,
           y ? (const T*)y->data_ptr() : nullptr,
           y ? place->data_ptr<int>() : nullptr, y ? gate->data_ptr<float>() : nullptr,
@@ -187,8 +188,9 @@ std::vector<torch::Tensor> residual_rmsnorm(
     };
     const bool vec = W % 4 == 0 && (!gate_pre || (gate_pre->stride(0) % 4 == 0 &&
                      (reinterpret_cast<uintptr_t>(gate_pre->data_ptr()) & 15) == 0));
-    if (vec) launch(residual_rmsnorm_kernel<T, 4>);
-    else launch(residual_rmsnorm_kernel<T, 1>);
+    if (vec && T_ <= 256 && W > 1024) launch(residual_rmsnorm_kernel<T, 4, 1024>, 1024);
+    else if (vec) launch(residual_rmsnorm_kernel<T, 4, 256>, 256);
+    else launch(residual_rmsnorm_kernel<T, 1, 256>, 256);
   });
   HIP_CHECK_KERNEL();
   return out;

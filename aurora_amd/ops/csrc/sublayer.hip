@@ -115,7 +115,8 @@ void embed_pairs(torch::Tensor ids, torch::Tensor table, double scale,
 // inputs read again for every tap (V = 1).
 template <typename T, int V, int TAPS>
 __global__ __launch_bounds__(256) void short_conv_kernel(
-    const T* __restrict__ h, const float* __restrict__ w, T* __restrict__ ring,
+    const T* __restrict__ h, const float* __restrict__ w /* [taps, W] */,
+    T* __restrict__ ring,
     const int* __restrict__ cu, const int* __restrict__ bseq, const int* __restrict__ boff,
     const int* __restrict__ starts, const int* __restrict__ slots, T* __restrict__ out,
     int W, int taps_) {
@@ -163,7 +164,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
 #pragma unroll
     for (int j = 0; j < TAPS; ++j)
 #pragma unroll
-      for (int v = 0; v < V; ++v) wt[j][v] = w[(long)(c + v) * TAPS + j];
+      for (int v = 0; v < V; ++v) wt[j][v] = w[(long)j * W + c + v];
 #pragma unroll
     for (int j = 1; j < TAPS; ++j) input(off - TAPS + j, win[j]);
     for (int t = 0; t < n; ++t) {
@@ -188,7 +189,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(
       for (int j = 0; j < taps; ++j) {
         input(off + t - keep + j, x);
 #pragma unroll
-        for (int v = 0; v < V; ++v) y[v] += w[(long)(c + v) * taps + j] * x[v];
+        for (int v = 0; v < V; ++v) y[v] += w[(long)j * W + c + v] * x[v];
       }
       store(off + t, y);
     }
@@ -208,10 +209,10 @@ void short_conv_add(torch::Tensor h, torch::Tensor w, torch::Tensor ring,
                     c10::optional<torch::Tensor> cu, c10::optional<torch::Tensor> bseq,
                     c10::optional<torch::Tensor> boff, torch::Tensor starts,
                     torch::Tensor slots, torch::Tensor out) {
-  const int T_ = h.size(0), W = h.size(1), taps = w.size(1), S = slots.numel();
+  const int T_ = h.size(0), W = h.size(1), taps = w.size(0), S = slots.numel();
   TORCH_CHECK(h.is_cuda() && h.is_contiguous() && out.is_contiguous() &&
               out.sizes() == h.sizes() && out.dtype() == h.dtype());
-  TORCH_CHECK(w.is_contiguous() && w.size(0) == W && w.dtype() == torch::kFloat32);
+  TORCH_CHECK(w.is_contiguous() && w.size(1) == W && w.dtype() == torch::kFloat32);
   TORCH_CHECK(taps >= 1 && taps <= CONV_MAX_TAPS, "a convolution of ", taps, " taps");
   TORCH_CHECK(ring.is_contiguous() && ring.dtype() == h.dtype() && ring.dim() == 3 &&
               ring.size(1) == taps - 1 && ring.size(2) == W, "convolution state");

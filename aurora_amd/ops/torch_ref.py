@@ -461,9 +461,9 @@ def embed_pairs(ids, table, scale, pairs, mul_prev, mul_cur, weight, eps, prev,
 
 
 def short_conv_add(h, w, ring, cu, starts, slots, out):
-    """out = h + causal convolution of h per channel; w [W, taps]. The ring
+    """out = h + causal convolution of h per channel; w [taps, W]. The ring
     [slots, taps - 1, W] holds position p's h at p mod (taps - 1)."""
-    taps = w.shape[1]
+    taps = w.shape[0]
     past = taps - 1
     for s in range(cu.numel() - 1):
         a, b, start, slot = int(cu[s]), int(cu[s + 1]), int(starts[s]), int(slots[s])
@@ -480,7 +480,7 @@ def short_conv_add(h, w, ring, cu, starts, slots, out):
                 ring[slot, (start + t) % past] = h[a + t].to(ring.dtype)
         y = full[past:].clone()
         for j in range(taps):
-            y += full[j:j + n] * w[:, j]
+            y += full[j:j + n] * w[j]
         out[a:b] = y.to(out.dtype)
 
 

@@ -406,7 +406,7 @@ def test_input_convolution_alone(device, taps, W):
         for a, b in _cuts(cuts):
             seg = _seg(b - a, device, a, single=a > 0 and b - a == 1)
             out = torch.empty(b - a, W, device=device)
-            ops.short_conv_add(h[a:b].to(device), w.to(device), ring, seg, out)
+            ops.short_conv_add(h[a:b].to(device), w.t().contiguous().to(device), ring, seg, out)
             got.append(out)
         err = (torch.cat(got).cpu() - want).abs().max(-1).values
         assert (err < 1e-5 * want.abs().max(-1).values.clamp(min=1)).all(), cuts

@@ -247,7 +247,7 @@ def test_embed_pairs(dtype, W):
 @pytest.mark.parametrize("W", [320, 50, 2056])
 @pytest.mark.parametrize("taps", [1, 2, 3, 4, 5, 6, 7, 16])
 def test_short_conv_and_its_fused_form(dtype, W, taps):
-    w, nw = rnd(W, taps, scale=0.5), rnd(W)
+    w, nw = rnd(taps, W, scale=0.5), rnd(W)
     ring = rnd(6, taps - 1, W, dtype=dtype)
     rg = ring.cuda()
     for lens, starts, slots, dec in (
