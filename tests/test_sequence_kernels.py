@@ -223,7 +223,7 @@ def test_routed_experts(dtype, T, W, F, E, top):
 # ------------------------------------- embeddings, input convolution, activation
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("W", [320, 50])
+@pytest.mark.parametrize("W", [288, 50])
 def test_embed_pairs(dtype, W):
     V, B = 200, 31
     table, pairs, w = rnd(V, W, dtype=dtype), rnd(B + 1, W, dtype=dtype), rnd(W)
@@ -244,7 +244,7 @@ def test_embed_pairs(dtype, W):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("W", [320, 50, 2056])
+@pytest.mark.parametrize("W", [288, 50, 2056])
 @pytest.mark.parametrize("taps", [1, 2, 3, 4, 5, 6, 7, 16])
 def test_short_conv_and_its_fused_form(dtype, W, taps):
     w, nw = rnd(taps, W, scale=0.5), rnd(W)
@@ -310,7 +310,7 @@ def test_head_linear(dtype, T, H, K, N):
 
 
 LATENT = [  # heads, dim, vdim, rank
-    (4, 64, 64, 128), (3, 20, 100, 50), (16, 128, 128, 512), (17, 64, 128, 256),
+    (5, 64, 64, 128), (3, 20, 100, 50), (16, 128, 128, 512), (17, 64, 128, 256),
     (40, 128, 64, 300), (1, 160, 72, 384), (6, 32, 32, 520), (2, 128, 128, 700), (33, 40, 24, 64)]
 
 
