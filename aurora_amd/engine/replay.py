@@ -97,7 +97,7 @@ def main(argv: Optional[List[str]] = None) -> int:
     ap.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
     ap.add_argument("--out", required=True, help="folder for <step>.f32 files")
     ap.add_argument("--max-tokens", type=int, required=True,
-                    help="most tokens that live requests hold at any time")
+                    help="capacity of the cache pool in tokens, over all unfinished requests")
     ap.add_argument("--device", choices=("auto", "cpu"), default="auto")
     args = ap.parse_args(argv)
     if args.device == "auto" and not torch.cuda.is_available():

@@ -181,7 +181,7 @@ def test_portions(rig, cuts):
 
 
 def test_unequal_batch(rig):
-    """Portions of some beside single tokens of others, requests that pause,
+    """Prompt portions and decoded tokens in one batch, requests that pause,
     start late and end early: each as if it were alone."""
     toks = {r: rig.tokens(n, i) for i, (r, n) in
             enumerate({"a": 70, "b": 33, "c": 90, "d": 5}.items())}
