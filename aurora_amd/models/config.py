@@ -55,9 +55,10 @@ class ModelSpec:
 
 # ---- layer-listed decoders -------------------------------------------------
 # A HybridSpec spells its layers out one by one: each has a mixer (attention
-# beside a recurrence, a recurrence or latent attention alone) and an optional
-# feed-forward. What all layers share (residual gates, the convolution of the
-# mixer's input, the norms' weight) are fields of the HybridSpec.
+# beside a recurrence, a recurrence or attention alone) and an optional
+# feed-forward. What all layers share (the norms' kind and place, residual gates,
+# the convolution of the mixer's input, depth averages) are fields of the
+# HybridSpec.
 
 @dataclass(frozen=True)
 class BiasedAttentionSpec:
@@ -114,7 +115,71 @@ class LatentAttentionSpec:
 
 
 @dataclass(frozen=True)
+class NormedAttentionSpec:
+    """Grouped-query attention over normed queries and keys."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    norm: str = "head"  # RMS over each "head", or over the "whole" projection
+    rot_dims: int = 0   # leading dimensions of a head that rotate; 0: none
+    rot_base: float = 1e4
+    #: query at position p times 1 + coef ln(floor((p + 1) / every) + 1)
+    q_temp: Optional[Tuple[float, int]] = None
+    #: values are the keys as projected, before norm and rotation
+    shared_kv: bool = False
+    #: a_h ln(1 + b_h (i - j)) off the score, with two learned numbers per head
+    log_bias: bool = False
+    sink: bool = False  # the softmax's denominator has one more term, 1
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError("query heads must be a multiple of key/value heads")
+        if self.shared_kv and self.vdim != self.dim:
+            raise ValueError("values that are the keys are as wide as the keys")
+        if self.rot_dims % 2 or self.rot_dims > self.dim:
+            raise ValueError(f"cannot rotate {self.rot_dims} of {self.dim} dimensions")
+
+
+@dataclass(frozen=True)
+class HeadDeltaSpec:
+    """Gated delta rule with a short convolution, one decay per head and a silu
+    gate as wide as the heads."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError("value heads must be a multiple of query/key heads")
+
+
+@dataclass(frozen=True)
+class MatrixMemorySpec:
+    """Matrix memory with exponential input and sigmoid forget gates (mLSTM);
+    both gates' pre-activations are soft-capped."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+
+PartSpec = Union[NormedAttentionSpec, HeadDeltaSpec, MatrixMemorySpec]
+
+
+@dataclass(frozen=True)
+class FusedMixerSpec:
+    """Parts side by side over one input; their scaled results add up. Each part
+    is (prefix of its tensors' names, spec, scale)."""
+    parts: Tuple[Tuple[str, PartSpec, float], ...]
+
+
+@dataclass(frozen=True)
 class MoESpec:
+    """Softmax-routed clamped GLU experts."""
     experts: int
     top: int
     ff: int
@@ -122,18 +187,40 @@ class MoESpec:
 
 
 @dataclass(frozen=True)
-class DenseSpec:
-    """Ungated two-matrix feed-forward with the xIELU activation."""
+class GroupedMoESpec:
+    """Sigmoid-routed GLU experts, chosen by corrected scores among the best
+    ``keep`` of ``groups`` groups of neighbours, beside a shared expert (of width
+    ``shared_ff``; 0: none) behind a sigmoid gate."""
+    experts: int
+    top: int
     ff: int
+    scale: float
+    groups: int = 1
+    keep: int = 1
+    shared_ff: int = 0
+
+    def __post_init__(self):
+        if self.experts % self.groups or not 1 <= self.keep <= self.groups \
+                or not 1 <= self.top <= self.keep * (self.experts // self.groups):
+            raise ValueError(f"cannot choose {self.top} of {self.experts} experts in the "
+                             f"best {self.keep} of {self.groups} groups")
 
 
-MixerSpec = Union[ParallelMixerSpec, RetentionSpec, LatentAttentionSpec]
+@dataclass(frozen=True)
+class DenseSpec:
+    """Ungated two-matrix feed-forward."""
+    ff: int
+    act: str = "xielu"  # or "gelu", the exact one
+
+
+MixerSpec = Union[ParallelMixerSpec, RetentionSpec, LatentAttentionSpec, FusedMixerSpec]
+MLPSpec = Union[MoESpec, GroupedMoESpec, DenseSpec]
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     mixer: MixerSpec
-    mlp: Union[MoESpec, DenseSpec, None]
+    mlp: Optional[MLPSpec]
 
 
 @dataclass(frozen=True)
@@ -172,8 +259,20 @@ class HybridSpec:
     residual_gates: bool = False
     #: what norms add to their stored weight
     norm_offset: float = 1.0
+    #: True: sublayers read the residual itself, and a layer norm with bias is
+    #: taken of each sublayer's result; False: an RMS norm of each one's input
+    output_norms: bool = False
+    #: what goes on after a layer is a learned sum of the embedding and of every
+    #: layer's result so far
+    depth_average: bool = False
 
     def __post_init__(self):
+        if self.output_norms and (self.loop or self.embedding or self.input_conv
+                                  or self.residual_gates):
+            raise ValueError("output norms come without loops, pair embeddings, input "
+                             "convolutions and residual gates")
+        if self.depth_average and not self.output_norms:
+            raise ValueError("depth averages come with output norms")
         for i, layer in enumerate(self.layers):
             j = getattr(layer.mixer, "kv_from", None)
             if j is None:
@@ -205,36 +304,62 @@ class HybridSpec:
 
     def param_count(self) -> int:
         w = self.hidden_size
-        n = 2 * self.vocab_size * w + w
+        norm = 2 * w if self.output_norms else w
+        n = 2 * self.vocab_size * w + norm
         if self.loop is not None:
             n += self.loop[2] * w
         if self.embedding is not None:
             n += (self.embedding.bigram.buckets + 2) * w
-        for layer in self.layers:
-            m = layer.mixer
+        for i, layer in enumerate(self.layers):
+            n += norm * (1 if layer.mlp is None else 2)
             n += self.input_conv * w
             if self.residual_gates:
                 n += (1 if layer.mlp is None else 2) * (w + 1) * w
-            if isinstance(m, RetentionSpec):
-                n += w * m.heads * (2 * m.dim + 3 * m.vdim) + w
-            elif isinstance(m, LatentAttentionSpec):
-                n += w * m.heads * (m.dim + m.vdim + 1) + w + m.heads
-                n += m.kv_rank * m.heads * (m.dim + m.vdim)
-                if m.kv_from is None:
-                    n += m.kv_rank * (w + 1)
-            else:
-                a, r = m.left, m.right
-                qkv = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)
-                n += (w + 1) * qkv + w * a.heads * a.vdim + w
-                ch = 2 * r.kv_heads * r.dim + r.heads * r.vdim
-                n += ch * (w + r.conv) + w * (r.heads + r.decay_rank + r.gate_rank)
-                n += r.heads * (r.dim * (r.decay_rank + 1) + r.vdim * r.gate_rank + 1)
-                n += r.vdim + w * r.heads * r.vdim
-            if isinstance(layer.mlp, DenseSpec):
-                n += w + 2 * w * layer.mlp.ff + 2
-            elif layer.mlp is not None:
-                n += w + layer.mlp.experts * (3 * w * layer.mlp.ff + w + 1)
+            if self.depth_average:
+                n += i + 2
+            n += _mixer_params(layer.mixer, w) + _mlp_params(layer.mlp, w)
         return n
+
+
+def _mixer_params(m: MixerSpec, w: int) -> int:
+    if isinstance(m, FusedMixerSpec):
+        return sum(_part_params(p, w) for _, p, _ in m.parts)
+    if isinstance(m, RetentionSpec):
+        return w * m.heads * (2 * m.dim + 3 * m.vdim)
+    if isinstance(m, LatentAttentionSpec):
+        n = w * m.heads * (m.dim + m.vdim + 1) + m.heads
+        n += m.kv_rank * m.heads * (m.dim + m.vdim)
+        return n + (m.kv_rank * (w + 1) if m.kv_from is None else 0)
+    a, r = m.left, m.right
+    qkv = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)
+    n = (w + 1) * qkv + w * a.heads * a.vdim
+    ch = 2 * r.kv_heads * r.dim + r.heads * r.vdim
+    n += ch * (w + r.conv) + w * (r.heads + r.decay_rank + r.gate_rank)
+    n += r.heads * (r.dim * (r.decay_rank + 1) + r.vdim * r.gate_rank + 1)
+    return n + r.vdim + w * r.heads * r.vdim
+
+
+def _part_params(p: PartSpec, w: int) -> int:
+    if isinstance(p, NormedAttentionSpec):
+        q, k = p.heads * p.dim, p.kv_heads * p.dim
+        n = w * (q + k + p.heads * p.vdim) + (2 * p.dim if p.norm == "head" else q + k)
+        return n + (0 if p.shared_kv else w * p.kv_heads * p.vdim) \
+            + (2 * p.heads if p.log_bias else 0)
+    if isinstance(p, HeadDeltaSpec):
+        ch = 2 * p.kv_heads * p.dim + p.heads * p.vdim
+        return ch * (w + p.conv) + 2 * p.heads * (w + 1) + p.vdim + 2 * w * p.heads * p.vdim
+    return 2 * w * p.heads * (p.dim + 1) + 2 * p.heads + p.heads * p.vdim * (3 * w + 1)
+
+
+def _mlp_params(f: Optional[MLPSpec], w: int) -> int:
+    if f is None:
+        return 0
+    if isinstance(f, DenseSpec):
+        return 2 * w * f.ff + (2 if f.act == "xielu" else 0)
+    n = f.experts * (3 * w * f.ff + w + 1)
+    if isinstance(f, GroupedMoESpec) and f.shared_ff:
+        n += w * (3 * f.shared_ff + 1)
+    return n
 
 
 AnySpec = Union[ModelSpec, HybridSpec]
@@ -313,8 +438,56 @@ def _senotar_spec(name: str, cfg: dict, shapes: Dict[str, Sequence[int]]) -> Hyb
             bigram["buckets"], bigram["mul_prev"], bigram["mul_cur"])))
 
 
+def _gakupel_spec(name: str, cfg: dict, shapes: Dict[str, Sequence[int]]) -> HybridSpec:
+    def attention(m: dict, **kw) -> NormedAttentionSpec:
+        return NormedAttentionSpec(heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"],
+                                   vdim=m["vdim"], scale=float(m["scale"]), **kw)
+
+    def mixer(i: int, kind: str, m: dict) -> FusedMixerSpec:
+        if kind == "attention":
+            rot = m["rot"]
+            return FusedMixerSpec((("", attention(
+                m, shared_kv=True, rot_dims=rot["dims"], rot_base=float(rot["base"])), 1.0),))
+        if kind == "delta":
+            return FusedMixerSpec((("", HeadDeltaSpec(
+                m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"]), 1.0),))
+        if kind == "parallel":
+            left, right = m["left"], m["right"]
+            temp = left["q_temp"]
+            return FusedMixerSpec((
+                ("left.", attention(left, norm="whole", log_bias=True, sink=True,
+                                    q_temp=(float(temp["coef"]), int(temp["every"]))),
+                 float(m["left_scale"])),
+                ("right.", MatrixMemorySpec(right["heads"], right["dim"], right["vdim"],
+                                            float(right["gate_cap"])),
+                 float(m["right_scale"]))))
+        raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+
+    def mlp(i: int, f: Optional[dict]) -> Optional[MLPSpec]:
+        if f is None:
+            return None
+        if f["kind"] == "dense":
+            return DenseSpec(f["ff"], "gelu")
+        if f["kind"] == "moe":
+            r = f["router"]
+            groups = r.get("groups") or {"count": 1, "keep": 1}
+            return GroupedMoESpec(
+                experts=r["experts"], top=r["top"], ff=f["expert"]["ff"],
+                scale=float(r["scale"]), groups=groups["count"], keep=groups["keep"],
+                shared_ff=(f.get("shared") or {"ff": 0})["ff"])
+        raise ValueError(f"layer {i}: unknown feed-forward {f['kind']!r}")
+
+    return HybridSpec(
+        name=name, arch="gakupel", hidden_size=cfg["width"], vocab_size=cfg["vocab"],
+        rms_eps=float(cfg["norm"]["eps"]), norm_offset=0.0, output_norms=True,
+        depth_average=True,
+        layers=tuple(LayerSpec(mixer(i, e["type"], e["mixer"]), mlp(i, e.get("mlp")))
+                     for i, e in enumerate(cfg["layers"])))
+
+
 #: config.json "architecture" -> reader(name, config, tensor shapes)
-_CONFIG_READERS = {"Kikalix": _kikalix_spec, "Senotar": _senotar_spec}
+_CONFIG_READERS = {"Kikalix": _kikalix_spec, "Senotar": _senotar_spec,
+                   "Gakupel": _gakupel_spec}
 
 
 def is_checkpoint_dir(path: str) -> bool:
@@ -492,3 +665,48 @@ register(senotar_spec(  # GPU smoke size
 register(senotar_spec(  # layer sizes of a 7B-class decoder
     "senotar-7b", "o" * 16 + "s" * 16, width=4096, vocab=32000, heads=32, dim=128,
     vdim=128, kv_rank=512, ff=14336))
+
+# ---- Gakupel presets ---------------------------------------------------------
+
+def gakupel_spec(name: str, pattern: str, *, width: int, vocab: int, heads: int,
+                 kv_heads: int, dim: int, l_dim: int, l_vdim: int, d_heads: int,
+                 d_kv_heads: int, d_dim: int, d_vdim: int, m_heads: int, m_dim: int,
+                 m_vdim: int, ff: int, experts: int, top: int, expert_ff: int,
+                 shared_ff: int, groups: int = 4, keep: int = 2, conv: int = 4,
+                 rot_dims: int = 0, max_position: int = 131072) -> HybridSpec:
+    """Layers of one size from a pattern: 'a' attention, 'd' delta rule, 'p'
+    attention beside a matrix memory; upper case: dense instead of routed."""
+    mixers = {
+        "a": FusedMixerSpec((("", NormedAttentionSpec(
+            heads, kv_heads, dim, dim, dim ** -0.5, rot_dims=rot_dims or dim,
+            shared_kv=True), 1.0),)),
+        "d": FusedMixerSpec((("", HeadDeltaSpec(d_heads, d_kv_heads, d_dim, d_vdim, conv),
+                              1.0),)),
+        "p": FusedMixerSpec((
+            ("left.", NormedAttentionSpec(
+                heads, kv_heads, l_dim, l_vdim, l_dim ** -0.5, norm="whole",
+                q_temp=(0.2, 1024), log_bias=True, sink=True), 0.7),
+            ("right.", MatrixMemorySpec(m_heads, m_dim, m_vdim, 15.0), 0.7)))}
+    moe = GroupedMoESpec(experts, top, expert_ff, 2.0, groups, keep, shared_ff)
+    return HybridSpec(
+        name=name, arch="gakupel", hidden_size=width, vocab_size=vocab,
+        max_position=max_position, norm_offset=0.0, output_norms=True, depth_average=True,
+        layers=tuple(LayerSpec(mixers[c.lower()], DenseSpec(ff, "gelu") if c.isupper() else moe)
+                     for c in pattern))
+
+
+register(gakupel_spec(  # CPU plumbing size
+    "tiny-gakupel", "Pad", width=64, vocab=512, heads=4, kv_heads=2, dim=16,
+    l_dim=12, l_vdim=20, d_heads=4, d_kv_heads=2, d_dim=16, d_vdim=8, m_heads=3, m_dim=8,
+    m_vdim=12, ff=96, experts=6, top=2, expert_ff=24, shared_ff=40, groups=3, rot_dims=8,
+    max_position=2048))
+register(gakupel_spec(  # GPU smoke size: the matrix-core kernels' head widths
+    "smoke-gakupel", "paDp", width=512, vocab=1024, heads=8, kv_heads=2, dim=64,
+    l_dim=128, l_vdim=64, d_heads=4, d_kv_heads=2, d_dim=128, d_vdim=128, m_heads=4,
+    m_dim=64, m_vdim=128, ff=1024, experts=16, top=2, expert_ff=128, shared_ff=256,
+    max_position=8192))
+register(gakupel_spec(  # layer sizes of a 7B-class decoder, 8 experts like mixtral-8x7b
+    "gakupel-8x7b", "pdaPpdap" * 4, width=4096, vocab=32000, heads=32, kv_heads=8, dim=128,
+    l_dim=128, l_vdim=128, d_heads=16, d_kv_heads=16, d_dim=128, d_vdim=256,
+    m_heads=16, m_dim=128, m_vdim=256, ff=14336, experts=8, top=2, expert_ff=14336,
+    shared_ff=14336, groups=4, keep=2))

@@ -1,11 +1,12 @@
-"""Layer-listed decoders (Kikalix, Senotar): mixers and feed-forwards chosen
-layer by layer, with a span of layers that may run several times.
+"""Layer-listed decoders (Kikalix, Senotar, Gakupel): mixers and feed-forwards
+chosen layer by layer, with a span of layers that may run several times.
 
 Same engine shape as the other decoders: packed varlen tokens, paged KV and
 per-step metadata. Two things differ. The residual stream is one fp32 tensor
 that every norm kernel updates in place (the preceding sub-layer's output, or
 the weighted expert rows, and the pass vector are added by the kernel that
-norms). And every layer RUN, not layer, owns a paged cache or recurrent state;
+norms; where norms are taken of the sub-layers' outputs, so are the normed
+output and the average over the depth). And every layer RUN, not layer, owns a paged cache or recurrent state;
 a mixer may instead read an earlier layer's cache. Beside the mixers', state is
 what an input convolution and a pair embedding remember of the last tokens.
 """
@@ -18,10 +19,20 @@ import torch.nn as nn
 
 from .. import ops
 from ..parallel import dist as pdist
-from .config import DenseSpec, HybridSpec, LatentAttentionSpec, ParallelMixerSpec
+from .config import (
+    DenseSpec,
+    FusedMixerSpec,
+    GroupedMoESpec,
+    HybridSpec,
+    LatentAttentionSpec,
+    ParallelMixerSpec,
+)
 from .llama import AttnMetadata
 from .mixers import (
+    DenseGeluMLP,
     DenseXieluMLP,
+    FusedMixer,
+    GroupedGLU,
     LatentAttention,
     ParallelMixer,
     RetentionMixer,
@@ -36,8 +47,15 @@ class HybridLayer(nn.Module):
         s = spec.layers[i]
         w = spec.hidden_size
         self.norm1 = _param(w, dtype=torch.float32)
-        if isinstance(s.mixer, ParallelMixerSpec):
-            self.mixer: nn.Module = ParallelMixer(s.mixer, w, spec.rms_eps, dtype)
+        self.norm1_bias = _param(w, dtype=torch.float32) if spec.output_norms else None
+        self.norm2_bias = None
+        # weights of the embedding's and every layer's result in what goes on
+        self.depth = _param(i + 2, dtype=torch.float32) if spec.depth_average else None
+        if isinstance(s.mixer, FusedMixerSpec):
+            self.mixer: nn.Module = FusedMixer(s.mixer, w, spec.rms_eps, dtype,
+                                               spec.max_position, rotations)
+        elif isinstance(s.mixer, ParallelMixerSpec):
+            self.mixer = ParallelMixer(s.mixer, w, spec.rms_eps, dtype)
         elif isinstance(s.mixer, LatentAttentionSpec):
             self.mixer = LatentAttention(s.mixer, w, spec.rms_eps, dtype)
         else:
@@ -56,7 +74,14 @@ class HybridLayer(nn.Module):
             self.mlp = None
             return
         self.norm2 = _param(w, dtype=torch.float32)
-        if isinstance(s.mlp, DenseSpec):
+        if spec.output_norms:
+            self.norm2_bias = _param(w, dtype=torch.float32)
+        if isinstance(s.mlp, GroupedMoESpec) or getattr(s.mlp, "act", None) == "gelu":
+            if spec.residual_gates:
+                raise ValueError(f"no residual gates around a {type(s.mlp).__name__}")
+            self.mlp = GroupedGLU(s.mlp, w, dtype) if isinstance(s.mlp, GroupedMoESpec) \
+                else DenseGeluMLP(s.mlp, w, dtype)
+        elif isinstance(s.mlp, DenseSpec):
             self.mlp = DenseXieluMLP(s.mlp, w, dtype, spec.residual_gates)
         elif spec.residual_gates:
             raise ValueError("routed experts have no residual gate")
@@ -88,6 +113,8 @@ class HybridForCausalLM(nn.Module):
             self.layers = nn.ModuleList(
                 [HybridLayer(spec, i, dtype, rotations) for i in range(spec.n_layers)])
             self.final_norm = _param(spec.hidden_size, dtype=torch.float32)
+            self.final_norm_bias = _param(spec.hidden_size, dtype=torch.float32) \
+                if spec.output_norms else None
             self.lm_head = _param(spec.vocab_size, spec.hidden_size, dtype=dtype)
             self.loop_step = _param(spec.loop[2], spec.hidden_size,
                                     dtype=torch.float32) if spec.loop else None
@@ -139,6 +166,8 @@ class HybridForCausalLM(nn.Module):
         """Normed hidden states [T, H]; ``trail``, if a list, receives the
         residual stream after every layer run."""
         segments = meta.segments(input_ids.shape[0])
+        if self.spec.output_norms:
+            return self._forward_output_normed(input_ids, kv_caches, meta, segments, trail)
         x = self._embed(input_ids, meta, segments)
         norm = {"eps": self.spec.rms_eps, "offset": self.spec.norm_offset,
                 "dtype": self.dtype}
@@ -167,6 +196,35 @@ class HybridForCausalLM(nn.Module):
                 trail.append(y)
         return ops.residual_rmsnorm(x, self.final_norm, **norm, **add)
 
+    def _forward_output_normed(self, input_ids, kv_caches, meta, segments, trail):
+        """Sublayers read the residual itself; one kernel per sublayer norms its
+        result, adds it, and after a layer takes the average over the depth, after
+        the last one the final norm as well."""
+        T, n = input_ids.shape[0], len(self._runs)
+        h = self.embed(input_ids)
+        if self.spec.depth_average:  # the embedding's and the layers' results
+            kept = torch.empty(n, T, h.shape[1], dtype=torch.float32, device=h.device)
+            src = kept[0].copy_(h)
+        else:
+            kept, src = None, h.float()
+        x = torch.empty_like(src)
+        norm = {"eps": self.spec.rms_eps, "dtype": self.dtype}
+        for run, (i, _, kv, st) in enumerate(self._runs):
+            layer = self.layers[i]
+            last = {} if kept is None else {"depth": (kept, layer.depth)}
+            if run == n - 1:
+                last["final"] = (self.final_norm, self.final_norm_bias)
+            y = layer.mixer(h, meta, segments, kv_caches[kv], meta.states[st])
+            h = ops.output_norm(src, x, layer.norm1, layer.norm1_bias, delta=y, **norm,
+                                **(last if layer.mlp is None else {}))
+            if layer.mlp is not None:
+                h = ops.output_norm(x, x, layer.norm2, layer.norm2_bias, **layer.mlp(h),
+                                    **norm, **last)
+            src = x
+            if trail is not None:
+                trail.append(x.clone())
+        return h
+
     @torch.inference_mode()
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
         return ops.linear(hidden, self.lm_head).float()
@@ -189,6 +247,8 @@ class HybridForCausalLM(nn.Module):
         """Weights held as they are stored (or views of them), by name."""
         out = {"embed": self.embed.weight.data, "final.norm": self.final_norm.data,
                "head": self.lm_head.data}
+        if self.final_norm_bias is not None:
+            out["final.norm.b"] = self.final_norm_bias.data
         if self.loop_step is not None:
             out["loop.step"] = self.loop_step.data
         if self.spec.embedding is not None:
@@ -197,6 +257,10 @@ class HybridForCausalLM(nn.Module):
             out[f"l{i}.norm1"] = layer.norm1.data
             if layer.mlp is not None:
                 out[f"l{i}.norm2"] = layer.norm2.data
+            for name, t in (("norm1.b", layer.norm1_bias), ("norm2.b", layer.norm2_bias),
+                            ("dwa", layer.depth)):
+                if t is not None:
+                    out[f"l{i}.{name}"] = t.data
             if layer.conv is not None:
                 out[f"l{i}.canon1"] = layer.conv.data.t()
             if layer.gate is not None:
@@ -246,7 +310,14 @@ class HybridForCausalLM(nn.Module):
         if self.spec.embedding is not None:
             self.pairs.copy_(randn(self.pairs.shape))
             self.embed_norm.copy_(norm_weight())
+        for bias in [self.final_norm_bias] + [b for layer in self.layers for b in
+                                              (layer.norm1_bias, layer.norm2_bias)]:
+            if bias is not None:
+                bias.copy_(randn((w,)) * 0.1)
         for layer in self.layers:
+            if layer.depth is not None:  # mostly the last, something of all
+                layer.depth.copy_(randn(tuple(layer.depth.shape)) * 0.1)
+                layer.depth[-1] += 1.0
             layer.norm1.copy_(norm_weight())
             layer.mixer.init_random(randn)
             if layer.conv is not None:

@@ -15,8 +15,13 @@ import torch.nn as nn
 from .. import ops
 from .config import (
     DenseSpec,
+    FusedMixerSpec,
+    GroupedMoESpec,
+    HeadDeltaSpec,
     LatentAttentionSpec,
+    MatrixMemorySpec,
     MoESpec,
+    NormedAttentionSpec,
     ParallelMixerSpec,
     RetentionSpec,
 )
@@ -334,6 +339,232 @@ class LatentAttention(nn.Module):
         return ops.linear(out, self.out_proj)
 
 
+class MixerPart(nn.Module):
+    """One of the mixers a ``FusedMixer`` runs side by side: its columns of the
+    common input projection, weights of its own, and heads for the common output
+    projection."""
+
+    #: names of the checkpoint's tensors beside projections and "o", with their
+    #: shapes; each is held as the fp32 parameter of the same place in ``own``
+    shapes: Dict[str, Tuple[int, ...]]
+
+    def __init__(self, spec, columns: Sequence[Tuple[str, int]], out_width: int,
+                 shapes: Dict[str, Tuple[int, ...]]):
+        super().__init__()
+        self.spec = spec
+        self.columns = list(columns)
+        self.out_width = out_width
+        self.shapes = shapes
+        self.own = nn.ParameterList([_param(*s, dtype=torch.float32)
+                                     for s in shapes.values()])
+        self._p = None
+
+    def kv_layout(self, dtype, device) -> List[Tuple[int, int, int]]:
+        return []
+
+    def state_layout(self, dtype) -> List[tuple]:
+        return []
+
+    def tensors(self) -> Dict[str, torch.Tensor]:
+        return dict(zip(self.shapes, self.own))
+
+    def random(self, name: str, randn) -> torch.Tensor:
+        """A random tensor of ``shapes``."""
+        return 1.0 + 0.1 * randn(self.shapes[name])
+
+    def params(self, at: Dict[str, int], eps: float):
+        """The kernels' sizes, columns and weights; built lazily, for the tensors
+        move with .to(device)."""
+        if self._p is None or self._device != self.own[0].device:
+            self._device = self.own[0].device
+            self._p = self.make_params(
+                at, {n: t.data for n, t in self.tensors().items()}, eps)
+        return self._p
+
+
+class NormedAttention(MixerPart):
+    """Grouped-query attention over normed queries and keys, with rotary
+    positions or a logarithmic distance bias, query temperature and sink."""
+
+    def __init__(self, spec: NormedAttentionSpec, max_position: int, rotations: dict):
+        H, G, d, e = spec.heads, spec.kv_heads, spec.dim, spec.vdim
+        columns = [("q", H * d), ("k", G * d)]
+        if not spec.shared_kv:
+            columns.append(("v", G * e))
+        if spec.norm not in ("head", "whole"):
+            raise ValueError(f"unknown norm of queries and keys {spec.norm!r}")
+        whole = spec.norm == "whole"
+        shapes = {"q.norm": (H * d if whole else d,), "k.norm": (G * d if whole else d,)}
+        if spec.log_bias:
+            shapes["r1"] = shapes["r2"] = (H,)
+        super().__init__(spec, columns, H * e, shapes)
+        cos_sin = None
+        if spec.rot_dims:
+            key = (spec.rot_dims, spec.rot_base)
+            if key not in rotations:  # one table for all layers that share it
+                rotations[key] = ops.torch_ref.rope_cos_sin_cache(
+                    spec.rot_dims, max_position, spec.rot_base)
+            cos_sin = rotations[key]
+        self.register_buffer("cos_sin", cos_sin, persistent=False)
+        zeros = torch.zeros(H, dtype=torch.float32)
+        self.register_buffer("flat", None if spec.log_bias else zeros, persistent=False)
+        self.register_buffer("sink", zeros.clone() if spec.sink else None, persistent=False)
+
+    def kv_layout(self, dtype, device):
+        s = self.spec
+        return [(s.kv_heads, *ops.cache_head_dims(s.dim, s.vdim, dtype, device))]
+
+    def random(self, name, randn):
+        # distances that matter, of every reach
+        return randn(self.shapes[name]).abs() if name in ("r1", "r2") \
+            else super().random(name, randn)
+
+    def make_params(self, at, t, eps):
+        s = self.spec
+        heads = ops.NormedHeadsParams(
+            s.heads, s.kv_heads, s.dim, s.vdim, at["q"], at["k"],
+            at["k" if s.shared_kv else "v"], t["q.norm"], t["k.norm"], s.norm == "whole",
+            eps, self.cos_sin, s.q_temp)
+        return heads, t.get("r1", self.flat), t.get("r2")
+
+    def forward(self, proj, at, eps, meta, segments, kv, state, out, col, scale):
+        s = self.spec
+        heads, slopes, rate = self.params(at, eps)
+        k_cache, v_cache = kv[0]
+        q = ops.normed_qkv(proj, heads, meta.positions, meta.slot_mapping, k_cache, v_cache)
+        for seg in segments:
+            ops.biased_attention(q, k_cache, v_cache, seg, s.scale, 0, slopes, out, col,
+                                 s.vdim, scale, rate, self.sink)
+
+
+class HeadDelta(MixerPart):
+    """Gated delta rule with one decay per head."""
+
+    def __init__(self, spec: HeadDeltaSpec):
+        H, ck, cv = spec.heads, spec.kv_heads * spec.dim, spec.heads * spec.vdim
+        super().__init__(
+            spec, [("q", ck), ("k", ck), ("v", cv), ("b", H), ("a", H), ("g", cv)], cv,
+            {"q.conv": (ck, spec.conv), "k.conv": (ck, spec.conv), "v.conv": (cv, spec.conv),
+             "A_log": (H,), "dt_bias": (H,), "norm": (spec.vdim,)})
+
+    def state_layout(self, dtype):
+        s = self.spec
+        channels = 2 * s.kv_heads * s.dim + s.heads * s.vdim
+        return [(((s.heads, s.dim, s.vdim), torch.float32), ((s.conv, channels), dtype))]
+
+    def random(self, name, randn):
+        x = randn(self.shapes[name])
+        return {"A_log": x * 0.5, "dt_bias": x - 3.0, "norm": 1.0 + 0.1 * x}.get(
+            name, x * self.spec.conv ** -0.5)
+
+    def make_params(self, at, t, eps):
+        s = self.spec
+        return ops.HeadDeltaParams(
+            s.heads, s.kv_heads, s.dim, s.vdim, s.conv, *(at[n] for n in "qkvbag"),
+            torch.cat([t[f"{n}.conv"] for n in "qkv"]), t["A_log"], t["dt_bias"], t["norm"],
+            eps)
+
+    def forward(self, proj, at, eps, meta, segments, kv, state, out, col, scale):
+        p = self.params(at, eps)
+        for seg in segments:
+            ops.head_delta_rule(proj, p, *state[0], seg, out, col, scale)
+
+
+class MatrixMemory(MixerPart):
+    """mLSTM: a decaying sum of key-value products with exponential input gates,
+    read through its normaliser."""
+
+    def __init__(self, spec: MatrixMemorySpec):
+        H, n, e = spec.heads, spec.heads * spec.dim, spec.heads * spec.vdim
+        super().__init__(
+            spec, [("q", n), ("k", n), ("v", e), ("i", H), ("f", H), ("g", e)], e,
+            {"i.b": (H,), "f.b": (H,), "norm": (e,)})
+
+    def state_layout(self, dtype):
+        s, f32 = self.spec, torch.float32
+        return [(((s.heads, s.dim, s.vdim), f32), ((s.heads, s.dim), f32), ((s.heads,), f32))]
+
+    def random(self, name, randn):
+        x = randn(self.shapes[name])
+        return {"i.b": x, "f.b": x + 4.0}.get(name, 1.0 + 0.1 * x)
+
+    def make_params(self, at, t, eps):
+        s = self.spec
+        return ops.MatrixMemoryParams(
+            s.heads, s.dim, s.vdim, *(at[n] for n in "qkvifg"), t["i.b"], t["f.b"],
+            t["norm"], s.gate_cap, eps)
+
+    def forward(self, proj, at, eps, meta, segments, kv, state, out, col, scale):
+        p = self.params(at, eps)
+        for seg in segments:
+            ops.matrix_memory(proj, p, *state[0], seg, out, col, scale)
+
+
+class FusedMixer(nn.Module):
+    """Parts side by side. All read one fused input projection and write their
+    scaled heads into one buffer, so the output projections and their sum are a
+    single product."""
+
+    def __init__(self, spec: FusedMixerSpec, hidden: int, eps: float, dtype,
+                 max_position: int, rotations: dict):
+        super().__init__()
+        self.eps = eps
+        self.names = [name for name, _, _ in spec.parts]
+        self.scales = [scale for _, _, scale in spec.parts]
+        make = {NormedAttentionSpec: lambda s: NormedAttention(s, max_position, rotations),
+                HeadDeltaSpec: HeadDelta, MatrixMemorySpec: MatrixMemory}
+        self.parts = nn.ModuleList([make[type(s)](s) for _, s, _ in spec.parts])
+        self.cols = FusedColumns([(name + n, w) for name, part in zip(self.names, self.parts)
+                                  for n, w in part.columns])
+        #: each part's columns under its own names
+        self.at = [{n: self.cols.at[name + n] for n, _ in part.columns}
+                   for name, part in zip(self.names, self.parts)]
+        self.in_proj = _param(self.cols.total, hidden, dtype=dtype)
+        self.out_proj = _param(hidden, sum(p.out_width for p in self.parts), dtype=dtype)
+
+    def kv_layout(self, dtype, device) -> List[Tuple[int, int, int]]:
+        return [e for p in self.parts for e in p.kv_layout(dtype, device)]
+
+    def state_layout(self, dtype) -> List[tuple]:
+        return [e for p in self.parts for e in p.state_layout(dtype)]
+
+    def load(self, get) -> None:
+        self.cols.pack({n: get(n) for n in self.cols.at}, self.in_proj)
+        for name, part in zip(self.names, self.parts):
+            for n, t in part.tensors().items():
+                t.copy_(get(name + n))
+        self.out_proj.copy_(torch.cat([get(name + "o") for name in self.names], dim=1))
+
+    def tensors(self) -> Dict[str, torch.Tensor]:
+        out = dict(self.cols.unpack(self.in_proj))
+        for name, part, o in zip(self.names, self.parts, self.out_proj.split(
+                [p.out_width for p in self.parts], dim=1)):
+            out.update({name + n: t for n, t in part.tensors().items()})
+            out[name + "o"] = o
+        return out
+
+    def init_random(self, randn) -> None:
+        hidden = self.out_proj.shape[0]
+        made = {}
+        for name, part in zip(self.names, self.parts):
+            made.update({name + n: part.random(n, randn) for n in part.shapes})
+            made[name + "o"] = randn((hidden, part.out_width)) * part.out_width ** -0.5
+        self.load(lambda n: made[n] if n in made
+                  else randn((self.cols.width[n], hidden)) * hidden ** -0.5)
+
+    def forward(self, h, meta, segments, kv, state):
+        proj = ops.linear(h, self.in_proj)
+        out = torch.empty(h.shape[0], self.out_proj.shape[1], dtype=h.dtype,
+                          device=h.device)
+        col = k0 = s0 = 0
+        for part, at, scale in zip(self.parts, self.at, self.scales):
+            k1 = k0 + len(part.kv_layout(h.dtype, h.device))
+            s1 = s0 + len(part.state_layout(h.dtype))
+            part(proj, at, self.eps, meta, segments, kv[k0:k1], state[s0:s1], out, col, scale)
+            col, k0, s0 = col + part.out_width, k1, s1
+        return ops.linear(out, self.out_proj)
+
+
 class DenseXieluMLP(nn.Module):
     """Two matrices around an xIELU. With ``gated``, the residual gate's
     projection of the same input shares the first product."""
@@ -381,6 +612,29 @@ class DenseXieluMLP(nn.Module):
         return add
 
 
+class DenseGeluMLP(nn.Module):
+    """Two matrices around an exact gelu."""
+
+    def __init__(self, spec: DenseSpec, hidden: int, dtype):
+        super().__init__()
+        self.up = _param(spec.ff, hidden, dtype=dtype)
+        self.down = _param(hidden, spec.ff, dtype=dtype)
+
+    def load(self, get) -> None:
+        self.up.copy_(get("up"))
+        self.down.copy_(get("down"))
+
+    def tensors(self) -> Dict[str, torch.Tensor]:
+        return {"up": self.up, "down": self.down}
+
+    def init_random(self, randn) -> None:
+        self.load(lambda n: randn(tuple(getattr(self, n).shape))
+                  * getattr(self, n).shape[1] ** -0.5)
+
+    def forward(self, h) -> Dict[str, object]:
+        return {"delta": ops.linear(ops.gelu(ops.linear(h, self.up)), self.down)}
+
+
 class RoutedGLU(nn.Module):
     """Top-k routed clamped-GLU experts with a biased fp32 router. Returns the
     chosen experts' rows unsummed; the next residual norm adds them up."""
@@ -425,3 +679,56 @@ class RoutedGLU(nn.Module):
         s = self.spec
         return {"moe": ops.moe_clamped_glu(h, self.router, self.router_bias, s.top,
                                            self.gate_up, self.down, s.limit, self.ALPHA)}
+
+
+class GroupedGLU(nn.Module):
+    """Sigmoid-routed GLU experts chosen among the best groups, beside a shared
+    expert whose gate is one more row of its first product. Returns the chosen
+    rows unsummed; the output norm adds everything up."""
+
+    def __init__(self, spec: GroupedMoESpec, hidden: int, dtype):
+        super().__init__()
+        self.spec = spec
+        E, ff, sf = spec.experts, spec.ff, spec.shared_ff
+        self.router = _param(E, hidden, dtype=dtype)
+        self.correction = _param(E, dtype=torch.float32)
+        self.gate_up = _param(E, 2 * ff, hidden, dtype=dtype)
+        self.down = _param(E, hidden, ff, dtype=dtype)
+        if sf:
+            # [gate; up; the shared gate's row; zeros]
+            self.shared_in = _param(-(-(2 * sf + 1) // 64) * 64, hidden, dtype=dtype)
+            self.shared_down = _param(hidden, sf, dtype=dtype)
+
+    def tensors(self) -> Dict[str, torch.Tensor]:
+        """Weights by the checkpoint's names; views that ``load`` fills."""
+        ff, sf = self.spec.ff, self.spec.shared_ff
+        out = {"router": self.router, "correction": self.correction}
+        for e in range(self.spec.experts):
+            out[f"e{e}.gate"] = self.gate_up[e, :ff]
+            out[f"e{e}.up"] = self.gate_up[e, ff:]
+            out[f"e{e}.down"] = self.down[e]
+        if sf:
+            out["shared.gate"], out["shared.up"] = self.shared_in[:sf], self.shared_in[sf:2 * sf]
+            out["shared.sg"] = self.shared_in[2 * sf:2 * sf + 1]
+            out["shared.down"] = self.shared_down
+        return out
+
+    def load(self, get) -> None:
+        for name, t in self.tensors().items():
+            t.copy_(get(name))
+
+    def init_random(self, randn) -> None:
+        tensors = self.tensors()
+        self.load(lambda n: randn(tuple(tensors[n].shape))
+                  * (0.1 if n == "correction" else tensors[n].shape[1] ** -0.5))
+
+    def forward(self, h) -> Dict[str, object]:
+        s = self.spec
+        add: Dict[str, object] = {"moe": ops.moe_grouped_glu(
+            h, self.router, self.correction, s.top, s.groups, s.keep, s.scale, self.gate_up,
+            self.down)}
+        if s.shared_ff:
+            z = ops.linear(h, self.shared_in)
+            add["delta"] = ops.linear(ops.silu_glu(z, s.shared_ff), self.shared_down)
+            add["gate"] = z[:, 2 * s.shared_ff]
+        return add

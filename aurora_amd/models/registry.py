@@ -34,6 +34,7 @@ _ARCHS = {
     "llama": (_llama, _load_llama),
     "kikalix": (_hybrid, _load_named),
     "senotar": (_hybrid, _load_named),
+    "gakupel": (_hybrid, _load_named),
 }
 
 

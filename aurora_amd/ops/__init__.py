@@ -242,7 +242,10 @@ def softmax_sample(logits, temperature, top_p, top_k, generator=None):
 
 from .sequence import (  # noqa: E402
     DeltaRuleParams,
+    HeadDeltaParams,
     LatentParams,
+    MatrixMemoryParams,
+    NormedHeadsParams,
     RetentionParams,
     Segment,
     bias_kv_write,
@@ -250,14 +253,21 @@ from .sequence import (  # noqa: E402
     cache_head_dims,
     delta_rule,
     embed_pairs,
+    gelu,
+    head_delta_rule,
     latent_attention,
     latent_head_width,
     latent_width,
     latent_write,
+    matrix_memory,
     moe_clamped_glu,
+    moe_grouped_glu,
+    normed_qkv,
+    output_norm,
     residual_rmsnorm,
     residual_rmsnorm_conv,
     retention,
     short_conv_add,
+    silu_glu,
     xielu,
 )

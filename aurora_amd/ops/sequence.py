@@ -1,6 +1,7 @@
 """Ops of the layer-listed decoders: biased window attention over paged KV,
-the gated delta rule, retention, routed clamped-GLU experts, latent attention,
-pair embeddings and the mixers' input convolution.
+gated delta rules, retention, matrix memories, routed GLU experts, latent
+attention, normed attention heads, pair embeddings, the mixers' input
+convolution and the residual's norms.
 
 Same dispatch rule as the rest of the package: GPU tensors run the gfx950
 kernels (bf16, or float32 throughout) and fail loudly without the extension;
@@ -66,6 +67,63 @@ class RetentionParams:
     decay: torch.Tensor    # [heads] fp32
     cos_sin: torch.Tensor  # [positions, rot_dims] fp32
     eps: float
+
+
+@dataclass
+class HeadDeltaParams:
+    """The gated delta rule with one decay per head and a silu gate."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+    q0: int
+    k0: int
+    v0: int
+    b0: int
+    a0: int
+    g0: int
+    conv_w: torch.Tensor   # [2*kv_heads*dim + heads*vdim, taps]
+    a_log: torch.Tensor    # [heads]
+    dt_bias: torch.Tensor  # [heads]
+    norm: torch.Tensor     # [vdim]
+    eps: float
+
+
+@dataclass
+class MatrixMemoryParams:
+    heads: int
+    dim: int
+    vdim: int
+    q0: int
+    k0: int
+    v0: int
+    i0: int
+    f0: int
+    g0: int
+    i_bias: torch.Tensor   # [heads]
+    f_bias: torch.Tensor   # [heads]
+    norm: torch.Tensor     # [heads * vdim]
+    cap: float
+    eps: float
+
+
+@dataclass
+class NormedHeadsParams:
+    """Normed queries and keys of an attention; v0 = k0: values are plain keys."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    q0: int
+    k0: int
+    v0: int
+    q_norm: torch.Tensor   # [dim], or [heads * dim] if ``whole``
+    k_norm: torch.Tensor
+    whole: bool            # one norm over all heads of a token
+    eps: float
+    cos_sin: Optional[torch.Tensor] = None  # [positions, rotated dims] fp32
+    temp: Optional[Tuple[float, int]] = None
 
 
 def latent_width(rank: int) -> int:
@@ -347,38 +405,43 @@ def bias_kv_write(proj, cols, bias, slots, k_cache, v_cache, heads, kv_heads, di
         heads, kv_heads, dim, vdim)
 
 
+def normed_qkv(proj, p: NormedHeadsParams, positions, slots, k_cache, v_cache):
+    """Queries of a fused projection; keys and values go to the cache."""
+    if not proj.is_cuda:
+        return torch_ref.normed_qkv(proj, p, positions, slots, k_cache, v_cache)
+    coef, every = p.temp or (0.0, 1)
+    return _hip("normed_qkv").normed_qkv(
+        proj, p.q0, p.k0, p.v0, p.q_norm, p.k_norm, p.whole, float(p.eps), p.cos_sin,
+        float(coef), every, positions, slots, k_cache, v_cache, p.heads, p.kv_heads,
+        p.dim, p.vdim)
+
+
 def biased_attention(q, k_cache, v_cache, seg: Segment, scale, window, slopes,
-                     out, col, vdim, out_scale):
+                     out, col, vdim, out_scale, log_rate=None, sink=None):
     """Attention of one segment's rows into out[rows, col:col+heads*vdim]."""
     qs, os_ = q[seg.rows], out[seg.rows]
+    extra = (scale, window, slopes, log_rate, sink, os_, col, vdim, out_scale)
     if not q.is_cuda:
         torch_ref.biased_attention_paged(
             qs, k_cache, v_cache, seg.block_tables, seg.cu_or_rows(qs.shape[0]),
-            seg.context_lens, scale, window, slopes, os_, col, vdim, out_scale)
+            seg.context_lens, scale, window, slopes, os_, col, vdim, out_scale,
+            log_rate, sink)
         return
     m = _hip("biased_attention")
     matrix = (q.dtype == torch.bfloat16 and q.shape[2] in MATRIX_HEAD_DIMS
               and v_cache.shape[3] in MATRIX_HEAD_DIMS)
     if matrix and seg.decode:
         m.biased_attention_decode(qs, k_cache, v_cache, seg.block_tables,
-                                  seg.context_lens, scale, window, slopes,
-                                  os_, col, vdim, out_scale)
+                                  seg.context_lens, *extra)
     elif matrix:
         rows = m.biased_prefill_rows(q.shape[1] // k_cache.shape[1])
         bseq, boff = seg.block_map(rows)
         m.biased_attention_prefill(qs, k_cache, v_cache, seg.block_tables, seg.cu,
-                                   seg.context_lens, bseq, boff, scale, window, slopes,
-                                   os_, col, vdim, out_scale)
+                                   seg.context_lens, bseq, boff, *extra)
     else:
-        if seg.decode:
-            m.biased_attention_rows(qs, k_cache, v_cache, seg.block_tables, None,
-                                    seg.context_lens, None, None, scale, window,
-                                    slopes, os_, col, vdim, out_scale)
-        else:
-            bseq, boff = seg.block_map(1)
-            m.biased_attention_rows(qs, k_cache, v_cache, seg.block_tables, seg.cu,
-                                    seg.context_lens, bseq, boff, scale, window,
-                                    slopes, os_, col, vdim, out_scale)
+        bseq, boff = (None, None) if seg.decode else seg.block_map(1)
+        m.biased_attention_rows(qs, k_cache, v_cache, seg.block_tables, seg.cu,
+                                seg.context_lens, bseq, boff, *extra)
 
 
 def delta_rule(proj, z, p: DeltaRuleParams, state, conv, seg: Segment,
@@ -398,6 +461,42 @@ def delta_rule(proj, z, p: DeltaRuleParams, state, conv, seg: Segment,
         m.delta_prefill(pr, zs, *w, *sizes, p.eps, state, conv, seg.cu,
                         *seg.chunk_map(), seg.starts,
                         seg.state_slots, os_, col, out_scale)
+
+
+def head_delta_rule(proj, p: HeadDeltaParams, state, conv, seg: Segment, out, col,
+                    out_scale):
+    pr, os_ = proj[seg.rows], out[seg.rows]
+    if not proj.is_cuda:
+        torch_ref.head_delta_rule(pr, p, state, conv, seg.cu_or_rows(pr.shape[0]),
+                                  seg.starts, seg.state_slots, os_, col, out_scale)
+        return
+    m = _hip("head_delta_rule")
+    args = (pr, p.conv_w, p.a_log, p.dt_bias, p.norm, p.heads, p.kv_heads, p.dim, p.vdim,
+            p.taps, p.q0, p.k0, p.v0, p.b0, p.a0, p.g0, p.eps, state, conv)
+    if seg.decode:
+        m.head_delta_decode(*args, seg.starts, seg.state_slots, os_, col, out_scale)
+    else:
+        m.head_delta_prefill(*args, seg.cu, *seg.chunk_map(), seg.starts, seg.state_slots,
+                             os_, col, out_scale)
+
+
+def matrix_memory(proj, p: MatrixMemoryParams, state, norm, top, seg: Segment, out, col,
+                  out_scale):
+    """``state``, ``norm`` and ``top`` hold every slot's memory, normaliser and
+    running maximum."""
+    pr, os_ = proj[seg.rows], out[seg.rows]
+    if not proj.is_cuda:
+        torch_ref.matrix_memory(pr, p, state, norm, top, seg.cu_or_rows(pr.shape[0]),
+                                seg.starts, seg.state_slots, os_, col, out_scale)
+        return
+    m = _hip("matrix_memory")
+    args = (pr, p.i_bias, p.f_bias, p.norm, p.heads, p.dim, p.vdim, p.q0, p.k0, p.v0,
+            p.i0, p.f0, p.g0, p.cap, p.eps, state, norm, top)
+    if seg.decode:
+        m.memory_decode(*args, seg.starts, seg.state_slots, os_, col, out_scale)
+    else:
+        m.memory_prefill(*args, seg.cu, *seg.chunk_map(), seg.starts, seg.state_slots,
+                         os_, col, out_scale)
 
 
 def retention(proj, p: RetentionParams, state, seg: Segment, out):
@@ -422,9 +521,48 @@ def moe_clamped_glu(h, router, bias, top: int, w_gate_up, w_down, limit: float,
     ``residual_rmsnorm``, which adds the weighted rows to the residual."""
     if not h.is_cuda:
         sel, weights = torch_ref.moe_route(h, router, bias, top)
-        y, place = torch_ref.moe_clamped_glu(h, sel, w_gate_up, w_down, limit, alpha)
-        return y, place, weights
-    m = _hip("moe_clamped_glu")
-    sel, weights = m.moe_route(h, router, bias, top)
-    y, place = m.moe_clamped_glu(h, sel, w_gate_up, w_down, float(limit), float(alpha))
+    else:
+        sel, weights = _hip("moe_route").moe_route(h, router, bias, top)
+    y, place = expert_rows(h, sel, w_gate_up, w_down, limit, alpha, 1.0)
     return y, place, weights
+
+
+def moe_grouped_glu(h, router, correction, top: int, groups: int, keep: int, scale: float,
+                    w_gate_up, w_down):
+    """Plain GLU experts chosen by corrected sigmoid scores among the best groups;
+    (y, place, weights) for ``output_norm``."""
+    route = torch_ref.moe_route_grouped if not h.is_cuda else \
+        _hip("moe_route_grouped").moe_route_grouped
+    sel, weights = route(h, router, correction, top, groups, keep, float(scale))
+    y, place = expert_rows(h, sel, w_gate_up, w_down, float("inf"), 1.0, 0.0)
+    return y, place, weights
+
+
+def expert_rows(h, sel, w_gate_up, w_down, limit: float, alpha: float, shift: float):
+    f = torch_ref.moe_clamped_glu if not h.is_cuda else \
+        _hip("moe_clamped_glu").moe_clamped_glu
+    return f(h, sel, w_gate_up, w_down, float(limit), float(alpha), float(shift))
+
+
+def output_norm(src, x, weight, bias, eps, delta=None, gate=None, moe=None, depth=None,
+                final=None, dtype=None):
+    """x = src + layer norm of a sub-layer's result (see ``torch_ref``), with the
+    depth average and the final norm that may follow it in the same kernel."""
+    if not src.is_cuda:
+        return torch_ref.output_norm(src, x, weight, bias, eps, delta, gate, moe, depth,
+                                     final, dtype)
+    y, place, share = moe if moe is not None else (None, None, None)
+    kept, coefs = depth if depth is not None else (None, None)
+    fw, fb = final if final is not None else (None, None)
+    return _hip("output_norm").output_norm(
+        src, x, weight, bias, delta, gate, y, place, share, kept, coefs, fw, fb, float(eps),
+        dtype == torch.bfloat16)
+
+
+def gelu(z):
+    """Rows of ``z`` may be strided."""
+    return torch_ref.gelu(z) if not z.is_cuda else _hip("gelu").gelu(z)
+
+
+def silu_glu(z, ff: int):
+    return torch_ref.silu_glu(z, ff) if not z.is_cuda else _hip("silu_glu").silu_glu(z, ff)

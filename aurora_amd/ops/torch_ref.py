@@ -297,10 +297,12 @@ def _paged_rows(cache, pages, L):
 
 def biased_attention_paged(q, k_cache, v_cache, block_tables, cu_seqlens_q,
                            context_lens, scale, window, slopes, out, col, vdim,
-                           out_scale):
-    """Causal paged attention with a window and a linear distance penalty
-    slope_h * (i - j); writes out[:, col : col + heads * vdim] times
-    out_scale. Decode is the case of one query per sequence."""
+                           out_scale, log_rate=None, sink=None):
+    """Causal paged attention with a window and a distance penalty slope_h *
+    (i - j), or with ``log_rate`` slope_h * ln(1 + rate_h (i - j)), and with
+    ``sink`` one more term e^sink_h of the denominator; writes
+    out[:, col : col + heads * vdim] times out_scale. Decode is the case of one
+    query per sequence."""
     T, Hq, _ = q.shape
     P = k_cache.shape[2]
     g = Hq // k_cache.shape[1]
@@ -315,12 +317,16 @@ def biased_attention_paged(q, k_cache, v_cache, block_tables, cu_seqlens_q,
         att = torch.einsum("qhd,hkd->hqk", q[a:b].float(), ks) * scale
         dist = (torch.arange(L - (b - a), L, device=q.device).unsqueeze(1)
                 - torch.arange(L, device=q.device).unsqueeze(0))
-        att = att - slopes.view(-1, 1, 1) * dist
+        far = dist.clamp(min=0) if log_rate is None else \
+            torch.log(1 + log_rate.view(-1, 1, 1) * dist.clamp(min=0))
+        att = att - slopes.view(-1, 1, 1) * far
         hidden = dist < 0
         if window:
             hidden = hidden | (dist >= window)
         att.masked_fill_(hidden, float("-inf"))
-        o = torch.einsum("hqk,hkd->qhd", att.softmax(-1), vs) * out_scale
+        if sink is not None:
+            att = torch.cat([att, sink.view(-1, 1, 1).expand(Hq, b - a, 1)], -1)
+        o = torch.einsum("hqk,hkd->qhd", att.softmax(-1)[..., :L], vs) * out_scale
         out[a:b, col:col + Hq * vdim] = o.reshape(b - a, -1).to(out.dtype)
 
 
@@ -334,7 +340,8 @@ def _head_rms(o, eps):
 
 def _delta_run(x, z, beta_in, p, start, S, conv):
     """One sequence's tokens from position ``start``: x [n, C] raw q|k|v
-    projections, S [H, d, e] and conv [taps, C] updated in place."""
+    projections, z [n, H*d | H] the decay's pre-activations, S [H, d, e] and conv
+    [taps, C] updated in place -> o / rms(o) times the norm's weight."""
     n = x.shape[0]
     H, G, d, e, taps = p.heads, p.kv_heads, p.dim, p.vdim, p.taps
     past = torch.zeros(taps - 1, x.shape[1])
@@ -350,7 +357,7 @@ def _delta_run(x, z, beta_in, p, start, S, conv):
     k = _l2_unit(y[:, G * d:2 * G * d].reshape(n, G, d))
     v = y[:, 2 * G * d:].reshape(n, H, e)
     q, k = (t.repeat_interleave(H // G, 1) for t in (q, k))
-    u = (z[:, :H * d].float() + p.dt_bias).reshape(n, H, d)
+    u = (z.float() + p.dt_bias).reshape(n, H, -1)
     decay = torch.exp(-p.a_log.exp().view(1, H, 1) * torch.nn.functional.softplus(u))
     beta = torch.sigmoid(beta_in.float())
     if start == 0:
@@ -361,8 +368,7 @@ def _delta_run(x, z, beta_in, p, start, S, conv):
         w = beta[t].unsqueeze(-1) * (v[t] - torch.einsum("hde,hd->he", S, k[t]))
         S.add_(k[t].unsqueeze(-1) * w.unsqueeze(1))
         o[t] = torch.einsum("hde,hd->he", S, q[t])
-    gate = torch.sigmoid(z[:, H * d:].float()).reshape(n, H, e)
-    return (_head_rms(o, p.eps) * p.norm * gate).reshape(n, H * e)
+    return (_head_rms(o, p.eps) * p.norm).reshape(n, H * e)
 
 
 def delta_rule(proj, z, p, state, conv, cu, starts, slots, out, col, out_scale):
@@ -375,9 +381,59 @@ def delta_rule(proj, z, p, state, conv, cu, starts, slots, out, col, out_scale):
         r = proj[a:b]
         x = torch.cat([r[:, p.q0:p.q0 + G * d], r[:, p.k0:p.k0 + G * d],
                        r[:, p.v0:p.v0 + p.heads * p.vdim]], 1)
-        y = _delta_run(x, z[a:b], r[:, p.b0:p.b0 + p.heads], p, int(starts[s]),
-                       state[slot], conv[slot])
+        nd = p.heads * d
+        y = _delta_run(x, z[a:b, :nd], r[:, p.b0:p.b0 + p.heads], p, int(starts[s]),
+                       state[slot], conv[slot]) * torch.sigmoid(z[a:b, nd:].float())
         out[a:b, col:col + p.heads * p.vdim] = (y * out_scale).to(out.dtype)
+
+
+def head_delta_rule(proj, p, state, conv, cu, starts, slots, out, col, out_scale):
+    """The rule with one decay per head and a silu gate, all from columns of the
+    projection."""
+    G, d, H, e = p.kv_heads, p.dim, p.heads, p.vdim
+    for s in range(len(slots)):
+        a, b, slot = int(cu[s]), int(cu[s + 1]), int(slots[s])
+        if slot < 0 or a == b:
+            continue
+        r = proj[a:b]
+        x = torch.cat([r[:, p.q0:p.q0 + G * d], r[:, p.k0:p.k0 + G * d],
+                       r[:, p.v0:p.v0 + H * e]], 1)
+        y = _delta_run(x, r[:, p.a0:p.a0 + H], r[:, p.b0:p.b0 + H], p, int(starts[s]),
+                       state[slot], conv[slot])
+        g = r[:, p.g0:p.g0 + H * e].float()
+        out[a:b, col:col + H * e] = (y * g * torch.sigmoid(g) * out_scale).to(out.dtype)
+
+
+def matrix_memory(proj, p, state, norm, top, cu, starts, slots, out, col, out_scale):
+    """S_t = e^{f + m - m_t} S + e^{i - m_t} k v', n_t alike with k alone, the
+    running maximum m_t = max(f + m, i); state [slots, H, d, e], norm [slots, H, d]
+    and top [slots, H] hold S, n and m."""
+    H, d, e = p.heads, p.dim, p.vdim
+    for s in range(len(slots)):
+        a, b, slot = int(cu[s]), int(cu[s + 1]), int(slots[s])
+        if slot < 0 or a == b:
+            continue
+        r, n = proj[a:b].float(), b - a
+        take = lambda c, w: r[:, c:c + H * w].reshape(n, H, w)  # noqa: E731
+        q, k, v = take(p.q0, d) * d ** -0.5, take(p.k0, d), take(p.v0, e)
+        i, f = (p.cap * torch.tanh((r[:, c:c + H] + bias) / p.cap)
+                for c, bias in ((p.i0, p.i_bias), (p.f0, p.f_bias)))
+        f = torch.nn.functional.logsigmoid(f)
+        S, N, M = state[slot], norm[slot], top[slot]
+        if int(starts[s]) == 0:
+            S.zero_(), N.zero_(), M.zero_()
+        o = torch.empty(n, H, e)
+        for t in range(n):
+            new = torch.maximum(f[t] + M, i[t])
+            keep, put = torch.exp(f[t] + M - new), torch.exp(i[t] - new)
+            M.copy_(new)
+            S.mul_(keep.view(H, 1, 1)).add_(torch.einsum("hd,he->hde", k[t] * put.view(H, 1), v[t]))
+            N.mul_(keep.view(H, 1)).add_(k[t] * put.view(H, 1))
+            den = torch.maximum((N * q[t]).sum(-1).abs(), torch.exp(-M))
+            o[t] = torch.einsum("hde,hd->he", S, q[t]) / (den + 1e-6).unsqueeze(-1)
+        y = _head_rms(o, p.eps).reshape(n, H * e) * p.norm
+        y = y * torch.sigmoid(r[:, p.g0:p.g0 + H * e])
+        out[a:b, col:col + H * e] = (y * out_scale).to(out.dtype)
 
 
 def retention(proj, p, state, cu, starts, slots, out):
@@ -416,9 +472,11 @@ def moe_route(h, router, bias, top: int):
     return sel.to(torch.int32), val.softmax(-1)
 
 
-def moe_clamped_glu(h, sel, w_gate_up, w_down, limit: float, alpha: float):
+def moe_clamped_glu(h, sel, w_gate_up, w_down, limit: float, alpha: float,
+                    shift: float = 1.0):
     """Every chosen expert's output, unweighted: (y [T*top, W], place [T, top])
-    with place giving the row of each choice."""
+    with place giving the row of each choice. Without a limit, alpha 1 and shift 0
+    make the activation silu(gate) * up."""
     T, top = sel.shape
     ff = w_down.shape[2]
     y = h.new_empty(T * top, h.shape[1])
@@ -431,7 +489,7 @@ def moe_clamped_glu(h, sel, w_gate_up, w_down, limit: float, alpha: float):
         gu = h[tok[rows]].float() @ w_gate_up[e].float().t()
         g = gu[:, :ff].clamp(max=limit)
         u = gu[:, ff:].clamp(-limit, limit)
-        a = (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(h.dtype)
+        a = (g * torch.sigmoid(alpha * g) * (u + shift)).to(h.dtype)
         y[rows] = (a.float() @ w_down[e].float().t()).to(h.dtype)
     return y, torch.arange(T * top, dtype=torch.int32).view(T, top)
 
@@ -526,3 +584,100 @@ def xielu(z, act):
     p, q = torch.nn.functional.softplus(act.float())
     low = (0.5 + q) * (torch.expm1(x.clamp(max=0)) - x)
     return (torch.where(x > 0, p * x * x, low) + 0.5 * x).to(z.dtype)
+
+
+# ---- layer-listed decoders: normed attention heads, output norms, grouped routing
+
+def normed_qkv(proj, p, positions, slots, k_cache, v_cache):
+    """Columns of a fused projection -> normed, rotated and scaled queries [T,
+    heads, DK], and normed, rotated keys and plain values in the paged cache,
+    whose head widths may exceed the model's (zero filled)."""
+    T = proj.shape[0]
+    DK, DV = k_cache.shape[3], v_cache.shape[3]
+
+    def heads(c0, h, w, d, weight):
+        x = proj[:, c0:c0 + h * d].float()
+        if weight is not None:
+            x = (x if p.whole else x.view(T, h, d))
+            x = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + p.eps) * weight
+        return x.reshape(T, h, d)
+
+    def place(x, width):
+        return torch.nn.functional.pad(x, (0, width - x.shape[2])).to(proj.dtype)
+
+    def rotated(x):
+        if p.cos_sin is None:
+            return x
+        cs = p.cos_sin[positions.long()].unsqueeze(1)
+        half = cs.shape[2] // 2
+        cos, sin = cs[..., :half], cs[..., half:]
+        u, w = x[..., :half], x[..., half:2 * half]
+        return torch.cat([u * cos - w * sin, w * cos + u * sin, x[..., 2 * half:]], -1)
+
+    q = rotated(heads(p.q0, p.heads, DK, p.dim, p.q_norm))
+    if p.temp is not None:
+        coef, every = p.temp
+        step = torch.div(positions.long() + 1, every, rounding_mode="floor") + 1
+        q = q * (1 + coef * torch.log(step.float())).view(T, 1, 1)
+    k = rotated(heads(p.k0, p.kv_heads, DK, p.dim, p.k_norm))
+    v = heads(p.v0, p.kv_heads, DV, p.vdim, None)
+    kv_cache_write(place(k, DK), place(v, DV), k_cache, v_cache, slots)
+    return place(q, DK)
+
+
+def _layer_norm(x, weight, bias, eps):
+    d = x - x.mean(-1, keepdim=True)
+    return d * torch.rsqrt(d.pow(2).mean(-1, keepdim=True) + eps) * weight + bias
+
+
+def output_norm(src, x, weight, bias, eps, delta=None, gate=None, moe=None, depth=None,
+                final=None, dtype=None):
+    """x = src + layer_norm(r), r the sub-layer's result: ``delta``, times the
+    sigmoid of one number per row, ``gate``, if given, and the chosen experts'
+    weighted rows. ``depth`` = (kept [n, T, W], coefs [i + 1]): the sum is kept as
+    entry i (if there is room), and x becomes the sum of coefs[j] times entry j.
+    Returns x in ``dtype``, with ``final`` = (weight, bias) its layer norm."""
+    r = torch.zeros_like(src)
+    if delta is not None:
+        y = delta.float()
+        r += y if gate is None else y * torch.sigmoid(gate.float()).unsqueeze(-1)
+    if moe is not None:
+        y, place, weights = moe
+        r += (y.float()[place.long()] * weights.unsqueeze(-1)).sum(1)
+    y = src + _layer_norm(r, weight, bias, eps)
+    if depth is not None:
+        kept, coefs = depth
+        i = coefs.numel() - 1
+        if i < kept.shape[0]:
+            kept[i] = y
+        y = coefs[i] * y + torch.einsum("j,jtw->tw", coefs[:i], kept[:i])
+    x.copy_(y)
+    return (x if final is None else _layer_norm(x, *final, eps)).to(dtype or x.dtype)
+
+
+def gelu(z):
+    """The exact one: z times the normal distribution function."""
+    x = z.float()
+    return (0.5 * x * (1 + torch.erf(x * 0.5 ** 0.5))).to(z.dtype)
+
+
+def silu_glu(z, ff):
+    """silu(gate) * up; z [T, 2 ff ...]: gate columns, then up columns."""
+    g, u = z[:, :ff].float(), z[:, ff:2 * ff].float()
+    return (g * torch.sigmoid(g) * u).to(z.dtype)
+
+
+def moe_route_grouped(h, router, correction, top: int, groups: int, keep: int, scale: float):
+    """Sigmoid scores; the ``top`` best corrected ones among the ``keep`` groups
+    whose two best corrected scores add up to most. -> (ids [T, top] int32, the
+    chosen plain scores' shares of their sum, times scale)."""
+    s = torch.sigmoid(h.float() @ router.float().t())
+    T, E = s.shape
+    choice = s + correction
+    per = choice.view(T, groups, E // groups)
+    best = per.topk(min(2, E // groups), dim=-1).values.sum(-1).topk(keep, dim=-1).indices
+    closed = torch.ones(T, groups, dtype=torch.bool).scatter_(1, best, False)
+    choice = per.masked_fill(closed.unsqueeze(-1), float("-inf")).view(T, E)
+    sel = choice.topk(top, dim=-1).indices
+    w = s.gather(1, sel)
+    return sel.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
