@@ -25,7 +25,11 @@
 #define TUNR 4  // tokens prefetched per group iteration (8 measured neutral)
 #endif
 
-template <int D, int DV, int G, bool FP8, bool BIAS>
+enum { NO_BIAS = 0, LINEAR_BIAS = 1, LOG_BIAS = 2 };
+
+// BIAS: a distance penalty per head (see attention_prefill.hip) and a window; sink:
+// one more term of the denominator per head, or null
+template <int D, int DV, int G, bool FP8, int BIAS>
 __global__ __launch_bounds__(256) void paged_decode_kernel(
     const __hip_bfloat16* __restrict__ q,   // [B, Hq, D]
     const void* __restrict__ kc,  // [NP, Hkv, P, D] bf16 | fp8 e4m3
@@ -37,7 +41,8 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
     int Hkv, int NG,                        // NG: head groups per kv head
     int P, int MP, int CS, float scale,
     long ostride, int dv, float oscale,
-    const float* __restrict__ slopes, int window) {
+    const float* __restrict__ slopes, const float* __restrict__ rates, int window,
+    const float* __restrict__ sink) {
   constexpr int GL = (D > DV ? D : DV) / 8;  // lanes per token-group
   constexpr int TPW = WAVE / GL;   // token-groups per wave
   constexpr int NW = 4;            // waves per workgroup
@@ -69,9 +74,12 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
       qf[g] = *reinterpret_cast<const shortx8*>(
           q + ((long)b * Hq + h0 + g) * D + sub * 8);
   }
-  float slope[G];
+  float slope[G], rate[G];
 #pragma unroll
-  for (int g = 0; g < G; ++g) slope[g] = BIAS ? slopes[h0 + g] : 0.f;
+  for (int g = 0; g < G; ++g) {
+    slope[g] = BIAS ? slopes[h0 + g] : 0.f;
+    rate[g] = BIAS == LOG_BIAS ? rates[h0 + g] : 0.f;
+  }
   // 16-B column of a key / value row this lane reads (lanes past the narrower
   // of the two re-read its last column and contribute nothing)
   const int ksub = min(sub * 8, D - 8), vsub = min(sub * 8, DV - 8);
@@ -127,7 +135,10 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
 #pragma unroll
       for (int g = 0; g < G; ++g) {
         s[g] = group_sum<GL>(dot8_bf16_fast(kf[u], qf[g])) * scale;
-        if constexpr (BIAS) s[g] -= slope[g] * (float)(L - 1 - t0 - u);
+        if constexpr (BIAS != NO_BIAS) {
+          const float dist = (float)(L - 1 - t0 - u);
+          s[g] -= slope[g] * (BIAS == LOG_BIAS ? __logf(1.f + rate[g] * dist) : dist);
+        }
         // defer-style rescale: the running max rarely grows, so the O/l
         // rescale (8*G VALU per token) is branch-skipped when it does not
         if (s[g] > m[g]) {
@@ -164,10 +175,12 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
   __syncthreads();
   for (int gd = tid; gd < G * DV; gd += blockDim.x) {
     const int g = gd / DV, d = gd % DV;
-    float M = -1e30f;
+    const bool ends = BIAS && CS == 1 && sink;  // the sink counts once
+    const float first = ends ? sink[h0 + g] : -1e30f;
+    float M = first;
 #pragma unroll 4
     for (int i = 0; i < NPART; ++i) M = fmaxf(M, s_m[g][i]);
-    float Lsum = 0.f, O = 0.f;
+    float Lsum = ends ? __expf(first - M) : 0.f, O = 0.f;
 #pragma unroll 4
     for (int i = 0; i < NPART; ++i) {
       const float w = __expf(s_m[g][i] - M);
@@ -196,14 +209,16 @@ template <int D>
 __global__ void decode_combine_kernel(const float* __restrict__ part,
                                       __hip_bfloat16* __restrict__ out,
                                       int CS, long BH, int Hq, long ostride,
-                                      int dv, float oscale) {
+                                      int dv, float oscale,
+                                      const float* __restrict__ sink) {
   const long bh = blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
   if (bh >= BH) return;
   const int lane = threadIdx.x % WAVE;
-  float M = -1e30f;
+  const float first = sink ? sink[bh % Hq] : -1e30f;
+  float M = first;
   for (int s = 0; s < CS; ++s)
     M = fmaxf(M, part[((long)s * BH + bh) * (D + 2) + D]);
-  float Lsum = 0.f;
+  float Lsum = sink ? __expf(first - M) : 0.f;
   for (int s = 0; s < CS; ++s) {
     const float* p = part + ((long)s * BH + bh) * (D + 2);
     Lsum += __expf(p[D] - M) * p[D + 1];
@@ -222,12 +237,12 @@ __global__ void decode_combine_kernel(const float* __restrict__ part,
 // query heads sharing one K/V stream: the largest tile that divides the group
 static int head_tile(int G) { return G % 8 == 0 ? 8 : G % 4 == 0 ? 4 : G % 2 == 0 ? 2 : 1; }
 
-template <int D, int DV, bool FP8, bool BIAS>
+template <int D, int DV, bool FP8, int BIAS>
 static void decode_launch(const torch::Tensor& q, const torch::Tensor& kc,
                           const torch::Tensor& vc, const torch::Tensor& bt,
                           const torch::Tensor& ctx, __hip_bfloat16* out, long ostride,
                           int dv, float scale, float oscale, const float* slopes,
-                          int window, int CS) {
+                          const float* rates, int window, const float* sink, int CS) {
   const int B = q.size(0), Hq = q.size(1);
   const int Hkv = kc.size(1), P = kc.size(2), MP = bt.size(1);
   const int G = Hq / Hkv, GT = head_tile(G);
@@ -242,7 +257,7 @@ static void decode_launch(const torch::Tensor& q, const torch::Tensor& kc,
                      0, stream, (const __hip_bfloat16*)q.data_ptr(),            \
                      kc.data_ptr(), vc.data_ptr(), out, pp, bt.data_ptr<int>(), \
                      ctx.data_ptr<int>(), Hkv, G / GT, P, MP, CS, scale,        \
-                     ostride, dv, oscale, slopes, window)
+                     ostride, dv, oscale, slopes, rates, window, sink)
   switch (GT) {
     case 8: LAUNCH(8); break;
     case 4: LAUNCH(4); break;
@@ -253,7 +268,7 @@ static void decode_launch(const torch::Tensor& q, const torch::Tensor& kc,
   if (CS > 1) {
     const long BH = (long)B * Hq;
     hipLaunchKernelGGL((decode_combine_kernel<DV>), dim3((BH + 3) / 4), dim3(256), 0,
-                       stream, pp, out, CS, BH, Hq, ostride, dv, oscale);
+                       stream, pp, out, CS, BH, Hq, ostride, dv, oscale, sink);
   }
   HIP_CHECK_KERNEL();
 }
@@ -274,8 +289,8 @@ torch::Tensor paged_attention_decode(torch::Tensor q, torch::Tensor kc,
   const long stride = (long)Hq * D;
   const bool fp8 = kc.dtype() == torch::kFloat8_e4m3fn;
 #define RUN(DD, F8) \
-  decode_launch<DD, DD, F8, false>(q, kc, vc, bt, ctx, o, stride, D, (float)scale, \
-                                   1.f, nullptr, 0, CS)
+  decode_launch<DD, DD, F8, NO_BIAS>(q, kc, vc, bt, ctx, o, stride, D, (float)scale, \
+                                     1.f, nullptr, nullptr, 0, nullptr, CS)
   if (D == 128) { if (fp8) RUN(128, true); else RUN(128, false); }
   else { if (fp8) RUN(64, true); else RUN(64, false); }
 #undef RUN
@@ -284,7 +299,9 @@ torch::Tensor paged_attention_decode(torch::Tensor q, torch::Tensor kc,
 
 void biased_attention_decode(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                              torch::Tensor bt, torch::Tensor ctx, double scale,
-                             long window, torch::Tensor slopes, torch::Tensor out,
+                             long window, torch::Tensor slopes,
+                             c10::optional<torch::Tensor> rates,
+                             c10::optional<torch::Tensor> sink, torch::Tensor out,
                              long col, long dv, double oscale) {
   TORCH_CHECK(q.is_cuda() && q.dtype() == torch::kBFloat16 && q.is_contiguous());
   const int B = q.size(0), Hq = q.size(1), D = q.size(2);
@@ -296,6 +313,8 @@ void biased_attention_decode(torch::Tensor q, torch::Tensor kc, torch::Tensor vc
   TORCH_CHECK(out.dtype() == torch::kBFloat16 && out.size(0) == B && out.stride(1) == 1 &&
               dv <= DV && col + Hq * dv <= out.size(1));
   TORCH_CHECK(slopes.numel() == Hq && slopes.dtype() == torch::kFloat32);
+  for (auto* t : {&rates, &sink})
+    TORCH_CHECK(!*t || ((*t)->numel() == Hq && (*t)->dtype() == torch::kFloat32));
   TORCH_CHECK(ctx.numel() == B && bt.size(0) == B && bt.dtype() == torch::kInt32 &&
               ctx.dtype() == torch::kInt32);
   if (B == 0) return;
@@ -303,14 +322,18 @@ void biased_attention_decode(torch::Tensor q, torch::Tensor kc, torch::Tensor vc
   int CS = std::max(1, std::min(8, 1024 / std::max(B * Hkv, 1)));
   if (window > 0) CS = std::max(1, std::min(CS, (int)((window + 63) / 64)));
   auto* o = (__hip_bfloat16*)out.data_ptr() + col;
-#define RUN(DD, DVV)                                                             \
-  decode_launch<DD, DVV, false, true>(q, kc, vc, bt, ctx, o, out.stride(0),      \
-                                      (int)dv, (float)scale, (float)oscale,      \
-                                      slopes.data_ptr<float>(), (int)window, CS)
-  if (D == 64 && DV == 64) RUN(64, 64);
-  else if (D == 64 && DV == 128) RUN(64, 128);
-  else if (D == 128 && DV == 64) RUN(128, 64);
-  else if (D == 128 && DV == 128) RUN(128, 128);
+  const float* rp = rates ? rates->data_ptr<float>() : nullptr;
+  const float* snk = sink ? sink->data_ptr<float>() : nullptr;
+#define RUN1(DD, DVV, BB)                                                        \
+  decode_launch<DD, DVV, false, BB>(q, kc, vc, bt, ctx, o, out.stride(0),        \
+                                    (int)dv, (float)scale, (float)oscale,        \
+                                    slopes.data_ptr<float>(), rp, (int)window, snk, CS)
+#define RUN(DD, DVV) if (rp) RUN1(DD, DVV, LOG_BIAS); else RUN1(DD, DVV, LINEAR_BIAS)
+  if (D == 64 && DV == 64) { RUN(64, 64); }
+  else if (D == 64 && DV == 128) { RUN(64, 128); }
+  else if (D == 128 && DV == 64) { RUN(128, 64); }
+  else if (D == 128 && DV == 128) { RUN(128, 128); }
   else TORCH_CHECK(false, "unsupported cache head widths ", D, ", ", DV);
 #undef RUN
+#undef RUN1
 }

@@ -19,11 +19,11 @@
 // feeds 8 waves of MFMA (GQA heads share the stage — staging bandwidth was
 // the 156-TF bound of the 4-wave/1-head structure).  KV tiles of 64 keys,
 // two 32-key MFMA steps each.
-// BIAS adds a per-head linear distance penalty and a sliding window (tiles
-// and MFMA steps wholly outside a wave's window are skipped), lets keys and
-// values differ in width, and writes scaled columns of a wider output. SINK
-// starts every row's softmax from a term without key or value and multiplies
-// the head by a sigmoid gate.
+// BIAS adds a per-head distance penalty, linear or logarithmic, and a sliding
+// window (tiles and MFMA steps wholly outside a wave's window are skipped), lets
+// keys and values differ in width, and writes scaled columns of a wider output. A
+// sink starts every row's softmax from a term without key or value; GATED takes
+// one and multiplies the head by a sigmoid gate.
 // Covers fresh prefill and append-prefill (chunked agent turns) since K/V
 // are read from the paged cache with an absolute-position causal bound.
 #include "common.h"
@@ -38,12 +38,14 @@ DEVINL unsigned int pack2_bf16(float lo, float hi) {
   return ((unsigned int)f32_to_bf16(hi) << 16) | f32_to_bf16(lo);
 }
 
+enum { NO_BIAS = 0, LINEAR_BIAS = 1, LOG_BIAS = 2 };
+
 union frag_u {
   unsigned int u[4];
   bf16x8 v;
 };
 
-template <int D, int DV, int HG, bool FP8, bool BIAS, bool SINK>  // HG = query heads per workgroup
+template <int D, int DV, int HG, bool FP8, int BIAS, bool GATED>  // HG = query heads per workgroup
 __global__ __launch_bounds__(512, 1) void prefill_kernel(
     const __hip_bfloat16* __restrict__ q,   // [T, qstride], heads D apart
     const void* __restrict__ kc,  // [NP, Hkv, P, D] bf16 | fp8 e4m3
@@ -56,8 +58,8 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
     const int* __restrict__ ctx_lens,       // [S]
     int Hq, int Hkv, int P, int MP, float scale,
     long qstride, long ostride, int dv, float oscale,
-    const float* __restrict__ slopes, int window,
-    const float* __restrict__ sink,         // [Hq]
+    const float* __restrict__ slopes, const float* __restrict__ rates, int window,
+    const float* __restrict__ sink,         // [Hq], or null unless GATED
     const __hip_bfloat16* __restrict__ gate, long gstride) {  // [T, gstride]
   constexpr int KVB = 64;           // keys staged per tile
   constexpr int NC = D / 16;        // Q^T fragments (MFMA K-chunks of QK^T)
@@ -114,7 +116,8 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   }
 
   const int q_abs = ctx - qlen + qrow;  // absolute position of this lane's q
-  float m = SINK ? sink[h] : -1e30f, l = SINK ? 1.f : 0.f;
+  const bool has_sink = GATED || (BIAS && sink);
+  float m = has_sink ? sink[h] : -1e30f, l = has_sink ? 1.f : 0.f;
   floatx16 o[NDT];
 #pragma unroll
   for (int dt = 0; dt < NDT; ++dt)
@@ -128,8 +131,10 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   // absolute position of the wave's first (smallest) q row
   const int q_abs_min = ctx - qlen + qoff + qsub * 32;
 
-  // this head's penalty per token of distance; first key any row here sees
+  // this head's penalty per token of distance, or of ln(1 + rate * distance);
+  // first key any row here sees
   const float slope = BIAS ? slopes[h] : 0.f;
+  const float rate = BIAS == LOG_BIAS ? rates[h] : 0.f;
   const int win = BIAS && window > 0 ? window : 0x3fffffff;
   const int tile0 = BIAS ? max(0, ctx - qlen + qoff - win + 1) / KVB : 0;
 
@@ -201,10 +206,11 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
       for (int r = 0; r < 16; ++r) {
         const int k_abs = ks + (r & 3) + 8 * (r >> 2) + 4 * half;
         float sv = st[r] * scale;
-        if constexpr (BIAS) {
+        if constexpr (BIAS != NO_BIAS) {
           // a row that has seen only masked keys yet holds weights of
           // exp(0); its first visible key rescales them to zero
-          sv -= slope * (float)(q_abs - k_abs);
+          const float dist = (float)(q_abs - k_abs);
+          sv -= slope * (BIAS == LOG_BIAS ? __logf(1.f + rate * dist) : dist);
           if (need_mask && (k_abs > q_abs || k_abs >= ctx || q_abs - k_abs >= win))
             sv = -1e30f;
         } else {
@@ -283,7 +289,7 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
   }
 
   // ---- epilogue: divide by l (per q row), transpose via LDS, store rows
-  if constexpr (SINK) {  // divided by l, times the gate
+  if constexpr (GATED) {  // divided by l, times the gate
     const long grow = (q_start + (qvalid ? qrow : 0)) * gstride + h;
     l *= 1.f + __expf(-bf16_to_f32(((const unsigned short*)gate)[grow]));
   }
@@ -382,7 +388,7 @@ torch::Tensor attention_prefill_paged(torch::Tensor q, torch::Tensor kc,
   dim3 grid(NB, Hq / HG), block(512);
   auto stream = CUR_STREAM;
 #define PLAUNCH1(DD, HGV, F8)                                                 \
-  hipLaunchKernelGGL((prefill_kernel<DD, DD, HGV, F8, false, false>), grid, block,   \
+  hipLaunchKernelGGL((prefill_kernel<DD, DD, HGV, F8, NO_BIAS, false>), grid, block,   \
                      (prefill_lds<DD, DD>()), stream,                         \
                      (const __hip_bfloat16*)q.data_ptr(),                     \
                      kc.data_ptr(), vc.data_ptr(),                            \
@@ -390,8 +396,8 @@ torch::Tensor attention_prefill_paged(torch::Tensor q, torch::Tensor kc,
                      bseq_t.data_ptr<int>(), boff_t.data_ptr<int>(),          \
                      cu_q.data_ptr<int>(), bt.data_ptr<int>(),                \
                      ctx.data_ptr<int>(), Hq, Hkv, P, MP, (float)scale,       \
-                     (long)Hq * D, (long)Hq * D, D, 1.f, nullptr, 0, nullptr, \
-                     nullptr, 0)
+                     (long)Hq * D, (long)Hq * D, D, 1.f, nullptr, nullptr, 0, \
+                     nullptr, nullptr, 0)
 #define PLAUNCH(DD, HGV)                                                      \
   if (fp8) { PLAUNCH1(DD, HGV, true); } else { PLAUNCH1(DD, HGV, false); }
 #define PLAUNCH_D(DD)                                                         \
@@ -418,7 +424,9 @@ long biased_prefill_rows(long G) { return 32 * (8 / heads_per_block((int)G)); }
 void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                               torch::Tensor bt, torch::Tensor cu_q, torch::Tensor ctx,
                               torch::Tensor bseq, torch::Tensor boff, double scale,
-                              long window, torch::Tensor slopes, torch::Tensor out,
+                              long window, torch::Tensor slopes,
+                              c10::optional<torch::Tensor> rates,
+                              c10::optional<torch::Tensor> sink, torch::Tensor out,
                               long col, long dv, double oscale) {
   TORCH_CHECK(q.is_cuda() && q.dtype() == torch::kBFloat16 && q.is_contiguous());
   const int T = q.size(0), Hq = q.size(1), D = q.size(2);
@@ -429,6 +437,8 @@ void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor v
   TORCH_CHECK(out.dtype() == torch::kBFloat16 && out.size(0) == T && out.stride(1) == 1 &&
               dv <= DV && col + Hq * dv <= out.size(1));
   TORCH_CHECK(slopes.numel() == Hq && slopes.dtype() == torch::kFloat32);
+  for (auto* t : {&rates, &sink})
+    TORCH_CHECK(!*t || ((*t)->numel() == Hq && (*t)->dtype() == torch::kFloat32));
   TORCH_CHECK(bseq.dtype() == torch::kInt32 && boff.dtype() == torch::kInt32 &&
               bseq.numel() == boff.numel() && cu_q.dtype() == torch::kInt32 &&
               cu_q.numel() == ctx.numel() + 1 && bt.size(0) == ctx.numel());
@@ -436,8 +446,10 @@ void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor v
   if (T == 0 || NB == 0) return;
   const int HG = heads_per_block(Hq / Hkv);
   dim3 grid(NB, Hq / HG), block(512);
-#define BLAUNCH(DD, DVV, HGV)                                                   \
-  hipLaunchKernelGGL((prefill_kernel<DD, DVV, HGV, false, true, false>), grid, block, \
+  const float* rp = rates ? rates->data_ptr<float>() : nullptr;
+  const float* snk = sink ? sink->data_ptr<float>() : nullptr;
+#define BLAUNCH1(DD, DVV, HGV, BB)                                              \
+  hipLaunchKernelGGL((prefill_kernel<DD, DVV, HGV, false, BB, false>), grid, block, \
                      (prefill_lds<DD, DVV>()), CUR_STREAM,                      \
                      (const __hip_bfloat16*)q.data_ptr(), kc.data_ptr(),        \
                      vc.data_ptr(), (__hip_bfloat16*)out.data_ptr() + col,      \
@@ -445,7 +457,10 @@ void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor v
                      cu_q.data_ptr<int>(), bt.data_ptr<int>(),                  \
                      ctx.data_ptr<int>(), Hq, Hkv, P, MP, (float)scale,         \
                      (long)Hq * D, out.stride(0), (int)dv, (float)oscale,       \
-                     slopes.data_ptr<float>(), (int)window, nullptr, nullptr, 0)
+                     slopes.data_ptr<float>(), rp, (int)window, snk, nullptr, 0)
+#define BLAUNCH(DD, DVV, HGV)                                                   \
+  if (rp) { BLAUNCH1(DD, DVV, HGV, LOG_BIAS); }                                 \
+  else { BLAUNCH1(DD, DVV, HGV, LINEAR_BIAS); }
 #define BLAUNCH_HG(DD, DVV)                    \
   switch (HG) {                                \
     case 1: BLAUNCH(DD, DVV, 1); break;        \
@@ -459,6 +474,7 @@ void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor v
   else TORCH_CHECK(false, "unsupported cache head widths ", D, ", ", DV);
 #undef BLAUNCH_HG
 #undef BLAUNCH
+#undef BLAUNCH1
   HIP_CHECK_KERNEL();
 }
 
@@ -489,14 +505,14 @@ void sink_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
   if (T == 0 || NB == 0) return;
   dim3 grid(NB, H), block(512);
 #define SLAUNCH(DD, DVV)                                                        \
-  hipLaunchKernelGGL((prefill_kernel<DD, DVV, 1, false, false, true>), grid,    \
+  hipLaunchKernelGGL((prefill_kernel<DD, DVV, 1, false, NO_BIAS, true>), grid,    \
                      block, (prefill_lds<DD, DVV>()), CUR_STREAM,               \
                      (const __hip_bfloat16*)q.data_ptr(), kc.data_ptr(),        \
                      vc.data_ptr(), (__hip_bfloat16*)out.data_ptr(),            \
                      bseq.data_ptr<int>(), boff.data_ptr<int>(),                \
                      cu_q.data_ptr<int>(), bt.data_ptr<int>(),                  \
                      ctx.data_ptr<int>(), H, H, P, MP, (float)scale,            \
-                     q.stride(0), out.stride(0), DV, 1.f, nullptr, 0,           \
+                     q.stride(0), out.stride(0), DV, 1.f, nullptr, nullptr, 0,  \
                      sink.data_ptr<float>(),                                    \
                      (const __hip_bfloat16*)gate.data_ptr(), gate.stride(0))
   if (D == 64 && DV == 64) { SLAUNCH(64, 64); }

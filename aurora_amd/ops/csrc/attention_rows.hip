@@ -1,6 +1,6 @@
 // Attention for any head width and for float32: one wave per (query row, head),
-// 64 keys at a time; with a distance bias and a window, or over shared latents
-// (keys that are also the values) with a sink.
+// 64 keys at a time; with a distance bias, a window and a sink, or over shared
+// latents (keys that are also the values).
 //
 // The matrix-core kernels (attention_prefill / attention_decode) serve bf16
 // heads up to 128 wide; this one serves everything else. Each lane scores its
@@ -21,6 +21,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(
     const int* __restrict__ bt, const int* __restrict__ cu,
     const int* __restrict__ ctx, const int* __restrict__ row_seq,
     const int* __restrict__ row_off, const float* __restrict__ slopes,
+    const float* __restrict__ rates,  // [Hq]: penalty of ln(1 + rate * distance)
     const float* __restrict__ sink,  // [Hq] each, or null
     T* __restrict__ out, long ostride, int T_, int Hq, int Hkv, int DK, int DV,
     int dv, int P, int MP, float scale, int window, float oscale) {
@@ -39,7 +40,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(
   const int len = cu ? cu[seq + 1] - cu[seq] : 1;
   const int pos = ctx[seq] - len + (row_off ? row_off[t] : 0);
   const int kvh = h / (Hq / Hkv);
-  const float slope = slopes ? slopes[h] : 0.f;
+  const float slope = slopes ? slopes[h] : 0.f, rate = rates ? rates[h] : 0.f;
   const int* pages = bt + (long)seq * MP;
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
   // a sink is one more term of the denominator
@@ -53,7 +54,8 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(
     const long row = ((long)pages[kk / P] * Hkv + kvh) * P + kk % P;
     float s = 0.f;
     for (int i = 0; i < DK; ++i) s += qv[i] * ldf(kc + row * DK + i);
-    s = seen ? s * scale - slope * (float)(pos - key) : -1e30f;
+    const float dist = (float)(pos - kk);
+    s = seen ? s * scale - slope * (rates ? logf(1.f + rate * dist) : dist) : -1e30f;
     const float mn = fmaxf(m, wave_max(s));
     const float alpha = expf(m - mn);
     const float p = seen ? expf(s - mn) : 0.f;
@@ -80,8 +82,10 @@ void biased_attention_rows(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                            torch::Tensor bt, c10::optional<torch::Tensor> cu,
                            torch::Tensor ctx, c10::optional<torch::Tensor> row_seq,
                            c10::optional<torch::Tensor> row_off, double scale,
-                           long window, torch::Tensor slopes, torch::Tensor out,
-                           long col, long dv, double oscale) {
+                           long window, torch::Tensor slopes,
+                           c10::optional<torch::Tensor> rates,
+                           c10::optional<torch::Tensor> sink, torch::Tensor out, long col,
+                           long dv, double oscale) {
   const int T_ = q.size(0), Hq = q.size(1), DK = q.size(2);
   const int Hkv = kc.size(1), P = kc.size(2), MP = bt.size(1), DV = vc.size(3);
   TORCH_CHECK(q.is_cuda() && q.is_contiguous() && kc.is_contiguous() &&
@@ -89,6 +93,8 @@ void biased_attention_rows(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
   TORCH_CHECK(kc.size(3) == DK && Hq % Hkv == 0 && dv <= DV && DV <= ROWS_MAX_DV,
               "head width ", DV, " not supported (at most ", ROWS_MAX_DV, ")");
   TORCH_CHECK(DK <= 2048 && slopes.numel() == Hq && slopes.dtype() == torch::kFloat32);
+  for (auto* t : {&rates, &sink})
+    TORCH_CHECK(!*t || ((*t)->numel() == Hq && (*t)->dtype() == torch::kFloat32));
   TORCH_CHECK(kc.dtype() == q.dtype() && vc.dtype() == q.dtype() && out.dtype() == q.dtype());
   TORCH_CHECK(out.size(0) == T_ && out.stride(1) == 1 && col + Hq * dv <= out.size(1));
   TORCH_CHECK(bt.dtype() == torch::kInt32 && ctx.dtype() == torch::kInt32);
@@ -109,7 +115,8 @@ void biased_attention_rows(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
         (attention_rows_kernel<T, ROWS_MAX_DV>), grid, dim3(256), 4 * DK * 4, CUR_STREAM, (const T*)q.data_ptr(),
         (const T*)kc.data_ptr(), (const T*)vc.data_ptr(), bt.data_ptr<int>(),
         cup, ctx.data_ptr<int>(), rsp, rop, slopes.data_ptr<float>(),
-        (const float*)nullptr, (T*)out.data_ptr() + col, out.stride(0), T_, Hq, Hkv, DK,
+        rates ? rates->data_ptr<float>() : nullptr,
+        sink ? sink->data_ptr<float>() : nullptr, (T*)out.data_ptr() + col, out.stride(0), T_, Hq, Hkv, DK,
         DV, (int)dv, P, MP, (float)scale, (int)window, (float)oscale);
   });
   HIP_CHECK_KERNEL();
@@ -146,7 +153,7 @@ void latent_attention_rows(torch::Tensor q, torch::Tensor cache, torch::Tensor b
           (const T*)cache.data_ptr(), (const T*)cache.data_ptr(), bt.data_ptr<int>(),
           cu ? cu->data_ptr<int>() : nullptr, ctx.data_ptr<int>(),
           cu ? row_seq->data_ptr<int>() : nullptr, cu ? row_off->data_ptr<int>() : nullptr,
-          (const float*)nullptr, sink.data_ptr<float>(), (T*)out.data_ptr(), (long)H * R, T_,
+          (const float*)nullptr, (const float*)nullptr, sink.data_ptr<float>(), (T*)out.data_ptr(), (long)H * R, T_,
           H, 1, R, R, R, P, MP, (float)scale, 0, 1.f);
     };
     if (R <= ROWS_MAX_DV) launch(attention_rows_kernel<T, ROWS_MAX_DV>);

@@ -61,16 +61,17 @@ long biased_prefill_rows(long G);
 void biased_attention_prefill(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                               torch::Tensor bt, torch::Tensor cu_q, torch::Tensor ctx,
                               torch::Tensor bseq, torch::Tensor boff, double scale,
-                              long window, torch::Tensor slopes, torch::Tensor out,
-                              long col, long dv, double oscale);
+                              long window, torch::Tensor slopes, OptT rates, OptT sink,
+                              torch::Tensor out, long col, long dv, double oscale);
 void biased_attention_decode(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                              torch::Tensor bt, torch::Tensor ctx, double scale, long window,
-                             torch::Tensor slopes, torch::Tensor out, long col, long dv,
-                             double oscale);
+                             torch::Tensor slopes, OptT rates, OptT sink,
+                             torch::Tensor out, long col, long dv, double oscale);
 void biased_attention_rows(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                            torch::Tensor bt, OptT cu, torch::Tensor ctx, OptT row_seq,
                            OptT row_off, double scale, long window, torch::Tensor slopes,
-                           torch::Tensor out, long col, long dv, double oscale);
+                           OptT rates, OptT sink, torch::Tensor out, long col, long dv,
+                           double oscale);
 void delta_prefill(torch::Tensor proj, torch::Tensor z, torch::Tensor conv_w,
                    torch::Tensor a_log, torch::Tensor dt_bias, torch::Tensor norm, long H,
                    long G, long d, long e, long taps, long q0, long k0, long v0, long b0,
@@ -96,7 +97,45 @@ std::vector<torch::Tensor> moe_route(torch::Tensor h, torch::Tensor router,
                                      torch::Tensor bias, long top);
 std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
                                            torch::Tensor w_gu, torch::Tensor w_dn,
-                                           double limit, double alpha);
+                                           double limit, double alpha, double shift);
+std::vector<torch::Tensor> moe_route_grouped(torch::Tensor h, torch::Tensor router,
+                                             torch::Tensor correction, long top,
+                                             long groups, long keep, double scale);
+torch::Tensor gelu(torch::Tensor z);
+torch::Tensor silu_glu(torch::Tensor z, long F);
+torch::Tensor output_norm(torch::Tensor src, torch::Tensor x, torch::Tensor weight,
+                          torch::Tensor bias, OptT delta, OptT gate, OptT y, OptT place,
+                          OptT share, OptT kept, OptT coefs, OptT fw, OptT fb, double eps,
+                          bool to_bf16);
+torch::Tensor normed_qkv(torch::Tensor proj, long q0, long k0, long v0, torch::Tensor qw,
+                         torch::Tensor kw, bool whole, double eps, OptT cos_sin, double coef,
+                         long every, torch::Tensor pos, torch::Tensor slots, torch::Tensor kc,
+                         torch::Tensor vc, long Hq, long Hkv, long d, long dv);
+void head_delta_prefill(torch::Tensor proj, torch::Tensor conv_w, torch::Tensor a_log,
+                        torch::Tensor dt_bias, torch::Tensor norm, long H, long G, long d,
+                        long e, long taps, long q0, long k0, long v0, long b0, long a0,
+                        long g0, double eps, torch::Tensor state, torch::Tensor ring,
+                        torch::Tensor cu, torch::Tensor cseq, torch::Tensor coff,
+                        torch::Tensor cfirst, torch::Tensor starts, torch::Tensor slots,
+                        torch::Tensor out, long col, double oscale);
+void head_delta_decode(torch::Tensor proj, torch::Tensor conv_w, torch::Tensor a_log,
+                       torch::Tensor dt_bias, torch::Tensor norm, long H, long G, long d,
+                       long e, long taps, long q0, long k0, long v0, long b0, long a0,
+                       long g0, double eps, torch::Tensor state, torch::Tensor ring,
+                       torch::Tensor starts, torch::Tensor slots, torch::Tensor out,
+                       long col, double oscale);
+void memory_prefill(torch::Tensor proj, torch::Tensor i_bias, torch::Tensor f_bias,
+                    torch::Tensor norm, long H, long d, long e, long q0, long k0, long v0,
+                    long i0, long f0, long g0, double cap, double eps, torch::Tensor state,
+                    torch::Tensor nstate, torch::Tensor mstate, torch::Tensor cu,
+                    torch::Tensor cseq, torch::Tensor coff, torch::Tensor cfirst,
+                    torch::Tensor starts, torch::Tensor slots, torch::Tensor out, long col,
+                    double oscale);
+void memory_decode(torch::Tensor proj, torch::Tensor i_bias, torch::Tensor f_bias,
+                   torch::Tensor norm, long H, long d, long e, long q0, long k0, long v0,
+                   long i0, long f0, long g0, double cap, double eps, torch::Tensor state,
+                   torch::Tensor nstate, torch::Tensor mstate, torch::Tensor starts,
+                   torch::Tensor slots, torch::Tensor out, long col, double oscale);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("rmsnorm", &rmsnorm, "fused RMSNorm (bf16, gfx950)");
@@ -133,15 +172,30 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("bias_kv_write", &bias_kv_write, "bias + head split + paged KV scatter");
   m.def("biased_prefill_rows", &biased_prefill_rows);
   m.def("biased_attention_prefill", &biased_attention_prefill,
-        "MFMA flash prefill with distance bias and window");
+        "MFMA flash prefill with distance bias, window and sink");
   m.def("biased_attention_decode", &biased_attention_decode,
-        "paged decode with distance bias and window");
+        "paged decode with distance bias, window and sink");
   m.def("biased_attention_rows", &biased_attention_rows,
-        "any head width / float32 attention with distance bias and window");
+        "any head width / float32 attention with distance bias, window and sink");
   m.def("delta_prefill", &delta_prefill, "gated delta rule, chunked");
   m.def("delta_decode", &delta_decode, "gated delta rule, one token per sequence");
   m.def("retention_prefill", &retention_prefill, "retention, chunked");
   m.def("retention_decode", &retention_decode, "retention, one token per sequence");
   m.def("moe_route", &moe_route, "fp32 router, top choice, softmax over the chosen");
+  m.def("moe_route_grouped", &moe_route_grouped,
+        "fp32 sigmoid router, top choice among the best groups");
   m.def("moe_clamped_glu", &moe_clamped_glu, "sorted grouped clamped-GLU experts");
+  m.def("head_delta_prefill", &head_delta_prefill,
+        "gated delta rule with a decay per head, chunked");
+  m.def("head_delta_decode", &head_delta_decode,
+        "gated delta rule with a decay per head, one token per sequence");
+  m.def("memory_prefill", &memory_prefill, "matrix memory (mLSTM), chunked");
+  m.def("memory_decode", &memory_decode, "matrix memory (mLSTM), one token per sequence");
+  m.def("output_norm", &output_norm,
+        "sub-layer result put together, layer norm, fp32 residual, depth average, "
+        "final norm");
+  m.def("normed_qkv", &normed_qkv,
+        "head norms + rotation + temperature + paged KV scatter");
+  m.def("gelu", &gelu, "exact gelu");
+  m.def("silu_glu", &silu_glu, "silu(gate) * up");
 }

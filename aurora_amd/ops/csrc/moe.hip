@@ -1,6 +1,9 @@
 // Routed experts with a clamped GLU:
+//     act = g sigmoid(alpha g) (u + shift),  g = min(gate, limit), u = clamp(up)
+// (without a limit, alpha 1 and shift 0: silu(gate) up), chosen by one of two routers:
 //     z = W_r h + b (fp32), the ``top`` largest, softmax over the chosen;
-//     act = g sigmoid(alpha g) (u + 1),  g = min(gate, limit), u = clamp(up)
+//     s = sigmoid(W_r h) (fp32), the ``top`` largest of s + c among the best groups of
+//     neighbours (by the sum of their two largest), weights s / sum s * scale
 // as route -> sort -> gathered up product with the activation in its epilogue
 // -> down product. Rows stay sorted by expert; the residual-norm kernel adds
 // each token's weighted rows, so no scatter pass exists. Nothing is read back
@@ -22,12 +25,13 @@ union mfrag {
 
 // ------------------------------------------------------------------- router
 
-// one workgroup per 16 tokens; its waves split the contraction
-template <typename T, bool MATRIX16>
+// one workgroup per 16 tokens; its waves split the contraction. GROUPED: bias is the
+// sigmoid scores' correction
+template <typename T, bool MATRIX16, bool GROUPED>
 __global__ __launch_bounds__(1024) void moe_route_kernel(
     const T* __restrict__ h, const T* __restrict__ router,
     const float* __restrict__ bias, int* __restrict__ sel, float* __restrict__ gate,
-    int T_, int W, int E, int top) {
+    int T_, int W, int E, int top, int groups, int keep, float scale) {
   extern __shared__ float logits[];  // [16][E]
   __shared__ float part[16][16][64];
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
@@ -78,13 +82,45 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(
       float z = 0.f;
 #pragma unroll
       for (int v = 0; v < 16; ++v) z += part[v][t][x];
-      if (e < E) logits[t * E + e] = z + bias[e];
+      if (e < E) logits[t * E + e] = GROUPED ? z : z + bias[e];
     }
     __syncthreads();
   }
   if (t0 + wave < T_) {
     const int t = wave;
     float* z = logits + t * E;
+    float* score = &part[wave][0][0];  // plain scores; from 512 on the groups'
+    if constexpr (GROUPED) {
+      float* gs = score + 512;
+      const int n = E / groups;
+      auto sync = [] {
+        __threadfence_block();
+        __builtin_amdgcn_wave_barrier();
+      };
+      for (int e = lane; e < E; e += WAVE) {
+        score[e] = sigmoid_f(z[e]);
+        z[e] = score[e] + bias[e];
+      }
+      sync();
+      for (int x = lane; x < groups; x += WAVE) {
+        float a = -INFINITY, b = -INFINITY;  // the two largest
+        for (int e = x * n; e < (x + 1) * n; ++e) {
+          const float c = z[e];
+          b = fmaxf(b, fminf(a, c));
+          a = fmaxf(a, c);
+        }
+        gs[x] = n > 1 ? a + b : a;
+      }
+      sync();
+      for (int x = lane; x < groups; x += WAVE) {
+        int better = 0;
+        for (int o = 0; o < groups; ++o)
+          better += gs[o] > gs[x] || (gs[o] == gs[x] && o < x);
+        if (better >= keep)
+          for (int e = x * n; e < (x + 1) * n; ++e) z[e] = -INFINITY;
+      }
+      sync();
+    }
     float first = 0.f, sum = 0.f;
     for (int n = 0; n < top; ++n) {
       float best = -INFINITY;
@@ -99,7 +135,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(
       }
       at = min(at, E - 1);  // all logits NaN: still a valid expert
       if (n == 0) first = best;
-      const float p = expf(best - first);
+      const float p = GROUPED ? score[at] : expf(best - first);
       sum += p;
       if (lane == n % WAVE) {
         sel[(long)(t0 + t) * top + n] = at;
@@ -110,12 +146,17 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(
       __builtin_amdgcn_wave_barrier();
     }
     // each lane rescales what it wrote
-    for (int n = lane; n < top; n += WAVE) gate[(long)(t0 + t) * top + n] /= sum;
+    for (int n = lane; n < top; n += WAVE) {
+      float& w = gate[(long)(t0 + t) * top + n];
+      w = GROUPED ? w / (sum + 1e-20f) * scale : w / sum;
+    }
   }
 }
 
-std::vector<torch::Tensor> moe_route(torch::Tensor h, torch::Tensor router,
-                                     torch::Tensor bias, long top) {
+template <bool GROUPED>
+static std::vector<torch::Tensor> route(const torch::Tensor& h, const torch::Tensor& router,
+                                        const torch::Tensor& bias, long top, long groups,
+                                        long keep, double scale) {
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.is_contiguous() &&
               router.is_contiguous() && router.dtype() == h.dtype());
   const long T_ = h.size(0), W = h.size(1), E = router.size(0);
@@ -129,14 +170,29 @@ std::vector<torch::Tensor> moe_route(torch::Tensor h, torch::Tensor router,
       hipLaunchKernelGGL(kern, dim3((T_ + 15) / 16), dim3(1024), 16 * E * 4, CUR_STREAM,
                          (const T*)h.data_ptr(), (const T*)router.data_ptr(),
                          bias.data_ptr<float>(), sel.data_ptr<int>(),
-                         gate.data_ptr<float>(), (int)T_, (int)W, (int)E, (int)top);
+                         gate.data_ptr<float>(), (int)T_, (int)W, (int)E, (int)top,
+                         (int)groups, (int)keep, (float)scale);
     };
     constexpr bool B16 = sizeof(T) == 2;
-    if (B16 && W % 8 == 0) launch(moe_route_kernel<T, B16>);
-    else launch(moe_route_kernel<T, false>);
+    if (B16 && W % 8 == 0) launch(moe_route_kernel<T, B16, GROUPED>);
+    else launch(moe_route_kernel<T, false, GROUPED>);
   });
   HIP_CHECK_KERNEL();
   return {sel, gate};
+}
+
+std::vector<torch::Tensor> moe_route(torch::Tensor h, torch::Tensor router,
+                                     torch::Tensor bias, long top) {
+  return route<false>(h, router, bias, top, 1, 1, 1.0);
+}
+
+std::vector<torch::Tensor> moe_route_grouped(torch::Tensor h, torch::Tensor router,
+                                             torch::Tensor correction, long top,
+                                             long groups, long keep, double scale) {
+  const long E = router.size(0);
+  TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups &&
+              top <= keep * (E / groups), "expert groups");
+  return route<true>(h, router, correction, top, groups, keep, scale);
 }
 
 // --------------------------------------------------------------------- sort
@@ -195,13 +251,13 @@ struct GroupArgs {
   void* y;             // [A, N]
   const int* table;
   int N, K;
-  float limit, alpha;
+  float limit, alpha, shift;
 };
 
-DEVINL float clamped_glu(float g, float u, float limit, float alpha) {
-  g = fminf(g, limit);
-  u = fminf(fmaxf(u, -limit), limit);
-  return g * (u + 1.f) / (1.f + expf(-alpha * g));
+DEVINL float clamped_glu(float g, float u, const GroupArgs& p) {
+  g = fminf(g, p.limit);
+  u = fminf(fmaxf(u, -p.limit), p.limit);
+  return g * (u + p.shift) / (1.f + expf(-p.alpha * g));
 }
 
 // Any size and float32: 32 rows x 64 columns, 16 of K at a time, through LDS as
@@ -251,7 +307,7 @@ __global__ __launch_bounds__(256) void grouped_any_kernel(GroupArgs p) {
   for (int x = tid; x < 32 * BN; x += 256) {
     const int r = x / BN, c = x % BN;
     if (r >= cnt || n0 + c >= p.N) continue;
-    const float v = GLU ? clamped_glu(cs[r][c], cs[r][32 + c], p.limit, p.alpha) : cs[r][c];
+    const float v = GLU ? clamped_glu(cs[r][c], cs[r][32 + c], p) : cs[r][c];
     stf((T*)p.y + (long)(row0 + r) * p.N + n0 + c, v);
   }
 }
@@ -373,8 +429,8 @@ __global__ __launch_bounds__(NTHR) void grouped_bf16_kernel(GroupArgs p) {
       for (int n = 0; n < NO; ++n) {
         const int c = n0 + (GLU ? wn / 2 : wn) + n * 16 + i;
         if (c >= p.N) continue;
-        const float v = GLU ? clamped_glu(acc[m][n][r], acc[m][n + (GLU ? NO : 0)][r],
-                                          p.limit, p.alpha) : acc[m][n][r];
+        const float v = GLU ? clamped_glu(acc[m][n][r], acc[m][n + (GLU ? NO : 0)][r], p)
+                            : acc[m][n][r];
         y[(long)(row0 + row) * p.N + c] = f32_to_bf16(v);
       }
     }
@@ -416,7 +472,7 @@ static void grouped(const GroupArgs& p, bool bf16, int tiles, int TM, long busy)
 
 std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
                                            torch::Tensor w_gu, torch::Tensor w_dn,
-                                           double limit, double alpha) {
+                                           double limit, double alpha, double shift) {
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.is_contiguous() && sel.is_contiguous() &&
               sel.dtype() == torch::kInt32 && sel.size(0) == h.size(0));
   const long T_ = h.size(0), W = h.size(1), top = sel.size(1), A = T_ * top;
@@ -440,7 +496,8 @@ std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
                      sel.data_ptr<int>(), (int)A, (int)E, (int)top, TM, tiles,
                      place.data_ptr<int>(), token.data_ptr<int>(), table.data_ptr<int>());
   GroupArgs p = {h.data_ptr(), token.data_ptr<int>(), w_gu.data_ptr(), act.data_ptr(),
-                 table.data_ptr<int>(), (int)F, (int)W, (float)limit, (float)alpha};
+                 table.data_ptr<int>(), (int)F, (int)W, (float)limit, (float)alpha,
+                 (float)shift};
   grouped<true>(p, bf16, tiles, TM, std::min(E, A));
   p.x = act.data_ptr();
   p.gather = nullptr;

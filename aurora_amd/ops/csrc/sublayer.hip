@@ -1,8 +1,8 @@
 // What surrounds the mixers of the layer-listed decoders: the embedding of
 // tokens and token pairs, the causal convolution added to a mixer's input, and
-// the xIELU activation.
+// the activations of the dense feed-forwards.
 //
-// Both kernels with a past keep it in state slots. Rows that read a sequence's
+// The two kernels with a past keep it in state slots. Rows that read a sequence's
 // past and the store of its new past belong to one thread (convolution, per
 // channel) or one workgroup (embedding, the portion's first row), so a portion
 // never races with itself. Slot -1 marks an idle row of a captured batch.
@@ -304,3 +304,64 @@ torch::Tensor xielu(torch::Tensor z, torch::Tensor act) {
   HIP_CHECK_KERNEL();
   return out;
 }
+
+// ------------------------------------------------------------- gelu, silu GLU
+
+// f(a, b) of the columns i and i + F of z [T, stride] (GLU), or f(a, 0)
+template <typename T, int V, bool GLU, typename Fn>
+__global__ __launch_bounds__(256) void activation_kernel(const T* __restrict__ z, long stride,
+                                                         T* __restrict__ out, long total,
+                                                         int F, Fn f) {
+  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * V;
+  if (i >= total) return;
+  const T* p = z + i / F * stride + i % F;
+  if constexpr (V % 4 == 0) {
+#pragma unroll
+    for (int v = 0; v < V; v += 4) {
+      floatx4 a = ld4(p + v), b = {0.f, 0.f, 0.f, 0.f};
+      if constexpr (GLU) b = ld4(p + F + v);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) a[j] = f(a[j], b[j]);
+      st4(out + i + v, a);
+    }
+  } else {
+    stf(out + i, f(ldf(p), GLU ? ldf(p + F) : 0.f));
+  }
+}
+
+struct ExactGelu {
+  DEVINL float operator()(float x, float) const {
+    return 0.5f * x * (1.f + erff(x * 0.70710678f));
+  }
+};
+struct SiluTimes {
+  DEVINL float operator()(float g, float u) const { return silu_f(g) * u; }
+};
+
+template <bool GLU, typename Fn>
+static torch::Tensor activate(const torch::Tensor& z, long F, Fn f) {
+  TORCH_CHECK(z.is_cuda() && z.dim() == 2 && z.stride(1) == 1 && F >= 1 &&
+              z.size(1) >= (GLU ? 2 : 1) * F);
+  const long T_ = z.size(0), total = T_ * F;
+  auto out = torch::empty({T_, F}, z.options());
+  if (total == 0) return out;
+  DISPATCH_ELEM(z.dtype() == torch::kBFloat16, {
+    constexpr int VW = 16 / sizeof(T);
+    auto launch = [&](auto kern, int v) {
+      hipLaunchKernelGGL(kern, dim3((total + 256 * v - 1) / (256 * v)), dim3(256), 0,
+                         CUR_STREAM, (const T*)z.data_ptr(), z.stride(0),
+                         (T*)out.data_ptr(), total, (int)F, f);
+    };
+    const bool vec = F % VW == 0 && z.stride(0) % VW == 0 &&
+                     (reinterpret_cast<uintptr_t>(z.data_ptr()) & 15) == 0;
+    if (vec) launch(activation_kernel<T, VW, GLU, Fn>, VW);
+    else launch(activation_kernel<T, 1, GLU, Fn>, 1);
+  });
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
+torch::Tensor gelu(torch::Tensor z) { return activate<false>(z, z.size(1), ExactGelu{}); }
+
+// z [T, 2 F or more]: gate columns, then up columns
+torch::Tensor silu_glu(torch::Tensor z, long F) { return activate<true>(z, F, SiluTimes{}); }

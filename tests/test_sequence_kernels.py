@@ -126,6 +126,61 @@ def test_biased_attention(dtype, H, G, d, e, window, decode):
     assert (og[:, :3] == 0).all() and (og[:, 3 + H * e:] == 0).all()
 
 
+NORMED = [  # heads, kv_heads, dim, vdim, rotated dims, shared keys, whole norm, log bias
+    (8, 2, 128, 128, 64, True, False, False), (4, 4, 64, 64, 64, True, False, False),
+    (8, 2, 96, 40, 0, False, True, True), (6, 3, 72, 100, 16, False, False, True),
+    (5, 1, 33, 33, 10, True, True, False), (14, 2, 112, 128, 0, False, True, True),
+    (2, 1, 160, 24, 96, False, False, True), (16, 1, 128, 64, 8, False, True, True)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,d,e,rot,shared,whole,log", NORMED)
+@pytest.mark.parametrize("decode", [False, True])
+def test_normed_attention(dtype, H, G, d, e, rot, shared, whole, log, decode):
+    """Normed, rotated heads through the cache, then attention with a logarithmic
+    distance bias and a sink, or with neither."""
+    P = 32
+    lens = [1] * 5 if decode else [150, 2, 33, 64]
+    starts = [0, 63, 500, 129, 1000] if decode else [0, 300, 129, 31]
+    seg, pages = _segment(lens, starts, P, decode=decode)
+    T = sum(lens)
+    DK, DV = ops.cache_head_dims(d, e, dtype, "cuda")
+    kc, vc = torch.zeros(pages, G, P, DK, dtype=dtype), torch.zeros(pages, G, P, DV, dtype=dtype)
+    kc[..., :d] = rnd(pages, G, P, d, dtype=dtype)
+    vc[..., :e] = rnd(pages, G, P, e, dtype=dtype)
+    q0, k0 = 8, 8 + -(-H * d // 8) * 8
+    v0 = k0 if shared else k0 + -(-G * d // 8) * 8
+    proj = rnd(T, -(-(v0 + G * e) // 8) * 8, dtype=dtype)
+    p = ops.NormedHeadsParams(
+        H, G, d, e, q0, k0, v0, 1 + rnd(H * d if whole else d, scale=0.3),
+        1 + rnd(G * d if whole else d, scale=0.3), whole, 1e-5,
+        torch_ref.rope_cos_sin_cache(rot, 2048, 1e4) if rot else None,
+        (0.3, 70) if log else None)
+    where = [(s, q) for s in range(len(lens)) for q in range(starts[s], starts[s] + lens[s])]
+    pos = torch.tensor([q for _, q in where], dtype=torch.int32)
+    slots = torch.tensor([int(seg.block_tables[s, q // P]) * P + q % P for s, q in where],
+                         dtype=torch.int32)
+    if decode:
+        slots[2] = -1  # an idle row writes nothing
+    kg, vg = kc.cuda(), vc.cuda()
+    q = ops.normed_qkv(proj, p, pos, slots, kc, vc)
+    qg = ops.normed_qkv(*gpu(proj), _params_to(p, "cuda"), *gpu(pos, slots), kg, vg)
+    close(qg, q, dtype)
+    close(kg, kc, dtype)
+    assert torch.equal(vg.cpu(), vc)
+    slopes, rate, sink = (rnd(H).abs(), rnd(H).abs(), rnd(H)) if log else \
+        (torch.zeros(H), None, None)
+    out = torch.zeros(T, 3 + H * e + 9, dtype=dtype)
+    og = out.cuda()
+    dev = [None if t is None else t.cuda() for t in (rate, sink)]
+    ops.biased_attention(qg, kg, vg, _to(seg, "cuda"), 2 * d ** -0.5, 0, slopes.cuda(),
+                         og, 3, e, 0.7, *dev)
+    ops.biased_attention(q.float(), kc.float(), vc.float(), seg, 2 * d ** -0.5, 0, slopes,
+                         out, 3, e, 0.7, rate, sink)
+    close(og, out, dtype)
+    assert (og[:, :3] == 0).all() and (og[:, 3 + H * e:] == 0).all()
+
+
 # -------------------------------------------------------------- recurrences
 
 def _delta(H, G, d, e, taps, dtype, strong):
@@ -174,6 +229,70 @@ def test_delta_rule(dtype, H, G, d, e, taps, strong):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,d,e,taps", DELTA)
+@pytest.mark.parametrize("strong", [False, True])
+def test_head_delta_rule(dtype, H, G, d, e, taps, strong):
+    up = lambda n: -(-n // 8) * 8  # noqa: E731
+    at = [0]
+    for n in (G * d, G * d, H * e, H, H, H * e):
+        at.append(at[-1] + up(n))
+    p = ops.HeadDeltaParams(
+        H, G, d, e, taps, *at[:6], rnd(2 * G * d + H * e, taps),
+        rnd(H, scale=0.3) + (2.0 if strong else -1.0), rnd(H) - 1.0, 1 + rnd(e, scale=0.1),
+        1e-5)
+    pg = _params_to(p, "cuda")
+    S, ring = rnd(6, H, d, e), rnd(6, taps, 2 * G * d + H * e, dtype=dtype)
+    Sg, rg = S.cuda(), ring.cuda()
+    for lens, starts, slots, dec in (
+            ([37, 2, 16, 1], [0, 5, 100, 0], [4, 0, 2, 5], False),
+            ([1, 1, 1, 1], [37, 7, 116, 1], [4, 0, 2, 5], True),
+            ([1, 1, 1, 1], [38, 8, 0, 0], [4, 0, -1, 3], True)):
+        seg, _ = _segment(lens, starts, 64, slots, dec)
+        proj = rnd(sum(lens), at[6], dtype=dtype)
+        out = torch.zeros(sum(lens), 2 + H * e, dtype=dtype)
+        og = out.cuda()
+        ops.head_delta_rule(proj, p, S, ring, seg, out, 2, 0.5)
+        ops.head_delta_rule(proj.cuda(), pg, Sg, rg, _to(seg, "cuda"), og, 2, 0.5)
+        close(og, out, dtype)
+        close(Sg, S, torch.float32, 3.0)
+        assert torch.equal(rg.cpu(), ring)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,d,e", [(4, 128, 128), (3, 32, 48), (3, 20, 7), (2, 256, 256),
+                                   (1, 48, 30), (2, 16, 15), (1, 1, 1), (2, 64, 300)])
+@pytest.mark.parametrize("forget", [5.0, -6.0])
+def test_matrix_memory(dtype, H, d, e, forget):
+    """Portions short and long (more tokens than the gates' scan takes at once), then
+    single tokens; memories that keep nearly all or nothing."""
+    up = lambda n: -(-n // 8) * 8  # noqa: E731
+    at = [0]
+    for n in (H * d, H * d, H * e, H, H, H * e):
+        at.append(at[-1] + up(n))
+    p = ops.MatrixMemoryParams(H, d, e, *at[:6], rnd(H) + 1, rnd(H) + forget,
+                               1 + rnd(H * e, scale=0.2), 7.0, 1e-5)
+    pg = _params_to(p, "cuda")
+    S, N, M = rnd(6, H, d, e), rnd(6, H, d) + 2, rnd(6, H).abs()
+    Sg, Ng, Mg = gpu(S, N, M)
+    for lens, starts, slots, dec in (
+            ([37, 2, 16, 1, 1100], [0, 5, 100, 0, 1], [4, 0, 2, 5, 1], False),
+            ([1, 1, 1, 1], [37, 7, 116, 1], [4, 0, 2, 5], True),
+            ([1, 1, 1, 1], [38, 8, 0, 0], [4, 0, -1, 3], True)):
+        seg, _ = _segment(lens, starts, 64, slots, dec)
+        proj = rnd(sum(lens), at[6], dtype=dtype)
+        out = torch.zeros(sum(lens), 2 + H * e, dtype=dtype)
+        og = out.cuda()
+        ops.matrix_memory(proj, p, S, N, M, seg, out, 2, 0.5)
+        ops.matrix_memory(proj.cuda(), pg, Sg, Ng, Mg, _to(seg, "cuda"), og, 2, 0.5)
+        close(og, out, dtype, 3.0)
+        close(Mg, M, torch.float32)
+        close(Sg, S, torch.float32, 6.0)
+        close(Ng, N, torch.float32, 6.0)
+        for a, b in ((Sg, S), (Ng, N), (Mg, M)):  # the next step starts from equal ones
+            a.copy_(b)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,d,e,rot", [(4, 128, 128, 128), (3, 32, 48, 32), (3, 20, 12, 8),
                                        (2, 256, 256, 64), (1, 48, 30, 48)])
 def test_retention(dtype, H, d, e, rot):
@@ -215,9 +334,86 @@ def test_routed_experts(dtype, T, W, F, E, top):
     assert torch.equal(sg.cpu().sort(-1).values, sel.sort(-1).values)
     close(wg, wt, torch.float32)
     y, place = torch_ref.moe_clamped_glu(h, sel, gu, dn, 0.9, 1.702)
-    yg, pg = m.moe_clamped_glu(*gpu(h), sel.cuda(), *gpu(gu, dn), 0.9, 1.702)
+    yg, pg = m.moe_clamped_glu(*gpu(h), sel.cuda(), *gpu(gu, dn), 0.9, 1.702, 1.0)
     assert sorted(pg.flatten().tolist()) == list(range(T * top))
     close(yg.cpu()[pg.cpu().long()], y[place.long()], dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,W,E,groups,keep,top", [
+    (40, 64, 12, 2, 1, 2), (5, 50, 6, 6, 3, 3), (33, 128, 512, 8, 4, 10), (17, 72, 70, 1, 1, 4),
+    (64, 320, 9, 3, 2, 6), (1, 8, 1, 1, 1, 1), (20, 64, 130, 65, 7, 14)])
+def test_grouped_router(dtype, T, W, E, groups, keep, top):
+    h, router = rnd(T, W, dtype=dtype), rnd(E, W, dtype=dtype, scale=2 * W ** -0.5)
+    corr = rnd(E, scale=0.3) - 1.0  # choice scores of both signs
+    args = (top, groups, keep, 2.5)
+    sel, wt = torch_ref.moe_route_grouped(h, router, corr, *args)
+    sg, wg = sequence._hip("test").moe_route_grouped(*gpu(h, router, corr), *args)
+    assert torch.equal(sg.cpu().sort(-1).values, sel.sort(-1).values)
+    order = (x.argsort(-1) for x in (sg.cpu(), sel))
+    close(wg.cpu().gather(1, next(order)), wt.gather(1, next(order)), torch.float32)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,W,F,E,top", [(64, 128, 64, 7, 2), (5, 50, 20, 3, 3)])
+def test_plain_glu_experts(dtype, T, W, F, E, top):
+    h = rnd(T, W, dtype=dtype, scale=8.0)  # beyond any clamp
+    gu, dn = rnd(E, 2 * F, W, dtype=dtype, scale=W ** -0.5), rnd(E, W, F, dtype=dtype, scale=F ** -0.5)
+    sel = torch.rand(T, E).topk(top).indices.int()
+    args = (float("inf"), 1.0, 0.0)
+    y, place = sequence.expert_rows(h, sel, gu, dn, *args)
+    yg, pg = sequence.expert_rows(*gpu(h, sel, gu, dn), *args)
+    close(yg.cpu()[pg.cpu().long()], y[place.long()], dtype)
+
+
+# --------------------------------------------------------------- output norms
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,W", [(7, 512), (5, 50), (3, 2052), (300, 1028)])
+@pytest.mark.parametrize("kind", ["delta", "moe", "both"])
+@pytest.mark.parametrize("depth", [0, 1, 6])
+@pytest.mark.parametrize("final", [False, True])
+def test_output_norm(dtype, T, W, kind, depth, final):
+    src, w, b = rnd(T, W), 1 + rnd(W, scale=0.2), rnd(W)
+    top, args = 3, {}
+    if kind != "moe":
+        args["delta"] = rnd(T, W, dtype=dtype) + 3.0  # a mean that matters
+    if kind != "delta":
+        args["moe"] = (rnd(T * top, W, dtype=dtype),
+                       torch.randperm(T * top).view(T, top).int(),
+                       torch.rand(T, top).softmax(-1))
+    if kind == "both":
+        args["gate"] = rnd(T, 11, dtype=dtype)[:, 4]
+    if final:
+        args["final"] = (1 + rnd(W, scale=0.2), rnd(W))
+    dev = {k: tuple(gpu(*v)) if isinstance(v, tuple) else v.cuda() for k, v in args.items()}
+    room = (depth + 1, depth)[final]  # the last result is not kept
+    kept = rnd(room, T, W)
+    kg = kept.cuda()
+    if depth:
+        coefs = rnd(depth + 1)
+        args["depth"], dev["depth"] = (kept, coefs), (kg, coefs.cuda())
+    x, xg = torch.empty(T, W), torch.empty(T, W, device="cuda")
+    want = torch_ref.output_norm(src, x, w, b, 1e-5, dtype=dtype, **args)
+    got = ops.output_norm(src.cuda(), xg, w.cuda(), b.cuda(), 1e-5, dtype=dtype, **dev)
+    close(got, want, dtype)
+    close(xg, x, torch.float32)
+    if depth:
+        close(kg, kept, torch.float32)
+    # in place
+    xg = src.cuda()
+    ops.output_norm(xg, xg, w.cuda(), b.cuda(), 1e-5, dtype=dtype, **dev)
+    close(xg, x, torch.float32)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("F", [256, 36, 5])
+def test_gelu_and_silu_glu(dtype, F):
+    z = torch.cat([rnd(9, 2 * F + 3), rnd(9, 2 * F + 3, scale=1e-3),
+                   rnd(9, 2 * F + 3, scale=8.0)]).to(dtype)
+    close(ops.silu_glu(z.cuda(), F), ops.silu_glu(z.float(), F), dtype)
+    for x in (z, z[:, :F], z[:, :2 * F].contiguous()):
+        close(ops.gelu(x.cuda()), ops.gelu(x.float()), dtype)
 
 
 # ------------------------------------- embeddings, input convolution, activation
