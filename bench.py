@@ -66,7 +66,7 @@ def parse_args():
                     help="layers per model in --mode layers")
     ap.add_argument("--size", default="all",
                     help="one of the --mode layers sizes, or all")
-    ap.add_argument("--design", choices=("kikalix", "senotar"), default="kikalix",
+    ap.add_argument("--design", choices=("kikalix", "senotar", "gakupel"), default="kikalix",
                     help="design of --mode layers")
     ap.add_argument("--rag", type=int, default=int(os.environ.get("BENCH_RAG", "1")),
                     help="per-turn on-GPU RAG retrieval + input-rail check (1=on)")
@@ -425,6 +425,12 @@ SENOTAR_SIZES = {
     "2048-5632": (2048, 16, 4, 512, 5632),
     "1024-2816": (1024, 16, 4, 256, 2816),
 }
+#: width, heads, kv heads, experts, top, expert ff, shared ff, dense ff
+GAKUPEL_SIZES = {
+    "4096-8x14336": (4096, 32, 8, 8, 2, 14336, 3584, 14336),
+    "2048-64x1408": (2048, 16, 4, 64, 6, 1408, 2816, 5632),
+    "1024-16x512": (1024, 8, 2, 16, 2, 512, 1024, 2816),
+}
 PREFILL_SEQS, PREFILL_LEN, DECODE_SEQS, DECODE_STEPS = 4, 2048, 64, 32
 
 
@@ -460,6 +466,26 @@ def senotar_pair(size: str, n_layers: int):
         name=f"llama-{size}", hidden_size=w, n_layers=n_layers, n_heads=h, n_kv_heads=kv,
         head_dim=d, intermediate_size=ff, vocab_size=32000, max_position=8192)
     return senotar, llama
+
+
+def gakupel_pair(size: str, n_layers: int):
+    """(Gakupel spec, Kikalix spec without a window) of one size: a recurrence in as
+    many layers, experts in as many as have them, heads and states of equal size."""
+    from aurora_amd.models.config import HybridSpec, gakupel_spec, kikalix_layers
+    w, h, kv, experts, top, ff, shared, dense = GAKUPEL_SIZES[size]
+    d = w // h
+    gakupel = gakupel_spec(
+        f"gakupel-{size}", ("pdaP" * n_layers)[:n_layers], width=w, vocab=32000, heads=h,
+        kv_heads=kv, dim=d, l_dim=d, l_vdim=d, d_heads=h // 2, d_kv_heads=h // 2, d_dim=d,
+        d_vdim=d, m_heads=h // 2, m_dim=d, m_vdim=2 * d, ff=dense, experts=experts, top=top,
+        expert_ff=ff, shared_ff=shared, groups=4, keep=2, max_position=8192)
+    kikalix = HybridSpec(
+        name=f"kikalix-{size}", hidden_size=w, vocab_size=32000, max_position=8192,
+        layers=kikalix_layers(
+            ("pppr" * n_layers)[:n_layers], heads=h, kv_heads=kv, dim=d, vdim=d, window=0,
+            d_heads=h // 2, d_kv_heads=h // 2, d_dim=d, d_vdim=d, rank=128, r_heads=h // 2,
+            r_dim=d, r_vdim=2 * d, experts=experts, top=top, ff=ff))
+    return gakupel, kikalix
 
 
 def layer_bench_engine(spec, seed: int = 0):
@@ -506,7 +532,8 @@ def layer_bench_once(eng, rng):
 
 def main_layers(args):
     table, pair = {"kikalix": (LAYER_SIZES, layer_pair),
-                   "senotar": (SENOTAR_SIZES, senotar_pair)}[args.design]
+                   "senotar": (SENOTAR_SIZES, senotar_pair),
+                   "gakupel": (GAKUPEL_SIZES, gakupel_pair)}[args.design]
     sizes = list(table) if args.size == "all" else [args.size]
     result = {}
     for size in sizes:

@@ -62,16 +62,18 @@ def attend(q, k, v, scale, bias=None, sink=False):
     is taken off the scores; a sink adds one to the softmax's denominator."""
     T, H, _ = q.shape
     group = H // k.shape[1]
-    out = torch.zeros(T, H, v.shape[2], dtype=q.dtype)
+    dist = torch.arange(T, dtype=q.dtype).unsqueeze(1) - torch.arange(T, dtype=q.dtype)
+    out = []
     for h in range(H):
-        for i in range(T):
-            s = (k[:i + 1, h // group] @ q[i, h]) * scale
-            if bias is not None:
-                s = s - bias(h, torch.arange(i, -1, -1, dtype=q.dtype))
-            top = max(float(s.max()), 0.0)
-            p = torch.exp(s - top)
-            out[i, h] = (p / (p.sum() + (math.exp(-top) if sink else 0.0))) @ v[:i + 1, h // group]
-    return out
+        s = (q[:, h] @ k[:, h // group].T) * scale
+        if bias is not None:
+            s = s - bias(h, dist.clamp(min=0))
+        s = s.masked_fill(dist < 0, -math.inf)
+        top = s.max(-1, keepdim=True).values.clamp(min=0)
+        p = torch.exp(s - top)
+        whole = p.sum(-1, keepdim=True) + (torch.exp(-top) if sink else 0.0)
+        out.append((p / whole) @ v[:, h // group])
+    return torch.stack(out, 1)
 
 
 # --------------------------------------------------------------------- mixers
