@@ -38,6 +38,7 @@ DEVINL unsigned int pack2_bf16(float lo, float hi) {
   return ((unsigned int)f32_to_bf16(hi) << 16) | f32_to_bf16(lo);
 }
 
+#define LN2 0.69314718f  // the hardware's logarithm has base 2
 enum { NO_BIAS = 0, LINEAR_BIAS = 1, LOG_BIAS = 2 };
 
 union frag_u {
@@ -133,7 +134,7 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
 
   // this head's penalty per token of distance, or of ln(1 + rate * distance);
   // first key any row here sees
-  const float slope = BIAS ? slopes[h] : 0.f;
+  const float slope = BIAS ? slopes[h] * (BIAS == LOG_BIAS ? LN2 : 1.f) : 0.f;
   const float rate = BIAS == LOG_BIAS ? rates[h] : 0.f;
   const int win = BIAS && window > 0 ? window : 0x3fffffff;
   const int tile0 = BIAS ? max(0, ctx - qlen + qoff - win + 1) / KVB : 0;
@@ -200,6 +201,9 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
       }
       // ---- mask + scale (S^T reg r holds key row R = (r&3)+8*(r>>2)+4*half)
       float p[16];
+      // distance of key row 4 * half, and the logarithm's argument there
+      const float dist0 = (float)(q_abs - ks - 4 * half);
+      const float arg0 = 1.f + rate * dist0;
       const bool need_mask = (ks + 31 > q_abs_min) || (ks + 31 >= ctx) ||
                              (BIAS && q_abs_min + 31 - ks >= win);
 #pragma unroll
@@ -209,8 +213,9 @@ __global__ __launch_bounds__(512, 1) void prefill_kernel(
         if constexpr (BIAS != NO_BIAS) {
           // a row that has seen only masked keys yet holds weights of
           // exp(0); its first visible key rescales them to zero
-          const float dist = (float)(q_abs - k_abs);
-          sv -= slope * (BIAS == LOG_BIAS ? __logf(1.f + rate * dist) : dist);
+          const float step = (float)((r & 3) + 8 * (r >> 2));
+          sv -= slope * (BIAS == LOG_BIAS ? __builtin_amdgcn_logf(arg0 - rate * step)
+                                          : dist0 - step);
           if (need_mask && (k_abs > q_abs || k_abs >= ctx || q_abs - k_abs >= win))
             sv = -1e30f;
         } else {

@@ -217,7 +217,7 @@ __global__ __launch_bounds__(1024) void memory_gates_kernel(RecArgs a,
 // Workspace of one (chunk, head), fp32: Q~, K~ (delta rules) and K^ in the order the
 // scan's lanes load them, 256 values per 16 channels: [tile][lane][4], where
 // lane 16 g + i holds channels 4g .. 4g+3 of token i (Q~, K~) or tokens
-// 4g .. 4g+3 of channel i (K^); e^{b_C} [dp]; A, T (delta rules) [16][16]
+// 4g .. 4g+3 of channel i (K^); e^{b_C} [dp], one of them but for DELTA; A, T (delta rules) [16][16]
 struct ChunkSpace {
   float *q, *k, *kt, *g, *a, *t;
   int dp;
@@ -401,7 +401,8 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(
         *reinterpret_cast<floatx4*>(w.k + wt) = k * fq[i];
     }
     *reinterpret_cast<floatx4*>(w.q + wt) = qe;
-    if (i == 0) *reinterpret_cast<floatx4*>(w.g + ws * dp + c0) = ge;
+    if (i == 0 && (MODE == DELTA || c0 == 0))
+      *reinterpret_cast<floatx4*>(w.g + ws * dp + c0) = ge;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       if constexpr (MODE == DELTA) {
@@ -464,9 +465,11 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(
   }
 }
 
-// NTW: 16-channel tiles of the state per wave (key channels <= 64 * NTW)
+// NTW: 16-channel tiles of the state per wave (key channels <= 64 * NTW). A memory's
+// extra column tile makes one workgroup more than fit at two per CU in the usual
+// sizes: it takes three, with one operand set less in flight.
 template <int MODE, int NTW>
-__global__ __launch_bounds__(256, NTW <= 2 ? 2 : 1) void chunk_scan_kernel(
+__global__ __launch_bounds__(256, NTW > 2 ? 1 : MODE == MEMORY ? 3 : 2) void chunk_scan_kernel(
     RecArgs a, const int* __restrict__ cu, const int* __restrict__ cfirst,
     ChunkSpace w, const float* __restrict__ vf, float* __restrict__ of,
     float* __restrict__ den, int S) {
@@ -500,10 +503,12 @@ __global__ __launch_bounds__(256, NTW <= 2 ? 2 : 1) void chunk_scan_kernel(
                  : cn ? nstate[row] : state[(long)row * a.e + col];
     }
 
-  // one chunk's operands; three sets, so that a chunk's loads have two chunks'
-  // time to arrive
+  // one chunk's operands; in three sets, a chunk's loads have two chunks' time to
+  // arrive
+  constexpr int SETS = MODE == MEMORY ? 2 : 3;
+  constexpr int NG = MODE == DELTA ? NTW : 1;  // decays per channel, or one
   struct Frags {
-    floatx4 q[NTW], k[NTW], t[NTW], gd[NTW], v, am, tm;
+    floatx4 q[NTW], k[NTW], t[NTW], gd[NG], v, am, tm;
   };
   const int nch = (len + CHUNK - 1) / CHUNK;
   const long base = cu[s];
@@ -518,8 +523,9 @@ __global__ __launch_bounds__(256, NTW <= 2 ? 2 : 1) void chunk_scan_kernel(
       f.q[x] = ld4(w.q + o);
       if (is_delta(MODE)) f.k[x] = ld4(w.k + o);
       f.t[x] = ld4(w.kt + o);
-      f.gd[x] = ld4(w.g + ws * dp + tile * 16 + 4 * g);
+      if constexpr (MODE == DELTA) f.gd[x] = ld4(w.g + ws * dp + tile * 16 + 4 * g);
     }
+    if constexpr (MODE != DELTA) f.gd[0][0] = w.g[ws * dp];
 #pragma unroll
     for (int r = 0; r < 4; ++r)
       f.v[r] = vf[(base + c * CHUNK + min(4 * g + r, n - 1)) * HE + h * a.e +
@@ -530,15 +536,16 @@ __global__ __launch_bounds__(256, NTW <= 2 ? 2 : 1) void chunk_scan_kernel(
   auto step = [&](int c, Frags& f) {
     const int n = min(CHUNK, len - c * CHUNK);
     const long row0 = base + c * CHUNK;
-    floatx4 qa[NTW], ka[NTW], ta[NTW], gd[NTW];
+    floatx4 qa[NTW], ka[NTW], ta[NTW], gd[NG];
 #pragma unroll
     for (int x = 0; x < NTW; ++x) {
       const float in = wave * NTW + x < RT ? 1.f : 0.f;
       qa[x] = f.q[x];  // meets a zero state where the tile is not there
       if (is_delta(MODE)) ka[x] = f.k[x];
       ta[x] = f.t[x] * in;
-      gd[x] = f.gd[x];
+      if constexpr (MODE == DELTA) gd[x] = f.gd[x];
     }
+    const float g0 = MODE == DELTA ? 0.f : f.gd[0][0];
     floatx4 u;
 #pragma unroll
     for (int r = 0; r < 4; ++r)
@@ -586,21 +593,23 @@ __global__ __launch_bounds__(256, NTW <= 2 ? 2 : 1) void chunk_scan_kernel(
     }
 #pragma unroll
     for (int x = 0; x < NTW; ++x) {
-      st[x] *= gd[x];
+      if constexpr (MODE == DELTA) st[x] *= gd[x];
+      else st[x] *= g0;
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         st[x] = __builtin_amdgcn_mfma_f32_16x16x4f32(ta[x][r], u[r], st[x], 0, 0, 0);
     }
-    if (c + 3 < nch) fetch(c + 3, f);
+    if (c + SETS < nch) fetch(c + SETS, f);
   };
   Frags f0, f1, f2;
   fetch(0, f0);
   if (nch > 1) fetch(1, f1);
-  if (nch > 2) fetch(2, f2);
-  for (int c = 0; c < nch; c += 3) {
+  if (SETS > 2 && nch > 2) fetch(2, f2);
+  for (int c = 0; c < nch; c += SETS) {
     step(c, f0);
     if (c + 1 < nch) step(c + 1, f1);
-    if (c + 2 < nch) step(c + 2, f2);
+    if constexpr (SETS > 2)
+      if (c + 2 < nch) step(c + 2, f2);
   }
 #pragma unroll
   for (int x = 0; x < NTW; ++x)

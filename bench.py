@@ -26,7 +26,7 @@ Two modes:
 
 * ``--mode layers``: prefill and decode throughput of a few full-width layers
   of a layer-listed decoder (``--design``: Kikalix beside a Mixtral-style model,
-  Senotar beside a Llama-style one) and as many of the other of equal width,
+  Senotar beside a Llama-style one, Gakupel beside Kikalix) and as many of the other of equal width,
   heads, experts and feed-forward (random weights), each through its engine's
   own batch building, kernels and decode graphs, the two timed in turn.
 
