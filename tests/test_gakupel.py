@@ -162,7 +162,11 @@ def weights(cfg, seed=0, decided=False):
         E = f["router"]["experts"]
         t[p + "router"], t[p + "correction"] = lin(E, w, 1.5), n(E, s=0.2) - 0.8
         if decided:
-            t[p + "correction"] = torch.randperm(E, generator=gen) * 2.0 - E
+            # groups one above the other, so that their sums are far apart as well
+            c = f["router"]["groups"]["count"]
+            rank = torch.argsort(torch.rand(c, E // c, generator=gen)) * 2.0
+            t[p + "correction"] = (rank + torch.randperm(c, generator=gen).view(c, 1)
+                                   * (4.0 * (E // c))).flatten() - 2 * E
         for e in range(E):
             glu(f"{p}e{e}.", f["expert"]["ff"])
         glu(p + "shared.", f["shared"]["ff"])
