@@ -57,8 +57,32 @@ class ModelSpec:
 # A HybridSpec spells its layers out one by one: each has a mixer (attention
 # beside a recurrence, a recurrence or attention alone) and an optional
 # feed-forward. What all layers share (the norms' kind and place, residual gates,
-# the convolution of the mixer's input, depth averages) are fields of the
+# the convolution of a sublayer's input, depth averages) are fields of the
 # HybridSpec.
+
+@dataclass(frozen=True)
+class YarnSpec:
+    """Frequencies stretched for longer contexts: pairs that turn fewer than
+    ``slow`` times within ``original`` positions by ``factor``, pairs that turn more
+    than ``fast`` times not at all, those between in part."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass(frozen=True)
+class RotationSpec:
+    """Rotary positions of neighbours: dimensions 2i and 2i + 1 of the first ``dims``
+    turn by position * base^(-2i/dims)."""
+    dims: int
+    base: float
+    yarn: Optional[YarnSpec] = None
+
+    def __post_init__(self):
+        if self.dims < 2 or self.dims % 2:
+            raise ValueError(f"cannot rotate {self.dims} dimensions")
+
 
 @dataclass(frozen=True)
 class BiasedAttentionSpec:
@@ -104,14 +128,20 @@ class RetentionSpec:
 
 @dataclass(frozen=True)
 class LatentAttentionSpec:
-    """Attention without positions over one cached latent per token, with a
-    sink in the softmax and a gate per head."""
+    """Attention over one cached latent per token."""
     heads: int
     dim: int
     vdim: int
     kv_rank: int
     scale: float
     kv_from: Optional[int] = None  # layer whose latents it reads; None: its own
+    q_rank: int = 0     # width of the normed latent queries come from; 0: none
+    #: beside the ``dim`` dimensions without positions a head has rot.dims rotated
+    #: ones, whose key all heads share; None: no positions
+    rot: Optional[RotationSpec] = None
+    window: int = 0     # keys a query sees, itself included; 0 = all before it
+    sink: bool = True   # a learned term of the softmax's denominator per head
+    gate: bool = True   # a sigmoid gate per head
 
 
 @dataclass(frozen=True)
@@ -143,6 +173,35 @@ class NormedAttentionSpec:
 
 
 @dataclass(frozen=True)
+class ConvAttentionSpec:
+    """Grouped-query attention whose projections pass a short causal convolution."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    conv: int                  # taps
+    rot: RotationSpec
+    #: values turn with their own position and every head's result back by the
+    #: query's, pair m by base^(-2m/vdim) per position; 0: they do not turn
+    value_base: float = 0.0
+    window: int = 0            # keys a query sees, itself included; 0: no window
+    chunk: int = 0             # keys of the query's chunk of positions alone; 0: no chunks
+    sink: bool = False         # the softmax's denominator has one more term, 1
+    gate: bool = False         # a sigmoid gate as wide as the heads
+
+    def __post_init__(self):
+        if self.heads % self.kv_heads:
+            raise ValueError("query heads must be a multiple of key/value heads")
+        if self.rot.dims > self.dim:
+            raise ValueError(f"cannot rotate {self.rot.dims} of {self.dim} dimensions")
+        if self.value_base and self.vdim % 2:
+            raise ValueError(f"cannot rotate {self.vdim} value dimensions")
+        if self.conv < 1:
+            raise ValueError(f"a convolution of {self.conv} taps")
+
+
+@dataclass(frozen=True)
 class HeadDeltaSpec:
     """Gated delta rule with a short convolution, one decay per head and a silu
     gate as wide as the heads."""
@@ -167,7 +226,7 @@ class MatrixMemorySpec:
     gate_cap: float
 
 
-PartSpec = Union[NormedAttentionSpec, HeadDeltaSpec, MatrixMemorySpec]
+PartSpec = Union[NormedAttentionSpec, ConvAttentionSpec, HeadDeltaSpec, MatrixMemorySpec]
 
 
 @dataclass(frozen=True)
@@ -188,18 +247,25 @@ class MoESpec:
 
 @dataclass(frozen=True)
 class GroupedMoESpec:
-    """Sigmoid-routed GLU experts, chosen by corrected scores among the best
-    ``keep`` of ``groups`` groups of neighbours, beside a shared expert (of width
-    ``shared_ff``; 0: none) behind a sigmoid gate."""
+    """Experts chosen among the best ``keep`` of ``groups`` groups of neighbours,
+    beside a shared expert (of width ``shared_ff``; 0: none)."""
     experts: int
     top: int
     ff: int
-    scale: float
+    scale: float = 1.0
     groups: int = 1
     keep: int = 1
     shared_ff: int = 0
+    #: "sigmoid": corrected scores choose, groups by the sum of their two largest,
+    #: weights are the chosen plain scores' shares; "softmax": scores over all
+    #: experts choose and weigh, groups by their largest
+    scores: str = "sigmoid"
+    act: str = "silu_glu"  # or "relu2": two matrices around the square of relu
+    shared_gate: bool = True  # a sigmoid gate of one number per token
 
     def __post_init__(self):
+        if self.scores not in ("sigmoid", "softmax") or self.act not in ("silu_glu", "relu2"):
+            raise ValueError(f"unknown router {self.scores!r} or activation {self.act!r}")
         if self.experts % self.groups or not 1 <= self.keep <= self.groups \
                 or not 1 <= self.top <= self.keep * (self.experts // self.groups):
             raise ValueError(f"cannot choose {self.top} of {self.experts} experts in the "
@@ -255,10 +321,15 @@ class HybridSpec:
     embedding: Optional[EmbeddingSpec] = None
     #: taps of the causal convolution added to every mixer's input (0: none)
     input_conv: int = 0
+    #: the same for every feed-forward's input
+    ff_conv: int = 0
     #: each sublayer's result is scaled by a sigmoid gate of the sublayer's input
     residual_gates: bool = False
     #: what norms add to their stored weight
     norm_offset: float = 1.0
+    #: beside each sublayer's input, its result is RMS normed as well
+    result_norms: bool = False
+    logit_scale: float = 1.0
     #: True: sublayers read the residual itself, and a layer norm with bias is
     #: taken of each sublayer's result; False: an RMS norm of each one's input
     output_norms: bool = False
@@ -268,9 +339,12 @@ class HybridSpec:
 
     def __post_init__(self):
         if self.output_norms and (self.loop or self.embedding or self.input_conv
-                                  or self.residual_gates):
+                                  or self.ff_conv or self.residual_gates
+                                  or self.result_norms):
             raise ValueError("output norms come without loops, pair embeddings, input "
-                             "convolutions and residual gates")
+                             "convolutions, residual gates and further norms")
+        if self.result_norms and (self.residual_gates or self.norm_offset):
+            raise ValueError("result norms come without residual gates and offsets")
         if self.depth_average and not self.output_norms:
             raise ValueError("depth averages come with output norms")
         for i, layer in enumerate(self.layers):
@@ -279,9 +353,9 @@ class HybridSpec:
                 continue
             src = self.layers[j].mixer if 0 <= j < i else None
             if not isinstance(src, LatentAttentionSpec) or src.kv_from is not None \
-                    or src.kv_rank != layer.mixer.kv_rank:
+                    or (src.kv_rank, src.rot) != (layer.mixer.kv_rank, layer.mixer.rot):
                 raise ValueError(f"layer {i}: kv_from {j} is no earlier layer with "
-                                 "latents of its own and the same rank")
+                                 "latents of its own, the same rank and rotation")
         if self.loop is not None:
             start, stop, times = self.loop
             if not (0 <= start < stop <= len(self.layers) and times >= 1):
@@ -304,15 +378,15 @@ class HybridSpec:
 
     def param_count(self) -> int:
         w = self.hidden_size
-        norm = 2 * w if self.output_norms else w
-        n = 2 * self.vocab_size * w + norm
+        norm = 2 * w if self.output_norms or self.result_norms else w
+        n = 2 * self.vocab_size * w + (2 * w if self.output_norms else w)
         if self.loop is not None:
             n += self.loop[2] * w
         if self.embedding is not None:
             n += (self.embedding.bigram.buckets + 2) * w
         for i, layer in enumerate(self.layers):
             n += norm * (1 if layer.mlp is None else 2)
-            n += self.input_conv * w
+            n += self.input_conv * w + (0 if layer.mlp is None else self.ff_conv * w)
             if self.residual_gates:
                 n += (1 if layer.mlp is None else 2) * (w + 1) * w
             if self.depth_average:
@@ -327,9 +401,12 @@ def _mixer_params(m: MixerSpec, w: int) -> int:
     if isinstance(m, RetentionSpec):
         return w * m.heads * (2 * m.dim + 3 * m.vdim)
     if isinstance(m, LatentAttentionSpec):
-        n = w * m.heads * (m.dim + m.vdim + 1) + m.heads
+        rot = m.rot.dims if m.rot else 0
+        q = m.heads * (m.dim + rot)
+        n = m.q_rank * (w + 1 + q) if m.q_rank else w * q
+        n += w * m.heads * (m.vdim + m.gate) + (m.heads if m.sink else 0)
         n += m.kv_rank * m.heads * (m.dim + m.vdim)
-        return n + (m.kv_rank * (w + 1) if m.kv_from is None else 0)
+        return n + (m.kv_rank * (w + 1) + rot * w if m.kv_from is None else 0)
     a, r = m.left, m.right
     qkv = a.heads * a.dim + a.kv_heads * (a.dim + a.vdim)
     n = (w + 1) * qkv + w * a.heads * a.vdim
@@ -345,6 +422,9 @@ def _part_params(p: PartSpec, w: int) -> int:
         n = w * (q + k + p.heads * p.vdim) + (2 * p.dim if p.norm == "head" else q + k)
         return n + (0 if p.shared_kv else w * p.kv_heads * p.vdim) \
             + (2 * p.heads if p.log_bias else 0)
+    if isinstance(p, ConvAttentionSpec):
+        ch, e = p.heads * p.dim + p.kv_heads * (p.dim + p.vdim), p.heads * p.vdim
+        return ch * (w + p.conv) + w * e * (2 if p.gate else 1)
     if isinstance(p, HeadDeltaSpec):
         ch = 2 * p.kv_heads * p.dim + p.heads * p.vdim
         return ch * (w + p.conv) + 2 * p.heads * (w + 1) + p.vdim + 2 * w * p.heads * p.vdim
@@ -356,10 +436,11 @@ def _mlp_params(f: Optional[MLPSpec], w: int) -> int:
         return 0
     if isinstance(f, DenseSpec):
         return 2 * w * f.ff + (2 if f.act == "xielu" else 0)
-    n = f.experts * (3 * w * f.ff + w + 1)
-    if isinstance(f, GroupedMoESpec) and f.shared_ff:
-        n += w * (3 * f.shared_ff + 1)
-    return n
+    if isinstance(f, MoESpec):
+        return f.experts * (3 * w * f.ff + w + 1)
+    matrices = 3 if f.act == "silu_glu" else 2
+    n = f.experts * (matrices * w * f.ff + w + (f.scores == "sigmoid"))
+    return n + (w * (matrices * f.shared_ff + f.shared_gate) if f.shared_ff else 0)
 
 
 AnySpec = Union[ModelSpec, HybridSpec]
@@ -485,9 +566,55 @@ def _gakupel_spec(name: str, cfg: dict, shapes: Dict[str, Sequence[int]]) -> Hyb
                      for i, e in enumerate(cfg["layers"])))
 
 
+def _fezuzen_spec(name: str, cfg: dict, shapes: Dict[str, Sequence[int]]) -> HybridSpec:
+    def rotation(r: dict) -> RotationSpec:
+        y = r.get("scaling")
+        return RotationSpec(r["dims"], float(r["base"]), YarnSpec(
+            *(float(y[k]) for k in ("factor", "original", "fast", "slow"))) if y else None)
+
+    def size(m: dict) -> int:
+        return int((m.get("mask") or {}).get("size") or 0)
+
+    def mixer(i: int, kind: str, m: dict) -> MixerSpec:
+        if kind == "latent_attention":
+            if m["rot"]["dims"] != m["rot_dim"]:
+                raise ValueError(f"layer {i}: rotates {m['rot']['dims']} of {m['rot_dim']} "
+                                 "dimensions")
+            return LatentAttentionSpec(
+                heads=m["heads"], dim=m["dim"], vdim=m["vdim"], kv_rank=m["kv_rank"],
+                scale=float(m["scale"]), kv_from=m.get("kv_from"), q_rank=m["q_rank"],
+                rot=rotation(m["rot"]), window=size(m), sink=False, gate=False)
+        if kind == "attention":
+            return FusedMixerSpec((("", ConvAttentionSpec(
+                heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"],
+                scale=float(m["scale"]), conv=m["conv"], rot=rotation(m["rot"]),
+                value_base=float(m["rot"]["base"]), chunk=size(m), sink=True, gate=True), 1.0),))
+        raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+
+    def mlp(i: int, f: Optional[dict]) -> Optional[MLPSpec]:
+        if f is None:
+            return None
+        if f.get("kind", "moe") != "moe":
+            raise ValueError(f"layer {i}: unknown feed-forward {f['kind']!r}")
+        r = f["router"]
+        groups = r.get("groups") or {"count": 1, "keep": 1}
+        return GroupedMoESpec(
+            experts=r["experts"], top=r["top"], ff=f["expert"]["ff"], groups=groups["count"],
+            keep=groups["keep"], shared_ff=(f.get("shared") or {"ff": 0})["ff"],
+            scores="softmax", act="relu2", shared_gate=False)
+
+    taps = cfg["canon"]["taps"]
+    return HybridSpec(
+        name=name, arch="fezuzen", hidden_size=cfg["width"], vocab_size=cfg["vocab"],
+        rms_eps=float(cfg["norm"]["eps"]), norm_offset=0.0, result_norms=True,
+        input_conv=taps, ff_conv=taps, logit_scale=float(cfg["logit_scale"]),
+        layers=tuple(LayerSpec(mixer(i, e["type"], e["mixer"]), mlp(i, e.get("mlp")))
+                     for i, e in enumerate(cfg["layers"])))
+
+
 #: config.json "architecture" -> reader(name, config, tensor shapes)
 _CONFIG_READERS = {"Kikalix": _kikalix_spec, "Senotar": _senotar_spec,
-                   "Gakupel": _gakupel_spec}
+                   "Gakupel": _gakupel_spec, "Fezuzen": _fezuzen_spec}
 
 
 def is_checkpoint_dir(path: str) -> bool:
@@ -710,3 +837,52 @@ register(gakupel_spec(  # layer sizes of a 7B-class decoder, 8 experts like mixt
     l_dim=128, l_vdim=128, d_heads=16, d_kv_heads=16, d_dim=128, d_vdim=256,
     m_heads=16, m_dim=128, m_vdim=256, ff=14336, experts=8, top=2, expert_ff=14336,
     shared_ff=14336, groups=4, keep=2))
+
+# ---- Fezuzen presets ---------------------------------------------------------
+
+def fezuzen_spec(name: str, pattern: str, *, width: int, vocab: int, heads: int, dim: int,
+                 rot_dim: int, vdim: int, kv_rank: int, q_rank: int, window: int,
+                 a_heads: int, kv_heads: int, a_dim: int, a_vdim: int, chunk: int,
+                 experts: int, top: int, expert_ff: int, shared_ff: int, groups: int = 4,
+                 keep: int = 2, taps: int = 4, conv: int = 4, base: float = 5e5,
+                 max_position: int = 131072) -> HybridSpec:
+    """Layers of one size from a pattern: 'o' latent attention with latents of its
+    own, 's' reading the last 'o' layer's, 'a' convolved attention; upper case:
+    without a feed-forward."""
+    yarn = YarnSpec(4.0, max_position / 4, 32.0, 1.0)
+    layers, own = [], None
+    moe = GroupedMoESpec(experts, top, expert_ff, 1.0, groups, keep, shared_ff,
+                         "softmax", "relu2", False)
+    for i, c in enumerate(pattern):
+        if c in "oO":
+            own = i
+        if c in "aA":
+            mixer: MixerSpec = FusedMixerSpec((("", ConvAttentionSpec(
+                a_heads, kv_heads, a_dim, a_vdim, a_dim ** -0.5, conv,
+                RotationSpec(a_dim, base), value_base=base, chunk=chunk, sink=True,
+                gate=True), 1.0),))
+        else:
+            mixer = LatentAttentionSpec(
+                heads, dim, vdim, kv_rank, (dim + rot_dim) ** -0.5,
+                None if c in "oO" else own, q_rank, RotationSpec(rot_dim, base, yarn), window,
+                sink=False, gate=False)
+        layers.append(LayerSpec(mixer, None if c.isupper() else moe))
+    return HybridSpec(
+        name=name, arch="fezuzen", hidden_size=width, vocab_size=vocab, layers=tuple(layers),
+        max_position=max_position, norm_offset=0.0, result_norms=True, input_conv=taps,
+        ff_conv=taps, logit_scale=0.25)
+
+
+register(fezuzen_spec(  # CPU plumbing size
+    "tiny-fezuzen", "oaSo", width=64, vocab=512, heads=3, dim=16, rot_dim=8, vdim=24,
+    kv_rank=20, q_rank=28, window=30, a_heads=4, kv_heads=2, a_dim=16, a_vdim=12, chunk=24,
+    experts=6, top=2, expert_ff=24, shared_ff=40, groups=3, taps=3, max_position=2048))
+register(fezuzen_spec(  # GPU smoke size: the matrix-core kernels' head widths
+    "smoke-fezuzen", "oaso", width=512, vocab=1024, heads=8, dim=128, rot_dim=64, vdim=128,
+    kv_rank=256, q_rank=384, window=300, a_heads=8, kv_heads=2, a_dim=128, a_vdim=64,
+    chunk=200, experts=16, top=2, expert_ff=128, shared_ff=256, max_position=8192))
+register(fezuzen_spec(  # layer sizes of a 2048 wide decoder, 64 experts
+    "fezuzen-13b", "oasa" * 8, width=2048, vocab=32000, heads=16, dim=128, rot_dim=64,
+    vdim=128, kv_rank=512, q_rank=1536, window=4096, a_heads=16, kv_heads=4, a_dim=128,
+    a_vdim=128, chunk=8192, experts=64, top=6, expert_ff=1408, shared_ff=2816, groups=8,
+    keep=3))

@@ -1,14 +1,16 @@
-"""Layer-listed decoders (Kikalix, Senotar, Gakupel): mixers and feed-forwards
-chosen layer by layer, with a span of layers that may run several times.
+"""Layer-listed decoders (Kikalix, Senotar, Gakupel, Fezuzen): mixers and
+feed-forwards chosen layer by layer, with a span of layers that may run several
+times.
 
 Same engine shape as the other decoders: packed varlen tokens, paged KV and
 per-step metadata. Two things differ. The residual stream is one fp32 tensor
 that every norm kernel updates in place (the preceding sub-layer's output, or
 the weighted expert rows, and the pass vector are added by the kernel that
 norms; where norms are taken of the sub-layers' outputs, so are the normed
-output and the average over the depth). And every layer RUN, not layer, owns a paged cache or recurrent state;
-a mixer may instead read an earlier layer's cache. Beside the mixers', state is
-what an input convolution and a pair embedding remember of the last tokens.
+output and the average over the depth). And every layer RUN, not layer, owns a
+paged cache or recurrent state; a mixer may instead read an earlier layer's cache.
+Beside the mixers', state is what input convolutions and a pair embedding remember
+of the last tokens.
 """
 from __future__ import annotations
 
@@ -32,7 +34,7 @@ from .mixers import (
     DenseGeluMLP,
     DenseXieluMLP,
     FusedMixer,
-    GroupedGLU,
+    GroupedExperts,
     LatentAttention,
     ParallelMixer,
     RetentionMixer,
@@ -57,7 +59,8 @@ class HybridLayer(nn.Module):
         elif isinstance(s.mixer, ParallelMixerSpec):
             self.mixer = ParallelMixer(s.mixer, w, spec.rms_eps, dtype)
         elif isinstance(s.mixer, LatentAttentionSpec):
-            self.mixer = LatentAttention(s.mixer, w, spec.rms_eps, dtype)
+            self.mixer = LatentAttention(s.mixer, w, spec.rms_eps, dtype,
+                                         spec.max_position, rotations)
         else:
             m = s.mixer
             key = (m.rot_dims, m.rot_base)
@@ -68,6 +71,12 @@ class HybridLayer(nn.Module):
         # convolution of the mixer's input, residual gate of its output
         self.conv = _param(spec.input_conv, w, dtype=torch.float32) \
             if spec.input_conv else None
+        self.ff_conv = _param(spec.ff_conv, w, dtype=torch.float32) \
+            if spec.ff_conv and s.mlp is not None else None
+        # norms of the sublayers' results
+        self.post1 = _param(w, dtype=torch.float32) if spec.result_norms else None
+        self.post2 = _param(w, dtype=torch.float32) \
+            if spec.result_norms and s.mlp is not None else None
         self.gate = _param(w, w, dtype=dtype) if spec.residual_gates else None
         self.gate_bias = _param(w, dtype=torch.float32) if spec.residual_gates else None
         if s.mlp is None:
@@ -76,10 +85,13 @@ class HybridLayer(nn.Module):
         self.norm2 = _param(w, dtype=torch.float32)
         if spec.output_norms:
             self.norm2_bias = _param(w, dtype=torch.float32)
+        if isinstance(s.mlp, GroupedMoESpec) and s.mlp.shared_gate and s.mlp.shared_ff \
+                and not spec.output_norms:
+            raise ValueError("a shared expert's gate needs output norms")
         if isinstance(s.mlp, GroupedMoESpec) or getattr(s.mlp, "act", None) == "gelu":
             if spec.residual_gates:
                 raise ValueError(f"no residual gates around a {type(s.mlp).__name__}")
-            self.mlp = GroupedGLU(s.mlp, w, dtype) if isinstance(s.mlp, GroupedMoESpec) \
+            self.mlp = GroupedExperts(s.mlp, w, dtype) if isinstance(s.mlp, GroupedMoESpec) \
                 else DenseGeluMLP(s.mlp, w, dtype)
         elif isinstance(s.mlp, DenseSpec):
             self.mlp = DenseXieluMLP(s.mlp, w, dtype, spec.residual_gates)
@@ -89,11 +101,12 @@ class HybridLayer(nn.Module):
             self.mlp = RoutedGLU(s.mlp, w, dtype)
 
     def state_layout(self, dtype) -> List[tuple]:
-        """The input convolution's last inputs, if it has any, then the mixer's."""
+        """The input convolutions' last inputs, if there are any, then the mixer's."""
         own = []
-        if self.conv is not None:
-            taps, w = self.conv.shape
-            own = [(((taps - 1, w), dtype),)]
+        for conv in (self.conv, self.ff_conv):
+            if conv is not None:
+                taps, w = conv.shape
+                own.append((((taps - 1, w), dtype),))
         return own + self.mixer.state_layout(dtype)
 
 
@@ -172,24 +185,33 @@ class HybridForCausalLM(nn.Module):
         norm = {"eps": self.spec.rms_eps, "offset": self.spec.norm_offset,
                 "dtype": self.dtype}
         add: Dict[str, object] = {}  # what the next norm adds to the residual
+
+        def read(weight, conv, state):
+            """The sublayer's normed input, what it reads, and the mixer's state."""
+            if conv is None:
+                h = ops.residual_rmsnorm(x, weight, **norm, **add)
+                return h, h, state
+            h, u = ops.residual_rmsnorm_conv(x, weight, conv_w=conv, ring=state[0][0],
+                                             segments=segments, **norm, **add)
+            return h, u, state[1:]
+
         for i, step, kv, st in self._runs:
             layer = self.layers[i]
             state = meta.states[st]
             if step is not None:
                 add["step"] = self.loop_step[step]
-            if layer.conv is None:
-                h = u = ops.residual_rmsnorm(x, layer.norm1, **norm, **add)
-            else:
-                h, u = ops.residual_rmsnorm_conv(x, layer.norm1, conv_w=layer.conv,
-                                                 ring=state[0][0], segments=segments,
-                                                 **norm, **add)
-                state = state[1:]
+            h, u, state = read(layer.norm1, layer.conv, state)
+            ff_state, state = (state[:1], state[1:]) if layer.ff_conv is not None else ([], state)
             add = {"delta": layer.mixer(u, meta, segments, kv_caches[kv], state)}
             if layer.gate is not None:
                 add["gate"] = (ops.linear(h, layer.gate), layer.gate_bias)
+            if layer.post1 is not None:
+                add["post"] = layer.post1
             if layer.mlp is not None:
-                h = ops.residual_rmsnorm(x, layer.norm2, **norm, **add)
-                add = layer.mlp(h)
+                h, u, _ = read(layer.norm2, layer.ff_conv, ff_state)
+                add = layer.mlp(u)
+                if layer.post2 is not None:
+                    add["post"] = layer.post2
             if trail is not None:
                 y = x.clone()
                 ops.residual_rmsnorm(y, layer.norm1, **norm, **add)
@@ -227,7 +249,8 @@ class HybridForCausalLM(nn.Module):
 
     @torch.inference_mode()
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
-        return ops.linear(hidden, self.lm_head).float()
+        logits = ops.linear(hidden, self.lm_head).float()
+        return logits if self.spec.logit_scale == 1.0 else logits.mul_(self.spec.logit_scale)
 
     @torch.inference_mode()
     def load_tensors(self, get) -> None:
@@ -261,8 +284,12 @@ class HybridForCausalLM(nn.Module):
                             ("dwa", layer.depth)):
                 if t is not None:
                     out[f"l{i}.{name}"] = t.data
-            if layer.conv is not None:
-                out[f"l{i}.canon1"] = layer.conv.data.t()
+            for name, t in (("norm1b", layer.post1), ("norm2b", layer.post2)):
+                if t is not None:
+                    out[f"l{i}.{name}"] = t.data
+            for name, t in (("canon1", layer.conv), ("canon2", layer.ff_conv)):
+                if t is not None:
+                    out[f"l{i}.{name}"] = t.data.t()
             if layer.gate is not None:
                 out[f"l{i}.rg1"], out[f"l{i}.rg1.b"] = layer.gate.data, layer.gate_bias.data
         return out
@@ -320,8 +347,12 @@ class HybridForCausalLM(nn.Module):
                 layer.depth[-1] += 1.0
             layer.norm1.copy_(norm_weight())
             layer.mixer.init_random(randn)
-            if layer.conv is not None:
-                layer.conv.copy_(randn(layer.conv.shape) * 0.3)
+            for conv in (layer.conv, layer.ff_conv):
+                if conv is not None:
+                    conv.copy_(randn(conv.shape) * 0.3)
+            for post in (layer.post1, layer.post2):
+                if post is not None:
+                    post.copy_(norm_weight())
             if layer.gate is not None:
                 layer.gate.copy_(randn((w, w)) * w ** -0.5)
                 layer.gate_bias.copy_(randn((w,)))

@@ -14,6 +14,7 @@ import torch.nn as nn
 
 from .. import ops
 from .config import (
+    ConvAttentionSpec,
     DenseSpec,
     FusedMixerSpec,
     GroupedMoESpec,
@@ -24,11 +25,20 @@ from .config import (
     NormedAttentionSpec,
     ParallelMixerSpec,
     RetentionSpec,
+    RotationSpec,
 )
 
 
 def _param(*shape, dtype) -> nn.Parameter:
     return nn.Parameter(torch.zeros(*shape, dtype=dtype), requires_grad=False)
+
+
+def _rotation(rotations: dict, rot: RotationSpec, max_position: int) -> torch.Tensor:
+    """The cosines and sines of ``rot``, one table for all layers that share it."""
+    if rot not in rotations:
+        rotations[rot] = ops.torch_ref.rotation_table(rot.dims, max_position, rot.base,
+                                                      rot.yarn)
+    return rotations[rot]
 
 
 class FusedColumns:
@@ -248,94 +258,150 @@ class RetentionMixer(nn.Module):
 
 
 class LatentAttention(nn.Module):
-    """Attention without positions over one cached latent per token: keys and
-    values are per-head linear maps of it. The softmax has a sink, every head a
-    sigmoid gate. A layer may read an earlier layer's latents instead of its
-    own. Heads and latents are padded with zeros to the kernels' widths."""
+    """Attention over one cached latent per token: keys and values are per-head
+    linear maps of it, and a part of every key that the heads share may be rotated
+    by its position and cached beside it. Queries come straight from the input or
+    through a normed latent of their own; the softmax may have a sink, every head a
+    sigmoid gate, and there may be a window. A layer may read an earlier layer's
+    latents instead of its own. Heads and latents are padded with zeros to the
+    kernels' widths."""
 
-    def __init__(self, spec: LatentAttentionSpec, hidden: int, eps: float, dtype):
+    def __init__(self, spec: LatentAttentionSpec, hidden: int, eps: float, dtype,
+                 max_position: int, rotations: dict):
         super().__init__()
         self.spec = spec
         self.eps = eps
         H, R = spec.heads, ops.latent_width(spec.kv_rank)
-        self.D, self.E, self.R = D, E, R = (
-            ops.latent_head_width(spec.dim), ops.latent_head_width(spec.vdim), R)
-        own = [("dkv", spec.kv_rank)] if spec.kv_from is None else []
-        self.cols = FusedColumns([("q", H * D)] + own + [("g", H)])
+        rot = spec.rot.dims if spec.rot else 0
+        if rot:
+            D, self.tail, key = ops.latent_rotary_widths(spec.dim, rot)
+            cos_sin = _rotation(rotations, spec.rot, max_position)
+        else:
+            D, self.tail, key, cos_sin = ops.latent_head_width(spec.dim), 0, 0, None
+        E = ops.latent_head_width(spec.vdim)
+        self.D, self.E, self.R, self.row = D, E, R, R + key
+        self.own = spec.kv_from is None
+        columns = [("dq", spec.q_rank)] if spec.q_rank else [("q", H * (D + self.tail))]
+        if self.own:
+            columns += [("dkv", spec.kv_rank)] + ([("kr", rot)] if rot else [])
+        if spec.gate:
+            columns.append(("g", H))
+        self.cols = FusedColumns(columns)
+        f32 = torch.float32
         self.in_proj = _param(self.cols.total, hidden, dtype=dtype)
-        if own:
-            self.latent_norm = _param(spec.kv_rank, dtype=torch.float32)
+        if spec.q_rank:
+            self.q_norm = _param(spec.q_rank, dtype=f32)
+            self.uq = _param(H * (D + self.tail), spec.q_rank, dtype=dtype)
+        if self.own:
+            self.latent_norm = _param(spec.kv_rank, dtype=f32)
         self.uk = _param(H, D, R, dtype=dtype)
         self.uk_t = _param(H, R, D, dtype=dtype)
         self.uv = _param(H, E, R, dtype=dtype)
-        self.sink = _param(H, dtype=torch.float32)
+        self.sink = _param(H, dtype=f32) if spec.sink else None
         self.out_proj = _param(hidden, H * E, dtype=dtype)
+        self.register_buffer("cos_sin", cos_sin, persistent=False)
         self._p: Optional[ops.LatentParams] = None
 
     def kv_layout(self, dtype, device) -> List[Tuple[int, int, int]]:
-        return [(1, self.R, 0)] if self.spec.kv_from is None else []
+        return [(1, self.row, 0)] if self.own else []
 
     def state_layout(self, dtype) -> List[tuple]:
         return []
 
+    def _query_rows(self) -> torch.Tensor:
+        """The queries' weights [H, D + tail, in]."""
+        w = self.uq if self.spec.q_rank else self.cols.unpack(self.in_proj)["q"]
+        return w.unflatten(0, (self.spec.heads, self.D + self.tail))
+
     def load(self, get) -> None:
         s, H, dev = self.spec, self.spec.heads, self.uk.device
+        rot = s.rot.dims if s.rot else 0
 
         def heads(t, n):  # [H*n, ...] -> [H, n, ...]
             return t.to(dev).unflatten(0, (H, n))
 
-        q = torch.zeros(H, self.D, self.in_proj.shape[1], dtype=self.uk.dtype, device=dev)
-        q[:, :s.dim] = heads(get("q"), s.dim)
-        parts = {"q": q.flatten(0, 1), "g": get("g")}
-        if s.kv_from is None:
-            parts["dkv"] = get("dkv")
+        self.in_proj.zero_()
+        parts = self.cols.unpack(self.in_proj)
+        queries, q = self._query_rows(), heads(get("uq" if s.q_rank else "q"), s.dim + rot)
+        queries.zero_()
+        queries[:, :s.dim] = q[:, :s.dim].to(queries.dtype)
+        queries[:, self.D:self.D + rot] = q[:, s.dim:].to(queries.dtype)
+        if s.q_rank:
+            parts["dq"].copy_(get("dq"))
+            self.q_norm.copy_(get("dq.norm"))
+        if self.own:
+            dkv = get("dkv")
+            parts["dkv"].copy_(dkv[:s.kv_rank])
+            if rot:
+                parts["kr"].copy_(dkv[s.kv_rank:])
             self.latent_norm.copy_(get("dkv.norm"))
-        self.cols.pack(parts, self.in_proj)
+        if s.gate:
+            parts["g"].copy_(get("g"))
         self.uk.zero_()
         self.uv.zero_()
         self.uk[:, :s.dim, :s.kv_rank] = heads(get("uk"), s.dim).to(self.uk.dtype)
         self.uv[:, :s.vdim, :s.kv_rank] = heads(get("uv"), s.vdim).to(self.uv.dtype)
         self.uk_t.copy_(self.uk.transpose(1, 2))
-        self.sink.copy_(get("sink"))
+        if s.sink:
+            self.sink.copy_(get("sink"))
         self.out_proj.zero_()
         self.out_proj.unflatten(1, (H, self.E))[:, :, :s.vdim] = get("o").to(
             device=dev, dtype=self.out_proj.dtype).unflatten(1, (H, s.vdim))
 
     def tensors(self) -> Dict[str, torch.Tensor]:
         s, H = self.spec, self.spec.heads
-        out = dict(self.cols.unpack(self.in_proj))
-        out["q"] = out["q"].unflatten(0, (H, self.D))[:, :s.dim].flatten(0, 1)
-        if s.kv_from is None:
+        rot = s.rot.dims if s.rot else 0
+        parts, q = self.cols.unpack(self.in_proj), self._query_rows()
+        q = torch.cat([q[:, :s.dim], q[:, self.D:self.D + rot]], 1).flatten(0, 1)
+        out = {"uq": q, "dq": parts["dq"], "dq.norm": self.q_norm} if s.q_rank else {"q": q}
+        if self.own:
+            out["dkv"] = torch.cat([parts[n] for n in ("dkv", "kr") if n in parts])
             out["dkv.norm"] = self.latent_norm
+        if s.gate:
+            out["g"] = parts["g"]
         out["uk"] = self.uk[:, :s.dim, :s.kv_rank].flatten(0, 1)
         out["uv"] = self.uv[:, :s.vdim, :s.kv_rank].flatten(0, 1)
-        out["sink"] = self.sink
+        if s.sink:
+            out["sink"] = self.sink
         out["o"] = self.out_proj.unflatten(1, (H, self.E))[:, :, :s.vdim].flatten(1)
         return out
 
     def init_random(self, randn) -> None:
-        s, H, hidden = self.spec, self.spec.heads, self.in_proj.shape[1]
-        shapes = {"q": (H * s.dim, hidden), "dkv": (s.kv_rank, hidden), "g": (H, hidden),
-                  "uk": (H * s.dim, s.kv_rank), "uv": (H * s.vdim, s.kv_rank),
-                  "o": (hidden, H * s.vdim)}
-        self.load(lambda n: randn(shapes[n]) * shapes[n][1] ** -0.5 if n in shapes
-                  else 1.0 + 0.1 * randn((s.kv_rank,)) if n == "dkv.norm" else randn((H,)))
+        shapes = {n: tuple(t.shape) for n, t in self.tensors().items()}
+        self.load(lambda n: randn(shapes[n]) * shapes[n][1] ** -0.5 if len(shapes[n]) > 1
+                  else 1.0 + 0.1 * randn(shapes[n]) if n.endswith(".norm")
+                  else randn(shapes[n]))
+
+    def _params(self):
+        # built lazily: the tensors move with .to(device)
+        if self._p is None or self._p[0].uk.device != self.uk.device:
+            s, at = self.spec, self.cols.at
+            front = None
+            if s.q_rank or self.own:
+                front = ops.LatentFrontParams(
+                    at.get("dkv"), s.kv_rank, self.latent_norm.data if self.own else None,
+                    self.eps, at.get("kr", 0), self.R, self.cos_sin, at.get("dq", 0),
+                    s.q_rank, self.q_norm.data if s.q_rank else None)
+            self._p = (ops.LatentParams(
+                s.heads, self.D, self.E, s.scale, at.get("q", 0), at.get("g"), self.uk.data,
+                self.uk_t.data, self.uv.data, self.sink.data if s.sink else None, self.tail,
+                self.cos_sin, s.window), front)
+        return self._p
 
     def forward(self, h, meta, segments, kv, state):
-        s, at = self.spec, self.cols.at
-        if self._p is None or self._p.uk.device != self.uk.device:
-            self._p = ops.LatentParams(s.heads, self.D, self.E, s.scale, at["q"], at["g"],
-                                       self.uk.data, self.uk_t.data, self.uv.data,
-                                       self.sink.data)
-        cache = kv[0][0]
-        proj = ops.linear(h, self.in_proj)
-        if s.kv_from is None:
-            ops.latent_write(proj, at["dkv"], s.kv_rank, self.latent_norm, self.eps,
-                             meta.slot_mapping, cache)
+        p, front = self._params()
+        cache, H, width = kv[0][0], self.spec.heads, self.D + self.tail
+        proj, q = ops.linear(h, self.in_proj), None
+        if front is not None:
+            q = ops.latent_front(proj, front, meta.positions, meta.slot_mapping, cache)
+        if q is not None:
+            q = ops.linear(q, self.uq).unflatten(1, (H, width))
+        elif self.tail:
+            q = proj[:, p.q0:p.q0 + H * width].unflatten(1, (H, width))
         out = torch.empty(h.shape[0], self.out_proj.shape[1], dtype=h.dtype,
                           device=h.device)
         for seg in segments:
-            ops.latent_attention(proj, self._p, cache, seg, out)
+            ops.latent_attention(proj, p, cache, seg, out, q, meta.positions)
         return ops.linear(out, self.out_proj)
 
 
@@ -437,6 +503,56 @@ class NormedAttention(MixerPart):
                                  s.vdim, scale, rate, self.sink)
 
 
+class ConvAttention(MixerPart):
+    """Grouped-query attention over convolved projections with rotary positions on
+    queries and keys, and on values too if they turn; in windows or chunks, with a
+    sink, and a sigmoid gate of every output channel."""
+
+    def __init__(self, spec: ConvAttentionSpec, max_position: int, rotations: dict):
+        H, G, d, e = spec.heads, spec.kv_heads, spec.dim, spec.vdim
+        columns = [("q", H * d), ("k", G * d), ("v", G * e)]
+        shapes = {f"{n}.conv": (w, spec.conv) for n, w in columns}
+        if spec.gate:
+            columns.append(("g", H * e))
+        super().__init__(spec, columns, H * e, shapes)
+        self.register_buffer("turn", _rotation(rotations, spec.rot, max_position),
+                             persistent=False)
+        self.register_buffer("value_turn", _rotation(
+            rotations, RotationSpec(e, spec.value_base), max_position)
+            if spec.value_base else None, persistent=False)
+        self.register_buffer("sink", torch.zeros(H, dtype=torch.float32)
+                             if spec.sink else None, persistent=False)
+
+    def kv_layout(self, dtype, device):
+        s = self.spec
+        return [(s.kv_heads, *ops.cache_head_dims(s.dim, s.vdim, dtype, device))]
+
+    def state_layout(self, dtype):
+        s = self.spec
+        channels = s.heads * s.dim + s.kv_heads * (s.dim + s.vdim)
+        return [(((s.conv - 1, channels), dtype),)]
+
+    def random(self, name, randn):
+        return randn(self.shapes[name]) * self.spec.conv ** -0.5
+
+    def make_params(self, at, t, eps):
+        s = self.spec
+        return ops.ConvHeadsParams(
+            s.heads, s.kv_heads, s.dim, s.vdim, at["q"], at["k"], at["v"],
+            torch.cat([t[f"{n}.conv"] for n in "qkv"]).t().contiguous(), self.turn,
+            self.value_turn)
+
+    def forward(self, proj, at, eps, meta, segments, kv, state, out, col, scale):
+        s, (k_cache, v_cache) = self.spec, kv[0]
+        q = ops.conv_qkv(proj, self.params(at, eps), meta.slot_mapping, state[0][0], segments,
+                         k_cache, v_cache)
+        gate = proj[:, at["g"]:at["g"] + s.heads * s.vdim] if s.gate else None
+        for seg in segments:
+            ops.biased_attention(q, k_cache, v_cache, seg, s.scale, s.window, None, out, col,
+                                 s.vdim, scale, sink=self.sink, chunk=s.chunk,
+                                 turn=self.value_turn, gate=gate)
+
+
 class HeadDelta(MixerPart):
     """Gated delta rule with one decay per head."""
 
@@ -512,6 +628,7 @@ class FusedMixer(nn.Module):
         self.names = [name for name, _, _ in spec.parts]
         self.scales = [scale for _, _, scale in spec.parts]
         make = {NormedAttentionSpec: lambda s: NormedAttention(s, max_position, rotations),
+                ConvAttentionSpec: lambda s: ConvAttention(s, max_position, rotations),
                 HeadDeltaSpec: HeadDelta, MatrixMemorySpec: MatrixMemory}
         self.parts = nn.ModuleList([make[type(s)](s) for _, s, _ in spec.parts])
         self.cols = FusedColumns([(name + n, w) for name, part in zip(self.names, self.parts)
@@ -681,35 +798,43 @@ class RoutedGLU(nn.Module):
                                            self.gate_up, self.down, s.limit, self.ALPHA)}
 
 
-class GroupedGLU(nn.Module):
-    """Sigmoid-routed GLU experts chosen among the best groups, beside a shared
-    expert whose gate is one more row of its first product. Returns the chosen
-    rows unsummed; the output norm adds everything up."""
+class GroupedExperts(nn.Module):
+    """Experts chosen among the best groups, beside a shared expert whose gate, if it
+    has one, is one more row of its first product. Returns the chosen rows unsummed;
+    the next norm adds everything up."""
 
     def __init__(self, spec: GroupedMoESpec, hidden: int, dtype):
         super().__init__()
         self.spec = spec
         E, ff, sf = spec.experts, spec.ff, spec.shared_ff
+        self.first = ("gate", "up") if spec.act == "silu_glu" else ("up",)
+        n = len(self.first)
         self.router = _param(E, hidden, dtype=dtype)
-        self.correction = _param(E, dtype=torch.float32)
-        self.gate_up = _param(E, 2 * ff, hidden, dtype=dtype)
+        self.correction = _param(E, dtype=torch.float32) if spec.scores == "sigmoid" else None
+        self.up = _param(E, n * ff, hidden, dtype=dtype)
         self.down = _param(E, hidden, ff, dtype=dtype)
         if sf:
             # [gate; up; the shared gate's row; zeros]
-            self.shared_in = _param(-(-(2 * sf + 1) // 64) * 64, hidden, dtype=dtype)
+            self.shared_in = _param(-(-(n * sf + spec.shared_gate) // 64) * 64, hidden,
+                                    dtype=dtype)
             self.shared_down = _param(hidden, sf, dtype=dtype)
 
     def tensors(self) -> Dict[str, torch.Tensor]:
         """Weights by the checkpoint's names; views that ``load`` fills."""
-        ff, sf = self.spec.ff, self.spec.shared_ff
-        out = {"router": self.router, "correction": self.correction}
-        for e in range(self.spec.experts):
-            out[f"e{e}.gate"] = self.gate_up[e, :ff]
-            out[f"e{e}.up"] = self.gate_up[e, ff:]
+        s, ff, sf = self.spec, self.spec.ff, self.spec.shared_ff
+        out = {"router": self.router}
+        if self.correction is not None:
+            out["correction"] = self.correction
+        for e in range(s.experts):
+            for i, name in enumerate(self.first):
+                out[f"e{e}.{name}"] = self.up[e, i * ff:(i + 1) * ff]
             out[f"e{e}.down"] = self.down[e]
         if sf:
-            out["shared.gate"], out["shared.up"] = self.shared_in[:sf], self.shared_in[sf:2 * sf]
-            out["shared.sg"] = self.shared_in[2 * sf:2 * sf + 1]
+            for i, name in enumerate(self.first):
+                out[f"shared.{name}"] = self.shared_in[i * sf:(i + 1) * sf]
+            if s.shared_gate:
+                n = len(self.first) * sf
+                out["shared.sg"] = self.shared_in[n:n + 1]
             out["shared.down"] = self.shared_down
         return out
 
@@ -724,11 +849,17 @@ class GroupedGLU(nn.Module):
 
     def forward(self, h) -> Dict[str, object]:
         s = self.spec
+        glu, sf = s.act == "silu_glu", s.shared_ff
+        if (s.scores == "sigmoid") != glu:
+            raise NotImplementedError(f"{s.act} experts behind a {s.scores} router")
         add: Dict[str, object] = {"moe": ops.moe_grouped_glu(
-            h, self.router, self.correction, s.top, s.groups, s.keep, s.scale, self.gate_up,
-            self.down)}
-        if s.shared_ff:
+            h, self.router, self.correction, s.top, s.groups, s.keep, s.scale, self.up,
+            self.down) if glu else ops.moe_softmax_relu2(
+            h, self.router, s.top, s.groups, s.keep, s.scale, self.up, self.down)}
+        if sf:
             z = ops.linear(h, self.shared_in)
-            add["delta"] = ops.linear(ops.silu_glu(z, s.shared_ff), self.shared_down)
-            add["gate"] = z[:, 2 * s.shared_ff]
+            a = ops.silu_glu(z, sf) if glu else ops.relu2(z[:, :sf])
+            add["delta"] = ops.linear(a, self.shared_down)
+            if s.shared_gate:
+                add["gate"] = z[:, len(self.first) * sf]
         return add

@@ -35,6 +35,7 @@ _ARCHS = {
     "kikalix": (_hybrid, _load_named),
     "senotar": (_hybrid, _load_named),
     "gakupel": (_hybrid, _load_named),
+    "fezuzen": (_hybrid, _load_named),
 }
 
 

@@ -241,8 +241,10 @@ def softmax_sample(logits, temperature, top_p, top_k, generator=None):
 
 
 from .sequence import (  # noqa: E402
+    ConvHeadsParams,
     DeltaRuleParams,
     HeadDeltaParams,
+    LatentFrontParams,
     LatentParams,
     MatrixMemoryParams,
     NormedHeadsParams,
@@ -251,19 +253,24 @@ from .sequence import (  # noqa: E402
     bias_kv_write,
     biased_attention,
     cache_head_dims,
+    conv_qkv,
     delta_rule,
     embed_pairs,
     gelu,
     head_delta_rule,
     latent_attention,
+    latent_front,
     latent_head_width,
+    latent_rotary_widths,
     latent_width,
     latent_write,
     matrix_memory,
     moe_clamped_glu,
     moe_grouped_glu,
+    moe_softmax_relu2,
     normed_qkv,
     output_norm,
+    relu2,
     residual_rmsnorm,
     residual_rmsnorm_conv,
     retention,

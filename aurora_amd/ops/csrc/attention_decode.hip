@@ -15,7 +15,7 @@
 // Replaces the per-token provider round-trip of the reference agent loop
 // (reference: server/chat/backend/agent/llm.py:192) with an in-process
 // batched decode step.
-#include "common.h"
+#include "head_turn.h"
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 
@@ -25,10 +25,11 @@
 #define TUNR 4  // tokens prefetched per group iteration (8 measured neutral)
 #endif
 
-enum { NO_BIAS = 0, LINEAR_BIAS = 1, LOG_BIAS = 2 };
+enum { NO_BIAS = 0, LINEAR_BIAS = 1, LOG_BIAS = 2, FLAT_BIAS = 3 };
 
-// BIAS: a distance penalty per head (see attention_prefill.hip) and a window; sink:
-// one more term of the denominator per head, or null
+// BIAS: a distance penalty per head or none (see attention_prefill.hip), a window or
+// chunks of positions; sink: one more term of the denominator per head, or null;
+// FLAT_BIAS results may be turned back and gated
 template <int D, int DV, int G, bool FP8, int BIAS>
 __global__ __launch_bounds__(256) void paged_decode_kernel(
     const __hip_bfloat16* __restrict__ q,   // [B, Hq, D]
@@ -42,7 +43,7 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
     int P, int MP, int CS, float scale,
     long ostride, int dv, float oscale,
     const float* __restrict__ slopes, const float* __restrict__ rates, int window,
-    const float* __restrict__ sink) {
+    int chunk_of, const float* __restrict__ sink, HeadTurn turn) {
   constexpr int GL = (D > DV ? D : DV) / 8;  // lanes per token-group
   constexpr int TPW = WAVE / GL;   // token-groups per wave
   constexpr int NW = 4;            // waves per workgroup
@@ -55,7 +56,8 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
   const int cs = blockIdx.z;
   const int L = ctx_lens[b];
   // contiguous chunk of the visible context for this split
-  const int first = BIAS && window > 0 ? max(0, L - window) : 0;
+  int first = BIAS && window > 0 ? max(0, L - window) : 0;
+  if (BIAS && chunk_of > 0) first = max(first, L - 1 - (L - 1) % chunk_of);
   const int chunk = (L - first + CS - 1) / CS;
   const int t_lo = first + cs * chunk;
   const int t_hi = min(L, t_lo + chunk);
@@ -77,7 +79,7 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
   float slope[G], rate[G];
 #pragma unroll
   for (int g = 0; g < G; ++g) {
-    slope[g] = BIAS ? slopes[h0 + g] : 0.f;
+    slope[g] = BIAS && BIAS != FLAT_BIAS ? slopes[h0 + g] : 0.f;
     rate[g] = BIAS == LOG_BIAS ? rates[h0 + g] : 0.f;
   }
   // 16-B column of a key / value row this lane reads (lanes past the narrower
@@ -135,7 +137,7 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
 #pragma unroll
       for (int g = 0; g < G; ++g) {
         s[g] = group_sum<GL>(dot8_bf16_fast(kf[u], qf[g])) * scale;
-        if constexpr (BIAS != NO_BIAS) {
+        if constexpr (BIAS == LINEAR_BIAS || BIAS == LOG_BIAS) {
           const float dist = (float)(L - 1 - t0 - u);
           s[g] -= slope[g] * (BIAS == LOG_BIAS ? __logf(1.f + rate[g] * dist) : dist);
         }
@@ -189,9 +191,10 @@ __global__ __launch_bounds__(256) void paged_decode_kernel(
     }
     const long hq = (long)b * Hq + h0 + g;
     if (CS == 1) {
+      float y = O / Lsum * oscale;
+      if constexpr (BIAS == FLAT_BIAS) y = turned<bf16_t>(turn, y, b, L - 1, h0 + g, d, dv);
       if (!BIAS || d < dv)
-        *(unsigned short*)(out + b * ostride + (long)(h0 + g) * dv + d) =
-            f32_to_bf16(O / Lsum * oscale);
+        *(unsigned short*)(out + b * ostride + (long)(h0 + g) * dv + d) = f32_to_bf16(y);
     } else {
       // emit an un-normalised chunk partial: {o*w-sum, m, l}
       float* dst = part + ((long)cs * gridDim.x * Hq + hq) * (DV + 2);
@@ -210,7 +213,8 @@ __global__ void decode_combine_kernel(const float* __restrict__ part,
                                       __hip_bfloat16* __restrict__ out,
                                       int CS, long BH, int Hq, long ostride,
                                       int dv, float oscale,
-                                      const float* __restrict__ sink) {
+                                      const float* __restrict__ sink, HeadTurn turn,
+                                      const int* __restrict__ ctx_lens) {
   const long bh = blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
   if (bh >= BH) return;
   const int lane = threadIdx.x % WAVE;
@@ -229,8 +233,10 @@ __global__ void decode_combine_kernel(const float* __restrict__ part,
       const float* p = part + ((long)s * BH + bh) * (D + 2);
       O += __expf(p[D] - M) * p[d];
     }
-    *(unsigned short*)(out + bh / Hq * ostride + bh % Hq * dv + d) =
-        f32_to_bf16(O / Lsum * oscale);
+    float y = O / Lsum * oscale;
+    if (turn.cs || turn.gate)
+      y = turned<bf16_t>(turn, y, bh / Hq, ctx_lens[bh / Hq] - 1, bh % Hq, d, dv);
+    *(unsigned short*)(out + bh / Hq * ostride + bh % Hq * dv + d) = f32_to_bf16(y);
   }
 }
 
@@ -242,7 +248,8 @@ static void decode_launch(const torch::Tensor& q, const torch::Tensor& kc,
                           const torch::Tensor& vc, const torch::Tensor& bt,
                           const torch::Tensor& ctx, __hip_bfloat16* out, long ostride,
                           int dv, float scale, float oscale, const float* slopes,
-                          const float* rates, int window, const float* sink, int CS) {
+                          const float* rates, int window, int chunk, const float* sink,
+                          const HeadTurn& turn, int CS) {
   const int B = q.size(0), Hq = q.size(1);
   const int Hkv = kc.size(1), P = kc.size(2), MP = bt.size(1);
   const int G = Hq / Hkv, GT = head_tile(G);
@@ -257,7 +264,7 @@ static void decode_launch(const torch::Tensor& q, const torch::Tensor& kc,
                      0, stream, (const __hip_bfloat16*)q.data_ptr(),            \
                      kc.data_ptr(), vc.data_ptr(), out, pp, bt.data_ptr<int>(), \
                      ctx.data_ptr<int>(), Hkv, G / GT, P, MP, CS, scale,        \
-                     ostride, dv, oscale, slopes, rates, window, sink)
+                     ostride, dv, oscale, slopes, rates, window, chunk, sink, turn)
   switch (GT) {
     case 8: LAUNCH(8); break;
     case 4: LAUNCH(4); break;
@@ -268,7 +275,8 @@ static void decode_launch(const torch::Tensor& q, const torch::Tensor& kc,
   if (CS > 1) {
     const long BH = (long)B * Hq;
     hipLaunchKernelGGL((decode_combine_kernel<DV>), dim3((BH + 3) / 4), dim3(256), 0,
-                       stream, pp, out, CS, BH, Hq, ostride, dv, oscale, sink);
+                       stream, pp, out, CS, BH, Hq, ostride, dv, oscale, sink, turn,
+                       ctx.data_ptr<int>());
   }
   HIP_CHECK_KERNEL();
 }
@@ -290,7 +298,7 @@ torch::Tensor paged_attention_decode(torch::Tensor q, torch::Tensor kc,
   const bool fp8 = kc.dtype() == torch::kFloat8_e4m3fn;
 #define RUN(DD, F8) \
   decode_launch<DD, DD, F8, NO_BIAS>(q, kc, vc, bt, ctx, o, stride, D, (float)scale, \
-                                     1.f, nullptr, nullptr, 0, nullptr, CS)
+                                     1.f, nullptr, nullptr, 0, 0, nullptr, HeadTurn{}, CS)
   if (D == 128) { if (fp8) RUN(128, true); else RUN(128, false); }
   else { if (fp8) RUN(64, true); else RUN(64, false); }
 #undef RUN
@@ -299,9 +307,11 @@ torch::Tensor paged_attention_decode(torch::Tensor q, torch::Tensor kc,
 
 void biased_attention_decode(torch::Tensor q, torch::Tensor kc, torch::Tensor vc,
                              torch::Tensor bt, torch::Tensor ctx, double scale,
-                             long window, torch::Tensor slopes,
+                             long window, long chunk, c10::optional<torch::Tensor> slopes,
                              c10::optional<torch::Tensor> rates,
-                             c10::optional<torch::Tensor> sink, torch::Tensor out,
+                             c10::optional<torch::Tensor> sink,
+                             c10::optional<torch::Tensor> turn,
+                             c10::optional<torch::Tensor> gate, torch::Tensor out,
                              long col, long dv, double oscale) {
   TORCH_CHECK(q.is_cuda() && q.dtype() == torch::kBFloat16 && q.is_contiguous());
   const int B = q.size(0), Hq = q.size(1), D = q.size(2);
@@ -312,23 +322,28 @@ void biased_attention_decode(torch::Tensor q, torch::Tensor kc, torch::Tensor vc
               kc.is_contiguous() && vc.is_contiguous() && bt.is_contiguous());
   TORCH_CHECK(out.dtype() == torch::kBFloat16 && out.size(0) == B && out.stride(1) == 1 &&
               dv <= DV && col + Hq * dv <= out.size(1));
-  TORCH_CHECK(slopes.numel() == Hq && slopes.dtype() == torch::kFloat32);
-  for (auto* t : {&rates, &sink})
+  for (auto* t : {&slopes, &rates, &sink})
     TORCH_CHECK(!*t || ((*t)->numel() == Hq && (*t)->dtype() == torch::kFloat32));
+  const HeadTurn ht = head_turn(turn, gate, slopes || rates, q, Hq, dv);
   TORCH_CHECK(ctx.numel() == B && bt.size(0) == B && bt.dtype() == torch::kInt32 &&
               ctx.dtype() == torch::kInt32);
   if (B == 0) return;
   // a split of fewer than 64 visible keys is not worth its combine
   int CS = std::max(1, std::min(8, 1024 / std::max(B * Hkv, 1)));
-  if (window > 0) CS = std::max(1, std::min(CS, (int)((window + 63) / 64)));
+  for (long seen : {window, chunk})
+    if (seen > 0) CS = std::max(1, std::min(CS, (int)((seen + 63) / 64)));
   auto* o = (__hip_bfloat16*)out.data_ptr() + col;
   const float* rp = rates ? rates->data_ptr<float>() : nullptr;
+  const float* sp = slopes ? slopes->data_ptr<float>() : nullptr;
   const float* snk = sink ? sink->data_ptr<float>() : nullptr;
 #define RUN1(DD, DVV, BB)                                                        \
   decode_launch<DD, DVV, false, BB>(q, kc, vc, bt, ctx, o, out.stride(0),        \
                                     (int)dv, (float)scale, (float)oscale,        \
-                                    slopes.data_ptr<float>(), rp, (int)window, snk, CS)
-#define RUN(DD, DVV) if (rp) RUN1(DD, DVV, LOG_BIAS); else RUN1(DD, DVV, LINEAR_BIAS)
+                                    sp, rp, (int)window, (int)chunk, snk, ht, CS)
+#define RUN(DD, DVV)                         \
+  if (!sp) RUN1(DD, DVV, FLAT_BIAS);         \
+  else if (rp) RUN1(DD, DVV, LOG_BIAS);      \
+  else RUN1(DD, DVV, LINEAR_BIAS)
   if (D == 64 && DV == 64) { RUN(64, 64); }
   else if (D == 64 && DV == 128) { RUN(64, 128); }
   else if (D == 128 && DV == 64) { RUN(128, 64); }

@@ -3,7 +3,8 @@
 //
 // A head's score q.(uk c) is (uk' q).c, and its output uv (sum_j p_j c_j), so
 // attention can stay in the latents' space: all (token, head) rows of a
-// sequence attend to ONE key row that is also the value row. That is what
+// sequence attend to ONE key row that is also the value row. A rotated key part that
+// the heads share follows c in that row and scores like the rest of it. That is what
 // decoding does (a latent is read once for all heads; 2 R flops per byte and
 // head row, so it needs the matrix cores), and short prompt portions on a long
 // context. Long portions spell keys and values out and run the flash prefill
@@ -15,7 +16,7 @@
 //    the tile before is computed, and scores them: S^T = C Q^T, the rows'
 //    queries live in registers as B fragments;
 //  * the bf16 weights go through LDS (one barrier a tile), then every wave owns
-//    R / 4 columns of O += P C. The value fragments are columns of the row-major
+//    VR / 4 columns of O += P C, VR the row's width without the key part. The value fragments are columns of the row-major
 //    tile: ds_read_b64_tr_b16 transposes on the way to the registers.
 //    Contraction slot 8 g + j holds key 4 g + j (j < 4) or 16 + 4 g + j - 4, on
 //    both operands;
@@ -28,9 +29,10 @@
 //    moves, and only then the waves exchange maxima and rescale O, when a score
 //    exceeds it by more than LAT_SLACK, so weights stay below 2^LAT_SLACK.
 // Few rows: the context is split over blockIdx.y, partial sums are merged by
-// latent_combine_kernel. A row's softmax starts from its sink (split 0 only).
-// Scores, maxima and sinks are in units of log 2.
-#include "elem.h"
+// latent_combine_kernel. A row's softmax starts from its sink, if there is one (split
+// 0 only). A window leaves out the tiles before it. Scores, maxima and sinks are in
+// units of log 2.
+#include "head_turn.h"
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
 
@@ -101,18 +103,18 @@ DEVINL void await_columns(shortx4 (&ready)[4]) {
                : "memory");
 }
 
-template <int R, int MT>
+template <int R, int VR, int MT>
 __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
     const bf16_t* __restrict__ q,      // [T * H, R]
     const bf16_t* __restrict__ cache,  // [NP, P, R]
     const int* __restrict__ bt, int MP, const int* __restrict__ cu,
     const int* __restrict__ ctx, const int* __restrict__ bseq,
     const int* __restrict__ boff, const float* __restrict__ sink,
-    bf16_t* __restrict__ out,          // [T * H, R] (one split)
-    float* __restrict__ part,          // [CS, T * H, R] (several)
+    bf16_t* __restrict__ out,          // [T * H, VR] (one split)
+    float* __restrict__ part,          // [CS, T * H, VR] (several)
     float* __restrict__ part_ml,       // [CS, T * H, 2]
-    int H, int P, long rows_all, float scale) {
-  constexpr int NT = R / 64;           // 16-column tiles of O per wave
+    int H, int P, long rows_all, float scale, int window) {
+  constexpr int NT = VR / 64;          // 16-column tiles of O per wave
   constexpr int ROWS = 16 * MT;
   constexpr int SLICE = 16 * R * 2;    // bytes of a wave's 16 latents
   constexpr int TILE = 4 * SLICE;
@@ -134,9 +136,11 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
   const int start = ctx[seq] - n;
   const int first_pos = start + off / H;
   const int kend = start + (off + nrows - 1) / H + 1;  // keys any row here sees
+  const int win = window > 0 ? window : 0x3fffffff;
+  const int before = max(0, first_pos - win + 1) / LAT_KEYS;  // tiles nobody here sees
   const int ntiles = (kend + LAT_KEYS - 1) / LAT_KEYS;
-  const int per = (ntiles + gridDim.y - 1) / gridDim.y;
-  const int tile0 = blockIdx.y * per, tile1 = min(ntiles, tile0 + per);
+  const int per = (ntiles - before + gridDim.y - 1) / gridDim.y;
+  const int tile0 = before + blockIdx.y * per, tile1 = min(ntiles, tile0 + per);
   const int* pages = bt + (long)seq * MP;
   const float scale2 = scale * LOG2E;
 
@@ -189,8 +193,8 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
 #pragma unroll
     for (int k = 0; k < R / 32; ++k) qf[t][k].s = *(const shortx8*)(src + k * 32);
     pos[t] = start + (off + r) / H;
-    m[t] = blockIdx.y == 0 ? sink[(off + r) % H] * LOG2E : -1e30f;
-    l[t] = blockIdx.y == 0 && wave == 0 && g == 0 ? 1.f : 0.f;
+    m[t] = sink && blockIdx.y == 0 ? sink[(off + r) % H] * LOG2E : -1e30f;
+    l[t] = sink && blockIdx.y == 0 && wave == 0 && g == 0 ? 1.f : 0.f;
   }
   floatx4 o[MT][NT];
 #pragma unroll
@@ -239,7 +243,8 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
     });
     await_blocks(kf[R / 32], kf[R / 32 + 1]);
     score(st, kf[R / 32], kf[R / 32 + 1], R / 32 - 2);
-    const bool some_hidden = tile * LAT_KEYS + LAT_KEYS - 1 > first_pos;
+    const bool some_hidden = tile * LAT_KEYS + LAT_KEYS - 1 > first_pos ||
+                             kend - 1 - tile * LAT_KEYS >= win;
     const int key0 = tile * LAT_KEYS + wave * 16 + g * 4;
     short* pb = pbuf + (tile & 1) * (ROWS * LAT_PSTRIDE);
 #pragma unroll
@@ -248,7 +253,7 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
       if (some_hidden)
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          if (key0 + r > pos[t]) st[t][r] = -INFINITY;
+          if (key0 + r > pos[t] || pos[t] - key0 - r >= win) st[t][r] = -INFINITY;
     }
     auto weigh = [&](int t) {  // stores the weights, returns their sum
       floatx4 p;
@@ -354,11 +359,11 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
         const float inv = 1.f / sum;
 #pragma unroll
         for (int c = 0; c < NT; ++c)
-          stf(ob + row * R + (wave * NT + c) * 16 + col, o[t][c][r] * inv);
+          stf(ob + row * VR + (wave * NT + c) * 16 + col, o[t][c][r] * inv);
       }
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-    for (int i = tid; i < nrows * (R / 8); i += 256)
-      *(shortx8*)(out + row0 * R + (long)i * 8) = *(const shortx8*)(ob + i * 8);
+    for (int i = tid; i < nrows * (VR / 8); i += 256)
+      *(shortx8*)(out + row0 * VR + (long)i * 8) = *(const shortx8*)(ob + i * 8);
     return;
   }
   // (a split without keys has no sums, and nobody reads any)
@@ -371,7 +376,7 @@ __global__ __launch_bounds__(256, 1) void latent_attention_kernel(
       if (row >= nrows || tile0 >= tile1) continue;
 #pragma unroll
       for (int c = 0; c < NT; ++c)
-        part[(prow + row) * R + (wave * NT + c) * 16 + col] = o[t][c][r];
+        part[(prow + row) * VR + (wave * NT + c) * 16 + col] = o[t][c][r];
     }
   if (wave == 0 && g == 0)
 #pragma unroll
@@ -426,7 +431,7 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
                                c10::optional<torch::Tensor> cu, torch::Tensor ctx,
                                c10::optional<torch::Tensor> bseq,
                                c10::optional<torch::Tensor> boff, long rows, double scale,
-                               torch::Tensor sink) {
+                               c10::optional<torch::Tensor> sink, long VR, long window) {
   const int T = q.size(0), H = q.size(1), R = q.size(2), S = ctx.numel();
   const int P = cache.size(2), MP = bt.size(1);
   TORCH_CHECK(q.is_cuda() && q.dtype() == torch::kBFloat16 && q.is_contiguous());
@@ -435,7 +440,7 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
   TORCH_CHECK(cache.size(0) * P < (1L << 31), "cache slots");
   TORCH_CHECK(bt.is_contiguous() && bt.dtype() == torch::kInt32 && bt.size(0) == S &&
               ctx.dtype() == torch::kInt32);
-  TORCH_CHECK(sink.numel() == H && sink.dtype() == torch::kFloat32);
+  TORCH_CHECK(!sink || (sink->numel() == H && sink->dtype() == torch::kFloat32));
   TORCH_CHECK(rows == 16 || rows == 32);
   int blocks;
   if (cu) {
@@ -447,20 +452,22 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
     TORCH_CHECK(T == S);
     blocks = S * ((H + rows - 1) / rows);
   }
-  auto out = torch::empty_like(q);
+  auto out = torch::empty({T, H, VR}, q.options());
   if (T == 0 || blocks == 0) return out;
   // one workgroup per CU, or as many as its LDS holds
-  const int CS = std::max(1, std::min(LAT_SPLITS, (R > 256 ? 256 : 512) / blocks));
+  int CS = std::max(1, std::min(LAT_SPLITS, (R > 256 ? 256 : 512) / blocks));
+  // a split of its own for every tile that a window touches, at most
+  if (window > 0) CS = std::min<long>(CS, (window + LAT_KEYS - 2) / LAT_KEYS + 1);
   const long all = (long)T * H;
   torch::Tensor part, ml;
   if (CS > 1) {
-    part = torch::empty({CS, all, R}, q.options().dtype(torch::kFloat32));
+    part = torch::empty({CS, all, VR}, q.options().dtype(torch::kFloat32));
     ml = torch::empty({CS, all, 2}, q.options().dtype(torch::kFloat32));
   }
-#define LATENT(RR, MT)                                                                   \
+#define LATENT(RR, VV, MT)                                                               \
   do {                                                                                   \
-    auto kern = latent_attention_kernel<RR, MT>;                                         \
-    constexpr int lds = 2 * LAT_KEYS * RR * 2 + \
+    auto kern = latent_attention_kernel<RR, VV, MT>;                                     \
+    constexpr int lds = 2 * LAT_KEYS * (RR) * 2 + \
                         2 * 16 * MT * LAT_PSTRIDE * 2 + 4 * 16 * MT * 4 + 32;              \
     static const hipError_t once = hipFuncSetAttribute(                                  \
         (const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds);             \
@@ -469,41 +476,67 @@ torch::Tensor latent_attention(torch::Tensor q, torch::Tensor cache, torch::Tens
                        (const bf16_t*)q.data_ptr(), (const bf16_t*)cache.data_ptr(),     \
                        bt.data_ptr<int>(), MP, cu ? cu->data_ptr<int>() : nullptr,       \
                        ctx.data_ptr<int>(), cu ? bseq->data_ptr<int>() : nullptr,        \
-                       cu ? boff->data_ptr<int>() : nullptr, sink.data_ptr<float>(),     \
+                       cu ? boff->data_ptr<int>() : nullptr,                             \
+                       sink ? sink->data_ptr<float>() : nullptr,                         \
                        (bf16_t*)out.data_ptr(), CS > 1 ? part.data_ptr<float>() : nullptr, \
-                       CS > 1 ? ml.data_ptr<float>() : nullptr, H, P, all, (float)scale); \
+                       CS > 1 ? ml.data_ptr<float>() : nullptr, H, P, all, (float)scale,  \
+                       (int)window);                                                     \
   } while (0)
-#define LATENT_R(RR)                       \
-  if (R == RR) {                           \
-    if (rows == 16) LATENT(RR, 1);         \
-    else LATENT(RR, 2);                    \
+#define LATENT_W(RR, VV)                       \
+  if (R == RR && VR == VV) {                   \
+    if (rows == 16) LATENT(RR, VV, 1);         \
+    else LATENT(RR, VV, 2);                    \
   } else
+#define LATENT_R(VV) LATENT_W(VV, VV) LATENT_W((VV + 64), VV)
   LATENT_R(64) LATENT_R(128) LATENT_R(256) LATENT_R(384) LATENT_R(512)
-  TORCH_CHECK(false, "unsupported latent width ", R);
+  TORCH_CHECK(false, "unsupported latent widths ", R, ", ", VR);
 #undef LATENT_R
+#undef LATENT_W
 #undef LATENT
   if (CS > 1)
     hipLaunchKernelGGL(latent_combine_kernel, dim3(all), dim3(256), 0, CUR_STREAM,
                        part.data_ptr<float>(), ml.data_ptr<float>(), (bf16_t*)out.data_ptr(),
-                       all, CS, R);
+                       all, CS, (int)VR);
   HIP_CHECK_KERNEL();
   return out;
 }
 
 // ------------------------------------------------------------------ latents
 
-// norm of a token's latent in fp32 and its place in the cache: one wave per token
+template <typename T>
+struct FrontArgs {
+  const T* proj;         // [T, stride]
+  long stride;
+  int c0, rank;          // latents; c0 < 0: none
+  const float* weight;
+  int k0, key_at, rot;   // the rotated key part and its place in a row; rot 0: none
+  const float* cs;       // [positions, rot]
+  const int *pos, *slots;
+  T* cache;              // rows of C
+  int C;
+  int q0, q_rank;        // the queries' latent; q_rank 0: none
+  const float* q_weight;
+  T* cq;                 // [T, q_rank]
+  float eps;
+};
+
+// What latent attention does first, one wave per token and part: a token's latent is
+// normed in fp32 and goes to its place in the cache with the rotated key part behind
+// it; the queries' latent is normed.
 template <typename T, int V>
-__global__ __launch_bounds__(256) void latent_write_kernel(
-    const T* __restrict__ proj, long stride, int rank, const float* __restrict__ weight,
-    float eps, const int* __restrict__ slots, T* __restrict__ cache, int T_, int R) {
-  const int t = blockIdx.x * 4 + threadIdx.x / WAVE;
+__global__ __launch_bounds__(256) void latent_front_kernel(FrontArgs<T> a, int T_) {
+  const int w = blockIdx.x * 4 + threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  const int parts = (a.c0 >= 0) + (a.q_rank > 0);
+  const int t = w / parts;
   if (t >= T_) return;
-  const int lane = threadIdx.x % WAVE;
-  const int slot = slots[t];
+  const bool query = a.c0 < 0 || w % parts == 1;
+  const int slot = query ? 0 : a.slots[t];
   if (slot < 0) return;
-  const T* src = proj + t * stride;
-  T* dst = cache + (long)slot * R;
+  const int rank = query ? a.q_rank : a.rank;
+  const T* row = a.proj + t * a.stride;
+  const T* src = row + (query ? a.q0 : a.c0);
+  const float* weight = query ? a.q_weight : a.weight;
+  T* dst = query ? a.cq + (long)t * rank : a.cache + (long)slot * a.C;
   float ss = 0.f;
   for (int i = lane * V; i < rank; i += WAVE * V) {
     if constexpr (V == 4) {
@@ -515,38 +548,168 @@ __global__ __launch_bounds__(256) void latent_write_kernel(
       ss += v * v;
     }
   }
-  const float inv = rsqrtf(wave_sum(ss) / rank + eps);
-  for (int i = lane * V; i < R; i += WAVE * V) {
+  const float inv = rsqrtf(wave_sum(ss) / rank + a.eps);
+  const int width = query ? rank : a.C;
+  const float* cs = a.rot > 0 && !query ? a.cs + (long)a.pos[t] * a.rot : nullptr;
+  for (int i = lane * V; i < width; i += WAVE * V) {
+    const int k = i - a.key_at;  // within the key part
+    const bool key = cs && k >= 0 && k < a.rot;
     if constexpr (V == 4) {
       floatx4 y = {0.f, 0.f, 0.f, 0.f};
-      if (i < rank) y = ld4(src + i) * inv * ld4(weight + i);
+      if (i < rank) {
+        y = ld4(src + i) * inv * ld4(weight + i);
+      } else if (key) {
+        y = ld4(row + a.k0 + k);
+        float u0 = y[0], v0 = y[1], u1 = y[2], v1 = y[3];
+        turn_pair(u0, v0, cs[k / 2], cs[(a.rot + k) / 2]);
+        turn_pair(u1, v1, cs[k / 2 + 1], cs[(a.rot + k) / 2 + 1]);
+        y = floatx4{u0, v0, u1, v1};
+      }
       st4(dst + i, y);
     } else {
-      stf(dst + i, i < rank ? ldf(src + i) * inv * weight[i] : 0.f);
+      float y = 0.f;
+      if (i < rank) {
+        y = ldf(src + i) * inv * weight[i];
+      } else if (key) {
+        float u = ldf(row + a.k0 + (k & ~1)), v = ldf(row + a.k0 + (k | 1));
+        turn_pair(u, v, cs[k / 2], cs[a.rot / 2 + k / 2]);
+        y = k & 1 ? v : u;
+      }
+      stf(dst + i, y);
     }
   }
 }
 
-void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight, double eps,
-                  torch::Tensor slots, torch::Tensor cache) {
-  const int T_ = proj.size(0), R = cache.size(3);
-  TORCH_CHECK(proj.is_cuda() && proj.dim() == 2 && proj.stride(1) == 1 &&
-              col + rank <= proj.size(1) && rank <= R);
+// c0 < 0: the latents are another layer's; no cq: queries come without a latent
+void latent_front(torch::Tensor proj, long c0, long rank, c10::optional<torch::Tensor> weight,
+                  double eps, long k0, long key_at, c10::optional<torch::Tensor> cos_sin,
+                  c10::optional<torch::Tensor> pos, torch::Tensor slots, torch::Tensor cache,
+                  long q0, c10::optional<torch::Tensor> q_weight,
+                  c10::optional<torch::Tensor> cq) {
+  const int T_ = proj.size(0), C = cache.size(3);
+  TORCH_CHECK(proj.is_cuda() && proj.dim() == 2 && proj.stride(1) == 1);
   TORCH_CHECK(cache.is_contiguous() && cache.size(1) == 1 && cache.dtype() == proj.dtype());
-  TORCH_CHECK(weight.numel() == rank && weight.dtype() == torch::kFloat32);
-  TORCH_CHECK(slots.numel() == T_ && slots.dtype() == torch::kInt32);
-  if (T_ == 0) return;
+  auto norm = [&](const c10::optional<torch::Tensor>& w, long n) {
+    return w && w->numel() == n && w->dtype() == torch::kFloat32 && w->is_contiguous();
+  };
+  const bool own = c0 >= 0;
+  const int rot = own && cos_sin ? (int)cos_sin->size(1) : 0;
+  if (own) {
+    TORCH_CHECK(c0 + rank <= proj.size(1) && rank <= C && norm(weight, rank), "latents");
+    TORCH_CHECK(slots.numel() == T_ && slots.dtype() == torch::kInt32);
+  }
+  if (rot) {
+    TORCH_CHECK(cos_sin->dtype() == torch::kFloat32 && cos_sin->is_contiguous() &&
+                cos_sin->dim() == 2 && rot % 2 == 0 && key_at >= rank && key_at + rot <= C &&
+                k0 >= 0 && k0 + rot <= proj.size(1), "rotated key part");
+    TORCH_CHECK(pos && pos->numel() == T_ && pos->dtype() == torch::kInt32);
+  }
+  const int q_rank = cq ? (int)cq->size(1) : 0;
+  if (cq)
+    TORCH_CHECK(cq->is_contiguous() && cq->size(0) == T_ && cq->dtype() == proj.dtype() &&
+                q0 >= 0 && q0 + q_rank <= proj.size(1) && norm(q_weight, q_rank),
+                "queries' latent");
+  const long waves = (long)T_ * (own + (q_rank > 0));
+  if (waves == 0) return;
   DISPATCH_ELEM(proj.dtype() == torch::kBFloat16, {
+    FrontArgs<T> a = {};
+    a.proj = (const T*)proj.data_ptr();
+    a.stride = proj.stride(0);
+    a.c0 = own ? c0 : -1;
+    a.rank = rank;
+    if (own) a.weight = weight->data_ptr<float>();
+    a.key_at = rot ? key_at : C;
+    if (rot) {
+      a.k0 = k0;
+      a.rot = rot;
+      a.cs = cos_sin->data_ptr<float>();
+      a.pos = pos->data_ptr<int>();
+    }
+    if (own) a.slots = slots.data_ptr<int>();
+    a.cache = (T*)cache.data_ptr();
+    a.C = C;
+    if (q_rank) {
+      a.q0 = q0;
+      a.q_rank = q_rank;
+      a.q_weight = q_weight->data_ptr<float>();
+      a.cq = (T*)cq->data_ptr();
+    }
+    a.eps = eps;
     auto launch = [&](auto kern) {
-      hipLaunchKernelGGL(kern, dim3((T_ + 3) / 4), dim3(256), 0, CUR_STREAM,
-                         (const T*)proj.data_ptr() + col, proj.stride(0), (int)rank,
-                         weight.data_ptr<float>(), (float)eps, slots.data_ptr<int>(),
-                         (T*)cache.data_ptr(), T_, R);
+      hipLaunchKernelGGL(kern, dim3((waves + 3) / 4), dim3(256), 0, CUR_STREAM, a, T_);
     };
-    const bool vec = ((rank | col | proj.stride(0) | R) & 3) == 0 &&
+    const long units = proj.stride(0) | q_rank | (q_rank ? q0 : 0) |
+                       (own ? c0 | rank | C | a.key_at : 0) | (rot ? k0 | rot : 0);
+    const bool vec = (units & 3) == 0 &&
                      (reinterpret_cast<uintptr_t>(proj.data_ptr()) & 15) == 0;
-    if (vec) launch(latent_write_kernel<T, 4>);
-    else launch(latent_write_kernel<T, 1>);
+    if (vec) launch(latent_front_kernel<T, 4>);
+    else launch(latent_front_kernel<T, 1>);
+  });
+  HIP_CHECK_KERNEL();
+}
+
+// ------------------------------------------------------------- rotated dimensions
+
+// neighbouring pairs of x's first ``rot`` dimensions turn into out, zeros follow
+template <typename T>
+struct TurnHeads {
+  const T* x;
+  long xt, xh;
+  T* out;
+  long ot, oh;
+  const float* cs;  // [positions, rot]
+  const int* pos;
+  int rot, W;       // W: dimensions of out, even
+};
+
+template <typename T>
+DEVINL void turn_heads(const TurnHeads<T>& a, int t, int h, int pair) {
+  const int d = 2 * pair;
+  float u = 0.f, v = 0.f;
+  if (d < a.rot) {
+    const T* p = a.x + t * a.xt + h * a.xh + d;
+    const float* cs = a.cs + (long)a.pos[t] * a.rot + pair;
+    u = ldf(p);
+    v = ldf(p + 1);
+    turn_pair(u, v, cs[0], cs[a.rot / 2]);
+  }
+  T* p = a.out + t * a.ot + h * a.oh + d;
+  stf(p, u);
+  stf(p + 1, v);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void rotate_heads_kernel(TurnHeads<T> a, long total, int H) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int pairs = a.W / 2;
+  const long th = i / pairs;
+  turn_heads(a, (int)(th / H), (int)(th % H), (int)(i % pairs));
+}
+
+template <typename T>
+static TurnHeads<T> turn_args(const torch::Tensor& x, const torch::Tensor& pos,
+                              const torch::Tensor& cos_sin, const torch::Tensor& out) {
+  TORCH_CHECK(x.is_cuda() && x.dim() == 3 && out.dim() == 3 && out.dtype() == x.dtype() &&
+              out.size(0) == x.size(0) && out.size(1) == x.size(1) && x.stride(2) == 1 &&
+              out.stride(2) == 1, "rotated heads");
+  TORCH_CHECK(cos_sin.dtype() == torch::kFloat32 && cos_sin.is_contiguous() &&
+              cos_sin.dim() == 2 && cos_sin.size(1) % 2 == 0 && cos_sin.size(1) <= x.size(2) &&
+              cos_sin.size(1) <= out.size(2) && out.size(2) % 2 == 0, "rotation");
+  TORCH_CHECK(pos.numel() == x.size(0) && pos.dtype() == torch::kInt32 && pos.is_contiguous());
+  return {(const T*)x.data_ptr(), x.stride(0), x.stride(1), (T*)out.data_ptr(), out.stride(0),
+          out.stride(1), cos_sin.data_ptr<float>(), pos.data_ptr<int>(), (int)cos_sin.size(1),
+          (int)out.size(2)};
+}
+
+void rotate_heads(torch::Tensor x, torch::Tensor pos, torch::Tensor cos_sin,
+                  torch::Tensor out) {
+  DISPATCH_ELEM(x.dtype() == torch::kBFloat16, {
+    const TurnHeads<T> a = turn_args<T>(x, pos, cos_sin, out);
+    const long total = x.size(0) * x.size(1) * (a.W / 2);
+    if (total == 0) return;
+    hipLaunchKernelGGL((rotate_heads_kernel<T>), dim3((total + 255) / 256), dim3(256), 0,
+                       CUR_STREAM, a, total, (int)x.size(1));
   });
   HIP_CHECK_KERNEL();
 }
@@ -556,16 +719,22 @@ void latent_write(torch::Tensor proj, long col, long rank, torch::Tensor weight,
 // out[t, h, n] = sum_k x[t, h, k] w[h, n, k], times sigmoid(gate[t, h]). Waves
 // take 16 outputs each (KS 1) or split the contraction (KS 4); TT 16-token
 // tiles per workgroup. K and N are multiples of 32; STEPS: 32-wide steps of a
-// wave if known, all of whose loads are then in flight at once.
+// wave if known, all of whose loads are then in flight at once. With ``turn`` the last
+// block of a row of blocks turns the rotated dimensions of the same tokens and head.
 template <int TT, int KS, int STEPS>
 __global__ __launch_bounds__(256) void head_linear_kernel(
     const bf16_t* __restrict__ x, long xt, long xh, const bf16_t* __restrict__ w,
     const bf16_t* __restrict__ gate, long gt, bf16_t* __restrict__ out, long ot, long oh,
-    int T_, int N, int K) {
+    int T_, int N, int K, TurnHeads<bf16_t> turn) {
   __shared__ __attribute__((aligned(16))) float red[KS > 1 ? 4 : 1][TT][WAVE][4];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, g = lane >> 4;
   const int h = blockIdx.y, t0 = blockIdx.z * 16 * TT;
+  if (turn.x && blockIdx.x == gridDim.x - 1) {
+    const int pairs = turn.W / 2, n = min(16 * TT, T_ - t0) * pairs;
+    for (int i = threadIdx.x; i < n; i += 256) turn_heads(turn, t0 + i / pairs, h, i % pairs);
+    return;
+  }
   const int n0 = KS > 1 ? blockIdx.x * 16 : (blockIdx.x * 4 + wave) * 16;
   if (n0 >= N) return;  // KS 1 only: whole waves, no barrier follows
   const int steps = K / 32, lo = KS > 1 ? steps * wave / 4 : 0,
@@ -624,7 +793,9 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
 }
 
 void head_linear(torch::Tensor x, torch::Tensor w, c10::optional<torch::Tensor> gate,
-                 torch::Tensor out) {
+                 torch::Tensor out, c10::optional<torch::Tensor> turn_x,
+                 c10::optional<torch::Tensor> turn_pos, c10::optional<torch::Tensor> turn_cs,
+                 c10::optional<torch::Tensor> turn_out) {
   const int T_ = x.size(0), H = x.size(1), K = x.size(2), N = w.size(1);
   TORCH_CHECK(x.is_cuda() && x.dtype() == torch::kBFloat16 && w.dtype() == x.dtype() &&
               out.dtype() == x.dtype() && w.is_contiguous());
@@ -638,14 +809,21 @@ void head_linear(torch::Tensor x, torch::Tensor w, c10::optional<torch::Tensor> 
   if (gate)
     TORCH_CHECK(gate->size(0) == T_ && gate->size(1) == H && gate->stride(1) == 1 &&
                 gate->dtype() == x.dtype());
+  TurnHeads<bf16_t> turn = {};
+  if (turn_x) {
+    TORCH_CHECK(turn_pos && turn_cs && turn_out && turn_x->size(0) == T_ &&
+                turn_x->size(1) == H && turn_x->dtype() == x.dtype());
+    turn = turn_args<bf16_t>(*turn_x, *turn_pos, *turn_cs, *turn_out);
+  }
   if (T_ == 0) return;
   auto launch = [&](auto kern, int tt, int ks) {
-    const dim3 grid(ks > 1 ? N / 16 : (N + 63) / 64, H, (T_ + 16 * tt - 1) / (16 * tt));
+    const dim3 grid((ks > 1 ? N / 16 : (N + 63) / 64) + (turn.x ? 1 : 0), H,
+                    (T_ + 16 * tt - 1) / (16 * tt));
     hipLaunchKernelGGL(kern, grid, dim3(256), 0, CUR_STREAM, (const bf16_t*)x.data_ptr(),
                        x.stride(0), x.stride(1), (const bf16_t*)w.data_ptr(),
                        gate ? (const bf16_t*)gate->data_ptr() : nullptr,
                        gate ? gate->stride(0) : 0, (bf16_t*)out.data_ptr(), out.stride(0),
-                       out.stride(1), T_, N, K);
+                       out.stride(1), T_, N, K, turn);
   };
   // a long contraction for few tokens: split it over the waves
   const bool split = K >= 256 && T_ <= 64;

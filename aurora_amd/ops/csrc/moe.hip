@@ -1,9 +1,12 @@
-// Routed experts with a clamped GLU:
+// Routed experts with a clamped GLU,
 //     act = g sigmoid(alpha g) (u + shift),  g = min(gate, limit), u = clamp(up)
-// (without a limit, alpha 1 and shift 0: silu(gate) up), chosen by one of two routers:
+// (without a limit, alpha 1 and shift 0: silu(gate) up), or a squared relu, act =
+// max(up, 0)^2, chosen by one of three routers:
 //     z = W_r h + b (fp32), the ``top`` largest, softmax over the chosen;
 //     s = sigmoid(W_r h) (fp32), the ``top`` largest of s + c among the best groups of
-//     neighbours (by the sum of their two largest), weights s / sum s * scale
+//     neighbours (by the sum of their two largest), weights s / sum s * scale;
+//     s = softmax(W_r h) (fp32) over all, the ``top`` largest among the best groups (by
+//     their largest), weights s * scale
 // as route -> sort -> gathered up product with the activation in its epilogue
 // -> down product. Rows stay sorted by expert; the residual-norm kernel adds
 // each token's weighted rows, so no scatter pass exists. Nothing is read back
@@ -25,13 +28,16 @@ union mfrag {
 
 // ------------------------------------------------------------------- router
 
-// one workgroup per 16 tokens; its waves split the contraction. GROUPED: bias is the
-// sigmoid scores' correction
-template <typename T, bool MATRIX16, bool GROUPED>
+enum { CHOSEN_SOFTMAX = 0, GROUPED_SIGMOID = 1, GROUPED_SOFTMAX = 2 };
+
+// one workgroup per 16 tokens; its waves split the contraction. GROUPED_SIGMOID: bias
+// is the scores' correction; GROUPED_SOFTMAX: there is none
+template <typename T, bool MATRIX16, int ROUTER>
 __global__ __launch_bounds__(1024) void moe_route_kernel(
     const T* __restrict__ h, const T* __restrict__ router,
     const float* __restrict__ bias, int* __restrict__ sel, float* __restrict__ gate,
     int T_, int W, int E, int top, int groups, int keep, float scale) {
+  constexpr bool GROUPED = ROUTER != CHOSEN_SOFTMAX;
   extern __shared__ float logits[];  // [16][E]
   __shared__ float part[16][16][64];
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE;
@@ -97,9 +103,18 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(
         __threadfence_block();
         __builtin_amdgcn_wave_barrier();
       };
-      for (int e = lane; e < E; e += WAVE) {
-        score[e] = sigmoid_f(z[e]);
-        z[e] = score[e] + bias[e];
+      if constexpr (ROUTER == GROUPED_SIGMOID) {
+        for (int e = lane; e < E; e += WAVE) {
+          score[e] = sigmoid_f(z[e]);
+          z[e] = score[e] + bias[e];
+        }
+      } else {
+        float most = -INFINITY, all = 0.f;
+        for (int e = lane; e < E; e += WAVE) most = fmaxf(most, z[e]);
+        most = wave_max(most);
+        for (int e = lane; e < E; e += WAVE) all += score[e] = expf(z[e] - most);
+        all = wave_sum(all);
+        for (int e = lane; e < E; e += WAVE) score[e] /= all;
       }
       sync();
       for (int x = lane; x < groups; x += WAVE) {
@@ -109,7 +124,7 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(
           b = fmaxf(b, fminf(a, c));
           a = fmaxf(a, c);
         }
-        gs[x] = n > 1 ? a + b : a;
+        gs[x] = ROUTER == GROUPED_SIGMOID && n > 1 ? a + b : a;
       }
       sync();
       for (int x = lane; x < groups; x += WAVE) {
@@ -148,19 +163,22 @@ __global__ __launch_bounds__(1024) void moe_route_kernel(
     // each lane rescales what it wrote
     for (int n = lane; n < top; n += WAVE) {
       float& w = gate[(long)(t0 + t) * top + n];
-      w = GROUPED ? w / (sum + 1e-20f) * scale : w / sum;
+      w = ROUTER == GROUPED_SIGMOID ? w / (sum + 1e-20f) * scale
+          : ROUTER == GROUPED_SOFTMAX ? w * scale : w / sum;
     }
   }
 }
 
-template <bool GROUPED>
+template <int ROUTER>
 static std::vector<torch::Tensor> route(const torch::Tensor& h, const torch::Tensor& router,
-                                        const torch::Tensor& bias, long top, long groups,
-                                        long keep, double scale) {
+                                        const c10::optional<torch::Tensor>& bias, long top,
+                                        long groups, long keep, double scale) {
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.is_contiguous() &&
               router.is_contiguous() && router.dtype() == h.dtype());
   const long T_ = h.size(0), W = h.size(1), E = router.size(0);
-  TORCH_CHECK(router.size(1) == W && bias.numel() == E && bias.dtype() == torch::kFloat32);
+  TORCH_CHECK(router.size(1) == W);
+  TORCH_CHECK(ROUTER == GROUPED_SOFTMAX ? !bias : bias && bias->numel() == E &&
+              bias->dtype() == torch::kFloat32, "router bias");
   TORCH_CHECK(top >= 1 && top <= E && E <= 512, "1 <= top <= experts <= 512");
   auto sel = torch::empty({T_, top}, h.options().dtype(torch::kInt32));
   auto gate = torch::empty({T_, top}, h.options().dtype(torch::kFloat32));
@@ -169,13 +187,13 @@ static std::vector<torch::Tensor> route(const torch::Tensor& h, const torch::Ten
     auto launch = [&](auto kern) {
       hipLaunchKernelGGL(kern, dim3((T_ + 15) / 16), dim3(1024), 16 * E * 4, CUR_STREAM,
                          (const T*)h.data_ptr(), (const T*)router.data_ptr(),
-                         bias.data_ptr<float>(), sel.data_ptr<int>(),
+                         bias ? bias->data_ptr<float>() : nullptr, sel.data_ptr<int>(),
                          gate.data_ptr<float>(), (int)T_, (int)W, (int)E, (int)top,
                          (int)groups, (int)keep, (float)scale);
     };
     constexpr bool B16 = sizeof(T) == 2;
-    if (B16 && W % 8 == 0) launch(moe_route_kernel<T, B16, GROUPED>);
-    else launch(moe_route_kernel<T, false, GROUPED>);
+    if (B16 && W % 8 == 0) launch(moe_route_kernel<T, B16, ROUTER>);
+    else launch(moe_route_kernel<T, false, ROUTER>);
   });
   HIP_CHECK_KERNEL();
   return {sel, gate};
@@ -183,16 +201,18 @@ static std::vector<torch::Tensor> route(const torch::Tensor& h, const torch::Ten
 
 std::vector<torch::Tensor> moe_route(torch::Tensor h, torch::Tensor router,
                                      torch::Tensor bias, long top) {
-  return route<false>(h, router, bias, top, 1, 1, 1.0);
+  return route<CHOSEN_SOFTMAX>(h, router, bias, top, 1, 1, 1.0);
 }
 
+// sigmoid scores with a correction, softmax scores without
 std::vector<torch::Tensor> moe_route_grouped(torch::Tensor h, torch::Tensor router,
-                                             torch::Tensor correction, long top,
-                                             long groups, long keep, double scale) {
+                                             c10::optional<torch::Tensor> correction,
+                                             long top, long groups, long keep, double scale) {
   const long E = router.size(0);
   TORCH_CHECK(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups &&
               top <= keep * (E / groups), "expert groups");
-  return route<true>(h, router, correction, top, groups, keep, scale);
+  if (!correction) return route<GROUPED_SOFTMAX>(h, router, correction, top, groups, keep, scale);
+  return route<GROUPED_SIGMOID>(h, router, correction, top, groups, keep, scale);
 }
 
 // --------------------------------------------------------------------- sort
@@ -244,6 +264,9 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(
 
 // ------------------------------------------------------------ grouped product
 
+// what the product's epilogue does
+enum { NO_ACT = 0, GLU_ACT = 1, RELU2_ACT = 2 };
+
 struct GroupArgs {
   const void* x;       // rows [*, K]; row r of the sorted batch is x[gather[r]]
   const int* gather;   // null: x itself is sorted
@@ -262,8 +285,9 @@ DEVINL float clamped_glu(float g, float u, const GroupArgs& p) {
 
 // Any size and float32: 32 rows x 64 columns, 16 of K at a time, through LDS as
 // fp32 (GLU: 32 gate and the matching 32 up columns).
-template <typename T, bool GLU>
+template <typename T, int ACT>
 __global__ __launch_bounds__(256) void grouped_any_kernel(GroupArgs p) {
+  constexpr bool GLU = ACT == GLU_ACT;
   const int* tb = p.table + blockIdx.y * 3;
   const int e = tb[0];
   if (e < 0) return;
@@ -307,7 +331,8 @@ __global__ __launch_bounds__(256) void grouped_any_kernel(GroupArgs p) {
   for (int x = tid; x < 32 * BN; x += 256) {
     const int r = x / BN, c = x % BN;
     if (r >= cnt || n0 + c >= p.N) continue;
-    const float v = GLU ? clamped_glu(cs[r][c], cs[r][32 + c], p) : cs[r][c];
+    float v = GLU ? clamped_glu(cs[r][c], cs[r][32 + c], p) : cs[r][c];
+    if constexpr (ACT == RELU2_ACT) v = v > 0.f ? v * v : 0.f;
     stf((T*)p.y + (long)(row0 + r) * p.N + n0 + c, v);
   }
 }
@@ -319,8 +344,9 @@ __global__ __launch_bounds__(256) void grouped_any_kernel(GroupArgs p) {
 // outputs, so the activation is register to register.
 #define GK 64
 
-template <int TM, int TB, int NS, int NTHR, bool GLU>
+template <int TM, int TB, int NS, int NTHR, int ACT>
 __global__ __launch_bounds__(NTHR) void grouped_bf16_kernel(GroupArgs p) {
+  constexpr bool GLU = ACT == GLU_ACT;
   const int* tb = p.table + blockIdx.y * 3;
   const int e = tb[0];
   if (e < 0) return;
@@ -429,18 +455,19 @@ __global__ __launch_bounds__(NTHR) void grouped_bf16_kernel(GroupArgs p) {
       for (int n = 0; n < NO; ++n) {
         const int c = n0 + (GLU ? wn / 2 : wn) + n * 16 + i;
         if (c >= p.N) continue;
-        const float v = GLU ? clamped_glu(acc[m][n][r], acc[m][n + (GLU ? NO : 0)][r], p)
-                            : acc[m][n][r];
+        float v = GLU ? clamped_glu(acc[m][n][r], acc[m][n + (GLU ? NO : 0)][r], p)
+                      : acc[m][n][r];
+        if constexpr (ACT == RELU2_ACT) v = v > 0.f ? v * v : 0.f;
         y[(long)(row0 + row) * p.N + c] = f32_to_bf16(v);
       }
     }
 }
 
-template <int TM, int TB, int NS, int NTHR, bool GLU>
+template <int TM, int TB, int NS, int NTHR, int ACT>
 static void grouped_bf16(const GroupArgs& p, int tiles) {
-  constexpr int BN = GLU ? TB / 2 : TB;
+  constexpr int BN = ACT == GLU_ACT ? TB / 2 : TB;
   constexpr int lds = NS * (TM + TB) * GK * 2;
-  auto kern = grouped_bf16_kernel<TM, TB, NS, NTHR, GLU>;
+  auto kern = grouped_bf16_kernel<TM, TB, NS, NTHR, ACT>;
   if (lds > 64 * 1024) {
     static const hipError_t once = hipFuncSetAttribute(
         (const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, lds);
@@ -449,36 +476,38 @@ static void grouped_bf16(const GroupArgs& p, int tiles) {
   hipLaunchKernelGGL(kern, dim3((p.N + BN - 1) / BN, tiles), dim3(NTHR), lds, CUR_STREAM, p);
 }
 
-template <bool GLU>
+template <int ACT>
 static void grouped(const GroupArgs& p, bool bf16, int tiles, int TM, long busy) {
+  constexpr bool GLU = ACT == GLU_ACT;
   if (bf16 && p.K % GK == 0) {
     const long blocks = (p.N + (GLU ? 63 : 127)) / (GLU ? 64 : 128) * busy;
-    if (TM == 256) grouped_bf16<256, 256, 2, 512, GLU>(p, tiles);
-    else if (TM == 128) grouped_bf16<128, 128, 2, 256, GLU>(p, tiles);
-    else if (TM == 64) grouped_bf16<64, 128, 3, 256, GLU>(p, tiles);
+    if (TM == 256) grouped_bf16<256, 256, 2, 512, ACT>(p, tiles);
+    else if (TM == 128) grouped_bf16<128, 128, 2, 256, ACT>(p, tiles);
+    else if (TM == 64) grouped_bf16<64, 128, 3, 256, ACT>(p, tiles);
     // few rows: the weights' stream counts. Two workgroups per CU with four
     // stages each, or one with seven where there are not enough for two
-    else if (blocks >= 512) grouped_bf16<32, 128, 4, 256, GLU>(p, tiles);
-    else grouped_bf16<32, 128, 7, 256, GLU>(p, tiles);
+    else if (blocks >= 512) grouped_bf16<32, 128, 4, 256, ACT>(p, tiles);
+    else grouped_bf16<32, 128, 7, 256, ACT>(p, tiles);
     return;
   }
   TORCH_CHECK(TM == 32);
   const dim3 grid((p.N + (GLU ? 31 : 63)) / (GLU ? 32 : 64), tiles);
   if (bf16)
-    hipLaunchKernelGGL((grouped_any_kernel<bf16_t, GLU>), grid, dim3(256), 0, CUR_STREAM, p);
+    hipLaunchKernelGGL((grouped_any_kernel<bf16_t, ACT>), grid, dim3(256), 0, CUR_STREAM, p);
   else
-    hipLaunchKernelGGL((grouped_any_kernel<float, GLU>), grid, dim3(256), 0, CUR_STREAM, p);
+    hipLaunchKernelGGL((grouped_any_kernel<float, ACT>), grid, dim3(256), 0, CUR_STREAM, p);
 }
 
-std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
-                                           torch::Tensor w_gu, torch::Tensor w_dn,
-                                           double limit, double alpha, double shift) {
+template <int ACT>
+static std::vector<torch::Tensor> experts(const torch::Tensor& h, const torch::Tensor& sel,
+                                          const torch::Tensor& w_up, const torch::Tensor& w_dn,
+                                          double limit, double alpha, double shift) {
   TORCH_CHECK(h.is_cuda() && h.dim() == 2 && h.is_contiguous() && sel.is_contiguous() &&
               sel.dtype() == torch::kInt32 && sel.size(0) == h.size(0));
   const long T_ = h.size(0), W = h.size(1), top = sel.size(1), A = T_ * top;
-  const long E = w_gu.size(0), F = w_gu.size(1) / 2;
-  TORCH_CHECK(w_gu.is_contiguous() && w_dn.is_contiguous() && w_gu.dtype() == h.dtype() &&
-              w_dn.dtype() == h.dtype() && w_gu.size(2) == W && w_dn.size(0) == E &&
+  const long E = w_up.size(0), F = w_up.size(1) / (ACT == GLU_ACT ? 2 : 1);
+  TORCH_CHECK(w_up.is_contiguous() && w_dn.is_contiguous() && w_up.dtype() == h.dtype() &&
+              w_dn.dtype() == h.dtype() && w_up.size(2) == W && w_dn.size(0) == E &&
               w_dn.size(1) == W && w_dn.size(2) == F && E <= MAX_EXPERTS);
   auto i32 = h.options().dtype(torch::kInt32);
   auto y = torch::empty({A, W}, h.options()), place = torch::empty({T_, top}, i32);
@@ -487,7 +516,8 @@ std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
   // row tile: enough rows per weight read when experts are well filled
   const bool matrix = bf16 && W % GK == 0 && F % GK == 0;
   // and the large tile only where it leaves enough blocks for the chip
-  const bool large = A >= 512 * E && A / 256 * ((F + 127) / 128) >= 1024;
+  const long cols = ACT == GLU_ACT ? 128 : 256;
+  const bool large = A >= 512 * E && A / 256 * ((F + cols - 1) / cols) >= 1024;
   const int TM = !matrix || A < 48 * E ? 32 : A < 160 * E ? 64 : large ? 256 : 128;
   const int tiles = (int)(A / TM + std::min(E, A));
   auto token = torch::empty({A}, i32), table = torch::empty({tiles, 3}, i32);
@@ -495,17 +525,28 @@ std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
   hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, CUR_STREAM,
                      sel.data_ptr<int>(), (int)A, (int)E, (int)top, TM, tiles,
                      place.data_ptr<int>(), token.data_ptr<int>(), table.data_ptr<int>());
-  GroupArgs p = {h.data_ptr(), token.data_ptr<int>(), w_gu.data_ptr(), act.data_ptr(),
+  GroupArgs p = {h.data_ptr(), token.data_ptr<int>(), w_up.data_ptr(), act.data_ptr(),
                  table.data_ptr<int>(), (int)F, (int)W, (float)limit, (float)alpha,
                  (float)shift};
-  grouped<true>(p, bf16, tiles, TM, std::min(E, A));
+  grouped<ACT>(p, bf16, tiles, TM, std::min(E, A));
   p.x = act.data_ptr();
   p.gather = nullptr;
   p.w = w_dn.data_ptr();
   p.y = y.data_ptr();
   p.N = W;
   p.K = F;
-  grouped<false>(p, bf16, tiles, TM, std::min(E, A));
+  grouped<NO_ACT>(p, bf16, tiles, TM, std::min(E, A));
   HIP_CHECK_KERNEL();
   return {y, place};
+}
+
+std::vector<torch::Tensor> moe_clamped_glu(torch::Tensor h, torch::Tensor sel,
+                                           torch::Tensor w_gu, torch::Tensor w_dn,
+                                           double limit, double alpha, double shift) {
+  return experts<GLU_ACT>(h, sel, w_gu, w_dn, limit, alpha, shift);
+}
+
+std::vector<torch::Tensor> moe_relu2(torch::Tensor h, torch::Tensor sel, torch::Tensor w_up,
+                                     torch::Tensor w_dn) {
+  return experts<RELU2_ACT>(h, sel, w_up, w_dn, 0.0, 0.0, 0.0);
 }

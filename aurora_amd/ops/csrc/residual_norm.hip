@@ -4,7 +4,8 @@
 // also adds what came before: a sub-layer's output, scaled by its residual gate
 // if it has one, or the chosen experts' rows with their routing weights (so no
 // separate combine pass exists), and the vector that marks a pass of a repeated
-// span. In steps of single tokens it also adds the next mixer's input
+// span. What the sub-layer and the experts give together may be normed before it is
+// added. In steps of single tokens the kernel also adds the next sublayer's input
 // convolution to the result. One workgroup per row, the row lives in LDS
 // between the sum of squares and the scaling: x is read and written once,
 // everything else once.
@@ -37,14 +38,15 @@ struct ConvTail {
   T* out;          // [T, W]
 };
 
-// NTHR threads per row: 1024 where few wide rows would leave the chip waiting
-template <typename T, int V, int NTHR>
+// NTHR threads per row: 1024 where few wide rows would leave the chip waiting. POST:
+// the result is normed, times ``post``, before it is added
+template <typename T, int V, int NTHR, bool POST>
 __global__ __launch_bounds__(NTHR) void residual_rmsnorm_kernel(
     float* __restrict__ x, const float* __restrict__ weight,
     const T* __restrict__ delta, ResidualGate<T> rg, const T* __restrict__ y,
     const int* __restrict__ place, const float* __restrict__ gate, int top,
-    const float* __restrict__ step, T* __restrict__ out, ConvTail<T> cv, int W,
-    float eps, float offset) {
+    const float* __restrict__ post, const float* __restrict__ step, T* __restrict__ out,
+    ConvTail<T> cv, int W, float eps, float offset) {
   extern __shared__ __attribute__((aligned(16))) float row[];
   __shared__ float red[NTHR / WAVE];
   const long base = (long)blockIdx.x * W;
@@ -52,6 +54,40 @@ __global__ __launch_bounds__(NTHR) void residual_rmsnorm_kernel(
   const float* gt = gate + (long)blockIdx.x * top;
   const T* pre = rg.pre ? rg.pre + blockIdx.x * rg.stride : nullptr;
   float ss = 0.f;
+  if constexpr (POST) {
+    typedef __attribute__((ext_vector_type(V))) float vec;
+    auto loadf = [](const float* p) {
+      if constexpr (V == 4) return ld4(p);
+      else return vec(*p);
+    };
+    auto load = [](const T* p) {
+      if constexpr (V == 4) return ld4(p);
+      else return vec(ldf(p));
+    };
+    auto store = [](float* p, vec v) {
+      if constexpr (V == 4) st4(p, v);
+      else *p = v[0];
+    };
+    float rs = 0.f;
+    for (int i = threadIdx.x * V; i < W; i += NTHR * V) {
+      vec r = vec(0.f);
+      if (delta) r = load(delta + base + i);
+      if (y)
+        for (int j = 0; j < top; ++j) r += gt[j] * load(y + (long)pl[j] * W + i);
+      store(row + i, r);
+#pragma unroll
+      for (int j = 0; j < V; ++j) rs += r[j] * r[j];
+    }
+    const float rinv = rsqrtf(block_sum<NTHR / WAVE>(rs, red) / W + eps);
+    for (int i = threadIdx.x * V; i < W; i += NTHR * V) {  // what the thread wrote
+      vec v = loadf(x + base + i) + loadf(row + i) * rinv * loadf(post + i);
+      if (step) v += loadf(step + i);
+      store(row + i, v);
+      store(x + base + i, v);
+#pragma unroll
+      for (int j = 0; j < V; ++j) ss += v[j] * v[j];
+    }
+  } else
   for (int i = threadIdx.x * V; i < W; i += NTHR * V) {
     float v[V];
     if constexpr (V == 4) {
@@ -130,8 +166,8 @@ std::vector<torch::Tensor> residual_rmsnorm(
     torch::Tensor x, torch::Tensor weight, c10::optional<torch::Tensor> delta,
     c10::optional<torch::Tensor> gate_pre, c10::optional<torch::Tensor> gate_bias,
     c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> place,
-    c10::optional<torch::Tensor> gate, c10::optional<torch::Tensor> step,
-    c10::optional<torch::Tensor> conv_w, c10::optional<torch::Tensor> ring,
+    c10::optional<torch::Tensor> gate, c10::optional<torch::Tensor> post,
+    c10::optional<torch::Tensor> step, c10::optional<torch::Tensor> conv_w, c10::optional<torch::Tensor> ring,
     c10::optional<torch::Tensor> pos, c10::optional<torch::Tensor> slots, double eps,
     double offset, bool to_bf16) {
   TORCH_CHECK(x.is_cuda() && x.dim() == 2 && x.is_contiguous() &&
@@ -157,6 +193,9 @@ std::vector<torch::Tensor> residual_rmsnorm(
                 place->size(0) == T_ && place->sizes() == gate->sizes(), "expert rows");
     top = place->size(1);
   }
+  if (post)
+    TORCH_CHECK(post->numel() == W && post->dtype() == torch::kFloat32 &&
+                post->is_contiguous() && !gate_pre && (delta || y), "norm of the result");
   if (step) TORCH_CHECK(step->numel() == W && step->dtype() == torch::kFloat32);
   if (conv_w) {
     TORCH_CHECK(ring && pos && slots && conv_w->is_contiguous() && conv_w->size(1) == W &&
@@ -183,14 +222,21 @@ std::vector<torch::Tensor> residual_rmsnorm(
           weight.data_ptr<float>(), delta ? (const T*)delta->data_ptr() : nullptr, rg,
           y ? (const T*)y->data_ptr() : nullptr,
           y ? place->data_ptr<int>() : nullptr, y ? gate->data_ptr<float>() : nullptr,
-          top, step ? step->data_ptr<float>() : nullptr, (T*)out[0].data_ptr(), cv, W,
+          top, post ? post->data_ptr<float>() : nullptr, step ? step->data_ptr<float>() : nullptr, (T*)out[0].data_ptr(), cv, W,
           (float)eps, (float)offset);
     };
     const bool vec = W % 4 == 0 && (!gate_pre || (gate_pre->stride(0) % 4 == 0 &&
                      (reinterpret_cast<uintptr_t>(gate_pre->data_ptr()) & 15) == 0));
-    if (vec && T_ <= 256 && W > 1024) launch(residual_rmsnorm_kernel<T, 4, 1024>, 1024);
-    else if (vec) launch(residual_rmsnorm_kernel<T, 4, 256>, 256);
-    else launch(residual_rmsnorm_kernel<T, 1, 256>, 256);
+    const bool wide = vec && T_ <= 256 && W > 1024;
+    if (post) {
+      if (wide) launch(residual_rmsnorm_kernel<T, 4, 1024, true>, 1024);
+      else if (vec) launch(residual_rmsnorm_kernel<T, 4, 256, true>, 256);
+      else launch(residual_rmsnorm_kernel<T, 1, 256, true>, 256);
+    } else {
+      if (wide) launch(residual_rmsnorm_kernel<T, 4, 1024, false>, 1024);
+      else if (vec) launch(residual_rmsnorm_kernel<T, 4, 256, false>, 256);
+      else launch(residual_rmsnorm_kernel<T, 1, 256, false>, 256);
+    }
   });
   HIP_CHECK_KERNEL();
   return out;

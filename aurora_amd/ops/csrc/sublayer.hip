@@ -1,5 +1,5 @@
 // What surrounds the mixers of the layer-listed decoders: the embedding of
-// tokens and token pairs, the causal convolution added to a mixer's input, and
+// tokens and token pairs, the causal convolution added to a sublayer's input, and
 // the activations of the dense feed-forwards.
 //
 // The two kernels with a past keep it in state slots. Rows that read a sequence's
@@ -305,7 +305,7 @@ torch::Tensor xielu(torch::Tensor z, torch::Tensor act) {
   return out;
 }
 
-// ------------------------------------------------------------- gelu, silu GLU
+// ---------------------------------------------------- gelu, relu^2, silu GLU
 
 // f(a, b) of the columns i and i + F of z [T, stride] (GLU), or f(a, 0)
 template <typename T, int V, bool GLU, typename Fn>
@@ -332,6 +332,12 @@ __global__ __launch_bounds__(256) void activation_kernel(const T* __restrict__ z
 struct ExactGelu {
   DEVINL float operator()(float x, float) const {
     return 0.5f * x * (1.f + erff(x * 0.70710678f));
+  }
+};
+struct SquaredRelu {
+  DEVINL float operator()(float x, float) const {
+    const float y = fmaxf(x, 0.f);
+    return y * y;
   }
 };
 struct SiluTimes {
@@ -362,6 +368,8 @@ static torch::Tensor activate(const torch::Tensor& z, long F, Fn f) {
 }
 
 torch::Tensor gelu(torch::Tensor z) { return activate<false>(z, z.size(1), ExactGelu{}); }
+
+torch::Tensor relu2(torch::Tensor z) { return activate<false>(z, z.size(1), SquaredRelu{}); }
 
 // z [T, 2 F or more]: gate columns, then up columns
 torch::Tensor silu_glu(torch::Tensor z, long F) { return activate<true>(z, F, SiluTimes{}); }

@@ -1,7 +1,7 @@
 """Ops of the layer-listed decoders: biased window attention over paged KV,
-gated delta rules, retention, matrix memories, routed GLU experts, latent
-attention, normed attention heads, pair embeddings, the mixers' input
-convolution and the residual's norms.
+gated delta rules, retention, matrix memories, routed experts, latent
+attention, normed and convolved attention heads, pair embeddings, the
+sublayers' input convolution and the residual's norms.
 
 Same dispatch rule as the rest of the package: GPU tensors run the gfx950
 kernels (bf16, or float32 throughout) and fail loudly without the extension;
@@ -21,6 +21,10 @@ from . import torch_ref
 MATRIX_HEAD_DIMS = (64, 128)
 #: latent widths of the matrix-core latent attention kernel
 MATRIX_LATENT_WIDTHS = (64, 128, 256, 384, 512)
+#: columns of a cached latent row per 64 that hold the shared rotated key
+KEY_PART = 64
+#: widths of spelled-out latent-attention heads, rotated part included
+SPELLED_HEAD_DIMS = (64, 128, 192)
 #: widest latent of the kernel that serves float32 and everything else
 MAX_LATENT = 1024
 #: tokens per chunk of the recurrence kernels
@@ -138,6 +142,14 @@ def latent_head_width(dim: int) -> int:
     return next((w for w in MATRIX_HEAD_DIMS if w >= dim), -(-dim // 32) * 32)
 
 
+def latent_rotary_widths(dim: int, rot: int) -> Tuple[int, int, int]:
+    """Widths of a rotary latent-attention head: its unrotated and its rotated part
+    in the query rows, and the rotated key's columns in a cached row."""
+    d = -(-dim // 32) * 32
+    whole = next((w for w in SPELLED_HEAD_DIMS if w >= d + rot), d + -(-rot // 32) * 32)
+    return d, whole - d, -(-rot // KEY_PART) * KEY_PART
+
+
 @dataclass
 class LatentParams:
     """Sizes, projection columns and weights of latent attention; all head and
@@ -147,11 +159,46 @@ class LatentParams:
     vdim: int
     scale: float
     q0: int
-    g0: int
+    g0: Optional[int]   # None: no gate
     uk: torch.Tensor    # [heads, dim, R]
     uk_t: torch.Tensor  # [heads, R, dim]
     uv: torch.Tensor    # [heads, vdim, R]
-    sink: torch.Tensor  # [heads] fp32
+    sink: Optional[torch.Tensor]  # [heads] fp32
+    #: width of the rotated part behind a query's ``dim`` columns
+    tail: int = 0
+    cos_sin: Optional[torch.Tensor] = None  # [positions, rotated dims] fp32
+    window: int = 0
+
+
+@dataclass
+class LatentFrontParams:
+    """Columns of the input projection and weights of what latent attention does
+    first; ``c0`` is None where the latents are another layer's."""
+    c0: Optional[int]
+    rank: int
+    weight: Optional[torch.Tensor]    # [rank]
+    eps: float
+    k0: int = 0                       # the rotated key part
+    key_at: int = 0                   # its place in a cached row
+    cos_sin: Optional[torch.Tensor] = None
+    q0: int = 0                       # the queries' latent
+    q_rank: int = 0                   # 0: none
+    q_weight: Optional[torch.Tensor] = None
+
+
+@dataclass
+class ConvHeadsParams:
+    """Sizes, projection columns and weights of convolved, rotated attention heads."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    q0: int
+    k0: int
+    v0: int
+    conv_w: torch.Tensor   # [taps, heads*dim + kv_heads*(dim + vdim)], the last the present
+    turn: torch.Tensor     # [positions, rotated dims] fp32
+    value_turn: Optional[torch.Tensor] = None  # [positions, vdim] fp32
 
 
 @dataclass
@@ -223,22 +270,28 @@ class Segment:
             self._maps[("latent", heads)] = hit
         return hit
 
-    def latent_rows(self, cache):
-        """Every context token's latent, packed, and the place of sequence s's
-        token t among them as a table [s, t]; places are found once per step."""
+    def first_keys(self, window: int) -> List[int]:
+        """First key any row of each portion sees through a window (0: none)."""
+        return [max(0, c - (b - a) - window + 1) if window else 0 for a, b, c in
+                zip(self.cu_host, self.cu_host[1:], self.ctx_host)]
+
+    def latent_rows(self, cache, window: int = 0):
+        """Every visible context token's latent, packed, and the place of sequence
+        s's token t among them as a table [s, t] (0 where it is not visible); places
+        are found once per step."""
         P = cache.shape[2]
-        hit = self._maps.get("context")
+        hit = self._maps.get(("context", window))
         if hit is None:
             dev = cache.device
             table = torch.zeros(len(self.ctx_host), max(self.ctx_host), dtype=torch.int32)
             place, n = [], 0
-            for s, c in enumerate(self.ctx_host):
-                table[s, :c] = torch.arange(n, n + c, dtype=torch.int32)
-                n += c
-                t = torch.arange(c, device=dev)
+            for s, (lo, c) in enumerate(zip(self.first_keys(window), self.ctx_host)):
+                table[s, lo:c] = torch.arange(n, n + c - lo, dtype=torch.int32)
+                n += c - lo
+                t = torch.arange(lo, c, device=dev)
                 place.append(self.block_tables[s].long()[t // P] * P + t % P)
             hit = (torch.cat(place), table.to(dev))
-            self._maps["context"] = hit
+            self._maps["context", window] = hit
         return cache.view(-1, cache.shape[3]).index_select(0, hit[0]), hit[1]
 
 
@@ -248,32 +301,33 @@ def _hip(op: str):
 
 
 def residual_rmsnorm(x, weight, eps, delta=None, moe=None, step=None,
-                     offset: float = 1.0, dtype=None, gate=None):
+                     offset: float = 1.0, dtype=None, gate=None, post=None):
     if not x.is_cuda:
         return torch_ref.residual_rmsnorm(x, weight, eps, delta, moe, step, offset,
-                                          dtype, gate)
-    return _residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate)[0]
+                                          dtype, gate, post)
+    return _residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate, post)[0]
 
 
-def _residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate,
+def _residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate, post,
                       conv=(None, None, None, None)):
     y, place, share = moe if moe is not None else (None, None, None)
     pre, bias = gate if gate is not None else (None, None)
     return _hip("residual_rmsnorm").residual_rmsnorm(
-        x, weight, delta, pre, bias, y, place, share, step, *conv, float(eps),
+        x, weight, delta, pre, bias, y, place, share, post, step, *conv, float(eps),
         float(offset), dtype == torch.bfloat16)
 
 
 def residual_rmsnorm_conv(x, weight, eps, conv_w, ring, segments: List[Segment],
                           delta=None, moe=None, step=None, offset: float = 1.0,
-                          dtype=None, gate=None):
+                          dtype=None, gate=None, post=None):
     """``residual_rmsnorm`` and ``short_conv_add`` of its result: (h, h + conv).
     A step of single tokens does both in one kernel."""
     if x.is_cuda and len(segments) == 1 and segments[0].decode:
         seg = segments[0]
         return tuple(_residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype,
-                                       gate, (conv_w, ring, seg.starts, seg.state_slots)))
-    h = residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate)
+                                       gate, post,
+                                       (conv_w, ring, seg.starts, seg.state_slots)))
+    h = residual_rmsnorm(x, weight, eps, delta, moe, step, offset, dtype, gate, post)
     u = torch.empty_like(h)
     for seg in segments:
         short_conv_add(h, conv_w, ring, seg, u)
@@ -309,23 +363,55 @@ def embed_pairs(ids, table, scale, pairs, mul_prev: int, mul_cur: int, weight, e
 
 
 def latent_write(proj, col: int, rank: int, weight, eps, slots, cache):
+    latent_front(proj, LatentFrontParams(col, rank, weight, eps), None, slots, cache)
+
+
+def latent_front(proj, p: LatentFrontParams, positions, slots, cache):
+    """Normed latents and the rotated key part to the cache; returns the queries'
+    normed latent [T, q_rank], if there is one."""
+    turn = p.cos_sin if p.c0 is not None else None
     if not proj.is_cuda:
-        return torch_ref.latent_write(proj, col, rank, weight, eps, slots, cache)
-    _hip("latent_write").latent_write(proj, col, rank, weight, float(eps), slots, cache)
+        if p.c0 is not None:
+            torch_ref.latent_write(
+                proj, p.c0, p.rank, p.weight, p.eps, slots, cache, p.key_at, p.k0,
+                None if turn is None else turn[positions.long()])
+        return torch_ref.normed_columns(proj, p.q0, p.q_rank, p.q_weight, p.eps).to(
+            proj.dtype) if p.q_rank else None
+    cq = torch.empty(proj.shape[0], p.q_rank, dtype=proj.dtype, device=proj.device) \
+        if p.q_rank else None
+    _hip("latent_front").latent_front(
+        proj, -1 if p.c0 is None else p.c0, p.rank, p.weight, float(p.eps), p.k0, p.key_at,
+        turn, positions, slots, cache, p.q0, p.q_weight, cq)
+    return cq
 
 
-def head_linear(x, w, gate=None, out=None):
+def rotate_heads(x, positions, cos_sin, out):
+    """Neighbouring pairs of the first dimensions of x [T, H, n] turn by their row's
+    position, into out [T, H, w] (may be x), zero filled behind them."""
+    if not x.is_cuda:
+        n = cos_sin.shape[1]
+        y = torch_ref.rotate_pairs(x[..., :n].float(), cos_sin[positions.long()])
+        out[..., :n] = y.to(out.dtype)
+        out[..., n:] = 0
+        return
+    _hip("rotate_heads").rotate_heads(x, positions, cos_sin, out)
+
+
+def head_linear(x, w, gate=None, out=None, turn=None):
     """Per-head product: x [T, H, K] (rows may be strided), w [H, N, K] ->
-    [T, H, N], times sigmoid(gate [T, H]) if given."""
+    [T, H, N], times sigmoid(gate [T, H]) if given. ``turn``: the arguments of a
+    ``rotate_heads`` of equally many rows and heads to run in the same launch."""
     T, H, _ = x.shape
     if out is None:
         out = torch.empty(T, H, w.shape[1], dtype=x.dtype, device=x.device)
     if x.dtype == torch.bfloat16:
-        _hip("head_linear").head_linear(x, w, gate, out)
+        _hip("head_linear").head_linear(x, w, gate, out, *(turn or (None,) * 4))
         return out
     y = torch.bmm(x.transpose(0, 1).contiguous(), w.transpose(1, 2).contiguous())
     y = y.transpose(0, 1)
     out.copy_(y if gate is None else y * torch.sigmoid(gate).unsqueeze(-1))
+    if turn is not None:
+        rotate_heads(*turn)
     return out
 
 
@@ -334,58 +420,85 @@ EXPANDED_LIMIT = 1 << 31
 
 
 def expand_latents(seg: Segment, p: LatentParams, rank: int) -> bool:
-    """Whether it is faster to spell out every key and value of a prompt
+    """Whether it is faster to spell out every visible key and value of a prompt
     portion's context than to attend in the latents' own space, where a pair of
     tokens costs 2 rank instead of dim + vdim but a key costs nothing."""
-    if seg.decode or p.dim not in MATRIX_HEAD_DIMS or p.vdim not in MATRIX_HEAD_DIMS:
+    if seg.decode or p.vdim not in MATRIX_HEAD_DIMS or p.dim + p.tail not in (
+            SPELLED_HEAD_DIMS if p.tail else MATRIX_HEAD_DIMS):
+        return False
+    # the flash kernel comes with sink and gate, or with a rotated part and window
+    ends = p.sink is not None and p.g0 is not None
+    if not (p.sink is None and p.g0 is None if p.tail else ends and not p.window):
         return False
     width = p.dim + p.vdim
-    keys = sum(seg.ctx_host)
+    first = seg.first_keys(p.window)
+    keys = sum(seg.ctx_host) - sum(first)
     if keys * p.heads * width > EXPANDED_LIMIT:
         return False
-    pairs = sum((b - a) * (c - (b - a) / 2) for a, b, c in
-                zip(seg.cu_host, seg.cu_host[1:], seg.ctx_host))
+    seen = [(b - a) * (c - (b - a) / 2) for a, b, c in
+            zip(seg.cu_host, seg.cu_host[1:], seg.ctx_host)]
+    if p.window:
+        seen = [min(n, (b - a) * p.window) for n, a, b in
+                zip(seen, seg.cu_host, seg.cu_host[1:])]
+    pairs = sum(seen)
     rows = seg.cu_host[-1]
     # measured rates in flops per us: the latent kernel and the per-head products
     # around it; library products and the flash kernel, which also takes 0.4 us
     # per key and 10^3 of width at least
     latent = pairs * p.heads * 4 * rank / 6e8 + rows * p.heads * 2 * rank * width / 2e8
     product = keys * p.heads * 2 * rank * width / 6e8
-    flash = max(pairs * p.heads * 2 * width / 3e8, max(seg.ctx_host) * width * 4e-4)
+    longest = max(min(c, p.window + 256) if p.window else c for c in seg.ctx_host)
+    flash = max(pairs * p.heads * 2 * (width + p.tail) / 3e8, longest * width * 4e-4)
     return product + flash < latent
 
 
-def latent_attention(proj, p: LatentParams, cache, seg: Segment, out):
-    """One segment's rows of gated latent attention into out [rows, H * vdim]."""
+def latent_attention(proj, p: LatentParams, cache, seg: Segment, out, q=None,
+                     positions=None):
+    """One segment's rows of latent attention into out [rows, H * vdim]. Queries are
+    columns of ``proj``, or all rows' q [T, H, dim + tail], whose tails are still to
+    be rotated by ``positions``; they may be overwritten."""
     pr, o = proj[seg.rows], out[seg.rows]
-    T, H, R = pr.shape[0], p.heads, cache.shape[3]
-    q = pr[:, p.q0:p.q0 + H * p.dim].unflatten(1, (H, p.dim))
-    gate = pr[:, p.g0:p.g0 + H]
+    T, H, R, C = pr.shape[0], p.heads, p.uk.shape[2], cache.shape[3]
+    if q is None:
+        q = pr[:, p.q0:p.q0 + H * p.dim].unflatten(1, (H, p.dim))
+    else:
+        q, positions = q[seg.rows], positions[seg.rows]
+    gate = None if p.g0 is None else pr[:, p.g0:p.g0 + H]
+    plain, tail = q[..., :p.dim], q[..., p.dim:]
     if not proj.is_cuda:
+        if p.tail:
+            rotate_heads(tail, positions, p.cos_sin, tail)
         torch_ref.latent_attention(q, gate, p.uk, p.uv, p.sink, p.scale, cache,
                                    seg.block_tables, seg.cu_or_rows(T),
-                                   seg.context_lens, o)
+                                   seg.context_lens, o, p.window)
         return
     m = _hip("latent_attention")
-    matrix = proj.dtype == torch.bfloat16 and R in MATRIX_LATENT_WIDTHS
+    matrix = (proj.dtype == torch.bfloat16 and R in MATRIX_LATENT_WIDTHS
+              and C - R in (0, KEY_PART))
     if matrix and expand_latents(seg, p, R):
-        c, rows = seg.latent_rows(cache)
-        k = torch.nn.functional.linear(c, p.uk.flatten(0, 1))
-        v = torch.nn.functional.linear(c, p.uv.flatten(0, 1))
+        c, rows = seg.latent_rows(cache, p.window)
+        k = torch.nn.functional.linear(c[:, :R], p.uk.flatten(0, 1)).view(-1, H, 1, p.dim)
+        v = torch.nn.functional.linear(c[:, :R], p.uv.flatten(0, 1)).view(-1, H, 1, p.vdim)
         bseq, boff = seg.block_map(m.biased_prefill_rows(1))
-        m.sink_attention_prefill(q, k.view(-1, H, 1, p.dim), v.view(-1, H, 1, p.vdim),
-                                 rows, seg.cu, seg.context_lens, bseq, boff, p.scale,
-                                 p.sink, gate, o)
+        if p.tail:
+            rotate_heads(tail, positions, p.cos_sin, tail)
+            m.tailed_attention_prefill(q, k, v, c[:, R:], rows, seg.cu, seg.context_lens,
+                                       bseq, boff, p.scale, p.window, o)
+        else:
+            m.sink_attention_prefill(q, k, v, rows, seg.cu, seg.context_lens, bseq, boff,
+                                     p.scale, p.sink, gate, o)
         return
-    qa = head_linear(q, p.uk_t)
+    qa = torch.empty(T, H, C, dtype=q.dtype, device=q.device)
+    head_linear(plain, p.uk_t, out=qa[..., :R],
+                turn=(tail, positions, p.cos_sin, qa[..., R:]) if p.tail else None)
     if matrix:
         oc = m.latent_attention(qa, cache, seg.block_tables, seg.cu, seg.context_lens,
-                                *seg.latent_map(H), p.scale, p.sink)
+                                *seg.latent_map(H), p.scale, p.sink, R, p.window)
     else:
-        oc = torch.empty_like(qa)
+        oc = torch.empty(T, H, R, dtype=q.dtype, device=q.device)
         bseq, boff = (None, None) if seg.decode else seg.block_map(1)
         m.latent_attention_rows(qa, cache, seg.block_tables, seg.cu, seg.context_lens,
-                                bseq, boff, p.scale, p.sink, oc)
+                                bseq, boff, p.scale, p.sink, p.window, oc)
     head_linear(oc, p.uv, gate, o.unflatten(1, (H, p.vdim)))
 
 
@@ -416,17 +529,40 @@ def normed_qkv(proj, p: NormedHeadsParams, positions, slots, k_cache, v_cache):
         p.dim, p.vdim)
 
 
+def conv_qkv(proj, p: ConvHeadsParams, kv_slots, ring, segments: List[Segment], k_cache,
+             v_cache):
+    """Convolved and rotated queries [T, heads, DK]; keys and values go to the cache,
+    the last projections to the ring."""
+    q = torch.empty(proj.shape[0], p.heads, k_cache.shape[3], dtype=proj.dtype,
+                    device=proj.device)
+    for seg in segments:
+        pr, qs, ks = proj[seg.rows], q[seg.rows], kv_slots[seg.rows]
+        if not proj.is_cuda:
+            torch_ref.conv_qkv(pr, p, ks, ring, seg.cu_or_rows(pr.shape[0]), seg.starts,
+                               seg.state_slots, k_cache, v_cache, qs)
+            continue
+        m = _hip("conv_qkv")
+        bseq, boff = (None, None) if seg.decode else seg.block_map(m.conv_qkv_rows())
+        m.conv_qkv(pr, p.q0, p.k0, p.v0, p.conv_w, p.turn, p.value_turn, ring, ks, seg.cu,
+                   bseq, boff, seg.starts, seg.state_slots, k_cache, v_cache, qs, p.dim,
+                   p.vdim)
+    return q
+
+
 def biased_attention(q, k_cache, v_cache, seg: Segment, scale, window, slopes,
-                     out, col, vdim, out_scale, log_rate=None, sink=None):
-    """Attention of one segment's rows into out[rows, col:col+heads*vdim]."""
+                     out, col, vdim, out_scale, log_rate=None, sink=None, chunk: int = 0,
+                     turn=None, gate=None):
+    """Attention of one segment's rows into out[rows, col:col+heads*vdim]; ``turn``
+    and ``gate`` (all rows') act on the result and come without slopes."""
     qs, os_ = q[seg.rows], out[seg.rows]
-    extra = (scale, window, slopes, log_rate, sink, os_, col, vdim, out_scale)
+    gs = None if gate is None else gate[seg.rows]
     if not q.is_cuda:
         torch_ref.biased_attention_paged(
             qs, k_cache, v_cache, seg.block_tables, seg.cu_or_rows(qs.shape[0]),
             seg.context_lens, scale, window, slopes, os_, col, vdim, out_scale,
-            log_rate, sink)
+            log_rate, sink, chunk, turn, gs)
         return
+    extra = (scale, window, chunk, slopes, log_rate, sink, turn, gs, os_, col, vdim, out_scale)
     m = _hip("biased_attention")
     matrix = (q.dtype == torch.bfloat16 and q.shape[2] in MATRIX_HEAD_DIMS
               and v_cache.shape[3] in MATRIX_HEAD_DIMS)
@@ -531,11 +667,26 @@ def moe_grouped_glu(h, router, correction, top: int, groups: int, keep: int, sca
                     w_gate_up, w_down):
     """Plain GLU experts chosen by corrected sigmoid scores among the best groups;
     (y, place, weights) for ``output_norm``."""
-    route = torch_ref.moe_route_grouped if not h.is_cuda else \
-        _hip("moe_route_grouped").moe_route_grouped
-    sel, weights = route(h, router, correction, top, groups, keep, float(scale))
+    if not h.is_cuda:
+        sel, weights = torch_ref.moe_route_grouped(h, router, correction, top, groups, keep,
+                                                   float(scale))
+    else:
+        sel, weights = _hip("moe_route_grouped").moe_route_grouped(
+            h, router, correction, top, groups, keep, float(scale))
     y, place = expert_rows(h, sel, w_gate_up, w_down, float("inf"), 1.0, 0.0)
     return y, place, weights
+
+
+def moe_softmax_relu2(h, router, top: int, groups: int, keep: int, scale: float, w_up,
+                      w_down):
+    """Squared-relu experts chosen and weighed by a softmax over all of them, among
+    the groups of the best; (y, place, weights) for the next norm."""
+    if not h.is_cuda:
+        sel, weights = torch_ref.moe_route_softmax(h, router, top, groups, keep, scale)
+        return *torch_ref.moe_relu2(h, sel, w_up, w_down), weights
+    m = _hip("moe_relu2")
+    sel, weights = m.moe_route_grouped(h, router, None, top, groups, keep, float(scale))
+    return *m.moe_relu2(h, sel, w_up, w_down), weights
 
 
 def expert_rows(h, sel, w_gate_up, w_down, limit: float, alpha: float, shift: float):
@@ -562,6 +713,10 @@ def output_norm(src, x, weight, bias, eps, delta=None, gate=None, moe=None, dept
 def gelu(z):
     """Rows of ``z`` may be strided."""
     return torch_ref.gelu(z) if not z.is_cuda else _hip("gelu").gelu(z)
+
+
+def relu2(z):
+    return torch_ref.relu2(z) if not z.is_cuda else _hip("relu2").relu2(z)
 
 
 def silu_glu(z, ff: int):

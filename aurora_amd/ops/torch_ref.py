@@ -15,6 +15,7 @@ KV cache layout (chosen for the MI355X decode kernel's streaming reads):
 """
 from __future__ import annotations
 
+import math
 from typing import Optional, Tuple
 
 import torch
@@ -46,6 +47,37 @@ def rope_cos_sin_cache(
     freqs = torch.outer(t, inv_freq)  # [max_pos, half]
     cache = torch.cat([freqs.cos(), freqs.sin()], dim=-1).to(dtype)
     return cache
+
+
+def rotation_table(dims: int, max_pos: int, base: float, yarn=None) -> torch.Tensor:
+    """[max_pos, dims] fp32: the cosines, then the sines of every pair's angle. With
+    ``yarn`` (factor, original, fast, slow) the slow pairs turn ``factor`` times slower,
+    those between the two limits in part, and all entries grow by 0.1 ln(factor) + 1."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    freq = base ** (-2.0 * i / dims)
+    grow = 1.0
+    if yarn is not None:
+        lo, hi = (dims * math.log(yarn.original / (2 * math.pi * t)) / (2 * math.log(base))
+                  for t in (yarn.fast, yarn.slow))
+        lo, hi = max(math.floor(lo), 0), min(math.ceil(hi), dims - 1)
+        ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0, 1)
+        freq = freq / yarn.factor * ramp + freq * (1 - ramp)
+        grow += 0.1 * math.log(yarn.factor)
+    a = torch.outer(torch.arange(max_pos, dtype=torch.float64), freq)
+    return (torch.cat([a.cos(), a.sin()], -1) * grow).float()
+
+
+def rotate_pairs(x, cos_sin, back: bool = False):
+    """x [T, H, d] fp32, cos_sin [T, n]: the first n dimensions turn in neighbouring
+    pairs, or ``back``."""
+    n = cos_sin.shape[1]
+    c, s = cos_sin[:, None, :n // 2], cos_sin[:, None, n // 2:]
+    if back:
+        s = -s
+    u, v = x[..., 0:n:2], x[..., 1:n:2]
+    y = x.clone()
+    y[..., 0:n:2], y[..., 1:n:2] = u * c - v * s, v * c + u * s
+    return y
 
 
 def rope_apply(
@@ -254,16 +286,21 @@ def softmax_sample(
 # ---- layer-listed decoders: biased attention, recurrences, routed GLU --------
 
 def residual_rmsnorm(x, weight, eps, delta=None, moe=None, step=None,
-                     offset: float = 1.0, dtype=None, gate=None):
+                     offset: float = 1.0, dtype=None, gate=None, post=None):
     """x (fp32, updated in place) += delta (times the sigmoid of ``gate`` =
-    (pre-activation, bias), if given), or the routed experts' weighted sum,
-    then += step; returns rms(x) * (offset + weight) in ``dtype``."""
+    (pre-activation, bias), if given) and the routed experts' weighted sum, with
+    ``post`` both together normed and times it, then += step; returns rms(x) *
+    (offset + weight) in ``dtype``."""
+    r = torch.zeros_like(x)
     if delta is not None:
         y = delta.float()
-        x += y if gate is None else y * torch.sigmoid(gate[0].float() + gate[1])
+        r += y if gate is None else y * torch.sigmoid(gate[0].float() + gate[1])
     if moe is not None:
         y, place, weights = moe
-        x += (y.float()[place.long()] * weights.unsqueeze(-1)).sum(1)
+        r += (y.float()[place.long()] * weights.unsqueeze(-1)).sum(1)
+    if post is not None:
+        r *= torch.rsqrt(r.pow(2).mean(-1, keepdim=True) + eps) * post
+    x += r
     if step is not None:
         x += step.float()
     inv = torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
@@ -297,12 +334,15 @@ def _paged_rows(cache, pages, L):
 
 def biased_attention_paged(q, k_cache, v_cache, block_tables, cu_seqlens_q,
                            context_lens, scale, window, slopes, out, col, vdim,
-                           out_scale, log_rate=None, sink=None):
+                           out_scale, log_rate=None, sink=None, chunk=0, turn=None,
+                           gate=None):
     """Causal paged attention with a window and a distance penalty slope_h *
     (i - j), or with ``log_rate`` slope_h * ln(1 + rate_h (i - j)), and with
-    ``sink`` one more term e^sink_h of the denominator; writes
-    out[:, col : col + heads * vdim] times out_scale. Decode is the case of one
-    query per sequence."""
+    ``sink`` one more term e^sink_h of the denominator; with ``chunk`` only keys of
+    the query's chunk of positions are seen. ``turn`` [positions, vdim] rotates every
+    head's result back by the query's position, ``gate`` [T, heads * vdim] multiplies
+    it by a sigmoid; writes out[:, col : col + heads * vdim] times out_scale. Decode
+    is the case of one query per sequence."""
     T, Hq, _ = q.shape
     P = k_cache.shape[2]
     g = Hq // k_cache.shape[1]
@@ -315,19 +355,28 @@ def biased_attention_paged(q, k_cache, v_cache, block_tables, cu_seqlens_q,
         ks = _paged_rows(k_cache, pages, L).repeat_interleave(g, 0)
         vs = _paged_rows(v_cache, pages, L).repeat_interleave(g, 0)[..., :vdim]
         att = torch.einsum("qhd,hkd->hqk", q[a:b].float(), ks) * scale
-        dist = (torch.arange(L - (b - a), L, device=q.device).unsqueeze(1)
-                - torch.arange(L, device=q.device).unsqueeze(0))
-        far = dist.clamp(min=0) if log_rate is None else \
-            torch.log(1 + log_rate.view(-1, 1, 1) * dist.clamp(min=0))
-        att = att - slopes.view(-1, 1, 1) * far
+        at = torch.arange(L - (b - a), L, device=q.device).unsqueeze(1)
+        keys = torch.arange(L, device=q.device).unsqueeze(0)
+        dist = at - keys
+        if slopes is not None:
+            far = dist.clamp(min=0) if log_rate is None else \
+                torch.log(1 + log_rate.view(-1, 1, 1) * dist.clamp(min=0))
+            att = att - slopes.view(-1, 1, 1) * far
         hidden = dist < 0
         if window:
             hidden = hidden | (dist >= window)
+        if chunk:
+            hidden = hidden | (at // chunk != keys // chunk)
         att.masked_fill_(hidden, float("-inf"))
         if sink is not None:
             att = torch.cat([att, sink.view(-1, 1, 1).expand(Hq, b - a, 1)], -1)
         o = torch.einsum("hqk,hkd->qhd", att.softmax(-1)[..., :L], vs) * out_scale
-        out[a:b, col:col + Hq * vdim] = o.reshape(b - a, -1).to(out.dtype)
+        if turn is not None:
+            o = rotate_pairs(o, turn[L - (b - a):L], back=True)
+        o = o.reshape(b - a, -1)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[a:b].float())
+        out[a:b, col:col + Hq * vdim] = o.to(out.dtype)
 
 
 def _l2_unit(x):
@@ -542,38 +591,56 @@ def short_conv_add(h, w, ring, cu, starts, slots, out):
         out[a:b] = y.to(out.dtype)
 
 
-def latent_write(proj, col, rank, weight, eps, slots, cache):
-    """Normed latent of every token into the paged cache [pages, 1, P, R],
-    zero filled past ``rank``."""
-    c = proj[:, col:col + rank].float()
-    c = c * torch.rsqrt(c.pow(2).mean(-1, keepdim=True) + eps) * weight
-    P = cache.shape[2]
+def normed_columns(proj, col, width, weight, eps):
+    x = proj[:, col:col + width].float()
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * weight
+
+
+def latent_write(proj, col, rank, weight, eps, slots, cache, at=None, key_col=None,
+                 cos_sin=None):
+    """Normed latent of every token into the paged cache [pages, 1, P, R], zero
+    filled past ``rank``; with ``cos_sin`` [T, n] the rotated columns from key_col on
+    from ``at`` on."""
+    c = normed_columns(proj, col, rank, weight, eps)
+    P, R = cache.shape[2:]
+    rows = torch.nn.functional.pad(c, (0, R - rank))
+    if cos_sin is not None:
+        n = cos_sin.shape[1]
+        k = proj[:, None, key_col:key_col + n].float()
+        rows[:, at:at + n] = rotate_pairs(k, cos_sin)[:, 0]
     ok = slots >= 0
-    at = slots[ok].long()
-    cache[at // P, 0, at % P] = torch.nn.functional.pad(
-        c, (0, cache.shape[3] - rank)).to(cache.dtype)[ok]
+    to = slots[ok].long()
+    cache[to // P, 0, to % P] = rows.to(cache.dtype)[ok]
 
 
-def latent_attention(q, gate, uk, uv, sink, scale, cache, block_tables, cu, ctx, out):
-    """q [T, H, D], gate [T, H] pre-activations, uk [H, D, R], uv [H, E, R]:
+def latent_attention(q, gate, uk, uv, sink, scale, cache, block_tables, cu, ctx, out,
+                     window=0):
+    """q [T, H, D + n], gate [T, H] pre-activations or None, uk [H, D, R], uv [H, E, R]:
     causal attention of every head to keys uk c and values uv c of the cached
-    latents c, the sink in the denominator, times sigmoid(gate) -> out [T, H*E]."""
-    H = q.shape[1]
+    latents c, the sink, if any, in the denominator, times sigmoid(gate) -> out [T,
+    H*E]. The cache's columns from R on are more dimensions of every head's key; where
+    their number is not n, the surplus is zeros."""
+    H, D, R = uk.shape
     P = cache.shape[2]
+    n = min(q.shape[2] - D, cache.shape[3] - R)
+    q = q[..., :D + n]
     for s in range(cu.numel() - 1):
         a, b, L = int(cu[s]), int(cu[s + 1]), int(ctx[s])
         if a == b:
             continue
         c = _paged_rows(cache, block_tables[s, :(L + P - 1) // P].long(), L)[0]
-        k = torch.einsum("hdr,kr->hkd", uk.float(), c)
-        v = torch.einsum("her,kr->hke", uv.float(), c)
+        k = torch.einsum("hdr,kr->hkd", uk.float(), c[:, :R])
+        v = torch.einsum("her,kr->hke", uv.float(), c[:, :R])
+        k = torch.cat([k, c[:, R:R + n].expand(H, -1, -1)], -1)
         att = torch.einsum("qhd,hkd->hqk", q[a:b].float(), k) * scale
-        later = (torch.arange(L).unsqueeze(0)
-                 > torch.arange(L - (b - a), L).unsqueeze(1))
-        att.masked_fill_(later, float("-inf"))
-        att = torch.cat([att, sink.view(H, 1, 1).expand(H, b - a, 1)], -1)
-        o = torch.einsum("hqk,hke->qhe", att.softmax(-1)[..., :-1], v)
-        o = o * torch.sigmoid(gate[a:b].float()).unsqueeze(-1)
+        dist = torch.arange(L - (b - a), L).unsqueeze(1) - torch.arange(L).unsqueeze(0)
+        hidden = (dist < 0) | (dist >= window) if window else dist < 0
+        att.masked_fill_(hidden, float("-inf"))
+        if sink is not None:
+            att = torch.cat([att, sink.view(H, 1, 1).expand(H, b - a, 1)], -1)
+        o = torch.einsum("hqk,hke->qhe", att.softmax(-1)[..., :L], v)
+        if gate is not None:
+            o = o * torch.sigmoid(gate[a:b].float()).unsqueeze(-1)
         out[a:b] = o.reshape(b - a, -1).to(out.dtype)
 
 
@@ -681,3 +748,72 @@ def moe_route_grouped(h, router, correction, top: int, groups: int, keep: int, s
     sel = choice.topk(top, dim=-1).indices
     w = s.gather(1, sel)
     return sel.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
+
+
+# ---- layer-listed decoders: convolved attention heads, softmax routing, relu^2
+
+def conv_qkv(proj, p, kv_slots, ring, cu, starts, slots, k_cache, v_cache, q):
+    """Columns of a fused projection through the causal convolution; then queries and
+    keys turn in their first dimensions and values, with ``p.value_turn``, in all;
+    queries to q [T, heads, DK], keys and values to the paged cache, zero filled. The
+    ring [slots, taps - 1, C] holds position s's projections at s mod (taps - 1)."""
+    H, G, d, e = p.heads, p.kv_heads, p.dim, p.vdim
+    taps, C = p.conv_w.shape
+    past = taps - 1
+    for s in range(cu.numel() - 1):
+        a, b, start, slot = int(cu[s]), int(cu[s + 1]), int(starts[s]), int(slots[s])
+        n = b - a
+        if n == 0:
+            continue
+        x = torch.cat([proj[a:b, c:c + w] for c, w in
+                       ((p.q0, H * d), (p.k0, G * d), (p.v0, G * e))], 1)
+        full = torch.zeros(past + n, C)
+        full[past:] = x.float()
+        if slot >= 0:
+            for j in range(1, past + 1):
+                if start - j >= 0:
+                    full[past - j] = ring[slot, (start - j) % past].float()
+            for t in range(max(0, n - past), n):
+                ring[slot, (start + t) % past] = x[t].to(ring.dtype)
+        y = sum(full[j:j + n] * p.conv_w[j] for j in range(taps))
+        turn = p.turn[start:start + n]
+        yq = rotate_pairs(y[:, :H * d].reshape(n, H, d), turn)
+        yk = rotate_pairs(y[:, H * d:(H + G) * d].reshape(n, G, d), turn)
+        yv = y[:, (H + G) * d:].reshape(n, G, e)
+        if p.value_turn is not None:
+            yv = rotate_pairs(yv, p.value_turn[start:start + n])
+        place = lambda t, w: torch.nn.functional.pad(  # noqa: E731
+            t, (0, w - t.shape[2])).to(proj.dtype)
+        q[a:b] = place(yq, q.shape[2])
+        kv_cache_write(place(yk, k_cache.shape[3]), place(yv, v_cache.shape[3]), k_cache,
+                       v_cache, kv_slots[a:b])
+
+
+def relu2(z):
+    return z.float().clamp(min=0).pow(2).to(z.dtype)
+
+
+def moe_route_softmax(h, router, top: int, groups: int, keep: int, scale: float):
+    """The ``top`` best experts among the ``keep`` groups with the largest scores,
+    a softmax over all experts -> (ids [T, top] int32, chosen scores times scale)."""
+    z = h.float() @ router.float().t()
+    T, E = z.shape
+    per = z.view(T, groups, E // groups)
+    best = per.amax(-1).topk(keep, dim=-1).indices
+    closed = torch.ones(T, groups, dtype=torch.bool).scatter_(1, best, False)
+    sel = per.masked_fill(closed.unsqueeze(-1), float("-inf")).view(T, E).topk(top, dim=-1).indices
+    return sel.to(torch.int32), z.softmax(-1).gather(1, sel) * scale
+
+
+def moe_relu2(h, sel, w_up, w_down):
+    """Every chosen expert's output, unweighted, as ``moe_clamped_glu`` gives it."""
+    T, top = sel.shape
+    y = h.new_empty(T * top, h.shape[1])
+    flat = sel.reshape(-1).long()
+    tok = torch.arange(T * top) // top
+    for e in range(w_down.shape[0]):
+        rows = (flat == e).nonzero().flatten()
+        if rows.numel():
+            a = relu2((h[tok[rows]].float() @ w_up[e].float().t())).to(h.dtype)
+            y[rows] = (a.float() @ w_down[e].float().t()).to(h.dtype)
+    return y, torch.arange(T * top, dtype=torch.int32).view(T, top)

@@ -18,7 +18,7 @@ EXTENSIONS = {
     "_hip_ops": ["bindings.cpp", "elementwise.hip", "attention_decode.hip",
                  "attention_prefill.hip", "skinny_gemm.hip", "residual_norm.hip",
                  "attention_rows.hip", "recurrence.hip", "moe.hip", "sublayer.hip",
-                 "latent_attention.hip", "output_norm.hip"],
+                 "latent_attention.hip", "output_norm.hip", "conv_heads.hip"],
     # sentence encoder, vector search, one-shot all-reduce
     "_hip_aux": ["bindings_aux.cpp", "encoder.hip", "allreduce.hip"],
 }
