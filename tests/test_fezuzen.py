@@ -1,0 +1,974 @@
+"""The Fezuzen decoder through the engine against the plain oracle.
+
+Every model here is written as a checkpoint folder from its own small
+configuration and random weights, and loaded the way a user loads one. The CPU
+runs check the engine (caches, state slots, batches, schedules); the ``gpu`` runs
+check the same through the kernels, in float32 at a tight tolerance and in bf16
+at a loose one.
+"""
+import json
+import math
+import os
+import subprocess
+import sys
+
+import pytest
+import torch
+from safetensors.torch import save_file
+
+import decoder_rig
+import fezuzen_oracle as oracle
+from aurora_amd import ops
+from aurora_amd.engine.engine import EngineConfig, LLMEngine
+from aurora_amd.engine.replay import TraceReplayer
+from aurora_amd.engine.sampling_params import SamplingParams
+from aurora_amd.models.config import get_spec, spec_from_checkpoint
+from aurora_amd.ops import sequence, torch_ref
+
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+D64 = torch.float64
+
+
+# ----------------------------------------------------------- small checkpoints
+
+def latent(heads, dim, rot, vdim, rank, q_rank, window, base=1e4, scale=None, yarn=None,
+           kv_from=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank,
+         "q_rank": q_rank, "scale": (dim + rot) ** -0.5 if scale is None else scale,
+         "mask": {"size": window}, "rot": {"base": base, "dims": rot}}
+    if yarn is not None:
+        m["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), yarn))
+    return "latent_attention", m if kv_from is None else {**m, "kv_from": kv_from}
+
+
+def attention(heads, kv, dim, vdim, rot, conv, chunk, base=1e4, scale=None):
+    return "attention", {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv,
+                         "scale": dim ** -0.5 if scale is None else scale,
+                         "mask": {"size": chunk}, "rot": {"base": base, "dims": rot}}
+
+
+def moe(experts, top, groups, keep, ff, shared):
+    f = {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": shared},
+         "router": {"experts": experts, "top": top,
+                    "groups": {"count": groups, "keep": keep}}}
+    if not shared:
+        del f["shared"]
+    if groups == 1:
+        del f["router"]["groups"]
+    return f
+
+
+def config(name):
+    """Unlike models. ``plain``: even sizes, every kind of layer, every width of
+    spelled-out heads. ``odd``: sizes that fit no tile, unequal layers, layers without
+    a feed-forward, latents read across other layers, no groups, no shared expert.
+    ``single``: ones everywhere a one is allowed. ``large``: heads and latents wider
+    than the matrix-core kernels take, or more heads than a tile has rows."""
+    if name == "plain":
+        y = (4.0, 64, 8.0, 1.0)
+        layers = [(latent(4, 64, 32, 64, 64, 96, 40, yarn=y), moe(8, 2, 4, 2, 64, 128)),
+                  (attention(4, 2, 64, 64, 64, 4, 24), moe(8, 3, 2, 1, 64, 64)),
+                  (latent(2, 128, 32, 128, 64, 64, 56, yarn=y, kv_from=0), moe(8, 2, 4, 2, 64, 128)),
+                  (attention(6, 3, 128, 64, 32, 3, 37), moe(4, 4, 4, 4, 128, 64)),
+                  (latent(3, 32, 64, 128, 128, 32, 16), moe(8, 2, 4, 3, 64, 64))]
+        vocab, width, taps, eps, out = 333, 128, 4, 1e-5, 0.7
+    elif name == "odd":
+        layers = [(latent(3, 12, 6, 10, 20, 14, 17, 300.0, 0.4, (3.0, 40, 3.0, 0.4)),
+                   moe(9, 4, 3, 2, 20, 28)),
+                  (attention(3, 1, 21, 14, 6, 3, 7, 500.0, 0.3), None),
+                  (latent(5, 33, 6, 7, 20, 50, 50, 300.0, 0.2, (3.0, 40, 3.0, 0.4), 0),
+                   moe(6, 3, 6, 4, 36, 0)),
+                  (attention(4, 2, 10, 34, 10, 1, 64), moe(5, 2, 1, 1, 12, 52)),
+                  (latent(1, 40, 10, 70, 7, 9, 1000, 50.0), None),
+                  (attention(2, 2, 9, 70, 2, 6, 45, 1e6), moe(7, 7, 1, 1, 9, 33))]
+        vocab, width, taps, eps, out = 301, 90, 3, 1e-3, 1.3
+    elif name == "single":
+        layers = [(latent(1, 1, 2, 1, 1, 1, 1, yarn=(1.0, 1, 1.0, 1.0)), moe(1, 1, 1, 1, 1, 1)),
+                  (attention(1, 1, 2, 2, 2, 1, 1), None),
+                  (latent(1, 1, 2, 1, 1, 1, 2, kv_from=0, yarn=(1.0, 1, 1.0, 1.0)),
+                   moe(2, 1, 2, 1, 1, 0))]
+        vocab, width, taps, eps, out = 64, 32, 1, 1.0, 1.0  # else one number is a sign
+    else:
+        layers = [(latent(20, 128, 64, 64, 260, 300, 130), moe(70, 6, 10, 3, 64, 64)),
+                  (attention(8, 1, 136, 200, 100, 5, 90), None),
+                  (latent(33, 16, 64, 128, 260, 24, 33, kv_from=0), moe(16, 4, 4, 2, 192, 64)),
+                  (latent(2, 160, 100, 40, 530, 200, 61), None),
+                  (attention(4, 2, 96, 130, 96, 9, 1000), moe(8, 2, 2, 2, 64, 320))]
+        vocab, width, taps, eps, out = 128, 192, 6, 1e-5, 0.4
+    return {"architecture": "Fezuzen", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "canon": {"taps": taps}, "logit_scale": out,
+            "layers": [{"type": m[0], "mixer": m[1], "mlp": f} for m, f in layers]}
+
+
+def weights(cfg, seed=0, decided=False):
+    """Random tensors, sized so that every term of the design matters: scores of a few
+    units, gates half open, convolutions as large as what they are added to, sublayer
+    norms far from one. ``decided``: channel 0 of the residual is large and constant and
+    alone chooses the experts, whose scores it sets far apart."""
+    gen = torch.Generator().manual_seed(seed)
+
+    def n(*shape, s=1.0):
+        return torch.randn(*shape, generator=gen) * s
+
+    def lin(o, i, s=1.0):
+        return n(o, i, s=s * i ** -0.5)
+
+    w, taps = cfg["width"], cfg["canon"]["taps"]
+    t = {"embed": n(cfg["vocab"], w), "head": lin(cfg["vocab"], w), "final.norm": 1 + n(w, s=0.2)}
+
+    def norms(l, k):
+        t[l + f"norm{k}"], t[l + f"norm{k}b"] = 1 + n(w, s=0.2), 0.8 + n(w, s=0.3)
+        t[l + f"canon{k}"] = n(w, taps, s=0.5)
+
+    for i, layer in enumerate(cfg["layers"]):
+        l, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        norms(l, 1)
+        p, H, d, e = l + "mix.", m["heads"], m["dim"], m["vdim"]
+        if layer["type"] == "latent_attention":
+            r, qr, rot = m["kv_rank"], m["q_rank"], m["rot_dim"]
+            t[p + "dq"], t[p + "dq.norm"] = lin(qr, w), 1 + n(qr, s=0.3)
+            t[p + "uq"] = lin(H * (d + rot), qr, 2.0 / (m["scale"] * (d + rot) ** 0.5))
+            if m.get("kv_from") is None:
+                t[p + "dkv"], t[p + "dkv.norm"] = lin(r + rot, w), 1 + n(r, s=0.3)
+            t[p + "uk"], t[p + "uv"] = lin(H * d, r), lin(H * e, r)
+        else:
+            G = m["kv_heads"]
+            for x, c, s in (("q", H * d, 1.5 / (m["scale"] * d ** 0.5)), ("k", G * d, 1.0),
+                            ("v", G * e, 1.0)):
+                t[p + x], t[p + x + ".conv"] = lin(c, w, s), n(c, m["conv"], s=0.7)
+            t[p + "g"] = lin(H * e, w, 1.5)
+        t[p + "o"] = lin(w, H * e, 2.0)
+        if f is None:
+            continue
+        norms(l, 2)
+        p, E = l + "mlp.", f["router"]["experts"]
+        t[p + "router"] = lin(E, w, 1.5)
+        for x, ff in [(f"e{x}", f["expert"]["ff"]) for x in range(E)] + \
+                ([("shared", f["shared"]["ff"])] if "shared" in f else []):
+            t[p + x + ".up"], t[p + x + ".down"] = lin(ff, w, 1.5), lin(w, ff)
+        if decided:
+            t[p + "router"] *= 0.03
+            t[p + "router"][:, 0] = 0.15 * torch.randperm(E, generator=gen)
+    if decided:
+        t["embed"][:, 0] = 12.0
+        for name, x in t.items():
+            if "canon" in name or name.endswith(("norm1b", "norm2b")):
+                x[0] = 0.05
+    return {k: v.to(torch.bfloat16) for k, v in t.items()}
+
+
+def make_rig(path, name, device, dtype="float32"):
+    cfg = config(name)
+    return decoder_rig.Rig(path, cfg, weights(cfg, decided=dtype == "bfloat16"), oracle, device,
+                           dtype, 0.06)
+
+
+CASES = [pytest.param((n, d, t), id=f"{n}-{d}-{t}",
+                      marks=[pytest.mark.gpu] if d == "cuda" else [])
+         for n in ("plain", "odd", "single", "large")
+         for d, t in (("cpu", "float32"), ("cuda", "float32"), ("cuda", "bfloat16"))]
+
+
+@pytest.fixture(scope="module", params=CASES)
+def rig(request, tmp_path_factory):
+    name, device, dtype = request.param
+    if device == "cuda" and not torch.cuda.is_available():
+        pytest.skip("no GPU in this container")
+    return make_rig(tmp_path_factory.mktemp("ckpt"), name,
+                    "auto" if device == "cuda" else "cpu", dtype)
+
+
+@pytest.fixture(scope="module")
+def cpu_rig(tmp_path_factory):
+    return make_rig(tmp_path_factory.mktemp("ckpt"), "odd", "cpu")
+
+
+# --------------------------------------------------------------- whole models
+
+def test_whole_prompt(rig):
+    toks = rig.tokens(90, 0)
+    rig.check(rig.run(rig.replayer(), "a", toks, [90]), rig.logits(toks))
+
+
+def test_residual_after_every_layer(rig):
+    """The residual stream, layer by layer: a fault shows where it happens."""
+    toks = rig.tokens(37, 1)
+    want, got = oracle.forward(rig.cfg, rig.t, toks)[1], rig.trail(toks)
+    assert len(got) == len(want)
+    for a, b in zip(got, want):
+        rig.check(a, b, 3e-5 if rig.dtype == "float32" else 0.03)
+
+
+def test_token_by_token(rig):
+    toks = rig.tokens(90, 0)
+    rig.check(rig.run(rig.replayer(), "a", toks, [1] * 90), rig.logits(toks))
+
+
+@pytest.mark.parametrize("cuts", [[2] * 45, [7, 2, 16, 1, 33, 2, 29], [64, 2, 15, 9],
+                                  [1, 89], [17, 16, 1, 1, 1, 15, 39], [2, 1, 2, 85]], ids=str)
+def test_portions(rig, cuts):
+    toks = rig.tokens(90, 0)
+    rig.check(rig.run(rig.replayer(), "a", toks, cuts), rig.logits(toks))
+
+
+@pytest.mark.parametrize("n", [1, 2, 3])
+def test_first_tokens(rig, n):
+    """A sequence's first tokens, alone, as its whole prompt or one by one."""
+    toks = rig.tokens(n, 5)
+    rp = rig.replayer()
+    rig.check(rig.run(rp, "a", toks, [n]), rig.logits(toks))
+    rig.check(rig.run(rp, "b", toks, [1] * n), rig.logits(toks))
+
+
+def test_unequal_batch(rig):
+    """Prompt portions and decoded tokens in one batch, requests that pause,
+    start late and end early: each as if it were alone."""
+    toks = {r: rig.tokens(n, i) for i, (r, n) in
+            enumerate({"a": 70, "b": 33, "c": 90, "d": 5}.items())}
+    rig.run_plan(rig.replayer(max_tokens=320), toks, [
+        {"a": 40, "d": 5}, {"a": 1, "b": 20}, {"b": 1, "a": 1, "c": 50},
+        {"c": 2}, {"b": 1, "c": 1}, {"c": 17, "a": 1, "b": 11}, {"a": 27, "c": 20}])
+
+
+def test_reused_pages_and_slots(rig):
+    """One slot and a pool that only just fits, so every later request gets what
+    an earlier one left behind."""
+    rp = rig.replayer(max_tokens=96, requests=1)
+    free = rp.engine.kv.num_free()
+    for i, cuts in enumerate([[90], [5, 1, 1], [2] * 20, [1] * 12, [1], [64, 26]]):
+        toks = rig.tokens(sum(cuts), 10 + i)
+        rig.check(rig.run(rp, f"r{i}", toks, cuts), rig.logits(toks))
+        assert rp.engine.kv.num_free() == free and rp.engine.states.num_free() == 1
+
+
+def test_long_decoding(rig):
+    n = 200 if rig.device == "cpu" else 400
+    toks = rig.tokens(n, 3)
+    rig.check(rig.run(rig.replayer(), "a", toks, [20] + [1] * (n - 20)), rig.logits(toks))
+
+
+def test_greedy_generation(rig):
+    """Through add_request, the scheduler (prompts cut at 32 tokens, batches of
+    prompts beside decoding) and the sampler."""
+    eng = rig.engine(kv_cache_pages=64, max_num_seqs=3, max_batched_tokens=32,
+                     max_model_len=256)
+    prompts = [rig.tokens(n, 20 + n) for n in (3, 70, 25, 40)]
+    out = eng.generate(prompts, SamplingParams(max_tokens=12, **decoder_rig.GREEDY))
+    assert eng.states.num_free() == eng.states.num_slots
+    rig.check_greedy(prompts, out, 12)
+
+
+# ----------------------------------------------------- the engine's own workings
+
+def test_caches_and_states_of_the_layers(cpu_rig):
+    """A layer that borrows latents has no cache; every layer remembers its mixer's
+    last inputs, layers with a feed-forward those of that too, a convolved attention
+    its projections."""
+    eng = cpu_rig.engine(kv_cache_pages=8, max_num_seqs=1)
+    assert eng.kv.layout == [(1, 64 + 64, 0), (1, 21, 14), (2, 10, 34), (1, 64 + 64, 0),
+                             (2, 9, 70)]
+    shapes = [s[0].shape[1:] for s in eng.states.states]
+    x = (2, 90)
+    assert shapes == [x, x, x, (2, 3 * 21 + 21 + 14), x, x, x, x,
+                      (0, 40 + 2 * (10 + 34)), x, x, x, (5, 18 + 2 * (9 + 70))]
+
+
+def test_preemption_recomputes_state(cpu_rig):
+    eng = cpu_rig.engine(kv_cache_pages=6, max_num_seqs=2, max_model_len=80)
+    prompts = [cpu_rig.tokens(20, 40), cpu_rig.tokens(18, 41)]
+    out = eng.generate(prompts, SamplingParams(max_tokens=30, **decoder_rig.GREEDY))
+    assert eng.counters["preemptions"] > 0
+    for prompt, got in zip(prompts, out):
+        assert got == cpu_rig.logits(prompt + got)[len(prompt) - 1:-1].argmax(-1).tolist()
+    assert eng.kv.num_free() == 6 and eng.states.num_free() == eng.states.num_slots
+
+
+def test_session_continues_from_its_state(cpu_rig):
+    eng = cpu_rig.engine(kv_cache_pages=32, max_num_seqs=2, max_model_len=256)
+    first = cpu_rig.tokens(21, 50)
+    out = decoder_rig.turn(eng, "t1", first, 5, "s")
+    assert out == cpu_rig.greedy(first, 5)
+    before = eng.counters["prompt_tokens"]
+    second = first + out + cpu_rig.tokens(9, 51)
+    assert decoder_rig.turn(eng, "t2", second, 5, "s") == cpu_rig.greedy(second, 5)
+    assert eng.counters["prompt_tokens"] - before == len(second) - (len(first) + 4)
+    # departs from it: everything runs again
+    third = second[:15] + cpu_rig.tokens(9, 52)
+    assert decoder_rig.turn(eng, "t3", third, 5, "s") == cpu_rig.greedy(third, 5)
+
+
+def test_equal_prompts_share_no_pages(cpu_rig):
+    eng = cpu_rig.engine(kv_cache_pages=64, max_num_seqs=4, max_model_len=256)
+    prompt = cpu_rig.tokens(50, 70)
+    p = SamplingParams(max_tokens=4, **decoder_rig.GREEDY)
+    assert eng.generate([prompt] * 2, p) == [cpu_rig.greedy(prompt, 4)] * 2
+    assert eng.counters["prefix_cache_pages"] == 0
+
+
+def test_trace_run_program(cpu_rig, tmp_path):
+    toks = cpu_rig.tokens(12, 90)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": toks[:9], "want": [8, 0]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": toks[9:], "want": [2]}], "end": ["a"]}]
+    r = subprocess.run(
+        [sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", cpu_rig.path,
+         "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "64", "--device", "cpu"],
+        input="".join(json.dumps(s) + "\n" for s in steps), text=True, capture_output=True,
+        timeout=120)
+    assert r.returncode == 0, r.stderr
+    for step, rows in ((0, [8, 0]), (1, [11])):
+        raw = bytearray((tmp_path / f"{step}.f32").read_bytes())
+        cpu_rig.check(torch.frombuffer(raw, dtype=torch.float32).view(len(rows), -1),
+                      cpu_rig.logits(toks)[rows])
+
+
+# ------------------------------------------------------- config, loader, registry
+
+@pytest.mark.parametrize("name", ["plain", "odd", "single", "large"])
+def test_config_and_weights_round_trip(tmp_path, name):
+    from aurora_amd.models.loader import save_named_safetensors
+    from aurora_amd.models.registry import build_model
+
+    rig = make_rig(tmp_path, name, "cpu")
+    spec = spec_from_checkpoint(rig.path)
+    assert spec.arch == "fezuzen" and spec.n_layers == len(rig.cfg["layers"])
+    assert spec.param_count() == sum(v.numel() for v in rig.t.values())
+    m = build_model(spec, torch.float32, "cpu", rig.path)
+    again = m.named_tensors()
+    assert set(again) == set(rig.t)
+    for k, v in rig.t.items():
+        assert torch.equal(again[k], v.float()), k
+    (tmp_path / "copy").mkdir()
+    save_named_safetensors(m, str(tmp_path / "copy"))
+    m2 = build_model(spec, torch.float32, "cpu", str(tmp_path / "copy"))
+    assert all(torch.equal(again[k], v) for k, v in m2.named_tensors().items())
+
+
+def test_bad_configs_are_refused(tmp_path):
+    cfg = config("odd")
+    save_file(weights(cfg), str(tmp_path / "model.safetensors"))
+
+    def spec(change):
+        c = json.loads(json.dumps(cfg))
+        change(c["layers"])
+        (tmp_path / "config.json").write_text(json.dumps(c))
+        return get_spec(str(tmp_path))
+
+    assert spec(lambda ls: None).n_layers == 6
+    for change in (lambda ls: ls[0].update(type="other"),
+                   lambda ls: ls[0]["mlp"].update(kind="dense"),
+                   lambda ls: ls[0]["mixer"].update(rot_dim=8),
+                   lambda ls: ls[0]["mixer"]["rot"].update(dims=5),
+                   lambda ls: ls[1]["mixer"].update(kv_heads=2),
+                   lambda ls: ls[1]["mixer"].update(vdim=15),
+                   lambda ls: ls[1]["mixer"]["rot"].update(dims=22),
+                   lambda ls: ls[2]["mixer"].update(kv_from=2),    # itself
+                   lambda ls: ls[2]["mixer"].update(kv_from=4),    # a later layer
+                   lambda ls: ls[2]["mixer"].update(kv_from=1),    # another kind
+                   lambda ls: ls[4]["mixer"].update(kv_from=2),    # one that borrows
+                   lambda ls: ls[4]["mixer"].update(kv_from=0),    # another rank
+                   lambda ls: ls[2]["mixer"]["rot"].update(base=301.0),
+                   lambda ls: ls[0]["mlp"]["router"]["groups"].update(keep=4),
+                   lambda ls: ls[0]["mlp"]["router"].update(top=7)):
+        with pytest.raises(ValueError):
+            spec(change)
+
+
+def test_presets_run():
+    eng = LLMEngine(EngineConfig(model="tiny-fezuzen", device="cpu", seed=7))
+    p = SamplingParams(max_tokens=6, **decoder_rig.GREEDY)
+    prompts = [[5, 9, 2], list(range(40, 90)), [7] * 25]
+    assert eng.generate(prompts, p) == [eng.generate([x], p)[0] for x in prompts]
+
+
+@pytest.mark.gpu
+def test_captured_and_eager_decoding_agree():
+    """Replays of captured steps, with prompts, pauses and joins between them,
+    against the same steps run eagerly."""
+    from aurora_amd.models.registry import build_model
+
+    spec = get_spec("smoke-fezuzen")
+    model = build_model(spec, torch.bfloat16, "cuda", seed=3)
+    gen = torch.Generator().manual_seed(1)
+    toks = {r: torch.randint(0, spec.vocab_size, (700,), generator=gen).tolist() for r in "abc"}
+    plan = ([{"a": 400}, {"b": 333}] + [{"a": 1, "b": 1}] * 20 + [{"c": 50, "a": 1}]
+            + [{"a": 1, "b": 1, "c": 1}] * 20 + [{"b": 1}] * 5 + [{"c": 1, "a": 1}] * 20)
+
+    def run(graphs):
+        rp = TraceReplayer(LLMEngine(EngineConfig(
+            model=spec.name, page_size=64, kv_cache_pages=64, max_num_seqs=4, state_slots=4,
+            max_model_len=1024, use_hip_graphs=graphs), model=model))
+        at, out = dict.fromkeys(toks, 0), []
+        for step in plan:
+            entries = [(r, toks[r][at[r]:at[r] + n], [n - 1]) for r, n in step.items()]
+            for r, n in step.items():
+                at[r] += n
+            out.append(rp.step(entries).cpu())
+        return torch.cat(out)
+
+    a, b = run(True), run(False)
+    assert torch.isfinite(a).all()
+    # the batch is padded to its bucket in a captured step, so products may be
+    # tiled otherwise; nothing else differs
+    assert ((a - b).norm(dim=-1) / b.norm(dim=-1)).quantile(0.9) < 0.02
+
+
+# --------------------------------------------------------- each mechanism alone
+
+DEVICES = [pytest.param("cpu"), pytest.param("cuda", marks=pytest.mark.gpu)]
+DTYPES = pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16], ids=str)
+
+
+def only_float32_on_cpu(device, dtype):
+    if device == "cpu" and dtype != torch.float32:
+        pytest.skip("the CPU runs in float32")
+
+
+def _seg(n, device, start=0, pages=None, single=False, P=16):
+    """The segment of one sequence's next n tokens (``single``: as a decoded one)."""
+    pages = torch.arange(-(-(start + n) // P)) if pages is None else pages
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)  # noqa: E731
+    tail = () if single else (i32([0, n]), [0, n], [start + n])
+    return ops.Segment(slice(0, n), i32([pages.tolist()]), i32([start + n]), i32([start]),
+                       i32([0]), *tail)
+
+
+def _steps(cuts, device, pages, P=16):
+    """(first, past the last token, segment, cache slots, positions) of every portion."""
+    at = 0
+    for c in cuts:
+        a, b = at, at + c
+        i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=device)  # noqa: E731
+        yield (a, b, _seg(c, device, a, pages, single=a > 0 and c == 1, P=P),
+               i32([int(pages[t // P]) * P + t % P for t in range(a, b)]),
+               i32(list(range(a, b))))
+        at = b
+
+
+@pytest.mark.parametrize("dims", [2, 6, 64, 128])
+@pytest.mark.parametrize("base,scaling", [
+    (1e4, None), (5e5, None), (1e4, (4.0, 512, 32.0, 1.0)), (300.0, (3.0, 40, 3.0, 0.4)),
+    (1e6, (40.0, 4096, 32.0, 1.0)), (1e4, (1.0, 1, 1.0, 1.0)), (1e4, (8.0, 1e9, 2.0, 1.0))], ids=str)
+def test_rotation_table(dims, base, scaling):
+    """Angles and growth of every pair, at positions near and far; the limits of the
+    scaling fall inside, before and behind the pairs."""
+    from aurora_amd.models.config import YarnSpec
+    cfg = scaling and dict(zip(("factor", "original", "fast", "slow"), scaling))
+    freq, grow = oracle.frequencies(dims, base, cfg)
+    got = torch_ref.rotation_table(dims, 5000, base, YarnSpec(**cfg) if cfg else None)
+    for p in (0, 1, 17, 4999):
+        a = p * torch.tensor(freq, dtype=D64)
+        want = torch.cat([a.cos(), a.sin()]) * grow
+        assert (got[p] - want).abs().max() < 1e-6 * grow
+    if cfg and cfg["factor"] > 1 and cfg["original"] == 1e9:
+        assert freq[0] == pytest.approx(1.0)  # turns often enough to stay
+
+
+def _latents_attend(c, kr, q, uk, uv, *, scale, base, window, cuts, device, dtype, monkeypatch,
+                    expand=False, P=16):
+    """ops.latent_front and ops.latent_attention over the portions of ``cuts``. c [T,
+    rank] with unit rms (so that the norm leaves it), kr [T, rot] and q [T, H, d + rot]
+    before their rotation."""
+    T, H, _ = q.shape
+    rank, rot, d, e = c.shape[1], kr.shape[1], uk.shape[1], uv.shape[1]
+    monkeypatch.setattr(sequence, "expand_latents", lambda seg, *a: expand and not seg.decode)
+    R, (D, tail, key) = ops.latent_width(rank), ops.latent_rotary_widths(d, rot)
+    E = ops.latent_head_width(e)
+    pages = torch.randperm(-(-T // P))
+    cache = torch.full((len(pages), 1, P, R + key), 9.0, dtype=dtype, device=device)
+    ukp, uvp = torch.zeros(H, D, R), torch.zeros(H, E, R)
+    ukp[:, :d, :rank], uvp[:, :e, :rank] = uk, uv
+    qp = torch.zeros(T, H, D + tail)
+    qp[..., :d], qp[..., D:D + rot] = q[..., :d], q[..., d:]
+    mv = lambda t: t.to(dtype).to(device)  # noqa: E731
+    turn = torch_ref.rotation_table(rot, T, base).to(device)
+    p = ops.LatentParams(H, D, E, scale, 0, None, mv(ukp), mv(ukp.transpose(1, 2).contiguous()),
+                         mv(uvp), None, tail, turn, window)
+    k0 = -(-rank // 8) * 8
+    proj = torch.zeros(T, k0 + -(-rot // 8) * 8)
+    proj[:, :rank], proj[:, k0:k0 + rot] = c, kr
+    front = ops.LatentFrontParams(0, rank, torch.ones(rank, device=device), 0.0, k0, R, turn)
+    proj, qp = mv(proj), mv(qp)
+    out = torch.zeros(T, H * E, dtype=dtype, device=device)
+    for a, b, seg, slots, positions in _steps(cuts, device, pages, P):
+        ops.latent_front(proj[a:b], front, positions, slots, cache)
+        ops.latent_attention(proj[a:b], p, cache, seg, out[a:b], qp[a:b].clone(), positions)
+    return out.float().cpu().view(T, H, E)[..., :e]
+
+
+def _unit_rms(c):
+    return c / c.pow(2).mean(-1, keepdim=True).sqrt()
+
+
+LATENT_SIZES = [(4, 64, 40, 64, 32), (20, 32, 64, 100, 16), (3, 20, 12, 530, 6),
+                (2, 128, 128, 512, 64), (2, 96, 64, 256, 30)]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@DTYPES
+@pytest.mark.parametrize("H,d,e,rank,rot", LATENT_SIZES)
+def test_far_latents_stand_out(device, dtype, H, d, e, rank, rot, monkeypatch):
+    """One key whose score is far above the rest: the query's output is its value while
+    the window holds it, at pages' and tiles' borders, in a prompt, at a portion's start
+    and in decoding, and has nothing of it one token further on or while it is still to
+    come."""
+    only_float32_on_cpu(device, dtype)
+    T, i, window = 270, 260, 101
+    gen = torch.Generator().manual_seed(rank)
+    n = lambda *s: torch.randn(*s, generator=gen)  # noqa: E731
+    as_stored = lambda t: t.to(dtype).double()  # noqa: E731
+    c = _unit_rms(n(T, rank)).to(dtype).float()
+    kr = n(T, rot) * 0.3
+    uk, uv = n(H, d, rank) * rank ** -0.5, n(H, e, rank) * rank ** -0.5
+    freq, _ = oracle.frequencies(rot, 1e4)
+    edge = i - window + 1
+    for j in (edge - 2, edge - 1, edge, edge + 1, 0, 191, 192, 207, 208, 255, 256, 259, 260, 261):
+        q = torch.cat([n(T, H, d) * 0.3, n(T, H, rot) * 0.3], -1)
+        k_j = torch.einsum("hdr,r->hd", uk, c[j])
+        q[i, :, :d] = 80 * k_j / k_j.pow(2).sum(-1, keepdim=True)  # scores 80 on key j
+        k = torch.einsum("hdr,tr->thd", as_stored(uk), c.double())
+        v = torch.einsum("her,tr->the", as_stored(uv), c.double())
+        qs, ks = as_stored(q), oracle.turn(as_stored(kr)[:, None], freq, 1.0)
+        qs = torch.cat([qs[..., :d], oracle.turn(qs[..., d:], freq, 1.0)], -1)
+        k = torch.cat([k, ks.expand(T, H, rot)], -1)
+        want = oracle.attend(qs, k, v, 1.0, oracle.visible(T, {"size": window}, oracle.in_window),
+                             oracle.softmax)
+        hit = (want[i] - v[j]).abs().max()
+        assert (hit < 0.02 * v[j].abs().max()) == (edge <= j <= i)
+        tol = 1e-4 if dtype == torch.float32 else 0.03
+        spelled = dtype == torch.bfloat16 and e != 12 and sum(ops.latent_rotary_widths(d, rot)[:2]) <= 192
+        for cuts in ([T], [i, 1, 9], [i - 2, 12], [i + 1, 9]):
+            for expand in (False, True) if spelled else (False,):
+                got = _latents_attend(c, kr, q, uk, uv, scale=1.0, base=1e4, window=window,
+                                      cuts=cuts, device=device, dtype=dtype,
+                                      monkeypatch=monkeypatch, expand=expand)
+                err = (got - want).abs().amax((1, 2)) / want.abs().max()
+                assert err[i] < tol, (j, cuts, expand, float(err[i]))
+                if j == 0:
+                    assert err.max() < tol, (cuts, expand, err.argmax())
+        if device == "cpu" and j == 0:
+            break
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@DTYPES
+@pytest.mark.parametrize("window", [1, 2, 63, 64, 65, 100, 149, 0])
+def test_window_counts_its_keys(device, dtype, window, monkeypatch):
+    """Equal scores weigh every visible key alike: key t's value is e_t's first
+    coordinate, so the sums tell exactly which keys were seen."""
+    only_float32_on_cpu(device, dtype)
+    T, H, d, e, rank, rot = 150, 3, 32, 64, 64, 16
+    c = _unit_rms(torch.where(torch.arange(T)[:, None] % 7 < 3, 1.0, -1.0).expand(T, rank))
+    mark = torch.where(torch.arange(T) % 7 < 3, 1.0, -1.0).double()
+    uv = torch.ones(H, e, rank) / rank
+    seen = oracle.visible(T, {"size": window} if window else None, oracle.in_window).double()
+    want = (seen @ mark) / seen.sum(-1)
+    for cuts in ([T], [1] * 5 + [90, 1, 1, 2, 51]):
+        for expand in (False, True) if dtype == torch.bfloat16 else (False,):
+            got = _latents_attend(c, torch.randn(T, rot), torch.zeros(T, H, d + rot),
+                                  torch.randn(H, d, rank), uv, scale=0.3, base=50.0,
+                                  window=window, cuts=cuts, device=device, dtype=dtype,
+                                  monkeypatch=monkeypatch, expand=expand)
+            tol = 1e-5 if dtype == torch.float32 else 1e-2
+            assert (got - want.view(T, 1, 1)).abs().max() < tol, (cuts, expand)
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("own,q_rank,rot,rank", [(True, 96, 16, 64), (False, 33, 6, 20),
+                                                 (True, 7, 2, 5), (True, 0, 64, 512)])
+def test_latent_front_alone(device, own, q_rank, rot, rank):
+    T, P, eps = 21, 16, 1e-3
+    R = ops.latent_width(rank)
+    k0 = -(-rank // 8) * 8
+    q0 = k0 + -(-rot // 8) * 8
+    proj = torch.randn(T, -(-(q0 + q_rank) // 8) * 8) * 2
+    w, qw = torch.randn(rank), torch.randn(max(q_rank, 1))
+    pos = torch.randperm(500)[:T].to(torch.int32)
+    slots = torch.randperm(40)[:T].to(torch.int32)
+    slots[3] = -1
+    turn = torch_ref.rotation_table(rot, 500, 77.0)
+    cache = torch.full((3, 1, P, R + 64), 5.0, device=device)
+    p = ops.LatentFrontParams(0 if own else None, rank, w.to(device), eps, k0, R,
+                              turn.to(device), q0, q_rank, qw.to(device) if q_rank else None)
+    cq = ops.latent_front(proj.to(device), p, pos.to(device), slots.to(device), cache)
+    if q_rank:
+        want = oracle.rms_norm(proj[:, q0:q0 + q_rank].double(), qw.double(), eps)
+        assert (cq.cpu() - want).abs().max() < 1e-5 * want.abs().max()
+    want = torch.full((3 * P, R + 64), 5.0, dtype=D64)
+    if own:
+        c = oracle.rms_norm(proj[:, :rank].double(), w.double(), eps)
+        freq, _ = oracle.frequencies(rot, 77.0)
+        for t in range(T):
+            if slots[t] < 0:
+                continue
+            row = torch.zeros(R + 64, dtype=D64)
+            row[:rank] = c[t]
+            x = torch.zeros(int(pos[t]) + 1, 1, rot, dtype=D64)
+            x[-1, 0] = proj[t, k0:k0 + rot]
+            row[R:R + rot] = oracle.turn(x, freq, 1.0)[-1, 0]
+            want[slots[t]] = row
+    else:
+        assert cq is not None
+    assert (cache.cpu().view(3 * P, -1) - want).abs().max() < 2e-5 * want.abs().max()
+
+
+def _heads(dim, vdim, dtype, device):
+    return ops.cache_head_dims(dim, vdim, dtype, device)
+
+
+def _conv_attend(x, H, G, d, e, conv, cuts, device, dtype, *, rot, base, scale, chunk=0, window=0,
+                 sink=True, gate=None, turn_values=True, P=16):
+    """ops.conv_qkv and ops.biased_attention over the portions of ``cuts``; x [T, H d +
+    G d + G e] as projected, conv [that, taps], gate [T, H e]."""
+    T, C = x.shape
+    taps = conv.shape[1]
+    at = [0, -(-H * d // 8) * 8]
+    at.append(at[1] + -(-G * d // 8) * 8)
+    g0 = at[2] + -(-G * e // 8) * 8
+    proj = torch.zeros(T, -(-(g0 + H * e) // 8) * 8)
+    for c0, part in zip(at, x.split([H * d, G * d, G * e], 1)):
+        proj[:, c0:c0 + part.shape[1]] = part
+    if gate is not None:
+        proj[:, g0:g0 + H * e] = gate
+    proj = proj.to(dtype).to(device)
+    DK, DV = _heads(d, e, dtype, device)
+    pages = torch.randperm(-(-T // P))
+    kc, vc = (torch.full((len(pages), G, P, w), 9.0, dtype=dtype, device=device) for w in (DK, DV))
+    ring = torch.full((1, taps - 1, C), float("nan"), dtype=dtype, device=device)  # never read fresh
+    values = torch_ref.rotation_table(e, T, base).to(device) if turn_values else None
+    p = ops.ConvHeadsParams(H, G, d, e, *at, conv.t().contiguous().to(device),
+                            torch_ref.rotation_table(rot, T, base).to(device), values)
+    s = torch.zeros(H, device=device) if sink else None
+    out = torch.zeros(T, H * e + 8, dtype=dtype, device=device)
+    for a, b, seg, slots, _ in _steps(cuts, device, pages, P):
+        q = ops.conv_qkv(proj[a:b], p, slots, ring, [seg], kc, vc)
+        g = proj[a:b, g0:g0 + H * e] if gate is not None else None
+        ops.biased_attention(q, kc, vc, seg, scale, window, None, out[a:b], 8, e, 1.0, sink=s,
+                             chunk=chunk, turn=values, gate=g)
+    assert (out[:, :8] == 0).all()
+    return out[:, 8:].float().cpu().view(T, H, e)
+
+
+def _conv_want(x, H, G, d, e, conv, *, rot, base, scale, chunk=0, window=0, sink=True, gate=None,
+               turn_values=True):
+    T = x.shape[0]
+    y = oracle.causal_conv(x.double(), conv.double())
+    r = {"dims": rot, "base": base}
+    q, k, v = (t.reshape(T, h, w) for t, h, w in
+               zip(y.split([H * d, G * d, G * e], 1), (H, G, G), (d, d, e)))
+    q, k = oracle.rotate(q, r), oracle.rotate(k, r)
+    v = oracle.rotate_values(v, r) if turn_values else v
+    size, rule = (chunk, oracle.in_chunk) if chunk else (window, oracle.in_window)
+    o = oracle.attend(q, k, v, scale, oracle.visible(T, {"size": size} if size else None, rule),
+                      oracle.softmax_plus_one if sink else oracle.softmax)
+    o = oracle.turn_back(o, r) if turn_values else o
+    return o if gate is None else o * torch.sigmoid(gate.double()).view(T, H, e)
+
+
+HEADS = [(4, 2, 64, 64), (4, 4, 128, 64), (8, 1, 64, 128), (6, 2, 128, 128), (3, 1, 20, 14),
+         (2, 1, 160, 200), (5, 5, 33, 34)]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@DTYPES
+@pytest.mark.parametrize("H,G,d,e", HEADS)
+def test_far_keys_stand_out(device, dtype, H, G, d, e):
+    """One key far above the rest and above the sink: a query of its chunk has its value
+    (turned to the query's distance), the chunk's neighbours have nothing of it; in
+    prompts, at portions' starts and in decoding."""
+    only_float32_on_cpu(device, dtype)
+    T, chunk, rot = 270, 52, d - d % 2
+    gen = torch.Generator().manual_seed(d)
+    n = lambda *s: torch.randn(*s, generator=gen)  # noqa: E731
+    conv = torch.cat([torch.zeros(H * d + G * (d + e), 1), torch.ones(H * d + G * (d + e), 1)], 1)
+    kw = dict(rot=rot, base=100.0, scale=1.0, chunk=chunk)
+    for j, i in ((207, 208), (208, 208), (208, 259), (207, 259), (259, 259), (259, 260),
+                 (256, 259), (240, 255), (0, 51), (0, 52), (209, 211)):
+        x = n(T, H * d + G * (d + e)) * 0.3
+        k_j = x[j, H * d:(H + G) * d].reshape(G, d)
+        # the query's rotation undone, the key's done: the score is 80
+        freq, _ = oracle.frequencies(rot, 100.0)
+        turn = lambda t, p: oracle.turn(  # noqa: E731
+            torch.cat([torch.zeros(abs(p), *t.shape), t[None]]).double(), freq, 1.0,
+            1 if p >= 0 else -1)[-1]
+        target = turn(k_j.float(), j - i)
+        q_i = 80 * target / target.pow(2).sum(-1, keepdim=True)
+        x[i, :H * d] = q_i.repeat_interleave(H // G, 0).reshape(-1).float()
+        x = x.to(dtype).float()
+        want = _conv_want(x, H, G, d, e, conv, **kw)
+        v = x[j, (H + G) * d:].reshape(G, e).double()
+        vf, _ = oracle.frequencies(e, 100.0)
+        v = oracle.turn(torch.cat([torch.zeros(abs(i - j), G, e, dtype=D64), v[None]]), vf, 1.0,
+                        -1 if i >= j else 1)[-1].repeat_interleave(H // G, 0)
+        near = (want[i] - v).abs().max() < 0.02 * v.abs().max()
+        assert near == (j <= i and j // chunk == i // chunk), (j, i)
+        tol = 1e-4 if dtype == torch.float32 else 0.03
+        for cuts in ([T], [i, 1, T - i - 1] if 0 < i else [T], [i + 1, T - i - 1], [i - 2, T - i + 2]):
+            got = _conv_attend(x, H, G, d, e, conv, cuts, device, dtype, **kw)
+            err = (got - want).abs().amax((1, 2)) / want.abs().max()
+            assert err[i] < tol, (j, i, cuts, float(err[i]))
+        if device == "cpu" and j == 259:
+            break
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@DTYPES
+@pytest.mark.parametrize("H,G,d,e", HEADS)
+@pytest.mark.parametrize("size", [("chunk", 1), ("chunk", 33), ("chunk", 64), ("window", 50),
+                                  ("chunk", 0)], ids=str)
+def test_convolved_attention_alone(device, dtype, H, G, d, e, size):
+    """All of it at once, over portions, with every option on and off."""
+    only_float32_on_cpu(device, dtype)
+    T, taps = 150, {1: 1, 33: 4, 64: 3, 50: 9, 0: 2}[size[1]]
+    gen = torch.Generator().manual_seed(e + taps)
+    n = lambda *s: torch.randn(*s, generator=gen)  # noqa: E731
+    rot = max(2, d // 4 * 2) if size[1] == 33 else d - d % 2
+    for option in range(2):
+        x = n(T, H * d + G * (d + e)).to(dtype).float()
+        x[:, :H * d] *= 2
+        conv = n(x.shape[1], taps) * 0.6
+        gate = n(T, H * e).mul(2).to(dtype).float() if option == 0 else None
+        kw = dict(rot=rot, base=500.0, scale=d ** -0.5, sink=option == 0, gate=gate,
+                  turn_values=option == 0, **{size[0]: size[1]})
+        want = _conv_want(x, H, G, d, e, conv, **kw)
+        tol = 2e-5 if dtype == torch.float32 else 0.03
+        for cuts in ([T], [1] * 20 + [2, 17, 1, 64, 46], [2] * 75):
+            got = _conv_attend(x, H, G, d, e, conv, cuts, device, dtype, **kw)
+            err = (got - want).norm(dim=-1) / want.norm(dim=-1).mean()
+            assert err.max() < tol, (option, cuts, float(err.max()))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@DTYPES
+@pytest.mark.parametrize("d", [64, 40])
+def test_sink_and_turned_values_have_closed_forms(device, dtype, d):
+    """Zero scores weigh each of the chunk's keys 1 / (1 + their number); equal values
+    that turn by their own and back by the query's position cancel by what lies
+    between."""
+    only_float32_on_cpu(device, dtype)
+    T, chunk, base = 120, 30, 40.0
+    x = torch.zeros(T, 3 * d)
+    x[:, 2 * d::2] = 1.0  # value (1, 0, 1, 0, ...)
+    want = torch.zeros(T, d, dtype=D64)
+    for i in range(T):
+        for j in range(i // chunk * chunk, i + 1):
+            a = (i - j) * base ** (-2.0 * torch.arange(d // 2, dtype=D64) / d)
+            want[i, 0::2] += torch.cos(a)  # by -(i - j)
+            want[i, 1::2] += -torch.sin(a)
+        want[i] /= 1 + i % chunk + 1
+    for cuts in ([T], [29, 1, 1, 60, 1, 28]):
+        got = _conv_attend(x, 1, 1, d, d, torch.ones(3 * d, 1), cuts, device, dtype, rot=d,
+                           base=base, scale=0.3, chunk=chunk)
+        tol = 1e-5 if dtype == torch.float32 else 0.02
+        assert (got[:, 0] - want).abs().max() < tol
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("taps", [1, 2, 3, 4, 7, 16])
+def test_short_convolution_alone(device, taps):
+    """One projection far above the rest must show in the keys of exactly the tokens its
+    taps reach, across portions and in single tokens."""
+    T, hit, G, d = 40, 13, 2, 8
+    C = G * d * 3
+    x = torch.randn(T, C)
+    x[hit] *= 1000
+    w = torch.randn(C, taps)
+    want = oracle.causal_conv(x.double(), w.double())[:, G * d:2 * G * d]
+    turn = torch_ref.rotation_table(2, T, 1e9)
+    for cuts in ([T], [1] * T, [hit, 27], [hit + 1, 26], [2] * 20):
+        ring = torch.full((1, taps - 1, C), float("nan"), device=device)
+        kc, vc = (torch.zeros(3, G, 16, d, device=device) for _ in "kv")
+        p = ops.ConvHeadsParams(G, G, d, d, 0, G * d, 2 * G * d, w.t().contiguous().to(device),
+                                turn.to(device) * 0 + torch.tensor([1.0, 0.0], device=device))
+        pages = torch.tensor([2, 0, 1])
+        for a, b, seg, slots, _ in _steps(cuts, device, pages):
+            ops.conv_qkv(x[a:b].to(device), p, slots, ring, [seg], kc, vc)
+        got = kc[pages].permute(0, 2, 1, 3).reshape(48, -1)[:T].cpu()
+        assert (got - want).abs().max() < 2e-6 * want.abs().max(), cuts
+        # the ring holds the last taps - 1 projections by position
+        for t in range(max(0, T - taps + 1), T):
+            assert torch.equal(ring[0, t % (taps - 1)].cpu(), x[t])
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("E,groups,keep,top", [(8, 4, 2, 3), (12, 2, 1, 6), (6, 6, 2, 2),
+                                               (5, 1, 1, 5), (70, 10, 3, 6), (1, 1, 1, 1)])
+def test_softmax_routing_alone(device, E, groups, keep, top):
+    """Logits that are far apart; weights are shares of all experts, chosen or not, and
+    nothing outside the best groups is chosen however large its score."""
+    T, W = 40, 64
+    r = {"top": top, "groups": {"count": groups, "keep": keep}}
+    gen = torch.Generator().manual_seed(E)
+    z = torch.stack([torch.randperm(E, generator=gen) for _ in range(T)]) * (6.0 / E)
+    h = torch.randn(T, W, generator=gen)
+    router = torch.linalg.lstsq(h.double(), z.double()).solution.T if E < W - T else None
+    if router is None or (h.double() @ router.T - z).abs().max() > 1e-9:
+        # one coordinate per expert
+        W = E + 3
+        h = torch.cat([z, torch.zeros(T, 3)], 1)
+        router = torch.eye(E, W, dtype=D64)
+    if device == "cpu":
+        sel, share = torch_ref.moe_route_softmax(h, router.float(), top, groups, keep, 1.0)
+    else:
+        sel, share = sequence._hip("moe_route_grouped").moe_route_grouped(
+            h.to(device), router.float().to(device), None, top, groups, keep, 1.0)
+    for t in range(T):
+        s = oracle.softmax(z[t].double())
+        want = oracle.choose(s.tolist(), r)
+        assert sel[t].tolist() == want
+        assert (share[t].cpu() - s[want]).abs().max() < 1e-6
+    if keep < groups and E > groups:  # a group's best expert may beat its neighbours' sum
+        left_out = [t for t in range(T) if set(oracle.choose(z[t].tolist(), r)) !=
+                    set(z[t].topk(top).indices.tolist())]
+        assert left_out
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16], ids=str)
+@pytest.mark.parametrize("W,ff,E,top", [(64, 64, 8, 2), (50, 20, 5, 3), (128, 192, 4, 4)])
+def test_squared_relu_experts_alone(device, dtype, W, ff, E, top):
+    only_float32_on_cpu(device, dtype)
+    for T in (1, 3, 200):
+        gen = torch.Generator().manual_seed(T)
+        n = lambda *s: torch.randn(*s, generator=gen)  # noqa: E731
+        h = n(T, W).to(dtype)
+        up, down = ((n(E, a, b) * b ** -0.5).to(dtype) for a, b in ((ff, W), (W, ff)))
+        sel = torch.stack([torch.randperm(E, generator=gen)[:top] for _ in range(T)]).int()
+        f = torch_ref.moe_relu2 if device == "cpu" else sequence._hip("moe_relu2").moe_relu2
+        y, place = f(h.to(device), sel.to(device), up.to(device), down.to(device))
+        got = y.cpu()[place.cpu().long()].double()
+        for t in range(0, T, 17):
+            for i, e in enumerate(sel[t].tolist()):
+                want = oracle.expert(h[t].double(), {".up": up[e].double(), ".down": down[e].double()}, "")
+                assert (got[t, i] - want).norm() < (1e-5 if dtype == torch.float32 else 0.02) * want.norm() + 1e-12
+        z = n(T, ff + 5).to(dtype)
+        a = ops.relu2(z.to(device)[:, :ff]).cpu().double()
+        assert (a - oracle.relu_squared(z[:, :ff].double())).abs().max() <= \
+            (1e-6 if dtype == torch.float32 else 0.04) * 16
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("W", [64, 50, 1056])
+def test_result_norm_and_convolution_alone(device, W):
+    """x += norm(delta + experts' rows), then the norm of x and its convolution, over
+    portions and single tokens, with one row far above the rest."""
+    T, top, taps, eps = 30, 3, 4, 1e-3
+    gen = torch.Generator().manual_seed(W)
+    n = lambda *s: torch.randn(*s, generator=gen)  # noqa: E731
+    x, delta, y = n(T, W), n(T, W), n(T * top, W)
+    delta[11] *= 300
+    share, post, weight, conv = n(T, top), n(W), n(W), n(taps, W)
+    place = torch.randperm(T * top, generator=gen).view(T, top).int()
+    r = delta.double() + (y.double()[place.long()] * share.double().unsqueeze(-1)).sum(1)
+    want_x = x.double() + oracle.rms_norm(r, post.double(), eps)
+    h = oracle.rms_norm(want_x, weight.double(), eps)
+    want = h, oracle.with_past(h, conv.double().t())
+    for cuts in ([T], [1] * T, [11, 1, 18], [2, 9, 1, 1, 17]):
+        ring = torch.full((1, taps - 1, W), float("nan"), device=device)
+        got, at = [], 0
+        for c in cuts:
+            a, b = at, at + c
+            at = b
+            xs = x[a:b].to(device).clone()
+            hu = ops.residual_rmsnorm_conv(
+                xs, weight.to(device), eps, conv.to(device), ring,
+                [_seg(c, device, a, single=a > 0 and c == 1)], delta=delta[a:b].to(device),
+                moe=(y.to(device), place[a:b].contiguous().to(device),
+                     share[a:b].contiguous().to(device)),
+                offset=0.0, dtype=torch.float32, post=post.to(device))
+            assert (xs.cpu() - want_x[a:b]).abs().max() < 1e-5
+            got.append([t.cpu() for t in hu])
+        for k in range(2):
+            assert (torch.cat([g[k] for g in got]) - want[k]).abs().max() < 3e-5, (cuts, k)
+
+
+# ------------------------------------------------ the tests would notice a fault
+
+FAULTS = {
+    "late window": ("in_window", lambda f: lambda i, j, s: f(i, j, s + 1)),
+    "early window": ("in_window", lambda f: lambda i, j, s: f(i, j, max(s - 1, 1))),
+    "sliding chunk": ("in_chunk", lambda f: lambda i, j, s: oracle.in_window(i, j, s)),
+    "shifted chunk": ("in_chunk", lambda f: lambda i, j, s: f(i + 1, j + 1, s)),
+    "no sink": ("softmax_plus_one", lambda f: oracle.softmax),
+    "sink everywhere": ("softmax", lambda f: oracle.softmax_plus_one),
+    "still values": ("rotate_values", lambda f: lambda v, r: v),
+    "no turn back": ("turn_back", lambda f: lambda o, r: o),
+    "turned on": ("turn_back", lambda f: lambda o, r: oracle.rotate_values(o, r)),
+    "halves": ("turn", lambda f: lambda x, fr, g, sign=1: torch.cat([f(
+        x[..., :2 * len(fr)].unflatten(-1, (2, -1)).transpose(-1, -2).flatten(-2), fr, g, sign),
+        x[..., 2 * len(fr):]], -1)),
+    "no growth": ("frequencies", lambda f: lambda *a: (f(*a)[0], 1.0)),
+    "unscaled angles": ("frequencies", lambda f: lambda d, b, s=None: (f(d, b)[0], f(d, b, s)[1])),
+    "late key": ("attend", lambda f: lambda q, k, v, *a: f(q, k.roll(1, 0), v, *a)),
+    "no past": ("with_past", lambda f: lambda h, w: h),
+    "bare convolution": ("with_past", lambda f: lambda h, w: oracle.causal_conv(h, w)),
+    "turned taps": ("causal_conv", lambda f: lambda u, w: f(u, w.flip(1))),
+    "cut convolution": ("causal_conv", lambda f: lambda u, w: torch.cat([f(u[:64], w), f(u[64:], w)])),
+    "raw latents": ("latents", lambda f: lambda u, t, p, m, e: (
+        u @ t[p + "dkv"].T[:, :m["kv_rank"]], f(u, t, p, m, e)[1])),
+    "plain relu": ("relu_squared", lambda f: lambda z: z.clamp(min=0)),
+    "groups by sum": ("group_score", lambda f: lambda s: sum(sorted(s)[-2:])),
+    "shares of the chosen": ("share", lambda f: lambda s, c: [s[e] / sum(s[x] for x in c) for e in c]),
+}
+
+
+@pytest.mark.parametrize("fault", list(FAULTS))
+def test_a_planted_fault_shows(cpu_rig, monkeypatch, fault):
+    """Each of these changes in the oracle moves its logits far beyond the
+    tolerance, so the comparisons above cannot pass with such a fault."""
+    toks = cpu_rig.tokens(90, 0)
+    good = cpu_rig.logits(toks)
+    name, change = FAULTS[fault]
+    monkeypatch.setattr(oracle, name, change(getattr(oracle, name)))
+    bad = oracle.forward(cpu_rig.cfg, cpu_rig.t, toks)[0]
+    assert ((bad - good).norm(dim=-1) / good.norm(dim=-1)).max() > 5e-3
+
+
+@pytest.mark.parametrize("change", [
+    lambda c: c["norm"].update(eps=3e-3),
+    lambda c: c.update(logit_scale=1.2),
+    lambda c: c["layers"][0]["mixer"].update(scale=0.3),
+    lambda c: c["layers"][0]["mixer"]["mask"].update(size=18),
+    lambda c: c["layers"][4]["mixer"]["rot"].update(base=60.0),
+    lambda c: [c["layers"][i]["mixer"]["rot"]["scaling"].update(factor=5.0) for i in (0, 2)],
+    lambda c: [c["layers"][i]["mixer"]["rot"]["scaling"].update(original=400) for i in (0, 2)],
+    lambda c: [c["layers"][i]["mixer"]["rot"]["scaling"].update(fast=0.5) for i in (0, 2)],
+    lambda c: [c["layers"][i]["mixer"]["rot"]["scaling"].update(slow=2.0) for i in (0, 2)],
+    lambda c: c["layers"][2]["mixer"]["mask"].update(size=30),
+    lambda c: c["layers"][1]["mixer"]["mask"].update(size=8),
+    lambda c: c["layers"][1]["mixer"].update(scale=0.2),
+    lambda c: c["layers"][1]["mixer"]["rot"].update(dims=8),
+    lambda c: c["layers"][1]["mixer"]["rot"].update(base=400.0),
+    lambda c: c["layers"][3]["mixer"].pop("mask"),
+    lambda c: c["layers"][0]["mlp"]["router"].update(top=3),
+    lambda c: c["layers"][0]["mlp"]["router"]["groups"].update(keep=3),
+    lambda c: c["layers"][0]["mlp"].pop("shared")])
+def test_every_constant_is_read(cpu_rig, tmp_path, change):
+    """With one constant changed the oracle's logits move, and the engine's with them."""
+    cfg = json.loads(json.dumps(cpu_rig.cfg))
+    change(cfg)
+    toks = cpu_rig.tokens(90, 0)
+    other = decoder_rig.Rig(tmp_path, cfg, cpu_rig.t, oracle, "cpu")
+    good, want = cpu_rig.logits(toks), other.logits(toks)
+    assert ((want - good).norm(dim=-1) / good.norm(dim=-1)).max() > 1e-3
+    other.check(other.run(other.replayer(), "a", toks, [60, 2, 1, 27]), want)
+
+
+def test_closed_forms_of_the_oracle():
+    """Small cases worked out by hand."""
+    x = torch.tensor([[3.0, 4.0]], dtype=D64)
+    assert torch.allclose(oracle.rms_norm(x, torch.ones(2), 0.0), x / math.sqrt(12.5))
+    u = torch.arange(1.0, 5.0, dtype=D64).view(4, 1)
+    assert oracle.causal_conv(u, torch.tensor([[10.0, 1.0]])).flatten().tolist() == [1, 12, 23, 34]
+    y = oracle.rotate(torch.tensor([[[1.0, 0.0, 5.0]]] * 2, dtype=D64), {"dims": 2, "base": 7.0})
+    assert torch.allclose(y[1, 0], torch.tensor([math.cos(1), math.sin(1), 5.0], dtype=D64))
+    p = oracle.softmax_plus_one(torch.tensor([[0.0, math.log(2.0)]], dtype=D64))
+    assert torch.allclose(p, torch.tensor([[0.25, 0.5]], dtype=D64))
+    i, j = torch.arange(6).unsqueeze(1), torch.arange(6).unsqueeze(0)
+    assert oracle.in_window(i, j, 2).sum(-1).tolist() == [1, 2, 2, 2, 2, 2]
+    assert oracle.in_chunk(i, j, 4).sum(-1).tolist() == [1, 2, 3, 4, 1, 2]
+    f, g = oracle.frequencies(4, 100.0, {"factor": 2.0, "original": 2 * math.pi * 100, "fast": 100.0,
+                                         "slow": 1.0})
+    assert f == pytest.approx([1.0, 0.1 / 2 * 0.5 + 0.1 * 0.5]) and g == pytest.approx(
+        1 + 0.1 * math.log(2))
+    r = {"top": 2, "groups": {"count": 2, "keep": 1}}
+    assert oracle.choose([0.3, 0.3, 0.31, 0.09], r) == [2, 3]
