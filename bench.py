@@ -26,9 +26,10 @@ Two modes:
 
 * ``--mode layers``: prefill and decode throughput of a few full-width layers
   of a layer-listed decoder (``--design``: Kikalix beside a Mixtral-style model,
-  Senotar beside a Llama-style one, Gakupel beside Kikalix) and as many of the other of equal width,
-  heads, experts and feed-forward (random weights), each through its engine's
-  own batch building, kernels and decode graphs, the two timed in turn.
+  Senotar beside a Llama-style one, Gakupel beside Kikalix, Fezuzen beside
+  Gakupel) and as many of the other of equal width, heads, experts and
+  feed-forward (random weights), each through its engine's own batch building,
+  kernels and decode graphs, the two timed in turn.
 
 Data: synthetic alert payloads / token streams, random-init weights
 (no network in this environment).
@@ -66,7 +67,8 @@ def parse_args():
                     help="layers per model in --mode layers")
     ap.add_argument("--size", default="all",
                     help="one of the --mode layers sizes, or all")
-    ap.add_argument("--design", choices=("kikalix", "senotar", "gakupel"), default="kikalix",
+    ap.add_argument("--design", choices=("kikalix", "senotar", "gakupel", "fezuzen"),
+                    default="kikalix",
                     help="design of --mode layers")
     ap.add_argument("--rag", type=int, default=int(os.environ.get("BENCH_RAG", "1")),
                     help="per-turn on-GPU RAG retrieval + input-rail check (1=on)")
@@ -431,6 +433,13 @@ GAKUPEL_SIZES = {
     "2048-64x1408": (2048, 16, 4, 64, 6, 1408, 2816, 5632),
     "1024-16x512": (1024, 8, 2, 16, 2, 512, 1024, 2816),
 }
+#: width, heads, kv heads, latent rank, queries' rank, unrotated and rotated width of a
+#: latent-attention head, experts, top, expert ff, shared ff
+FEZUZEN_SIZES = {
+    "4096-8x14336": (4096, 32, 8, 512, 1536, 128, 64, 8, 2, 14336, 3584),
+    "2048-64x1408": (2048, 16, 4, 512, 1024, 128, 64, 64, 6, 1408, 2816),
+    "1024-16x512": (1024, 8, 2, 256, 512, 64, 32, 16, 2, 512, 1024),
+}
 PREFILL_SEQS, PREFILL_LEN, DECODE_SEQS, DECODE_STEPS = 4, 2048, 64, 32
 
 
@@ -488,6 +497,26 @@ def gakupel_pair(size: str, n_layers: int):
     return gakupel, kikalix
 
 
+def fezuzen_pair(size: str, n_layers: int):
+    """(Fezuzen spec, Gakupel spec) of one size: windows and chunks of half a prompt,
+    every second latent layer borrowing, beside full attention; routed experts and a
+    shared one in every layer of both."""
+    from aurora_amd.models.config import fezuzen_spec, gakupel_spec
+    w, h, kv, rank, q_rank, dim, rot, experts, top, ff, shared = FEZUZEN_SIZES[size]
+    d = w // h
+    fezuzen = fezuzen_spec(
+        f"fezuzen-{size}", ("oasa" * n_layers)[:n_layers], width=w, vocab=32000, heads=h,
+        dim=dim, rot_dim=rot, vdim=dim, kv_rank=rank, q_rank=q_rank, window=1024, a_heads=h,
+        kv_heads=kv, a_dim=d, a_vdim=d, chunk=1024, experts=experts, top=top, expert_ff=ff,
+        shared_ff=shared, groups=4, keep=2, max_position=8192)
+    gakupel = gakupel_spec(
+        f"gakupel-{size}", "a" * n_layers, width=w, vocab=32000, heads=h,
+        kv_heads=kv, dim=d, l_dim=d, l_vdim=d, d_heads=h, d_kv_heads=h, d_dim=d, d_vdim=d,
+        m_heads=h, m_dim=d, m_vdim=d, ff=ff, experts=experts, top=top, expert_ff=ff,
+        shared_ff=shared, groups=4, keep=2, max_position=8192)
+    return fezuzen, gakupel
+
+
 def layer_bench_engine(spec, seed: int = 0):
     from aurora_amd.engine.engine import EngineConfig, LLMEngine
     from aurora_amd.models.registry import build_model
@@ -533,7 +562,8 @@ def layer_bench_once(eng, rng):
 def main_layers(args):
     table, pair = {"kikalix": (LAYER_SIZES, layer_pair),
                    "senotar": (SENOTAR_SIZES, senotar_pair),
-                   "gakupel": (GAKUPEL_SIZES, gakupel_pair)}[args.design]
+                   "gakupel": (GAKUPEL_SIZES, gakupel_pair),
+                   "fezuzen": (FEZUZEN_SIZES, fezuzen_pair)}[args.design]
     sizes = list(table) if args.size == "all" else [args.size]
     result = {}
     for size in sizes:

@@ -160,7 +160,7 @@ def weights(cfg, seed=0, decided=False):
 def make_rig(path, name, device, dtype="float32"):
     cfg = config(name)
     return decoder_rig.Rig(path, cfg, weights(cfg, decided=dtype == "bfloat16"), oracle, device,
-                           dtype, 0.06)
+                           dtype, 0.1)
 
 
 CASES = [pytest.param((n, d, t), id=f"{n}-{d}-{t}",
@@ -730,7 +730,7 @@ def test_convolved_attention_alone(device, dtype, H, G, d, e, size):
         kw = dict(rot=rot, base=500.0, scale=d ** -0.5, sink=option == 0, gate=gate,
                   turn_values=option == 0, **{size[0]: size[1]})
         want = _conv_want(x, H, G, d, e, conv, **kw)
-        tol = 2e-5 if dtype == torch.float32 else 0.03
+        tol = 2e-5 if dtype == torch.float32 else 0.05
         for cuts in ([T], [1] * 20 + [2, 17, 1, 64, 46], [2] * 75):
             got = _conv_attend(x, H, G, d, e, conv, cuts, device, dtype, **kw)
             err = (got - want).norm(dim=-1) / want.norm(dim=-1).mean()
@@ -790,36 +790,32 @@ def test_short_convolution_alone(device, taps):
 
 
 @pytest.mark.parametrize("device", DEVICES)
+@DTYPES
 @pytest.mark.parametrize("E,groups,keep,top", [(8, 4, 2, 3), (12, 2, 1, 6), (6, 6, 2, 2),
                                                (5, 1, 1, 5), (70, 10, 3, 6), (1, 1, 1, 1)])
-def test_softmax_routing_alone(device, E, groups, keep, top):
+def test_softmax_routing_alone(device, dtype, E, groups, keep, top):
     """Logits that are far apart; weights are shares of all experts, chosen or not, and
     nothing outside the best groups is chosen however large its score."""
-    T, W = 40, 64
+    only_float32_on_cpu(device, dtype)
+    T, W = 40, -(-E // 8) * 8 if dtype == torch.bfloat16 else E + 3
     r = {"top": top, "groups": {"count": groups, "keep": keep}}
     gen = torch.Generator().manual_seed(E)
-    z = torch.stack([torch.randperm(E, generator=gen) for _ in range(T)]) * (6.0 / E)
-    h = torch.randn(T, W, generator=gen)
-    router = torch.linalg.lstsq(h.double(), z.double()).solution.T if E < W - T else None
-    if router is None or (h.double() @ router.T - z).abs().max() > 1e-9:
-        # one coordinate per expert
-        W = E + 3
-        h = torch.cat([z, torch.zeros(T, 3)], 1)
-        router = torch.eye(E, W, dtype=D64)
+    z = torch.stack([torch.randperm(E, generator=gen) for _ in range(T)]) / 8.0  # exact
+    h = torch.cat([z, torch.randn(T, W - E, generator=gen)], 1).to(dtype)
+    router = torch.eye(E, W).to(dtype)
     if device == "cpu":
-        sel, share = torch_ref.moe_route_softmax(h, router.float(), top, groups, keep, 1.0)
+        sel, share = torch_ref.moe_route_softmax(h, router, top, groups, keep, 0.5)
     else:
         sel, share = sequence._hip("moe_route_grouped").moe_route_grouped(
-            h.to(device), router.float().to(device), None, top, groups, keep, 1.0)
+            h.to(device), router.to(device), None, top, groups, keep, 0.5)
     for t in range(T):
         s = oracle.softmax(z[t].double())
         want = oracle.choose(s.tolist(), r)
         assert sel[t].tolist() == want
-        assert (share[t].cpu() - s[want]).abs().max() < 1e-6
-    if keep < groups and E > groups:  # a group's best expert may beat its neighbours' sum
-        left_out = [t for t in range(T) if set(oracle.choose(z[t].tolist(), r)) !=
-                    set(z[t].topk(top).indices.tolist())]
-        assert left_out
+        assert (share[t].cpu() - 0.5 * s[want]).abs().max() < 1e-6
+    if keep < groups and groups < E:  # the groups matter
+        assert any(oracle.choose(z[t].tolist(), r) != z[t].topk(top).indices.tolist()
+                   for t in range(T))
 
 
 @pytest.mark.parametrize("device", DEVICES)
