@@ -129,6 +129,9 @@ class HybridForCausalLM(nn.Module):
             self.final_norm_bias = _param(spec.hidden_size, dtype=torch.float32) \
                 if spec.output_norms else None
             self.lm_head = _param(spec.vocab_size, spec.hidden_size, dtype=dtype)
+            # fp32 and not a scalar, so that the product is fp32 too
+            self.register_buffer("logit_scale", torch.tensor([spec.logit_scale]).float()
+                                 if spec.logit_scale != 1.0 else None, persistent=False)
             self.loop_step = _param(spec.loop[2], spec.hidden_size,
                                     dtype=torch.float32) if spec.loop else None
             if spec.embedding is not None:
@@ -179,8 +182,9 @@ class HybridForCausalLM(nn.Module):
         """Normed hidden states [T, H]; ``trail``, if a list, receives the
         residual stream after every layer run."""
         segments = meta.segments(input_ids.shape[0])
+        states = meta.states or []  # a model need not have any
         if self.spec.output_norms:
-            return self._forward_output_normed(input_ids, kv_caches, meta, segments, trail)
+            return self._forward_output_normed(input_ids, kv_caches, meta, segments, states, trail)
         x = self._embed(input_ids, meta, segments)
         norm = {"eps": self.spec.rms_eps, "offset": self.spec.norm_offset,
                 "dtype": self.dtype}
@@ -197,7 +201,7 @@ class HybridForCausalLM(nn.Module):
 
         for i, step, kv, st in self._runs:
             layer = self.layers[i]
-            state = meta.states[st]
+            state = states[st]
             if step is not None:
                 add["step"] = self.loop_step[step]
             h, u, state = read(layer.norm1, layer.conv, state)
@@ -218,7 +222,7 @@ class HybridForCausalLM(nn.Module):
                 trail.append(y)
         return ops.residual_rmsnorm(x, self.final_norm, **norm, **add)
 
-    def _forward_output_normed(self, input_ids, kv_caches, meta, segments, trail):
+    def _forward_output_normed(self, input_ids, kv_caches, meta, segments, states, trail):
         """Sublayers read the residual itself; one kernel per sublayer norms its
         result, adds it, and after a layer takes the average over the depth, after
         the last one the final norm as well."""
@@ -236,7 +240,7 @@ class HybridForCausalLM(nn.Module):
             last = {} if kept is None else {"depth": (kept, layer.depth)}
             if run == n - 1:
                 last["final"] = (self.final_norm, self.final_norm_bias)
-            y = layer.mixer(h, meta, segments, kv_caches[kv], meta.states[st])
+            y = layer.mixer(h, meta, segments, kv_caches[kv], states[st])
             h = ops.output_norm(src, x, layer.norm1, layer.norm1_bias, delta=y, **norm,
                                 **(last if layer.mlp is None else {}))
             if layer.mlp is not None:
@@ -249,8 +253,8 @@ class HybridForCausalLM(nn.Module):
 
     @torch.inference_mode()
     def compute_logits(self, hidden: torch.Tensor) -> torch.Tensor:
-        logits = ops.linear(hidden, self.lm_head).float()
-        return logits if self.spec.logit_scale == 1.0 else logits.mul_(self.spec.logit_scale)
+        logits = ops.linear(hidden, self.lm_head)
+        return logits.float() if self.logit_scale is None else logits * self.logit_scale
 
     @torch.inference_mode()
     def load_tensors(self, get) -> None:

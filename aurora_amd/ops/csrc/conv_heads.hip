@@ -34,7 +34,7 @@ struct ConvHeadArgs {
 };
 
 // VEC: 16-byte accesses of V elements, and d, dv, DK, DV, columns and strides are
-// multiples of V; else V is 2 and a head's last channel may stand alone. TAPS 0: any
+// multiples of V (TAPS > 0 only so); else V is 2 and a head's last channel may stand alone. TAPS 0: any
 // number, inputs read again for every tap.
 template <typename T, int V, int TAPS, bool VEC>
 __global__ __launch_bounds__(256) void conv_qkv_kernel(ConvHeadArgs a) {
@@ -77,7 +77,6 @@ __global__ __launch_bounds__(256) void conv_qkv_kernel(ConvHeadArgs a) {
       for (int v = 0; v < V; ++v) x[v] = p && c + v < n ? ldf(p + v) : 0.f;
     }
   };
-  auto weight = [&](int j, int v) { return c + v < n ? a.w[(long)j * a.C + ch + v] : 0.f; };
   // rotation and place of local row t
   auto finish = [&](int t, float (&y)[V]) {
     const int turning = is_v ? (a.vcs ? a.dv : 0) : a.rot;
@@ -120,7 +119,12 @@ __global__ __launch_bounds__(256) void conv_qkv_kernel(ConvHeadArgs a) {
 #pragma unroll
     for (int j = 0; j < TAPS; ++j)
 #pragma unroll
-      for (int v = 0; v < V; ++v) wt[j][v] = weight(j, v);
+      for (int v = 0; v < V; v += 4) {
+        floatx4 y = {0.f, 0.f, 0.f, 0.f};
+        if (c < n) y = ld4(a.w + (long)j * a.C + ch + v);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) wt[j][v + i] = y[i];
+      }
 #pragma unroll
     for (int j = 1; j < TAPS; ++j) input(off - TAPS + j, win[j]);
     for (int t = 0; t < rows; ++t) {
@@ -146,7 +150,8 @@ __global__ __launch_bounds__(256) void conv_qkv_kernel(ConvHeadArgs a) {
       for (int j = 0; j < taps; ++j) {
         input(off + t - keep + j, x);
 #pragma unroll
-        for (int v = 0; v < V; ++v) y[v] += weight(j, v) * x[v];
+        for (int v = 0; v < V; ++v)
+          if (c + v < n) y[v] += a.w[(long)j * a.C + ch + v] * x[v];
       }
       finish(off + t, y);
     }

@@ -720,19 +720,22 @@ void rotate_heads(torch::Tensor x, torch::Tensor pos, torch::Tensor cos_sin,
 // take 16 outputs each (KS 1) or split the contraction (KS 4); TT 16-token
 // tiles per workgroup. K and N are multiples of 32; STEPS: 32-wide steps of a
 // wave if known, all of whose loads are then in flight at once. With ``turn`` the last
-// block of a row of blocks turns the rotated dimensions of the same tokens and head.
+// ``turners`` blocks of a row of blocks turn the rotated dimensions of the same tokens
+// and head.
 template <int TT, int KS, int STEPS>
 __global__ __launch_bounds__(256) void head_linear_kernel(
     const bf16_t* __restrict__ x, long xt, long xh, const bf16_t* __restrict__ w,
     const bf16_t* __restrict__ gate, long gt, bf16_t* __restrict__ out, long ot, long oh,
-    int T_, int N, int K, TurnHeads<bf16_t> turn) {
+    int T_, int N, int K, TurnHeads<bf16_t> turn, int turners) {
   __shared__ __attribute__((aligned(16))) float red[KS > 1 ? 4 : 1][TT][WAVE][4];
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
   const int col = lane & 15, g = lane >> 4;
   const int h = blockIdx.y, t0 = blockIdx.z * 16 * TT;
-  if (turn.x && blockIdx.x == gridDim.x - 1) {
+  const int part = (int)blockIdx.x - (int)(gridDim.x - turners);
+  if (part >= 0) {
     const int pairs = turn.W / 2, n = min(16 * TT, T_ - t0) * pairs;
-    for (int i = threadIdx.x; i < n; i += 256) turn_heads(turn, t0 + i / pairs, h, i % pairs);
+    for (int i = part * 256 + threadIdx.x; i < n; i += turners * 256)
+      turn_heads(turn, t0 + i / pairs, h, i % pairs);
     return;
   }
   const int n0 = KS > 1 ? blockIdx.x * 16 : (blockIdx.x * 4 + wave) * 16;
@@ -817,13 +820,14 @@ void head_linear(torch::Tensor x, torch::Tensor w, c10::optional<torch::Tensor> 
   }
   if (T_ == 0) return;
   auto launch = [&](auto kern, int tt, int ks) {
-    const dim3 grid((ks > 1 ? N / 16 : (N + 63) / 64) + (turn.x ? 1 : 0), H,
+    const int turners = turn.x ? (std::min(16 * tt, T_) * (turn.W / 2) + 255) / 256 : 0;
+    const dim3 grid((ks > 1 ? N / 16 : (N + 63) / 64) + turners, H,
                     (T_ + 16 * tt - 1) / (16 * tt));
     hipLaunchKernelGGL(kern, grid, dim3(256), 0, CUR_STREAM, (const bf16_t*)x.data_ptr(),
                        x.stride(0), x.stride(1), (const bf16_t*)w.data_ptr(),
                        gate ? (const bf16_t*)gate->data_ptr() : nullptr,
                        gate ? gate->stride(0) : 0, (bf16_t*)out.data_ptr(), out.stride(0),
-                       out.stride(1), T_, N, K, turn);
+                       out.stride(1), T_, N, K, turn, turners);
   };
   // a long contraction for few tokens: split it over the waves
   const bool split = K >= 256 && T_ <= 64;

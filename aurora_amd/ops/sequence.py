@@ -224,19 +224,24 @@ class Segment:
             return self.cu
         return torch.arange(n + 1, dtype=torch.int32, device=self.context_lens.device)
 
-    def block_map(self, rows_per_block: int) -> Tuple[torch.Tensor, torch.Tensor]:
+    def block_map(self, rows_per_block: int,
+                  chunk: int = 0) -> Tuple[torch.Tensor, torch.Tensor]:
         """(sequence, first row within it) of every block of rows; built once
-        per step and shared by all layers."""
-        hit = self._maps.get(rows_per_block)
+        per step and shared by all layers. With ``chunk`` the blocks are in the order
+        of how many keys of their chunk they see."""
+        hit = self._maps.get((rows_per_block, chunk))
         if hit is None:
-            seq, off = [], []
-            for s in range(len(self.cu_host) - 1):
-                for o in range(0, self.cu_host[s + 1] - self.cu_host[s], rows_per_block):
-                    seq.append(s)
-                    off.append(o)
-            t = torch.tensor([seq, off], dtype=torch.int32).to(self.context_lens.device)
+            blocks = []
+            for s, (a, b) in enumerate(zip(self.cu_host, self.cu_host[1:])):
+                blocks += [(s, o) for o in range(0, b - a, rows_per_block)]
+            if chunk:
+                first = [c - (b - a) for a, b, c in
+                         zip(self.cu_host, self.cu_host[1:], self.ctx_host)]
+                blocks.sort(key=lambda x: (first[x[0]] + x[1]) % chunk)
+            t = torch.tensor(blocks, dtype=torch.int32).view(-1, 2).t().contiguous().to(
+                self.context_lens.device)
             hit = (t[0], t[1])
-            self._maps[rows_per_block] = hit
+            self._maps[rows_per_block, chunk] = hit
         return hit
 
     def chunk_map(self) -> Tuple[torch.Tensor, torch.Tensor, torch.Tensor]:
@@ -571,7 +576,7 @@ def biased_attention(q, k_cache, v_cache, seg: Segment, scale, window, slopes,
                                   seg.context_lens, *extra)
     elif matrix:
         rows = m.biased_prefill_rows(q.shape[1] // k_cache.shape[1])
-        bseq, boff = seg.block_map(rows)
+        bseq, boff = seg.block_map(rows, chunk)
         m.biased_attention_prefill(qs, k_cache, v_cache, seg.block_tables, seg.cu,
                                    seg.context_lens, bseq, boff, *extra)
     else:

@@ -498,16 +498,16 @@ def gakupel_pair(size: str, n_layers: int):
 
 
 def fezuzen_pair(size: str, n_layers: int):
-    """(Fezuzen spec, Gakupel spec) of one size: windows and chunks of half a prompt,
-    every second latent layer borrowing, beside full attention; routed experts and a
-    shared one in every layer of both."""
+    """(Fezuzen spec, Gakupel spec) of one size: windows of half a prompt and chunks of
+    three quarters, every second latent layer borrowing, beside full attention; routed
+    experts and a shared one in every layer of both."""
     from aurora_amd.models.config import fezuzen_spec, gakupel_spec
     w, h, kv, rank, q_rank, dim, rot, experts, top, ff, shared = FEZUZEN_SIZES[size]
     d = w // h
     fezuzen = fezuzen_spec(
         f"fezuzen-{size}", ("oasa" * n_layers)[:n_layers], width=w, vocab=32000, heads=h,
         dim=dim, rot_dim=rot, vdim=dim, kv_rank=rank, q_rank=q_rank, window=1024, a_heads=h,
-        kv_heads=kv, a_dim=d, a_vdim=d, chunk=1024, experts=experts, top=top, expert_ff=ff,
+        kv_heads=kv, a_dim=d, a_vdim=d, chunk=1536, experts=experts, top=top, expert_ff=ff,
         shared_ff=shared, groups=4, keep=2, max_position=8192)
     gakupel = gakupel_spec(
         f"gakupel-{size}", "a" * n_layers, width=w, vocab=32000, heads=h,

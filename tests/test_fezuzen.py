@@ -41,10 +41,13 @@ def latent(heads, dim, rot, vdim, rank, q_rank, window, base=1e4, scale=None, ya
     return "latent_attention", m if kv_from is None else {**m, "kv_from": kv_from}
 
 
-def attention(heads, kv, dim, vdim, rot, conv, chunk, base=1e4, scale=None):
-    return "attention", {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv,
-                         "scale": dim ** -0.5 if scale is None else scale,
-                         "mask": {"size": chunk}, "rot": {"base": base, "dims": rot}}
+def attention(heads, kv, dim, vdim, rot, conv, chunk, base=1e4, scale=None, yarn=None):
+    m = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": vdim, "conv": conv,
+         "scale": dim ** -0.5 if scale is None else scale, "mask": {"size": chunk},
+         "rot": {"base": base, "dims": rot}}
+    if yarn is not None:  # of the keys alone
+        m["rot"]["scaling"] = dict(zip(("factor", "original", "fast", "slow"), yarn))
+    return "attention", m
 
 
 def moe(experts, top, groups, keep, ff, shared):
@@ -69,7 +72,8 @@ def config(name):
         layers = [(latent(4, 64, 32, 64, 64, 96, 40, yarn=y), moe(8, 2, 4, 2, 64, 128)),
                   (attention(4, 2, 64, 64, 64, 4, 24), moe(8, 3, 2, 1, 64, 64)),
                   (latent(2, 128, 32, 128, 64, 64, 56, yarn=y, kv_from=0), moe(8, 2, 4, 2, 64, 128)),
-                  (attention(6, 3, 128, 64, 32, 3, 37), moe(4, 4, 4, 4, 128, 64)),
+                  (attention(6, 3, 128, 64, 32, 3, 37, yarn=(3.0, 100, 8.0, 1.0)),
+                   moe(4, 4, 4, 4, 128, 64)),
                   (latent(3, 32, 64, 128, 128, 32, 16), moe(8, 2, 4, 3, 64, 64))]
         vocab, width, taps, eps, out = 333, 128, 4, 1e-5, 0.7
     elif name == "odd":
