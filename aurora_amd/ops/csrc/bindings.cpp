@@ -44,6 +44,7 @@ torch::Tensor xielu(torch::Tensor z, torch::Tensor act);
 void latent_front(torch::Tensor proj, long c0, long rank, OptT weight, double eps, long k0,
                   long key_at, OptT cos_sin, OptT pos, torch::Tensor slots,
                   torch::Tensor cache, long q0, OptT q_weight, OptT cq);
+torch::Tensor gather_latents(torch::Tensor cache, torch::Tensor rows);
 void rotate_heads(torch::Tensor x, torch::Tensor pos, torch::Tensor cos_sin,
                   torch::Tensor out);
 void head_linear(torch::Tensor x, torch::Tensor w, OptT gate, torch::Tensor out, OptT turn_x,
@@ -180,6 +181,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("xielu", &xielu, "xIELU activation");
   m.def("latent_front", &latent_front,
         "latent norm + rotated key part + paged scatter, norm of the queries' latent");
+  m.def("gather_latents", &gather_latents, "cached latent rows, packed");
   m.def("rotate_heads", &rotate_heads, "rotary positions of neighbouring pairs");
   m.def("head_linear", &head_linear,
         "per-head product with an optional gate, or beside rotated dimensions");

@@ -648,6 +648,31 @@ void latent_front(torch::Tensor proj, long c0, long rank, c10::optional<torch::T
   HIP_CHECK_KERNEL();
 }
 
+// cached rows, packed: 16 bytes per thread
+__global__ __launch_bounds__(256) void gather_latents_kernel(
+    const shortx8* __restrict__ cache, const int* __restrict__ rows, shortx8* __restrict__ out,
+    long total, int units) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int n = (int)(i / units);
+  out[i] = cache[(long)rows[n] * units + i % units];
+}
+
+torch::Tensor gather_latents(torch::Tensor cache, torch::Tensor rows) {
+  const long N = rows.numel(), C = cache.size(3);
+  TORCH_CHECK(cache.is_cuda() && cache.is_contiguous() && cache.size(1) == 1 &&
+              cache.dtype() == torch::kBFloat16 && C % 8 == 0, "latent cache");
+  TORCH_CHECK(rows.dtype() == torch::kInt32 && rows.is_contiguous());
+  auto out = torch::empty({N, C}, cache.options());
+  const long total = N * (C / 8);
+  if (total == 0) return out;
+  hipLaunchKernelGGL(gather_latents_kernel, dim3((total + 255) / 256), dim3(256), 0, CUR_STREAM,
+                     (const shortx8*)cache.data_ptr(), rows.data_ptr<int>(),
+                     (shortx8*)out.data_ptr(), total, (int)(C / 8));
+  HIP_CHECK_KERNEL();
+  return out;
+}
+
 // ------------------------------------------------------------- rotated dimensions
 
 // neighbouring pairs of x's first ``rot`` dimensions turn into out, zeros follow
@@ -660,31 +685,51 @@ struct TurnHeads {
   const float* cs;  // [positions, rot]
   const int* pos;
   int rot, W;       // W: dimensions of out, even
+  int unit;         // dimensions per thread: 8 in 16-byte accesses, or 2
+  __host__ __device__ int units() const { return W / unit; }
 };
 
 template <typename T>
-DEVINL void turn_heads(const TurnHeads<T>& a, int t, int h, int pair) {
-  const int d = 2 * pair;
+DEVINL void turn_heads(const TurnHeads<T>& a, int t, int h, int i) {
+  const int d = i * a.unit;
+  const T* p = a.x + t * a.xt + h * a.xh + d;
+  T* to = a.out + t * a.ot + h * a.oh + d;
+  const float* cs = a.cs + (long)a.pos[t] * a.rot + d / 2;
+  const bool turns = d < a.rot;
+  if (a.unit == 8) {
+    floatx4 y[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    if (turns) {
+      const floatx4 c = ld4(cs), s = ld4(cs + a.rot / 2);
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        const floatx4 x = ld4(p + 4 * k);
+        float u0 = x[0], v0 = x[1], u1 = x[2], v1 = x[3];
+        turn_pair(u0, v0, c[2 * k], s[2 * k]);
+        turn_pair(u1, v1, c[2 * k + 1], s[2 * k + 1]);
+        y[k] = floatx4{u0, v0, u1, v1};
+      }
+    }
+    st4(to, y[0]);
+    st4(to + 4, y[1]);
+    return;
+  }
   float u = 0.f, v = 0.f;
-  if (d < a.rot) {
-    const T* p = a.x + t * a.xt + h * a.xh + d;
-    const float* cs = a.cs + (long)a.pos[t] * a.rot + pair;
+  if (turns) {
     u = ldf(p);
     v = ldf(p + 1);
     turn_pair(u, v, cs[0], cs[a.rot / 2]);
   }
-  T* p = a.out + t * a.ot + h * a.oh + d;
-  stf(p, u);
-  stf(p + 1, v);
+  stf(to, u);
+  stf(to + 1, v);
 }
 
 template <typename T>
 __global__ __launch_bounds__(256) void rotate_heads_kernel(TurnHeads<T> a, long total, int H) {
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
   if (i >= total) return;
-  const int pairs = a.W / 2;
-  const long th = i / pairs;
-  turn_heads(a, (int)(th / H), (int)(th % H), (int)(i % pairs));
+  const int units = a.units();
+  const long th = i / units;
+  turn_heads(a, (int)(th / H), (int)(th % H), (int)(i % units));
 }
 
 template <typename T>
@@ -697,16 +742,20 @@ static TurnHeads<T> turn_args(const torch::Tensor& x, const torch::Tensor& pos,
               cos_sin.dim() == 2 && cos_sin.size(1) % 2 == 0 && cos_sin.size(1) <= x.size(2) &&
               cos_sin.size(1) <= out.size(2) && out.size(2) % 2 == 0, "rotation");
   TORCH_CHECK(pos.numel() == x.size(0) && pos.dtype() == torch::kInt32 && pos.is_contiguous());
-  return {(const T*)x.data_ptr(), x.stride(0), x.stride(1), (T*)out.data_ptr(), out.stride(0),
-          out.stride(1), cos_sin.data_ptr<float>(), pos.data_ptr<int>(), (int)cos_sin.size(1),
-          (int)out.size(2)};
+  TurnHeads<T> a = {(const T*)x.data_ptr(), x.stride(0), x.stride(1), (T*)out.data_ptr(),
+                    out.stride(0), out.stride(1), cos_sin.data_ptr<float>(),
+                    pos.data_ptr<int>(), (int)cos_sin.size(1), (int)out.size(2), 2};
+  const long strides = a.xt | a.xh | a.ot | a.oh | a.rot | a.W;
+  const uintptr_t at = reinterpret_cast<uintptr_t>(a.x) | reinterpret_cast<uintptr_t>(a.out);
+  if ((strides & 7) == 0 && (at & 15) == 0) a.unit = 8;
+  return a;
 }
 
 void rotate_heads(torch::Tensor x, torch::Tensor pos, torch::Tensor cos_sin,
                   torch::Tensor out) {
   DISPATCH_ELEM(x.dtype() == torch::kBFloat16, {
     const TurnHeads<T> a = turn_args<T>(x, pos, cos_sin, out);
-    const long total = x.size(0) * x.size(1) * (a.W / 2);
+    const long total = x.size(0) * x.size(1) * a.units();
     if (total == 0) return;
     hipLaunchKernelGGL((rotate_heads_kernel<T>), dim3((total + 255) / 256), dim3(256), 0,
                        CUR_STREAM, a, total, (int)x.size(1));
@@ -733,9 +782,9 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   const int h = blockIdx.y, t0 = blockIdx.z * 16 * TT;
   const int part = (int)blockIdx.x - (int)(gridDim.x - turners);
   if (part >= 0) {
-    const int pairs = turn.W / 2, n = min(16 * TT, T_ - t0) * pairs;
+    const int units = turn.units(), n = min(16 * TT, T_ - t0) * units;
     for (int i = part * 256 + threadIdx.x; i < n; i += turners * 256)
-      turn_heads(turn, t0 + i / pairs, h, i % pairs);
+      turn_heads(turn, t0 + i / units, h, i % units);
     return;
   }
   const int n0 = KS > 1 ? blockIdx.x * 16 : (blockIdx.x * 4 + wave) * 16;
@@ -820,7 +869,7 @@ void head_linear(torch::Tensor x, torch::Tensor w, c10::optional<torch::Tensor> 
   }
   if (T_ == 0) return;
   auto launch = [&](auto kern, int tt, int ks) {
-    const int turners = turn.x ? (std::min(16 * tt, T_) * (turn.W / 2) + 255) / 256 : 0;
+    const int turners = turn.x ? (std::min(16 * tt, T_) * turn.units() + 255) / 256 : 0;
     const dim3 grid((ks > 1 ? N / 16 : (N + 63) / 64) + turners, H,
                     (T_ + 16 * tt - 1) / (16 * tt));
     hipLaunchKernelGGL(kern, grid, dim3(256), 0, CUR_STREAM, (const bf16_t*)x.data_ptr(),

@@ -295,9 +295,9 @@ class Segment:
                 n += c - lo
                 t = torch.arange(lo, c, device=dev)
                 place.append(self.block_tables[s].long()[t // P] * P + t % P)
-            hit = (torch.cat(place), table.to(dev))
+            hit = (torch.cat(place).to(torch.int32), table.to(dev))
             self._maps["context", window] = hit
-        return cache.view(-1, cache.shape[3]).index_select(0, hit[0]), hit[1]
+        return _hip("gather_latents").gather_latents(cache, hit[0]), hit[1]
 
 
 def _hip(op: str):
