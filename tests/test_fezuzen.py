@@ -70,7 +70,7 @@ def config(name):
     if name == "plain":
         y = (4.0, 64, 8.0, 1.0)
         layers = [(latent(4, 64, 32, 64, 64, 96, 40, yarn=y), moe(8, 2, 4, 2, 64, 128)),
-                  (attention(4, 2, 64, 64, 64, 4, 24), moe(8, 3, 2, 1, 64, 64)),
+                  (attention(8, 2, 64, 64, 64, 4, 24), moe(8, 3, 2, 1, 64, 64)),
                   (latent(2, 128, 32, 128, 64, 64, 56, yarn=y, kv_from=0), moe(8, 2, 4, 2, 64, 128)),
                   (attention(6, 3, 128, 64, 32, 3, 37, yarn=(3.0, 100, 8.0, 1.0)),
                    moe(4, 4, 4, 4, 128, 64)),
